@@ -4,5 +4,7 @@ from .dokanex import DokanexConfig
 from .llama import LlamaConfig, RopeScaling
 from .muretar import MuretarConfig
 from .rorevik import RorevikConfig
+from .semezen import SemezenConfig
 
-__all__ = ["ConfigReader", "architecture_name", "read_config_json", "LlamaConfig", "RopeScaling", "DafidraConfig", "RorevikConfig", "DokanexConfig", "MuretarConfig"]
+__all__ = ["ConfigReader", "architecture_name", "read_config_json", "LlamaConfig", "RopeScaling", "DafidraConfig", "RorevikConfig", "DokanexConfig", "MuretarConfig",
+           "SemezenConfig"]

@@ -230,11 +230,12 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 2
       float inv = 1.0f / st.l[0];
       if (OPT) {
         if (opt.sinks) inv = sink_inverse(st.l[0], st.m[0] * (scale * PI_LOG2E), opt.sinks[head]);
-        if (opt.gate) inv *= opt.gate[row * nh + head];
+        if (opt.gate && !opt.gate_stride) inv *= opt.gate[row * nh + head];
         inv *= opt.out_mult;
       }
 #pragma unroll
       for (int db = 0; db < HD / 16; ++db) {
+        if (OPT && opt.gate_stride) st.o[db][0] *= feature_gates(opt, row, head * HD + db * 16 + lg * 4);
         uint2 w;
         w.x = pack_bf16x2(st.o[db][0][0] * inv, st.o[db][0][1] * inv);
         w.y = pack_bf16x2(st.o[db][0][2] * inv, st.o[db][0][3] * inv);
@@ -261,10 +262,10 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 2
 // Merge the key ranges of one (request, head) by one wave: lane d owns features d, d + 64, ..
 // Ranges are added in range order; an empty range (m = -inf) counts nothing.
 // sink2: the head's sink in base-2 units, joining the sum of weights once (-inf: none); gate: a
-// factor for the finished output.
+// factor for the finished output; features: gates per feature, still to go through a sigmoid (null: none).
 template <int HD>
 __device__ inline void combine_ranges(bf16_t* __restrict__ o, const float* base, int splits, int lane, float sink2 = -INFINITY,
-                                      float gate = 1.0f) {
+                                      float gate = 1.0f, const float* features = nullptr) {
   const int rec = HD + 4;
   constexpr int NF = (HD + 63) / 64;     // features per lane
   // lane s holds range s (splits <= 64): maxima, weights and the total in parallel
@@ -296,7 +297,10 @@ __device__ inline void combine_ranges(bf16_t* __restrict__ o, const float* base,
   }
 #pragma unroll
   for (int i = 0; i < NF; ++i)
-    if (lane + i * 64 < HD) o[lane + i * 64] = from_float<bf16_t>(range_finish(acc[i], l_tot) * gate);
+    if (lane + i * 64 < HD) {
+      const float f = features ? gate / (1.0f + __expf(-features[lane + i * 64])) : gate;
+      o[lane + i * 64] = from_float<bf16_t>(range_finish(acc[i], l_tot) * f);
+    }
 }
 
 // One wave per (request, head).
@@ -312,7 +316,8 @@ __global__ __launch_bounds__(64) void attention_combine_kernel(bf16_t* __restric
   const long out_row = rows ? rows[blockIdx.y] : q_start[r];
   combine_ranges<HD>(out + out_row * out_stride + (long)head * HD, part + ((long)blockIdx.y * nh + head) * splits * (HD + 4),
                      splits, threadIdx.x, opt.sinks ? opt.sinks[head] * PI_LOG2E : -INFINITY,
-                     (opt.gate ? opt.gate[out_row * nh + head] : 1.0f) * opt.out_mult);
+                     (opt.gate && !opt.gate_stride ? opt.gate[out_row * nh + head] : 1.0f) * opt.out_mult,
+                     opt.gate_stride ? opt.gate + out_row * opt.gate_stride + (long)head * HD : nullptr);
 }
 
 // One wave per (row of `part`, head): rows are a launch's requests (results to the requests'
@@ -424,12 +429,13 @@ extern "C" int pi_attention_decode(void* out, long out_stride, const void* q, lo
                                    const void* v_cache, const int* block_table, int table_width, const int* q_start,
                                    const int* kv_len, const int* req_ids, int R, int nh, int nkv, int hd, int page_size,
                                    float scale, int window, long num_pages, int splits, void* part, long part_elems,
-                                   const float* slopes, const float* sinks, const float* gate, float softcap, float out_mult,
-                                   int chunk, hipStream_t stream) {
+                                   const float* slopes, const float* sinks, const float* gate, long gate_stride, float softcap,
+                                   float out_mult, int chunk, hipStream_t stream) {
   PI_REQUIRE(chunk >= 0, "attention_decode: chunk must be >= 0, got %d", chunk);
+  PI_REQUIRE(gate_stride == 0 || (gate && gate_stride % 4 == 0 && (uintptr_t)gate % 16 == 0), "attention_decode: gates per feature must lie in 16-byte groups");
   return launch_decode(false, DecodeSource{}, out, out_stride, q, q_stride, k_cache, v_cache, block_table, table_width, q_start,
                        kv_len, req_ids, R, nh, nkv, hd, page_size, scale, window, num_pages, splits, part, part_elems, true, stream,
-                       AttnOptions{slopes, sinks, gate, softcap, out_mult, chunk});
+                       AttnOptions{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk});
 }
 
 // The same for a step of single tokens only (T == R tokens, request r at row q_start[r]),
@@ -478,7 +484,8 @@ extern "C" int pi_attention_decode_fused(void* out, long out_stride, const void*
 // Merge partial results that the tile kernel wrote for `Z` tokens whose tiles' keys were cut in
 // `cuts` shares: part [Z, nh, cuts, hd + 4]; token z's result goes to row rows[z] of out.
 extern "C" int pi_attention_combine_rows(void* out, long out_stride, const int* rows, int Z, const void* part, int nh, int hd,
-                                         int cuts, const float* sinks, const float* gate, float out_mult, hipStream_t stream) {
+                                         int cuts, const float* sinks, const float* gate, long gate_stride, float out_mult,
+                                         hipStream_t stream) {
   PI_REQUIRE(Z > 0 && Z <= 65535 && nh > 0 && cuts >= 2 && cuts <= 64 && rows && part, "attention_combine_rows: bad arguments (%d tokens, %d heads, %d cuts)", Z, nh, cuts);
-  return launch_combine(out, out_stride, nullptr, nullptr, rows, Z, part, nh, hd, cuts, stream, AttnOptions{nullptr, sinks, gate, 0.f, out_mult});
+  return launch_combine(out, out_stride, nullptr, nullptr, rows, Z, part, nh, hd, cuts, stream, AttnOptions{nullptr, sinks, gate, 0.f, out_mult, gate_stride});
 }

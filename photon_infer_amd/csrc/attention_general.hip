@@ -16,7 +16,8 @@
 //   * a distance bias: slope[head] * (p - t) is taken off the scaled score of key t;
 //   * a sink per head: exp(sink[head]) joins the denominator once; it has no key and no value,
 //     is not scaled and gets no bias;
-//   * an output gate: head h's output at token t is multiplied by gate[t, h] (float32);
+//   * an output gate: head h's output at token t is multiplied by gate[t, h] (float32); or, with gate_stride > 0, feature d
+//     of it by sigmoid(gate[t * gate_stride + h * vd + d]);
 //   * a cap on the scores: the scaled score s becomes softcap * tanh(s / softcap) (0: none), before any bias;
 //   * a factor on every output (out_mult; 1: none), applied in float32 before the one rounding.
 //
@@ -37,7 +38,7 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
     const T* __restrict__ v_cache, const int* __restrict__ block_table, int table_width,
     const int* __restrict__ req_of_token, const int* __restrict__ positions, int nh, int nkv, int hd, int page_size,
     float scale, int window, long num_pages, float* __restrict__ part, int vd, const float* __restrict__ slopes,
-    const float* __restrict__ sinks, const float* __restrict__ gate, float softcap, float out_mult, int chunk) {
+    const float* __restrict__ sinks, const float* __restrict__ gate, long gate_stride, float softcap, float out_mult, int chunk) {
   __shared__ float qs[NACC * PI_WAVE];
   __shared__ float ps[PI_WAVE];
   __shared__ long voff[PI_WAVE];   // values are stored [page, kv_head, head_dim, slot]
@@ -163,11 +164,14 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
     for (int i = 0; i < NACC; ++i) acc[i] *= corr;
   }
   T* o = out + t * out_stride + (long)h * vd;
-  const float inv = out_mult * (gate ? gate[t * nh + h] : 1.0f) / l;
+  const float inv = out_mult * (gate && !gate_stride ? gate[t * nh + h] : 1.0f) / l;
 #pragma unroll
   for (int i = 0; i < NACC; ++i) {
     const int d = lane + i * PI_WAVE;
-    if (d < vd) o[d] = from_float<T>(acc[i] * inv);
+    if (d < vd) {
+      const float f = gate_stride ? 1.0f / (1.0f + expf(-gate[t * gate_stride + (long)h * vd + d])) : 1.0f;
+      o[d] = from_float<T>(acc[i] * inv * f);
+    }
   }
 }
 
@@ -176,7 +180,7 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
 template <typename T, int NACC>
 __global__ __launch_bounds__(PI_WAVE) void merge_key_ranges_kernel(T* __restrict__ out, long out_stride, const float* __restrict__ part,
                                                                    int nh, int hd, int splits, const float* __restrict__ sinks,
-                                                                   const float* __restrict__ gate, float out_mult) {
+                                                                   const float* __restrict__ gate, long gate_stride, float out_mult) {
   const long t = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x;
   const float* base = part + ((long)t * nh + h) * splits * (hd + 2);
@@ -197,11 +201,14 @@ __global__ __launch_bounds__(PI_WAVE) void merge_key_ranges_kernel(T* __restrict
     }
   }
   T* o = out + t * out_stride + (long)h * hd;
-  const float inv = out_mult * (gate ? gate[t * nh + h] : 1.0f) / l;
+  const float inv = out_mult * (gate && !gate_stride ? gate[t * nh + h] : 1.0f) / l;
 #pragma unroll
   for (int i = 0; i < NACC; ++i) {
     const int d = lane + i * PI_WAVE;
-    if (d < hd) o[d] = from_float<T>(acc[i] * inv);
+    if (d < hd) {
+      const float f = gate_stride ? 1.0f / (1.0f + expf(-gate[t * gate_stride + (long)h * hd + d])) : 1.0f;
+      o[d] = from_float<T>(acc[i] * inv * f);
+    }
   }
 }
 
@@ -221,7 +228,7 @@ extern "C" int pi_paged_attention_general(void* out, long out_stride, const void
                                           const void* v_cache, int dtype, const int* block_table, int table_width,
                                           const int* req_of_token, const int* positions, int T, int nh, int nkv, int hd,
                                           int page_size, float scale, int window, long num_pages, int splits, void* part,
-                                          long part_elems, int vd, const float* slopes, const float* sinks, const float* gate,
+                                          long part_elems, int vd, const float* slopes, const float* sinks, const float* gate, long gate_stride,
                                           float softcap, float out_mult, int chunk, hipStream_t stream) {
   PI_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention: heads %d must be a positive multiple of kv heads %d", nh, nkv);
   PI_REQUIRE(hd > 0 && hd <= PI_MAX_HEAD_DIM, "attention: head_dim %d must be at most %d", hd, PI_MAX_HEAD_DIM);
@@ -241,36 +248,36 @@ extern "C" int pi_paged_attention_general(void* out, long out_stride, const void
     if (dtype == PI_F32)
       hipLaunchKernelGGL((paged_attention_general_kernel<float, PI_ATTN_WIDE>), grid, block, 0, stream, (float*)out, out_stride, (const float*)q,
                          q_stride, (const float*)k_cache, (const float*)v_cache, block_table, table_width, req_of_token,
-                         positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, softcap, out_mult, chunk);
+                         positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
     else if (dtype == PI_BF16)
       hipLaunchKernelGGL((paged_attention_general_kernel<bf16_t, PI_ATTN_WIDE>), grid, block, 0, stream, (bf16_t*)out, out_stride,
                          (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, table_width,
-                         req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, softcap, out_mult, chunk);
+                         req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
     else
       return pi_fail("attention: unsupported dtype %d", dtype);
     if (pi_check_launch("paged_attention_general")) return -1;
     if (splits == 1) return 0;
     if (dtype == PI_F32)
-      hipLaunchKernelGGL((merge_key_ranges_kernel<float, PI_ATTN_WIDE>), dim3(T, nh), block, 0, stream, (float*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, out_mult);
+      hipLaunchKernelGGL((merge_key_ranges_kernel<float, PI_ATTN_WIDE>), dim3(T, nh), block, 0, stream, (float*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, gate_stride, out_mult);
     else
-      hipLaunchKernelGGL((merge_key_ranges_kernel<bf16_t, PI_ATTN_WIDE>), dim3(T, nh), block, 0, stream, (bf16_t*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, out_mult);
+      hipLaunchKernelGGL((merge_key_ranges_kernel<bf16_t, PI_ATTN_WIDE>), dim3(T, nh), block, 0, stream, (bf16_t*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, gate_stride, out_mult);
     return pi_check_launch("merge_key_ranges");
   }
   if (dtype == PI_F32)
     hipLaunchKernelGGL((paged_attention_general_kernel<float, 4>), grid, block, 0, stream, (float*)out, out_stride, (const float*)q,
                        q_stride, (const float*)k_cache, (const float*)v_cache, block_table, table_width, req_of_token,
-                       positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, softcap, out_mult, chunk);
+                       positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
   else if (dtype == PI_BF16)
     hipLaunchKernelGGL((paged_attention_general_kernel<bf16_t, 4>), grid, block, 0, stream, (bf16_t*)out, out_stride,
                        (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, table_width,
-                       req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, softcap, out_mult, chunk);
+                       req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
   else
     return pi_fail("attention: unsupported dtype %d", dtype);
   if (pi_check_launch("paged_attention_general")) return -1;
   if (splits == 1) return 0;
   if (dtype == PI_F32)
-    hipLaunchKernelGGL((merge_key_ranges_kernel<float, 4>), dim3(T, nh), block, 0, stream, (float*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, out_mult);
+    hipLaunchKernelGGL((merge_key_ranges_kernel<float, 4>), dim3(T, nh), block, 0, stream, (float*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, gate_stride, out_mult);
   else
-    hipLaunchKernelGGL((merge_key_ranges_kernel<bf16_t, 4>), dim3(T, nh), block, 0, stream, (bf16_t*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, out_mult);
+    hipLaunchKernelGGL((merge_key_ranges_kernel<bf16_t, 4>), dim3(T, nh), block, 0, stream, (bf16_t*)out, out_stride, (const float*)part, nh, vd, splits, sinks, gate, gate_stride, out_mult);
   return pi_check_launch("merge_key_ranges");
 }

@@ -53,7 +53,8 @@ struct AttnState {
 // Options of a head beyond plain softmax attention, each off when its pointer is null:
 //   slopes [heads]: slope * (p - t) is taken off the scaled score of key t for the query at p;
 //   sinks  [heads]: exp(sink) joins the softmax's denominator once (no key, no value, no scale, no bias);
-//   gate   [tokens, heads] float32: multiplies the head's output;
+//   gate   [tokens, heads] float32: multiplies the head's output; with gate_stride > 0 instead float32 rows
+//          [heads * HD] that far apart, one gate per feature, still to go through a sigmoid;
 //   softcap > 0: the scaled score s becomes softcap * tanh(s / softcap), before any bias;
 //   out_mult: a factor on every output.
 struct AttnOptions {
@@ -62,9 +63,16 @@ struct AttnOptions {
   const float* gate;
   float softcap = 0.f;
   float out_mult = 1.f;
+  long gate_stride = 0;   // > 0: gates per feature
   int chunk = 0;          // C > 0: a token sees the keys of its own chunk of C positions only (a bound like the window's: no option of the arithmetic)
   bool any() const { return slopes || sinks || gate || softcap > 0.f || out_mult != 1.f; }
 };
+
+// the factors that the gates of four neighbouring features (as projected) put on them
+__device__ inline f32x4_t feature_gates(const AttnOptions& opt, long row, long col) {
+  const float4 g = *reinterpret_cast<const float4*>(opt.gate + row * opt.gate_stride + col);
+  return f32x4_t{1.0f / (1.0f + __expf(-g.x)), 1.0f / (1.0f + __expf(-g.y)), 1.0f / (1.0f + __expf(-g.z)), 1.0f / (1.0f + __expf(-g.w))};
+}
 
 // The first key a token at position pos sees: 0, or pos - window + 1, or the start of pos's chunk (the later of them).
 __device__ inline int first_seen_key(int pos, int window, int chunk) {

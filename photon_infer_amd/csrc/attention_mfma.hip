@@ -183,12 +183,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
       float inv = 1.0f / st.l[c];
       if (OPT) {
         if (opt.sinks) inv = sink_inverse(st.l[c], st.m[c] * scale_log2, opt.sinks[heads[c]]);
-        if (opt.gate) inv *= opt.gate[rows[c] * nh + heads[c]];
+        if (opt.gate && !opt.gate_stride) inv *= opt.gate[rows[c] * nh + heads[c]];
         inv *= opt.out_mult;
       }
       bf16_t* o = out + rows[c] * out_stride + (long)heads[c] * HD + lg * 4;
 #pragma unroll
       for (int db = 0; db < HD / 16; ++db) {
+        if (OPT && opt.gate_stride) st.o[db][c] *= feature_gates(opt, rows[c], heads[c] * HD + db * 16 + lg * 4);
         uint2 w;
         w.x = pack_bf16x2(st.o[db][c][0] * inv, st.o[db][c][1] * inv);
         w.y = pack_bf16x2(st.o[db][c][2] * inv, st.o[db][c][3] * inv);
@@ -217,8 +218,8 @@ extern "C" int pi_attention_prefill_mfma(void* out, long out_stride, const void*
                                          const int* kv_len, const int* tile_req, const int* tile_q0, const int* tile_cut,
                                          const int* tile_z0, void* part, const int* order, int rounds, int seats, int nh,
                                          int nkv, int hd, int page_size, float scale, int window, long num_pages,
-                                         const float* slopes, const float* sinks, const float* gate, float softcap,
-                                         float out_mult, int chunk, hipStream_t stream) {
+                                         const float* slopes, const float* sinks, const float* gate, long gate_stride,
+                                         float softcap, float out_mult, int chunk, hipStream_t stream) {
   PI_REQUIRE(chunk >= 0, "attention_prefill: chunk must be >= 0, got %d", chunk);
   PI_REQUIRE(rounds > 0 && seats > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_prefill: bad sizes rounds=%d seats=%d heads=%d kv_heads=%d", rounds, seats, nh, nkv);
   PI_REQUIRE(hd >= 16 && hd <= 256 && hd % 16 == 0, "attention_prefill: head_dim %d is not a multiple of 16 up to 256", hd);
@@ -230,7 +231,8 @@ extern "C" int pi_attention_prefill_mfma(void* out, long out_stride, const void*
   PI_REQUIRE(out_stride % 4 == 0 && q_stride % 8 == 0 && ((uintptr_t)q % 16 == 0) && ((uintptr_t)out % 8 == 0), "attention_prefill: q / out rows must be 16- / 8-byte aligned");
   const size_t lds = tiles_lds_bytes(hd);
   const dim3 grid(nkv, seats), block(256);
-  const AttnOptions opt{slopes, sinks, gate, softcap, out_mult, chunk};
+  PI_REQUIRE(gate_stride == 0 || (gate && gate_stride % 4 == 0 && (uintptr_t)gate % 16 == 0), "attention_prefill: gates per feature must lie in 16-byte groups");
+  const AttnOptions opt{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk};
   const bool with_options = opt.any();
   PI_REQUIRE(!with_options || scale > 0.f, "attention_prefill: a distance bias or a cap needs a positive scale");
 #define GO(H, C, N)                    \

@@ -69,6 +69,9 @@ __device__ inline void load4(const bf16_t* p, float v[4]) {
   v[2] = __uint_as_float(q.y << 16); v[3] = __uint_as_float(q.y & 0xffff0000u);
 }
 
+// x Phi(x), Phi the normal distribution function: the exact (erf) gelu
+__device__ inline float gelu_exact(float x) { return 0.5f * x * (1.0f + erff(x * 0.70710678118654752f)); }
+
 // ---- wave64 reductions (every lane gets the result)
 __device__ inline float wave_sum(float v) {
 #pragma unroll

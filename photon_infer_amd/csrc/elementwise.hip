@@ -5,14 +5,15 @@
 PI_DEFINE_MODULE(core)
 
 // ------------------------------------------------------------------ embedding
-// out[t, :] = float(table[ids[t], :]) * scale.  An id outside [0, V) fills the row with NaN:
+// out[t, c, :] = float(table[ids[t], :]) * scale for every copy c (grid y; one unless the stream is several side by
+// side).  An id outside [0, V) fills the row with NaN:
 // loud in every later result, and no access outside the table.
 template <typename TW>
 __global__ void embedding_kernel(float* __restrict__ out, const TW* __restrict__ table,
                                  const int* __restrict__ ids, int D, int V, float scale) {
   const long t = blockIdx.x;
   const int id = ids[t];
-  float* o = out + t * D;
+  float* o = out + (t * gridDim.y + blockIdx.y) * D;
   if (id < 0 || id >= V) {
     for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = __builtin_nanf("");
     return;
@@ -26,14 +27,14 @@ __global__ void embedding_kernel(float* __restrict__ out, const TW* __restrict__
 }
 
 extern "C" int pi_embedding(float* out, const void* table, int table_dtype, const int* ids, int T, int D,
-                            int V, float scale, hipStream_t stream) {
-  PI_REQUIRE(T >= 0 && D > 0 && V > 0, "embedding: bad sizes T=%d D=%d V=%d", T, D, V);
+                            int V, float scale, int copies, hipStream_t stream) {
+  PI_REQUIRE(T >= 0 && D > 0 && V > 0 && copies > 0 && copies <= 65535, "embedding: bad sizes T=%d D=%d V=%d copies=%d", T, D, V, copies);
   if (T == 0) return 0;
   const int threads = D >= 256 ? 256 : 64;
   if (table_dtype == PI_F32)
-    hipLaunchKernelGGL(embedding_kernel<float>, dim3(T), dim3(threads), 0, stream, out, (const float*)table, ids, D, V, scale);
+    hipLaunchKernelGGL(embedding_kernel<float>, dim3(T, copies), dim3(threads), 0, stream, out, (const float*)table, ids, D, V, scale);
   else if (table_dtype == PI_BF16)
-    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(T), dim3(threads), 0, stream, out, (const bf16_t*)table, ids, D, V, scale);
+    hipLaunchKernelGGL(embedding_kernel<bf16_t>, dim3(T, copies), dim3(threads), 0, stream, out, (const bf16_t*)table, ids, D, V, scale);
   else
     return pi_fail("embedding: unsupported table dtype %d", table_dtype);
   return pi_check_launch("embedding");
@@ -291,34 +292,36 @@ extern "C" int pi_swiglu(void* out, const void* gu, int dtype, int T, int I, int
   return pi_check_launch("swiglu");
 }
 
-// ------------------------------------------------------------------ squared relu
-// out = max(in, 0)^2, from the float32 results of a product into the activation type: the square is
-// taken before the one rounding.
-template <typename TO>
-__global__ void relu_squared_kernel(TO* __restrict__ out, const float* __restrict__ in, long n) {
+// ------------------------------------------------------------------ activations of feed-forwards without a gate
+// out = act(in), act = max(v, 0)^2 or the exact gelu, from the float32 results of a product (a tensor, or its pieces
+// still split over k) into the activation type: the activation is taken before the one rounding.
+enum { ACT_RELU2 = 0, ACT_GELU = 1 };
+template <typename TO, int ACT>
+__global__ void activation_kernel(TO* __restrict__ out, const float* __restrict__ in, long n, int splits) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
-  const float v = fmaxf(in[i], 0.f);
-  out[i] = from_float<TO>(v * v);
+  const float v = splits > 1 ? split_sum(in, splits, n, i) : in[i];
+  const float r = fmaxf(v, 0.f);
+  out[i] = from_float<TO>(ACT == ACT_GELU ? gelu_exact(v) : r * r);
 }
 
-extern "C" int pi_relu_squared(void* out, int out_dtype, const float* in, long n, hipStream_t stream) {
-  PI_REQUIRE(n >= 0 && out && in, "squared relu: bad arguments");
+extern "C" int pi_activation(void* out, int out_dtype, const float* in, long n, int splits, int act, hipStream_t stream) {
+  PI_REQUIRE(n >= 0 && out && in && splits >= 1, "activation: bad arguments");
+  PI_REQUIRE(act == ACT_RELU2 || act == ACT_GELU, "activation: unknown activation %d", act);
   if (n == 0) return 0;
   const long blocks = (n + 255) / 256;
-  PI_REQUIRE(blocks < 2147483647L, "squared relu: too many elements (%ld)", n);
-  if (out_dtype == PI_F32)
-    hipLaunchKernelGGL(relu_squared_kernel<float>, dim3((unsigned)blocks), dim3(256), 0, stream, (float*)out, in, n);
-  else if (out_dtype == PI_BF16)
-    hipLaunchKernelGGL(relu_squared_kernel<bf16_t>, dim3((unsigned)blocks), dim3(256), 0, stream, (bf16_t*)out, in, n);
-  else
-    return pi_fail("squared relu: unsupported dtype %d", out_dtype);
-  return pi_check_launch("relu_squared");
+  PI_REQUIRE(blocks < 2147483647L, "activation: too many elements (%ld)", n);
+#define ACT_GO(TO, A) hipLaunchKernelGGL((activation_kernel<TO, A>), dim3((unsigned)blocks), dim3(256), 0, stream, (TO*)out, in, n, splits)
+  if (out_dtype == PI_F32) { if (act == ACT_GELU) ACT_GO(float, ACT_GELU); else ACT_GO(float, ACT_RELU2); }
+  else if (out_dtype == PI_BF16) { if (act == ACT_GELU) ACT_GO(bf16_t, ACT_GELU); else ACT_GO(bf16_t, ACT_RELU2); }
+  else return pi_fail("activation: unsupported dtype %d", out_dtype);
+#undef ACT_GO
+  return pi_check_launch("activation");
 }
 
 // ------------------------------------------------------------------ clamped gated unit with biases
 // g = min(gate + bg, limit), u = clamp(up + bu, -limit, limit), out = g * sigmoid(alpha * g) * (u + 1).
-// The gate and up products lie in halves of a row ([gate | up]) in TI; biases and arithmetic are
+// The gate and up products lie in halves of a row ([gate | up]) in TI; biases (bg null: none) and arithmetic are
 // float32.  Optionally the stream's row gets a bias added on the way (x[t, :] += xb): the bias of
 // the product that follows, which then only accumulates.
 template <typename TO, typename TI, typename TB>
@@ -332,8 +335,8 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(TO* __restrict__ out, 
     // block == 0: [gate | up] in halves, biases bg and bu; block == b: gate and up interleaved in blocks of b
     // columns, and so are the biases, all in bg
     const int gc = block ? (i / block) * 2 * block + i % block : i, uc = block ? gc + block : I + i;
-    const float g = fminf(to_float(row[gc]) + to_float(block ? bg[gc] : bg[i]), limit);
-    const float u = fminf(fmaxf(to_float(row[uc]) + to_float(block ? bg[uc] : bu[i]), -limit), limit);
+    const float g = fminf(to_float(row[gc]) + (bg ? to_float(block ? bg[gc] : bg[i]) : 0.f), limit);
+    const float u = fminf(fmaxf(to_float(row[uc]) + (bg ? to_float(block ? bg[uc] : bu[i]) : 0.f), -limit), limit);
     out[t * I + i] = from_float<TO>(g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
   }
   if (x && i < D) x[t * D + i] += to_float(xb[i]);

@@ -30,10 +30,10 @@ PI_DEFINE_MODULE(bf16)
 #define BK 64
 #define TILE_ELEMS (BM * BK)                // a tile's slab in LDS: rows of 128 bytes
 
-enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ACCUM = 2, EPI_SWIGLU = 3, EPI_CLAMPED_GLU = 4, EPI_RELU2 = 5 };
+enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ACCUM = 2, EPI_SWIGLU = 3, EPI_CLAMPED_GLU = 4, EPI_RELU2 = 5, EPI_GELU = 6 };
 
-// results that leave as bfloat16, one per input column: as they are, or through max(c, 0)^2
-#define EPI_HALF(E) ((E) == EPI_BF16 || (E) == EPI_RELU2)
+// results that leave as bfloat16, one per input column: as they are, through max(c, 0)^2, or through the exact gelu
+#define EPI_HALF(E) ((E) == EPI_BF16 || (E) == EPI_RELU2 || (E) == EPI_GELU)
 
 // the gated epilogues store one output column per pair of input columns, in bfloat16
 #define EPI_GATED(E) ((E) == EPI_SWIGLU || (E) == EPI_CLAMPED_GLU)
@@ -97,11 +97,12 @@ __device__ inline void store_rows32(float* patch, const f32x16_t& acc0, const f3
       const f32x4_t u0 = *reinterpret_cast<const f32x4_t*>(g + 16), u1 = *reinterpret_cast<const f32x4_t*>(g + 20);
       float o[8];
       if (EPI == EPI_CLAMPED_GLU) {
-        const float* bg = glu.bias + col0 + j * 32 + q * 8;      // col0: the corner's first input column
+        const bool biased = glu.bias != nullptr;
+        const float* bg = glu.bias + (biased ? col0 + j * 32 + q * 8 : 0);      // col0: the corner's first input column
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          o[e] = clamped_glu_mul(g0[e], u0[e], bg[e], bg[16 + e], glu.limit, glu.alpha);
-          o[4 + e] = clamped_glu_mul(g1[e], u1[e], bg[4 + e], bg[20 + e], glu.limit, glu.alpha);
+          o[e] = clamped_glu_mul(g0[e], u0[e], biased ? bg[e] : 0.f, biased ? bg[16 + e] : 0.f, glu.limit, glu.alpha);
+          o[4 + e] = clamped_glu_mul(g1[e], u1[e], biased ? bg[4 + e] : 0.f, biased ? bg[20 + e] : 0.f, glu.limit, glu.alpha);
         }
       } else {
 #pragma unroll
@@ -130,6 +131,10 @@ __device__ inline void store_rows32(float* patch, const f32x16_t& acc0, const f3
           a[e] = fmaxf(a[e], 0.f); a[e] *= a[e];
           b[e] = fmaxf(b[e], 0.f); b[e] *= b[e];
         }
+      }
+      if (EPI == EPI_GELU) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { a[e] = gelu_exact(a[e]); b[e] = gelu_exact(b[e]); }
       }
       bf16_t* dst = out + (row0 + r) * ld + c;
       if (wide && c + 8 <= cols_left) {
@@ -557,11 +562,12 @@ extern "C" int pi_gemm_mfma_group_tile_rows() { return BM; }
 
 // C[row, :] = A[row, :] . W[group of row]^T over a device-side list of `tiles` row tiles (see the
 // kernel); W is [groups, N, K] with `group_stride` elements from one group's matrix to the next.
-// epilogue: 0 store bf16, 1 store f32, 3 SwiGLU (every group's rows interleaved by 16; C is [rows, N / 2] bf16).
+// epilogue: 0 store bf16, 1 store f32, 3 SwiGLU (every group's rows interleaved by 16; C is [rows, N / 2] bf16), 4 the clamped
+// gated unit without biases (rows as for 3; `limit` and `alpha`), 5 max(c, 0)^2 as bf16.
 template <int EPI>
 static int launch_grouped(void* C, long ldc, const void* A, long lda, const void* W, long ldw, long group_stride,
                           const int* group_of_tile, const int* tile_row0, const int* tile_rows, int tiles, int N, int K,
-                          long group_a_step, long group_c_step, hipStream_t stream) {
+                          long group_a_step, long group_c_step, hipStream_t stream, GluArgs glu = GluArgs{nullptr, 0.f, 0.f}) {
   static bool configured = false;
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_mfma_kernel<EPI>),
@@ -572,13 +578,14 @@ static int launch_grouped(void* C, long ldc, const void* A, long lda, const void
   const int tiles_n = ceil_div(N, BN);
   hipLaunchKernelGGL((gemm_mfma_kernel<EPI>), dim3((unsigned)tiles * tiles_n, 1), dim3(256), kLdsBytes, stream, C, ldc,
                      (const bf16_t*)A, lda, (const bf16_t*)W, ldw, BM, N, K, tiles_n, K, group_of_tile, tile_row0, tile_rows,
-                     group_stride, group_a_step, group_c_step, GluArgs{nullptr, 0.f, 0.f});
+                     group_stride, group_a_step, group_c_step, glu);
   return pi_check_launch("gemm_mfma_grouped");
 }
 
 extern "C" int pi_gemm_mfma_grouped(void* C, int epilogue, long ldc, const void* A, long lda, const void* W, long ldw,
                                     long group_stride, const int* group_of_tile, const int* tile_row0, const int* tile_rows,
-                                    int tiles, int N, int K, long group_a_step, long group_c_step, hipStream_t stream) {
+                                    int tiles, int N, int K, long group_a_step, long group_c_step, float limit, float alpha,
+                                    hipStream_t stream) {
   PI_REQUIRE(tiles >= 0 && N > 0 && K > 0, "gemm_mfma_grouped: bad sizes tiles=%d N=%d K=%d", tiles, N, K);
   PI_REQUIRE(group_a_step >= 0 && group_c_step >= 0 && group_a_step % 8 == 0 && group_c_step % 8 == 0,
              "gemm_mfma_grouped: a group's columns in the rows (%ld, %ld) must start at multiples of 8", group_a_step, group_c_step);
@@ -587,13 +594,14 @@ extern "C" int pi_gemm_mfma_grouped(void* C, int epilogue, long ldc, const void*
   PI_REQUIRE(256 * lda < (1L << 29) && 256 * ldw < (1L << 29), "gemm_mfma_grouped: row strides (%ld, %ld) are too long", lda, ldw);
   PI_REQUIRE(ldc > 0 && ldc < (1L << 23), "gemm_mfma_grouped: the result's row stride (%ld) is too long", ldc);
   PI_REQUIRE(((uintptr_t)A % 16 == 0) && ((uintptr_t)W % 16 == 0), "gemm_mfma_grouped: operands must be 16-byte aligned");
-  PI_REQUIRE(epilogue != EPI_SWIGLU || N % 32 == 0, "gemm_mfma_grouped: the SwiGLU epilogue needs N (%d) to be a multiple of 32", N);
+  PI_REQUIRE(!EPI_GATED(epilogue) || N % 32 == 0, "gemm_mfma_grouped: the gated epilogues need N (%d) to be a multiple of 32", N);
   PI_REQUIRE((long)tiles * ceil_div(N, BN) < 2147483647L, "gemm_mfma_grouped: too many tiles");
   PI_REQUIRE(group_of_tile && tile_row0 && tile_rows, "gemm_mfma_grouped: the tile list is missing");
   if (tiles == 0) return 0;
   switch (epilogue) {
     case EPI_BF16: return launch_grouped<EPI_BF16>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
     case EPI_F32: return launch_grouped<EPI_F32>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
+    case EPI_CLAMPED_GLU: return launch_grouped<EPI_CLAMPED_GLU>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream, GluArgs{nullptr, limit, alpha});
     case EPI_RELU2: return launch_grouped<EPI_RELU2>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
     case EPI_SWIGLU: return launch_grouped<EPI_SWIGLU>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
   }
@@ -607,7 +615,7 @@ extern "C" int pi_gemm_mfma_pieces(int K, int splits) {
 }
 
 // epilogue: 0 store bf16, 1 store f32, 2 add into f32, 3 SwiGLU (W rows interleaved by 16; C is [M, N / 2] bf16),
-// 5 store max(c, 0)^2 as bf16
+// 5 store max(c, 0)^2 as bf16, 6 store the exact gelu of c as bf16
 extern "C" int pi_gemm_mfma(void* C, int epilogue, long ldc, const void* A, long lda, const void* W, long ldw, int M,
                             int N, int K, int splits, hipStream_t stream) {
   PI_REQUIRE(M > 0 && N > 0 && K > 0, "gemm_mfma: bad sizes M=%d N=%d K=%d", M, N, K);
@@ -626,6 +634,7 @@ extern "C" int pi_gemm_mfma(void* C, int epilogue, long ldc, const void* A, long
     case EPI_F32: return launch<EPI_F32>(C, ldc, A, lda, W, ldw, M, N, K, splits, stream);
     case EPI_ACCUM: return launch<EPI_ACCUM>(C, ldc, A, lda, W, ldw, M, N, K, splits, stream);
     case EPI_RELU2: return launch<EPI_RELU2>(C, ldc, A, lda, W, ldw, M, N, K, splits, stream);
+    case EPI_GELU: return launch<EPI_GELU>(C, ldc, A, lda, W, ldw, M, N, K, splits, stream);
     case EPI_SWIGLU: return launch<EPI_SWIGLU>(C, ldc, A, lda, W, ldw, M, N, K, splits, stream);
   }
   return pi_fail("gemm_mfma: unknown epilogue %d", epilogue);

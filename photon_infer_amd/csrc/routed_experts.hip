@@ -3,7 +3,7 @@
 // count ever travels to the host, so a step's launches depend on its number of tokens only.
 //
 // Routing, per token, from float32 router logits z [E]:
-//   s = softmax(z) over all experts;
+//   s = softmax(z) over all experts, or sigmoid(z) of each on its own;
 //   experts form `groups` equal groups of neighbours, a group's score is its largest s, and
 //   only experts of the `keep` best groups may be chosen (groups <= 1: all may);
 //   the `top` allowed experts with the largest s are chosen, weights = their s (as they are,
@@ -32,7 +32,7 @@ __device__ inline void wave_argmax(float& v, int& idx) {
 
 __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ logits,
                                                         long logits_stride, int E, int top, int groups, int keep, int renorm,
-                                                        const float* __restrict__ correction, float renorm_eps) {
+                                                        const float* __restrict__ correction, float renorm_eps, int sigmoid) {
   __shared__ float s[RE_MAX_EXPERTS];
   __shared__ float c[RE_MAX_EXPERTS];      // what the choice goes by
   __shared__ unsigned char allowed[RE_MAX_EXPERTS];
@@ -40,21 +40,31 @@ __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, f
   const long t = blockIdx.x;
   const int lane = threadIdx.x;
   const float* z = logits + t * logits_stride;
-  float mx = -INFINITY;
-  for (int e = lane; e < E; e += PI_WAVE) mx = fmaxf(mx, z[e]);
-  mx = wave_max(mx);
-  float sum = 0.f;
-  for (int e = lane; e < E; e += PI_WAVE) {
-    const float v = expf(z[e] - mx);
-    s[e] = v;
-    sum += v;
-  }
-  sum = wave_sum(sum);
-  const float inv = 1.0f / sum;
-  for (int e = lane; e < E; e += PI_WAVE) {
-    s[e] *= inv;
-    c[e] = correction ? s[e] + correction[e] : s[e];
-    allowed[e] = (groups <= 1) ? 1 : 0;
+  if (sigmoid) {
+    // the sigmoid grows with z, so without a correction the choice goes by z itself: large logits whose scores round
+    // to the same number keep their order
+    for (int e = lane; e < E; e += PI_WAVE) {
+      s[e] = 1.0f / (1.0f + expf(-z[e]));
+      c[e] = correction ? s[e] + correction[e] : z[e];
+      allowed[e] = (groups <= 1) ? 1 : 0;
+    }
+  } else {
+    float mx = -INFINITY;
+    for (int e = lane; e < E; e += PI_WAVE) mx = fmaxf(mx, z[e]);
+    mx = wave_max(mx);
+    float sum = 0.f;
+    for (int e = lane; e < E; e += PI_WAVE) {
+      const float v = expf(z[e] - mx);
+      s[e] = v;
+      sum += v;
+    }
+    sum = wave_sum(sum);
+    const float inv = 1.0f / sum;
+    for (int e = lane; e < E; e += PI_WAVE) {
+      s[e] *= inv;
+      c[e] = correction ? s[e] + correction[e] : s[e];
+      allowed[e] = (groups <= 1) ? 1 : 0;
+    }
   }
   __syncthreads();
   if (groups > 1) {
@@ -112,13 +122,13 @@ __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, f
 }
 
 extern "C" int pi_route(int* ids, float* weights, const float* logits, long logits_stride, int T, int E, int top, int groups,
-                        int keep, int renorm, const float* correction, float renorm_eps, hipStream_t stream) {
+                        int keep, int renorm, const float* correction, float renorm_eps, int sigmoid, hipStream_t stream) {
   PI_REQUIRE(T >= 0 && E > 0 && E <= RE_MAX_EXPERTS, "routing: %d experts (at most %d)", E, RE_MAX_EXPERTS);
   PI_REQUIRE(top > 0 && top <= E, "routing: %d choices among %d experts", top, E);
   PI_REQUIRE(groups <= 1 || (E % groups == 0 && keep > 0 && keep <= groups), "routing: %d experts in %d groups, %d kept", E, groups, keep);
   PI_REQUIRE(groups <= 1 || (long)keep * (E / groups) >= top, "routing: %d kept groups of %d experts hold fewer than %d choices", keep, groups > 0 ? E / groups : 0, top);
   if (T == 0) return 0;
-  hipLaunchKernelGGL(route_kernel, dim3(T), dim3(PI_WAVE), 0, stream, ids, weights, logits, logits_stride, E, top, groups, keep, renorm, correction, renorm_eps);
+  hipLaunchKernelGGL(route_kernel, dim3(T), dim3(PI_WAVE), 0, stream, ids, weights, logits, logits_stride, E, top, groups, keep, renorm, correction, renorm_eps, sigmoid);
   return pi_check_launch("route");
 }
 
@@ -199,21 +209,29 @@ extern "C" int pi_group_entries(const int* ids, int N, int E, int* row_entry, in
 
 extern "C" int pi_group_tile_rows() { return RE_TILE; }
 
-// rows[row, :] = src[row_entry[row] / top, :]   (activations copied into expert order)
+// rows[row, :] = src[row_entry[row] / top, :]   (activations copied into expert order), times the entry's weight when
+// weights are given (routing that weighs an expert's input instead of its output)
 template <typename T>
-__global__ void gather_rows_kernel(T* __restrict__ out, const T* __restrict__ src, const int* __restrict__ row_entry, int top, int D) {
+__global__ void gather_rows_kernel(T* __restrict__ out, const T* __restrict__ src, const int* __restrict__ row_entry, int top, int D,
+                                   const float* __restrict__ weights) {
   const long row = blockIdx.x;
   const long t = row_entry[row] / top;
+  if (weights) {
+    const float w = weights[row_entry[row]];
+    for (int d = threadIdx.x; d < D; d += blockDim.x) out[row * D + d] = from_float<T>(to_float(src[t * D + d]) * w);
+    return;
+  }
   for (int d = threadIdx.x; d < D; d += blockDim.x) out[row * D + d] = src[t * D + d];
 }
 
-extern "C" int pi_gather_rows(void* out, const void* src, int dtype, const int* row_entry, int N, int top, int D, hipStream_t stream) {
+extern "C" int pi_gather_rows(void* out, const void* src, int dtype, const int* row_entry, int N, int top, int D, const float* weights,
+                              hipStream_t stream) {
   PI_REQUIRE(N >= 0 && top > 0 && D > 0, "gather: bad sizes");
   if (N == 0) return 0;
   if (dtype == PI_F32)
-    hipLaunchKernelGGL(gather_rows_kernel<float>, dim3(N), dim3(256), 0, stream, (float*)out, (const float*)src, row_entry, top, D);
+    hipLaunchKernelGGL(gather_rows_kernel<float>, dim3(N), dim3(256), 0, stream, (float*)out, (const float*)src, row_entry, top, D, weights);
   else if (dtype == PI_BF16)
-    hipLaunchKernelGGL(gather_rows_kernel<bf16_t>, dim3(N), dim3(256), 0, stream, (bf16_t*)out, (const bf16_t*)src, row_entry, top, D);
+    hipLaunchKernelGGL(gather_rows_kernel<bf16_t>, dim3(N), dim3(256), 0, stream, (bf16_t*)out, (const bf16_t*)src, row_entry, top, D, weights);
   else
     return pi_fail("gather: unsupported dtype %d", dtype);
   return pi_check_launch("gather_rows");
@@ -300,7 +318,7 @@ extern "C" int pi_grouped_gemm_general(void* C, int c_dtype, long ldc, const voi
 }
 
 // out[t, :] (+)= sum_j weights[t, j] * y[entry_row[t * top + j], :], choices in order (float32); a choice whose
-// id is num_real or more (ids given) stands for the token's own activations h[t, :] instead
+// id is num_real or more (ids given) stands for the token's own activations h[t, :] instead; weights null: a plain sum
 template <typename TH>
 __global__ void combine_choices_kernel(float* __restrict__ out, const float* __restrict__ y, const float* __restrict__ weights,
                                        const int* __restrict__ entry_row, int top, int D, int accumulate, const int* __restrict__ ids,
@@ -312,7 +330,7 @@ __global__ void combine_choices_kernel(float* __restrict__ out, const float* __r
   for (int j = 0; j < top; ++j) {
     const bool own = ids && ids[t * top + j] >= num_real;
     const float v = own ? to_float(h[t * D + d]) : y[(long)entry_row[t * top + j] * D + d];
-    acc = fmaf(weights[t * top + j], v, acc);
+    acc = weights ? fmaf(weights[t * top + j], v, acc) : acc + v;
   }
   out[t * D + d] = accumulate ? out[t * D + d] + acc : acc;
 }

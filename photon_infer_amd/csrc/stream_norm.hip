@@ -613,3 +613,237 @@ extern "C" int pi_qk_norm_kv_write(void* q_out, long q_stride, float* gate_out, 
 #undef QKN_GO
   return pi_check_launch("qk_norm_kv_write");
 }
+
+// ---------------------------------------------------------------- queries and keys rotated, then normalised per head; values are the keys
+// Projection rows (float32, a tensor or the pieces of a product split over k) hold [q: nh*hd | k: nkv*hd | gates: ng].
+//   q, k <- + bias (by column; null: none), rotated by the token's angles on the first rd features of each head
+//           (halves paired, or neighbours), then every head divided by the root mean square of its hd entries
+//   values: the keys with their bias, neither rotated nor normalised
+// Queries go to q_out, keys to the key pages [page, kv head, slot, hd], values to the value pages [page, kv head, hd, slot].
+// Pieces only: the gates' columns are summed into gate_out (float32 [T, ng]) as they are, for whoever applies them.
+// Everything is float32 until the one rounding on store.
+struct QkRopeArgs {
+  const float* proj;       // [T, stride], or null: the pieces
+  long stride;
+  const float* part;       // [splits, T, stride]
+  int splits;
+  long plane;
+  const float* bias;       // [(nh + nkv) * hd] or null
+  const float* table;      // [T, rd]: cosines, then sines
+  int rd, interleaved;
+  float eps;
+  int T, nh, nkv, hd, ng;
+  const int* positions;
+  const int* req_of_token;
+  const int* block_table;
+  int table_width, page_size;
+  long num_pages;
+  float* gate_out;
+};
+
+__device__ inline float qkr_value(const QkRopeArgs& a, long t, int col) {
+  const float v = a.part ? split_sum(a.part, a.splits, a.plane, t * a.stride + col) : a.proj[t * a.stride + col];
+  return a.bias ? v + a.bias[col] : v;
+}
+
+// four neighbouring columns; rows and columns are whole 16-byte groups
+__device__ inline float4 qkr_value4(const QkRopeArgs& a, long t, int col, bool with_bias) {
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (a.part) {
+    const float* p = a.part + t * a.stride + col;
+    for (int s0 = 0; s0 < a.splits; s0 += 8) {       // eight pieces' loads in flight, added in split order
+      float4 l[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) l[u] = s0 + u < a.splits ? *reinterpret_cast<const float4*>(p + (s0 + u) * a.plane) : make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) { v.x += l[u].x; v.y += l[u].y; v.z += l[u].z; v.w += l[u].w; }
+    }
+  } else {
+    v = *reinterpret_cast<const float4*>(a.proj + t * a.stride + col);
+  }
+  if (with_bias && a.bias) {
+    const float4 b = *reinterpret_cast<const float4*>(a.bias + col);
+    v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
+  }
+  return v;
+}
+
+// page and slot of a token's position; false: no page (the host checks tables; nothing is written outside the pool)
+__device__ inline bool qkr_place(const QkRopeArgs& a, long t, long& page, int& slot) {
+  const int pos = a.positions[t], blk = pos / a.page_size;
+  slot = pos % a.page_size;
+  page = blk < a.table_width ? a.block_table[(long)a.req_of_token[t] * a.table_width + blk] : -1;
+  return page >= 0 && page < a.num_pages;
+}
+
+// Blocks [0, head_blocks): heads of queries and keys, LANES lanes per (token, head) with four features each (LANES 0:
+// a wave per (token, head), features 64 apart, for sizes that are no whole 16-byte groups); then value_blocks: a
+// thread per (PT neighbouring tokens, kv head, feature); then the gates of pieces, four columns per thread.
+template <typename T, int LANES, int PT>
+__global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T* __restrict__ q_out, long q_stride, T* __restrict__ k_cache,
+                                                                 T* __restrict__ v_cache, int head_blocks, int value_blocks) {
+  const int hd = a.hd, half = a.rd / 2;
+  if ((int)blockIdx.x < head_blocks) {
+    constexpr int L = LANES ? LANES : PI_WAVE;
+    const long item = ((long)blockIdx.x * 256 + threadIdx.x) / L;
+    const int lane = threadIdx.x % L, heads = a.nh + a.nkv;
+    const int u = (int)(item % heads);
+    const long t = item / heads;
+    if (t >= a.T) return;                            // whole groups of lanes leave together
+    const int col = u * hd;                          // key heads follow the query heads in the row
+    T* dst;
+    if (u < a.nh) {
+      dst = q_out + t * q_stride + col;
+    } else {
+      long page;
+      int slot;
+      if (!qkr_place(a, t, page, slot)) return;
+      dst = k_cache + ((page * a.nkv + (u - a.nh)) * a.page_size + slot) * hd;
+    }
+    const float* cs = a.table + t * a.rd;
+    if constexpr (LANES > 0) {
+      const int d = 4 * lane;
+      const bool in = d < hd;
+      const float4 v4 = in ? qkr_value4(a, t, col + d, true) : make_float4(0.f, 0.f, 0.f, 0.f);
+      float v[4] = {v4.x, v4.y, v4.z, v4.w}, o[4];
+      float ss = fmaf(v[3], v[3], fmaf(v[2], v[2], fmaf(v[1], v[1], v[0] * v[0])));      // a rotation keeps it
+#pragma unroll
+      for (int off = L / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, PI_WAVE);
+      const float r = 1.0f / sqrtf(ss / hd + a.eps);
+      const bool by_lanes = !a.interleaved && half % 4 == 0;      // a feature's partner is the same feature of another lane
+      float other[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) other[e] = 0.f;
+      if (by_lanes && a.rd > 0) {
+        const int partner = (int)(threadIdx.x % PI_WAVE) + (d < half ? half / 4 : (d < a.rd ? -half / 4 : 0));
+#pragma unroll
+        for (int e = 0; e < 4; ++e) other[e] = __shfl(v[e], partner, PI_WAVE);
+      }
+      if (!in) return;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = d + e;
+        o[e] = v[e];
+        if (i < a.rd) {
+          const int j = a.interleaved ? i / 2 : (i < half ? i : i - half);
+          const bool low = a.interleaved ? (i & 1) == 0 : i < half;
+          const float b = a.interleaved ? v[e ^ 1] : (by_lanes ? other[e] : qkr_value(a, t, col + (low ? i + half : i - half)));
+          float lo, hi;
+          rope_pair(low ? v[e] : b, low ? b : v[e], cs[j], cs[half + j], lo, hi);
+          o[e] = low ? lo : hi;
+        }
+        o[e] *= r;
+      }
+      store4<T>(dst + d, make_float4(o[0], o[1], o[2], o[3]));
+    } else {
+      float ss = 0.f;
+      for (int i = lane; i < hd; i += PI_WAVE) {
+        const float v = qkr_value(a, t, col + i);
+        ss = fmaf(v, v, ss);
+      }
+      const float r = 1.0f / sqrtf(wave_sum(ss) / hd + a.eps);
+      for (int i = lane; i < hd; i += PI_WAVE) {
+        float v = qkr_value(a, t, col + i);
+        if (i < a.rd) {
+          const int j = a.interleaved ? i / 2 : (i < half ? i : i - half);
+          const bool low = a.interleaved ? (i & 1) == 0 : i < half;
+          const float b = qkr_value(a, t, col + (a.interleaved ? i ^ 1 : (low ? i + half : i - half)));
+          float lo, hi;
+          rope_pair(low ? v : b, low ? b : v, cs[j], cs[half + j], lo, hi);
+          v = low ? lo : hi;
+        }
+        dst[i] = from_float<T>(v * r);
+      }
+    }
+    return;
+  }
+  if ((int)blockIdx.x < head_blocks + value_blocks) {
+    const long idx = ((long)blockIdx.x - head_blocks) * 256 + threadIdx.x;
+    const int row = a.nkv * hd;
+    const int c = (int)(idx % row), g = c / hd, d = c % hd;
+    const long t0 = idx / row * PT;
+    if (t0 >= a.T) return;
+    const int n = (int)min((long)PT, a.T - t0);
+    T val[PT];
+    int pos[PT], req[PT];
+#pragma unroll
+    for (int i = 0; i < PT; ++i) {
+      const long t = t0 + (i < n ? i : 0);
+      val[i] = from_float<T>(qkr_value(a, t, a.nh * hd + c));
+      pos[i] = a.positions[t];
+      req[i] = a.req_of_token[t];
+    }
+    if constexpr (PT == 4 && sizeof(T) == 2) {
+      // four neighbours in one page: one 8-byte store
+      if (n == 4 && a.page_size % 4 == 0 && pos[0] % 4 == 0 && req[1] == req[0] && req[2] == req[0] && req[3] == req[0] &&
+          pos[1] == pos[0] + 1 && pos[2] == pos[0] + 2 && pos[3] == pos[0] + 3) {
+        long page;
+        int slot;
+        if (!qkr_place(a, t0, page, slot)) return;
+        const uint16_t* b = reinterpret_cast<const uint16_t*>(val);
+        *reinterpret_cast<uint2*>(v_cache + ((page * a.nkv + g) * hd + d) * a.page_size + slot) =
+            make_uint2((uint32_t)b[0] | ((uint32_t)b[1] << 16), (uint32_t)b[2] | ((uint32_t)b[3] << 16));
+        return;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < PT; ++i) {
+      long page;
+      int slot;
+      if (i < n && qkr_place(a, t0 + i, page, slot)) v_cache[((page * a.nkv + g) * hd + d) * a.page_size + slot] = val[i];
+    }
+    return;
+  }
+  const long idx = ((long)blockIdx.x - head_blocks - value_blocks) * 256 + threadIdx.x;
+  const int per = (a.ng + 3) / 4;
+  const long t = idx / per;
+  const int c = (int)(idx % per) * 4;
+  if (t >= a.T) return;
+  const int col = (a.nh + a.nkv) * hd + c;
+  if constexpr (LANES > 0) {
+    if (a.ng % 4 == 0) {
+      *reinterpret_cast<float4*>(a.gate_out + t * a.ng + c) = qkr_value4(a, t, col, false);
+      return;
+    }
+  }
+  for (int e = 0; e < 4 && c + e < a.ng; ++e) a.gate_out[t * a.ng + c + e] = split_sum(a.part, a.splits, a.plane, t * a.stride + col + e);
+}
+
+extern "C" int pi_qk_rope_norm_write(void* q_out, long q_stride, int dtype, const float* proj, long stride, const float* part, int splits,
+                                     const float* bias, const float* table, int rd, int interleaved, float eps, int T, int nh, int nkv,
+                                     int hd, int ng, float* gate_out, const int* positions, const int* req_of_token, void* k_cache,
+                                     void* v_cache, const int* block_table, int table_width, int page_size, long num_pages,
+                                     hipStream_t stream) {
+  PI_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && hd > 0 && hd <= 640 && ng >= 0, "qk rope norm: bad sizes T=%d heads=%d kv_heads=%d head_dim=%d", T, nh, nkv, hd);
+  PI_REQUIRE((proj != nullptr) != (part != nullptr) && (!part || splits >= 1), "qk rope norm: give the projection as a tensor or as pieces");
+  PI_REQUIRE(stride >= (long)(nh + nkv) * hd + (part ? ng : 0), "qk rope norm: rows of %ld hold no queries, keys and gates", stride);
+  PI_REQUIRE(rd >= 0 && rd <= hd && rd % 2 == 0 && (rd == 0 || table), "qk rope norm: rotation of %d features", rd);
+  PI_REQUIRE(q_out && positions && req_of_token && k_cache && v_cache && block_table && table_width > 0 && page_size > 0 && num_pages > 0,
+             "qk rope norm: bad cache geometry");
+  PI_REQUIRE(!part || ng == 0 || gate_out, "qk rope norm: gates in pieces need a place");
+  PI_REQUIRE(dtype == PI_F32 || dtype == PI_BF16, "qk rope norm: unsupported dtype %d", dtype);
+  if (T == 0) return 0;
+  QkRopeArgs a{proj, stride, part, splits, (long)T * stride, bias, table, rd, interleaved, eps, T, nh, nkv, hd, ng, positions, req_of_token,
+               block_table, table_width, page_size, num_pages, gate_out};
+  const int bytes = dtype == PI_F32 ? 16 : 8;
+  bool wide = hd % 4 == 0 && hd <= 256 && stride % 4 == 0 && q_stride % 4 == 0 && (uintptr_t)q_out % bytes == 0 && (uintptr_t)k_cache % bytes == 0;
+  for (const void* p : {(const void*)proj, (const void*)part, (const void*)bias, (const void*)gate_out}) wide = wide && (uintptr_t)p % 16 == 0;
+  const int lanes = !wide ? 0 : (hd <= 64 ? 16 : (hd <= 128 ? 32 : 64));
+  const bool four = T >= 16 && (uintptr_t)v_cache % 8 == 0;
+  const long items = (long)T * (nh + nkv), values = (long)ceil_div(T, four ? 4 : 1) * nkv * hd, gates = part ? (long)T * ceil_div(ng, 4) : 0;
+  const long hb = (items * (lanes ? lanes : PI_WAVE) + 255) / 256, vb = (values + 255) / 256, gb = (gates + 255) / 256;
+  PI_REQUIRE(hb + vb + gb < 2147483647L, "qk rope norm: too many tokens (%d)", T);
+  const dim3 grid((unsigned)(hb + vb + gb)), block(256);
+#define QR_GO(TT, L_, P_) hipLaunchKernelGGL((qk_rope_norm_write_kernel<TT, L_, P_>), grid, block, 0, stream, a, (TT*)q_out, q_stride, (TT*)k_cache, (TT*)v_cache, (int)hb, (int)vb)
+#define QR_PICK(TT)                                                            \
+  do {                                                                         \
+    if (lanes == 0) { if (four) QR_GO(TT, 0, 4); else QR_GO(TT, 0, 1); }       \
+    else if (lanes == 16) { if (four) QR_GO(TT, 16, 4); else QR_GO(TT, 16, 1); } \
+    else if (lanes == 32) { if (four) QR_GO(TT, 32, 4); else QR_GO(TT, 32, 1); } \
+    else { if (four) QR_GO(TT, 64, 4); else QR_GO(TT, 64, 1); }                \
+  } while (0)
+  if (dtype == PI_F32) QR_PICK(float); else QR_PICK(bf16_t);
+#undef QR_PICK
+#undef QR_GO
+  return pi_check_launch("qk_rope_norm_write");
+}

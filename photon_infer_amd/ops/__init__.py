@@ -102,9 +102,13 @@ def check_general_attention_sizes(num_heads: int, num_kv_heads: int, head_dim: i
 def embedding(out: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, scale: float = 1.0,
               pos_table: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None) -> None:
     """out[t, :] = float32(table[ids[t], :]) * scale; with a learned position table,
-    out[t, :] = table[ids[t], :] * scale + pos_table[positions[t], :]."""
+    out[t, :] = table[ids[t], :] * scale + pos_table[positions[t], :].  ``out`` [T, n, D]: n equal
+    copies of every row (not with a position table)."""
     _gpu(out, table, ids, pos_table, positions)
-    T, D = out.shape
+    copies = out.shape[1] if out.dim() == 3 else 1
+    if out.dim() not in (2, 3) or (out.dim() == 3 and pos_table is not None):
+        raise KernelError(f"embedding: output of shape {tuple(out.shape)}")
+    T, D = out.shape[0], out.shape[-1]
     if out.dtype != torch.float32 or not out.is_contiguous():
         raise KernelError("embedding: output must be contiguous float32")
     if table.dim() != 2 or table.shape[1] != D or not table.is_contiguous():
@@ -118,7 +122,7 @@ def embedding(out: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, scale: 
                   positions.data_ptr(), float(scale), T, D, table.shape[0], pos_table.shape[0], _stream())
         return
     _lib.call("core", "pi_embedding", out.data_ptr(), table.data_ptr(), _dt(table), ids.data_ptr(), T, D,
-              table.shape[0], float(scale), _stream())
+              table.shape[0], float(scale), copies, _stream())
 
 
 def softcap_(x: torch.Tensor, cap: float) -> None:
@@ -164,11 +168,13 @@ def rmsnorm(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, eps: float
 # workspace), and a block arrangement must materialize before it hands the stream to a part that
 # does not read it through ``rmsnorm``.
 def materialize(x: torch.Tensor, ws: Optional[KernelWorkspace]) -> torch.Tensor:
-    """Apply an update of ``x`` that is still pending in ``ws``, if there is one."""
-    p = ws.take_pending(x) if ws is not None else None
-    if p is not None:
+    """Apply an update of ``x`` that is still pending in ``ws``, if there is one (a result whose pieces are unadded is
+    written)."""
+    p = ws.pending if ws is not None else None
+    if p is not None and p.is_for(x):
         from . import fast
-        fast.reduce_into(x, p, accumulate=True)
+        ws.pending = None
+        fast.reduce_into(x, p.pieces, accumulate=p.accumulate)
         ws.counts["applied"] += 1
     return x
 
@@ -222,9 +228,9 @@ def gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, accumulate: bool =
     """out[M, N] (+)= a[M, K] @ w[N, K]^T with float32 accumulation.
 
     ``ws``: where a product split over k keeps its pieces (without one, memory of this call's own).
-    ``may_defer`` (with ``accumulate`` and ``ws``): the caller promises that ``out`` is next read
-    by ``rmsnorm`` or ``materialize`` with the same workspace; a product that was split over k may
-    then stay in pieces there."""
+    ``may_defer`` (with ``ws``): the caller promises that ``out`` is next read by ``rmsnorm`` or ``materialize``
+    - a result that is not accumulated: by ``hyper_streams`` or ``materialize`` - with the same workspace; a
+    product that was split over k may then stay in pieces there."""
     if isinstance(a, KeyRanges):
         # attention's output of a decode step, its key ranges not merged yet: the weight-streaming
         # kernel merges them as it reads; anything else gets them merged first
@@ -237,7 +243,7 @@ def gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, accumulate: bool =
             materialize(out, ws)
         from . import fast
         if _FAST and fast.gemm_from_ranges(out, a, w, accumulate, w.shape[0], _rows(w, "gemm w"), _rows(out, "gemm out"),
-                                           may_defer and accumulate and out.is_contiguous(), ws):
+                                           may_defer and out.dtype == torch.float32 and out.is_contiguous(), ws):
             return
         merged = torch.empty((a.tokens, a.heads * a.head_dim), dtype=torch.bfloat16, device=out.device)
         fast.merge_ranges(merged, a)
@@ -258,7 +264,7 @@ def gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, accumulate: bool =
         materialize(out, ws)
     if _FAST and a.dtype == torch.bfloat16 and w.dtype == torch.bfloat16:
         from . import fast
-        if fast.gemm(out, a, w, accumulate, M, N, K, lda, ldw, ldc, may_defer and accumulate and out.is_contiguous(), ws):
+        if fast.gemm(out, a, w, accumulate, M, N, K, lda, ldw, ldc, may_defer and out.dtype == torch.float32 and out.is_contiguous(), ws):
             return
     _lib.call("core", "pi_gemm_general", out.data_ptr(), _dt(out), ldc, a.data_ptr(), _dt(a), lda, w.data_ptr(),
               _dt(w), ldw, M, N, K, int(accumulate), _stream())
@@ -433,7 +439,8 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
                     page_size: int, scale: float, window: int = 0, ws: Optional[KernelWorkspace] = None, *,
                     value_dim: Optional[int] = None, slopes: Optional[torch.Tensor] = None,
                     sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0) -> None:
+                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0,
+                    feature_gate: Optional[torch.Tensor] = None) -> None:
     """Causal attention of every token of the step over its request's pages.
 
     ``ctx`` carries ``positions`` and ``req_of_token`` ([T] int32), the step's shape on the host
@@ -445,7 +452,9 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
     (float32 [heads]: exp(sink) joins the softmax's denominator once), ``gate`` (float32
     [T, heads]: multiplies a head's output), ``softcap`` (c > 0: the scaled score s becomes c * tanh(s / c)),
     ``out_scale`` (a factor on every output, applied in float32 before the one rounding), ``chunk`` (C > 0: positions
-    are cut into chunks of C, counted from 0, and a token sees the keys of its own chunk only).
+    are cut into chunks of C, counted from 0, and a token sees the keys of its own chunk only), ``feature_gate``
+    (float32 [T, heads * value_dim], rows may lie apart; instead of ``gate``: feature i of the output is multiplied by
+    sigmoid(feature_gate[t, i]), in float32 before the one rounding).
     """
     _gpu(out, q, k_cache, v_cache, block_table, ctx.positions, ctx.req_of_token)
     chunk = int(chunk or 0)
@@ -456,6 +465,12 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
     softcap, out_scale = float(softcap or 0.0), float(out_scale)
     if softcap < 0.0:
         raise KernelError(f"attention: a cap on the scores must be positive, got {softcap}")
+    gate_stride = 0
+    if feature_gate is not None:
+        if gate is not None:
+            raise KernelError("attention: gates per head and per feature do not go together")
+        gate_stride, gate = _f32_rows(feature_gate, T, num_heads * vd, "attention gates"), feature_gate
+        _gpu(feature_gate)
     plain = value_dim is None and slopes is None and sinks is None and gate is None and softcap == 0.0 and out_scale == 1.0
     if plain:
         check_attention_sizes(num_heads, num_kv_heads, head_dim)
@@ -463,7 +478,8 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
         check_general_attention_sizes(num_heads, num_kv_heads, head_dim, vd)
         _f32_vector(slopes, num_heads, "attention slopes")
         _f32_vector(sinks, num_heads, "attention sinks")
-        _f32_vector(gate, T * num_heads, "attention gate")
+        if not gate_stride:
+            _f32_vector(gate, T * num_heads, "attention gate")
     if q.shape[1] != num_heads * head_dim or out.shape != (T, num_heads * vd) or out.dtype != q.dtype:
         raise KernelError(f"attention: q {tuple(q.shape)} / out {tuple(out.shape)} do not match {num_heads} x {head_dim} (values {vd})")
     pages = _check_cache(k_cache, v_cache, num_kv_heads, head_dim, page_size, q.dtype, vd)
@@ -477,7 +493,7 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
         # the matrix-core kernels take heads whose values are as wide as their keys, options included
         from . import fast
         if fast.paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_kv_heads, head_dim,
-                                page_size, scale, window, pages, ws, slopes, sinks, gate, softcap, out_scale, chunk):
+                                page_size, scale, window, pages, ws, slopes, sinks, gate, softcap, out_scale, chunk, gate_stride):
             return
     # a step of few tokens over long contexts: its keys cut into ranges, merged by a second kernel
     # (as many as the context-length bucket asks for, so that a step gives the same bits eagerly and replayed)
@@ -488,7 +504,7 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
               _rows(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), _dt(q), block_table.data_ptr(),
               block_table.shape[1], ctx.req_of_token.data_ptr(), ctx.positions.data_ptr(), T, num_heads,
               num_kv_heads, head_dim, page_size, float(scale), int(window), pages, ranges, _ptr(part),
-              0 if part is None else part.numel(), vd, _ptr(slopes), _ptr(sinks), _ptr(gate), softcap, out_scale, chunk, _stream())
+              0 if part is None else part.numel(), vd, _ptr(slopes), _ptr(sinks), _ptr(gate), gate_stride, softcap, out_scale, chunk, _stream())
 
 
 def general_attention_ranges(tokens: int, num_heads: int, max_kv_len: int) -> int:
@@ -617,33 +633,53 @@ def diff_combine(out: torch.Tensor, attn: torch.Tensor, lam: float, eps: float, 
               int(heads), int(kv_heads), int(value_dim), int(split), _stream())
 
 
-EPI_RELU2 = 5        # the matrix-core products' epilogue: max(c, 0)^2 rounded to bfloat16
+ACTIVATIONS = {"relu2": 0, "gelu": 1}     # of feed-forwards without a gate: max(z, 0)^2; z Phi(z), Phi the normal distribution function
 
 
-def gemm_relu_squared(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, ws: Optional[KernelWorkspace] = None) -> None:
-    """out[M, N] = max(a @ w^T, 0)^2, the square taken on the product's float32 result.  With bfloat16 operands and more
-    rows than the weight-streaming products take, product and activation are one kernel."""
+def _activation_kind(activation: str) -> int:
+    if activation not in ACTIVATIONS:
+        raise KernelError(f"activation '{activation}' is not known ({', '.join(sorted(ACTIVATIONS))})")
+    return ACTIVATIONS[activation]
+
+
+def gemm_activation(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, activation: str, ws: Optional[KernelWorkspace] = None) -> None:
+    """out[M, N] = activation(a @ w^T), taken on the product's float32 result.  With bfloat16 operands and more
+    rows than the weight-streaming products take, product and activation are one kernel; with fewer, the activation's
+    kernel adds the pieces of a product that was split over k."""
     _gpu(out, a, w)
+    _activation_kind(activation)
     M, N = out.shape
     if w.shape[0] != N or a.shape != (M, w.shape[1]):
-        raise KernelError(f"gemm_relu_squared: shapes do not agree: a {tuple(a.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
+        raise KernelError(f"gemm_activation: shapes do not agree: a {tuple(a.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
     if M == 0:
         return
     if _FAST and a.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and out.is_contiguous():
         from . import fast
-        if fast.gemm_relu_squared(out, a, w, M, N, a.shape[1], _rows(a, "gemm a"), _rows(w, "gemm w")):
+        if fast.gemm_activation(out, a, w, activation, M, N, a.shape[1], _rows(a, "gemm a"), _rows(w, "gemm w")):
             return
-    u = torch.empty((M, N), dtype=torch.float32, device=a.device)
-    gemm(u, a, w, ws=ws)
-    relu_squared(out, u)
+    activate(out, qkv_projection(a, w, torch.float32, ws), activation)
 
 
-def relu_squared(out: torch.Tensor, a: torch.Tensor) -> None:
-    """out = max(a, 0)^2 from float32 ``a`` into ``out`` (any type), squared before the one rounding."""
-    _gpu(out, a)
-    if a.dtype != torch.float32 or out.shape != a.shape or not (a.is_contiguous() and out.is_contiguous()):
-        raise KernelError("squared relu: expected a contiguous float32 input and an output of its shape")
-    _lib.call("core", "pi_relu_squared", out.data_ptr(), _dt(out), a.data_ptr(), a.numel(), _stream())
+def gemm_relu_squared(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, ws: Optional[KernelWorkspace] = None) -> None:
+    """out[M, N] = max(a @ w^T, 0)^2 (``gemm_activation``)."""
+    gemm_activation(out, a, w, "relu2", ws)
+
+
+def activate(out: torch.Tensor, a, activation: str) -> None:
+    """out = activation(a) from float32 ``a`` (a tensor, or ``Partials``: a product still split over k) into ``out``
+    (any type), taken before the one rounding."""
+    kind = _activation_kind(activation)
+    pieces = a if isinstance(a, Partials) else None
+    _gpu(out, pieces.part if pieces is not None else a)
+    if pieces is not None:
+        if tuple(out.shape) != (pieces.M, pieces.N) or not out.is_contiguous():
+            raise KernelError(f"activation: pieces [{pieces.M}, {pieces.N}] do not match the output {tuple(out.shape)}")
+        src, splits = pieces.part, pieces.splits
+    else:
+        if a.dtype != torch.float32 or out.shape != a.shape or not (a.is_contiguous() and out.is_contiguous()):
+            raise KernelError("activation: expected a contiguous float32 input and an output of its shape")
+        src, splits = a, 1
+    _lib.call("core", "pi_activation", out.data_ptr(), _dt(out), src.data_ptr(), out.numel(), splits, kind, _stream())
 
 
 def branch_norm_add(x: torch.Tensor, a: torch.Tensor, w_outer: torch.Tensor, eps: float, mult: float,
@@ -713,6 +749,43 @@ def qk_norm_kv_write(q_out: torch.Tensor, gate_out: Optional[torch.Tensor], proj
               _ptr(v_cache), _ptr(block_table), block_table.shape[1] if k_cache is not None else 0, page_size, pages,
               pieces.part.data_ptr() if pieces is not None else None, pieces.splits if pieces is not None else 0,
               pieces.M * pieces.N if pieces is not None else 0, int(bool(per_head)), int(bool(has_kv)), _stream())
+
+
+def qk_rope_norm_write(q_out: torch.Tensor, proj, bias: Optional[torch.Tensor], rotary, ctx, eps: float, num_heads: int, num_kv_heads: int,
+                       head_dim: int, num_gates: int, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                       page_size: int) -> Optional[torch.Tensor]:
+    """From float32 projection rows [q heads | k heads | gates] (a tensor, or ``Partials``), with ``bias`` (float32, one per
+    column of q and k, or None) added: queries and keys rotated (``rotary`` as for ``rope_kv_write``), then every head divided
+    by its root mean square, queries into ``q_out``, keys into their pages; the keys as projected, neither rotated nor
+    normalised, into the value pages.  Returns the gates' columns as they are, float32 [T, num_gates]: a view of a
+    projection that is a tensor, otherwise their pieces summed (None without gates)."""
+    pieces = proj if isinstance(proj, Partials) else None
+    _gpu(q_out, pieces.part if pieces is not None else proj, bias, k_cache, v_cache, block_table)
+    check_general_attention_sizes(num_heads, num_kv_heads, head_dim, head_dim)
+    T, QK = q_out.shape[0], (num_heads + num_kv_heads) * head_dim
+    if pieces is not None:
+        if pieces.M != T or pieces.N < QK + num_gates:
+            raise KernelError(f"qk rope norm: pieces [{pieces.M}, {pieces.N}] do not hold q, k and gates of {T} tokens")
+    else:
+        _f32_rows(proj, T, QK + num_gates, "qk rope norm projection")
+    if q_out.shape[1] != num_heads * head_dim:
+        raise KernelError(f"qk rope norm: q has {q_out.shape[1]} columns, expected {num_heads * head_dim}")
+    _f32_vector(bias, QK, "qk rope norm bias")
+    pages = _check_cache(k_cache, v_cache, num_kv_heads, head_dim, page_size, q_out.dtype)
+    if block_table.dim() != 2 or block_table.dtype != torch.int32 or not block_table.is_contiguous():
+        raise KernelError("qk rope norm: block table must be contiguous int32 [requests, width]")
+    _i32(ctx.positions, "positions", T)
+    _i32(ctx.req_of_token, "req_of_token", T)
+    table_ptr, rdim, inter, _keep = _rotary_args(rotary, ctx.positions, T)
+    gates = None
+    if num_gates:
+        gates = torch.empty((T, num_gates), dtype=torch.float32, device=q_out.device) if pieces is not None else proj[:, QK:QK + num_gates]
+    _lib.call("core", "pi_qk_rope_norm_write", q_out.data_ptr(), _rows(q_out, "q"), _dt(q_out), None if pieces is not None else proj.data_ptr(),
+              pieces.N if pieces is not None else _rows(proj, "projection"), pieces.part.data_ptr() if pieces is not None else None,
+              pieces.splits if pieces is not None else 0, _ptr(bias), table_ptr, rdim, int(bool(inter)), float(eps), T, num_heads, num_kv_heads,
+              head_dim, num_gates, _ptr(gates) if pieces is not None else None, ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(),
+              k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, pages, _stream())
+    return gates
 
 
 # ----------------------------------------------------------------------------- attention through a latent
@@ -862,21 +935,23 @@ def head_norm_gate(y: torch.Tensor, o: torch.Tensor, gates: torch.Tensor, weight
 
 # ----------------------------------------------------------------------------- routed experts
 def route(logits: torch.Tensor, top: int, groups: int = 1, keep: int = 1, renorm: bool = False,
-          correction: Optional[torch.Tensor] = None, renorm_eps: float = 0.0):
+          correction: Optional[torch.Tensor] = None, renorm_eps: float = 0.0, scoring: str = "softmax"):
     """Choose ``top`` experts per row of float32 router logits: (ids int32 [T, top], weights float32
-    [T, top]).  Scores are the softmax over all experts; with ``groups`` > 1 only experts of the
+    [T, top]).  Scores are the softmax over all experts, or (``scoring`` "sigmoid") every logit's own sigmoid; with ``groups`` > 1 only experts of the
     ``keep`` groups with the largest best score may be chosen; weights are the chosen scores
     (divided by their sum + ``renorm_eps`` when ``renorm``).  ``correction`` (float32 [E]): the choice goes
     by score + correction, the weights by the scores alone."""
     _gpu(logits, correction)
     T, E = logits.shape
+    if scoring not in ("softmax", "sigmoid"):
+        raise KernelError(f"routing: scores '{scoring}' are not known (softmax, sigmoid)")
     _f32_vector(correction, E, "routing correction")
     if logits.dtype != torch.float32:
         raise KernelError("routing: logits must be float32")
     ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _lib.call("core", "pi_route", ids.data_ptr(), weights.data_ptr(), logits.data_ptr(), _rows(logits, "router logits"), T, E,
-              int(top), int(groups), int(keep), int(bool(renorm)), _ptr(correction), float(renorm_eps), _stream())
+              int(top), int(groups), int(keep), int(bool(renorm)), _ptr(correction), float(renorm_eps), int(scoring == "sigmoid"), _stream())
     return ids, weights
 
 
@@ -917,18 +992,21 @@ def group_entries(ids: torch.Tensor, num_experts: int, tile: Optional[int] = Non
     return ExpertRows(row_entry, entry_row, te, t0, tr, ids.shape[1], tile)
 
 
-def gather_rows(src: torch.Tensor, rows: ExpertRows) -> torch.Tensor:
-    """The tokens' activations copied into expert order: [entries, D]."""
-    _gpu(src)
+def gather_rows(src: torch.Tensor, rows: ExpertRows, weights: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The tokens' activations copied into expert order: [entries, D].  ``weights`` (float32, one per entry): times the
+    entry's weight (float32 product, rounded once)."""
+    _gpu(src, weights)
+    if weights is not None:
+        _f32_vector(weights, rows.rows, "gather weights")
     if src.dim() != 2 or not src.is_contiguous():
         raise KernelError("gather: activations must be contiguous 2-D")
     out = torch.empty((rows.rows, src.shape[1]), dtype=src.dtype, device=src.device)
     _lib.call("core", "pi_gather_rows", out.data_ptr(), src.data_ptr(), _dt(src), rows.row_entry.data_ptr(), rows.rows, rows.top,
-              src.shape[1], _stream())
+              src.shape[1], _ptr(weights), _stream())
     return out
 
 
-def _grouped_fast(out, a, w, rows: ExpertRows, epilogue: int) -> bool:
+def _grouped_fast(out, a, w, rows: ExpertRows, epilogue: int, limit: float = 0.0, alpha: float = 0.0) -> bool:
     """The matrix-core grouped product, when the operands are what it takes."""
     if not (_FAST and a.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and _lib.build.MODULES["bf16"]):
         return False
@@ -939,7 +1017,7 @@ def _grouped_fast(out, a, w, rows: ExpertRows, epilogue: int) -> bool:
         return False
     _lib.call("bf16", "pi_gemm_mfma_grouped", out.data_ptr(), epilogue, _rows(out, "out"), a.data_ptr(), _rows(a, "a"), w.data_ptr(),
               K, w.shape[1] * K, rows.tile_expert.data_ptr(), rows.tile_row0.data_ptr(), rows.tile_rows.data_ptr(),
-              rows.tile_expert.numel(), w.shape[1], K, 0, 0, _stream())
+              rows.tile_expert.numel(), w.shape[1], K, 0, 0, float(limit), float(alpha), _stream())
     return True
 
 
@@ -976,6 +1054,24 @@ def grouped_gemm_swiglu(out: torch.Tensor, a: torch.Tensor, w_gate_up: torch.Ten
     swiglu(out, gu, block)
 
 
+def grouped_gemm_clamped_glu(out: torch.Tensor, a: torch.Tensor, w_gate_up: torch.Tensor, rows: ExpertRows, limit: float, alpha: float,
+                             block: int = 0) -> None:
+    """out[row] = the clamped gated unit (``clamped_glu``, no biases) of a[row] with the row's expert's matrices, laid out as
+    for ``grouped_gemm_swiglu``.  With bfloat16 operands and blocks of 16 product and unit are one kernel; otherwise the
+    product's float32 result goes through the unit's own kernel."""
+    _gpu(out, a, w_gate_up)
+    F2 = w_gate_up.shape[1]
+    if out.shape != (rows.rows, F2 // 2) or out.dtype != a.dtype:
+        raise KernelError(f"grouped clamped unit: out {tuple(out.shape)} does not match {rows.rows} x {F2 // 2}")
+    if rows.rows == 0:
+        return
+    if block == 16 and F2 % 32 == 0 and out.is_contiguous() and _grouped_fast(out, a, w_gate_up, rows, 4, limit, alpha):
+        return
+    gu = torch.empty((rows.rows, F2), dtype=torch.float32, device=a.device)
+    grouped_gemm(gu, a, w_gate_up, rows)
+    clamped_glu(out, gu, None, None, limit, alpha, block=block)
+
+
 def grouped_gemm_relu_squared(out: torch.Tensor, a: torch.Tensor, w_up: torch.Tensor, rows: ExpertRows) -> None:
     """out[row] = max(a[row] @ W^T, 0)^2 with the row's expert's matrix; ``w_up`` is [experts, F, K].  The square is taken on
     the product's float32 result."""
@@ -984,29 +1080,32 @@ def grouped_gemm_relu_squared(out: torch.Tensor, a: torch.Tensor, w_up: torch.Te
         raise KernelError(f"grouped squared relu: out {tuple(out.shape)} does not match {rows.rows} x {w_up.shape[1]}")
     if rows.rows == 0:
         return
-    if out.dtype == torch.bfloat16 and out.is_contiguous() and _grouped_fast(out, a, w_up, rows, EPI_RELU2):
+    if out.dtype == torch.bfloat16 and out.is_contiguous() and _grouped_fast(out, a, w_up, rows, 5):
         return
     u = torch.empty((rows.rows, w_up.shape[1]), dtype=torch.float32, device=a.device)
     grouped_gemm(u, a, w_up, rows)
-    relu_squared(out, u)
+    activate(out, u, "relu2")
 
 
-def combine_choices(out: torch.Tensor, y: torch.Tensor, weights: torch.Tensor, rows: ExpertRows, accumulate: bool = False,
+def combine_choices(out: torch.Tensor, y: torch.Tensor, weights: Optional[torch.Tensor], rows: ExpertRows, accumulate: bool = False,
                     ids: Optional[torch.Tensor] = None, num_real: int = 0, h: Optional[torch.Tensor] = None) -> None:
-    """out[t] (+)= sum over the token's choices of weight * y[row of (t, choice)], in choice order (float32).
+    """out[t] (+)= sum over the token's choices of weight * y[row of (t, choice)], in choice order (float32; ``weights``
+    None: a plain sum, without identity experts).
     With ``ids`` (int32 [T, top]), ``num_real`` and the tokens' activations ``h`` [T, D]: a choice whose id is
     ``num_real`` or more is an identity expert and contributes weight * h[t]."""
     _gpu(out, y, weights, ids, h)
     if ids is not None:
+        if weights is None:
+            raise KernelError("combine: identity experts need weights")
         _i32(ids, "expert ids", weights.numel())
         if h is None or h.shape != out.shape or not h.is_contiguous():
             raise KernelError("combine: identity experts need the tokens' activations, contiguous and as wide as the output")
     T, D = out.shape
     if out.dtype != torch.float32 or y.dtype != torch.float32 or not (out.is_contiguous() and y.is_contiguous()) or y.shape != (rows.rows, D):
         raise KernelError(f"combine: expected float32 out [{T}, {D}] and y [{rows.rows}, {D}]")
-    if weights.dtype != torch.float32 or not weights.is_contiguous() or weights.numel() != rows.rows:
+    if weights is not None and (weights.dtype != torch.float32 or not weights.is_contiguous() or weights.numel() != rows.rows):
         raise KernelError("combine: one float32 weight per entry is needed")
-    _lib.call("core", "pi_combine_choices", out.data_ptr(), y.data_ptr(), weights.data_ptr(), rows.entry_row.data_ptr(), T, rows.top, D,
+    _lib.call("core", "pi_combine_choices", out.data_ptr(), y.data_ptr(), _ptr(weights), rows.entry_row.data_ptr(), T, rows.top, D,
               int(bool(accumulate)), _ptr(ids), int(num_real), _ptr(h), _dt(h) if h is not None else PI_F32, _stream())
 
 
@@ -1151,19 +1250,25 @@ def delta_scan(o: torch.Tensor, qkv: torch.Tensor, a: torch.Tensor, dt_bias: tor
               kv_heads, key_dim, value_dim, float(q_scale), float(unit_eps), SCAN_KINDS[kind], float(tau), _stream())
 
 
-def clamped_glu(out: torch.Tensor, gate_up: torch.Tensor, gate_bias: torch.Tensor, up_bias: Optional[torch.Tensor], limit: float,
+def clamped_glu(out: torch.Tensor, gate_up: torch.Tensor, gate_bias: Optional[torch.Tensor], up_bias: Optional[torch.Tensor], limit: float,
                 alpha: float, x: Optional[torch.Tensor] = None, x_bias: Optional[torch.Tensor] = None, block: int = 0) -> None:
     """out = g * sigmoid(alpha * g) * (u + 1) with g = min(gate + gate_bias, limit) and
     u = clamp(up + up_bias, -limit, limit).  ``block`` = 0: ``gate_up`` [T, 2I] holds the two products in halves;
     ``block`` = b: gate and up interleaved in blocks of b columns, and ``gate_bias`` [2I] holds both biases in the
-    same order (``up_bias`` None).  With ``x`` (the float32 stream) and ``x_bias``: x[t, :] += x_bias as well, the
+    same order (``up_bias`` None).  No biases at all: both None.  With ``x`` (the float32 stream) and ``x_bias``: x[t, :] += x_bias as well, the
     bias of the product that follows."""
     _gpu(out, gate_up, gate_bias, up_bias, x, x_bias)
     T, I = out.shape
     if gate_up.shape != (T, 2 * I) or not (out.is_contiguous() and gate_up.is_contiguous()):
         raise KernelError(f"clamped unit: expected contiguous gate_up [{T}, {2 * I}], got {tuple(gate_up.shape)}")
-    if block < 0 or (block and (I % block or up_bias is not None or gate_bias.numel() != 2 * I)):
+    if block < 0 or (block and (I % block or up_bias is not None or (gate_bias is not None and gate_bias.numel() != 2 * I))):
         raise KernelError(f"clamped unit: interleave block {block} needs {I} % block == 0 and one bias vector of {2 * I}")
+    if gate_bias is None:
+        if up_bias is not None or x is not None:
+            raise KernelError("clamped unit: without the gate's biases there are no others")
+        _lib.call("core", "pi_clamped_glu", out.data_ptr(), _dt(out), gate_up.data_ptr(), _dt(gate_up), None, None, None, PI_F32, float(limit),
+                  float(alpha), T, I, None, 0, int(block), _stream())
+        return
     biases = [gate_bias] + ([up_bias] if not block else []) + ([x_bias] if x is not None else [])
     if any(b is None or b.dtype != gate_bias.dtype or not b.is_contiguous() for b in biases) or (not block and (gate_bias.numel() != I or up_bias.numel() != I)):
         raise KernelError(f"clamped unit: biases must be contiguous [{I}] of one type")
@@ -1218,3 +1323,92 @@ def gemm_clamped_glu(out: torch.Tensor, a: torch.Tensor, w_gate_up: torch.Tensor
         clamped_glu(out, gu, bias, None, limit, alpha, x, x_bias, block=block)
     else:
         clamped_glu(out, gu, bias[:I], bias[I:], limit, alpha, x, x_bias)
+
+
+# ----------------------------------------------------------------------------- several streams side by side
+HYPER_MAX_STREAMS = 16
+
+
+def hyper_streams(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, post: Optional[torch.Tensor] = None, h_dtype: Optional[torch.dtype] = None,
+                  read: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None, eps: float = 0.0,
+                  rows: Optional[torch.Tensor] = None, shift: Optional[torch.Tensor] = None, state: Optional[torch.Tensor] = None,
+                  ctx=None, ws: Optional[KernelWorkspace] = None) -> Optional[torch.Tensor]:
+    """The streams ``x`` (float32 [T, n, D]) around their sublayers; either half may be left out:
+
+    * ``y`` (float32 [T, D], a sublayer's result; when its product is still in pieces in ``ws`` they are added here) and
+      ``post`` (float32: out [n], then mix [n, n] by [from, to]): ``X_t <- sum_s mix[s, t] X_s + out[t] * y``;
+    * ``read`` (float32 [n]), ``norm`` (float32 [D]), ``eps`` and ``h_dtype``: returns ``h = rms(sum_s read[s] X_s) * norm``
+      of the new streams in that type - of the rows ``rows`` (int32) only, if given: the streams are then not
+      written back.
+
+    ``shift`` (float32 [D]) with ``state`` (float32 [slots, >= D]) and ``ctx``: h is moved towards the h of the request's token
+    before, ``h + (h_before - h) * shift``; the state row holds the h of the last token of the step before and takes this
+    step's last.  Shift and update together are for steps of single tokens."""
+    pieces = ws.take_result(y) if y is not None and ws is not None else None
+    _gpu(x, y, post, read, norm, rows, shift, state)
+    if x.dim() != 3 or x.dtype != torch.float32 or not x.is_contiguous():
+        raise KernelError(f"hyper streams: the streams must be contiguous float32 [T, n, D], got {x.dtype} {tuple(x.shape)}")
+    T, n, D = x.shape
+    if n > HYPER_MAX_STREAMS:
+        raise KernelError(f"hyper streams: {n} streams are more than {HYPER_MAX_STREAMS}")
+    if y is not None:
+        _f32_vector(post, n + n * n, "hyper streams mix")
+        if pieces is not None:
+            ws.counts["added_by_streams"] += 1
+            if (pieces.M, pieces.N) != (T, D):
+                raise KernelError(f"hyper streams: pieces [{pieces.M}, {pieces.N}] of a result [{T}, {D}]")
+        elif y.dtype != torch.float32 or not y.is_contiguous() or tuple(y.shape) != (T, D):
+            raise KernelError(f"hyper streams: the result must be contiguous float32 [{T}, {D}]")
+    h, M = None, T
+    if h_dtype is not None:
+        _f32_vector(read, n, "hyper streams reading weights")
+        _f32_vector(norm, D, "hyper streams norm weight")
+        if rows is not None:
+            M = rows.numel()
+            _i32(rows, "hyper streams rows", M)
+        h = torch.empty((M, D), dtype=h_dtype, device=x.device)
+    elif y is None:
+        raise KernelError("hyper streams: nothing to do")
+    if shift is not None:
+        _f32_vector(shift, D, "hyper streams shift")
+        _state_rows(state, D, "hyper streams")
+        _i32(ctx.q_start, "q_start", ctx.R + 1)
+        _i32(ctx.slots, "slots", ctx.R)
+        _i32(ctx.req_of_token, "req_of_token", T)
+    _lib.call("core", "pi_hyper_streams", x.data_ptr(), n, D, T, _ptr(y) if pieces is None else None, pieces.part.data_ptr() if pieces is not None else None,
+              pieces.splits if pieces is not None else 0, _ptr(post), int(rows is None), _ptr(h), _dt(h) if h is not None else PI_F32, _ptr(read), _ptr(norm),
+              float(eps), _ptr(rows), M, _ptr(shift), _ptr(state), state.stride(0) if state is not None else 0, state.shape[0] if state is not None else 0,
+              _ptr(ctx.q_start) if shift is not None else None, _ptr(ctx.slots) if shift is not None else None,
+              _ptr(ctx.req_of_token) if shift is not None else None, int(bool(getattr(ctx, "all_decode", False))) if shift is not None else 0, _stream())
+    return h
+
+
+def min_gru(out: torch.Tensor, proj, bias: torch.Tensor, ctx, state: torch.Tensor, width: int) -> None:
+    """The minGRU recurrence over the step's tokens, request by request, from and into the requests' state rows (``state``
+    float32 [slots, >= width], rows ``ctx.slots``): from float32 projection rows [z | u | gate] (a tensor, or ``Partials``)
+    and ``bias`` (float32: of z, then of u), ``S <- (1 - z) S + z c`` with ``z = sigmoid(z + bias)``, ``c = u`` + 1/2 where
+    ``u + bias`` >= 0 and its sigmoid below; ``out`` [T, width] = S * silu(gate) in any type."""
+    pieces = proj if isinstance(proj, Partials) else None
+    _gpu(out, pieces.part if pieces is not None else proj, bias, state)
+    T, W = out.shape[0], int(width)
+    if pieces is not None:
+        if pieces.M != T or pieces.N < 3 * W:
+            raise KernelError(f"min gru: pieces [{pieces.M}, {pieces.N}] do not hold three times {W} columns of {T} tokens")
+        stride = pieces.N
+    else:
+        stride = _f32_rows(proj, T, 3 * W, "min gru projection")
+    if out.dim() != 2 or out.shape[1] != W:
+        raise KernelError(f"min gru: output must be [{T}, {W}], got {tuple(out.shape)}")
+    _f32_vector(bias, 2 * W, "min gru bias")
+    _state_rows(state, W, "min gru")
+    _i32(ctx.q_start, "q_start", ctx.R + 1)
+    _i32(ctx.slots, "slots", ctx.R)
+    longest = int(getattr(ctx, "max_q_len", 0) or T)
+    lib = _lib.load("core")
+    lib.pi_min_gru_work_floats.restype = ctypes.c_long
+    floats = int(lib.pi_min_gru_work_floats(T, ctx.R, longest, W))
+    work = torch.empty(floats, dtype=torch.float32, device=out.device) if floats else None
+    _lib.call("core", "pi_min_gru", out.data_ptr(), _dt(out), _rows(out, "min gru out"), None if pieces is not None else proj.data_ptr(), stride,
+              pieces.part.data_ptr() if pieces is not None else None, pieces.splits if pieces is not None else 0, bias.data_ptr(),
+              ctx.q_start.data_ptr(), ctx.slots.data_ptr(), ctx.R, T, longest, state.data_ptr(), state.stride(0), state.shape[0], W, _ptr(work),
+              floats, _stream())

@@ -27,7 +27,6 @@ from . import _lib
 from .workspace import GEMM_PART_FLOATS, KernelWorkspace, KeyRanges, Partials, PendingUpdate
 
 EPI_BF16, EPI_F32, EPI_ACCUM, EPI_SWIGLU = 0, 1, 2, 3
-EPI_RELU2 = 5
 SKINNY_MAX_ROWS = 128          # up to this many tokens the weight-streaming kernels serve a product (measured against the tile kernel)
 ROWS_PER_BLOCK = 32            # weight rows per block of the skinny kernel
 BLOCKS_PER_UNIT = 2            # blocks of it wanted per compute unit to keep HBM busy (measured: 512 on 256 units; 384 and 768 are slower)
@@ -110,7 +109,7 @@ def flush(ws: Optional[KernelWorkspace]) -> None:
     if ws is None or ws.pending is None:
         return
     p, ws.pending = ws.pending, None
-    reduce_into(p.target, p.pieces, accumulate=True)
+    reduce_into(p.target, p.pieces, accumulate=p.accumulate)
     ws.counts["flushed"] += 1
 
 
@@ -186,7 +185,7 @@ def gemm(out, a, w, accumulate, M, N, K, lda, ldw, ldc, may_defer=False, ws: Opt
         # stay in the workspace for the next norm of this stream
         splits = _tile_splits(M, N, K) if may_defer else 1
         if splits > 1:
-            ws.pending = PendingUpdate(out, _tiles_in_pieces(a, w, M, N, K, lda, ldw, splits, ws))
+            ws.pending = PendingUpdate(out, _tiles_in_pieces(a, w, M, N, K, lda, ldw, splits, ws), accumulate)
             ws.counts["deferred"] += 1
             return True
         _lib.call("bf16", "pi_gemm_mfma", out.data_ptr(), epilogue, ldc, a.data_ptr(), lda, w.data_ptr(), ldw, M, N, K, 1,
@@ -195,7 +194,7 @@ def gemm(out, a, w, accumulate, M, N, K, lda, ldw, ldc, may_defer=False, ws: Opt
     pieces = _skinny(out.data_ptr(), epilogue, ldc, a, w, M, N, K, lda, ldw, _skinny_splits(M, N, K), ws)
     if pieces is not None:
         if may_defer:
-            ws.pending = PendingUpdate(out, pieces)          # the next norm of this stream adds them
+            ws.pending = PendingUpdate(out, pieces, accumulate)          # the next norm of this stream adds them
             ws.counts["deferred"] += 1
         else:
             _lib.call("bf16", "pi_splitk_reduce", out.data_ptr(), epilogue, ldc, pieces.part.data_ptr(), pieces.splits,
@@ -218,7 +217,7 @@ def ranges_product_ok(tokens: int, head_dim: int, weight_bytes: int = 0) -> bool
 def merge_ranges(out: torch.Tensor, kr: KeyRanges) -> None:
     """The merged attention output, bfloat16 [tokens, heads * head_dim], by the merging kernel."""
     _lib.call("bf16", "pi_attention_combine_rows", out.data_ptr(), out.stride(0), kr.rows.data_ptr(), kr.tokens,
-              kr.part.data_ptr(), kr.heads, kr.head_dim, kr.count, None, None, 1.0, _stream())
+              kr.part.data_ptr(), kr.heads, kr.head_dim, kr.count, None, None, 0, 1.0, _stream())
 
 
 def gemm_from_ranges(out, kr: KeyRanges, w, accumulate, N, ldw, ldc, may_defer, ws: Optional[KernelWorkspace]) -> bool:
@@ -249,7 +248,7 @@ def gemm_from_ranges(out, kr: KeyRanges, w, accumulate, N, ldw, ldc, may_defer, 
         if ws is not None:
             ws.counts["split_products"] += 1
         if may_defer and ws is not None:
-            ws.pending = PendingUpdate(out, pieces)
+            ws.pending = PendingUpdate(out, pieces, accumulate)
             ws.counts["deferred"] += 1
         else:
             _lib.call("bf16", "pi_splitk_reduce", out.data_ptr(), epilogue, ldc, pieces.part.data_ptr(), pieces.splits, M, N,
@@ -281,12 +280,15 @@ def gemm_pieces(a, w, ws: Optional[KernelWorkspace]) -> Optional[Partials]:
     return _skinny(0, EPI_F32, N, a, w, M, N, K, lda, ldw, splits, ws)
 
 
-def gemm_relu_squared(out, a, w, M, N, K, lda, ldw) -> bool:
-    """out [M, N] bfloat16 = max(a @ w^T, 0)^2 as the tile product's epilogue; only for more rows than the
+EPI_OF_ACTIVATION = {"relu2": 5, "gelu": 6}
+
+
+def gemm_activation(out, a, w, activation, M, N, K, lda, ldw) -> bool:
+    """out [M, N] bfloat16 = activation(a @ w^T) as the tile product's epilogue; only for more rows than the
     weight-streaming products take (those have no such epilogue)."""
     if not _gemm_ok(a, w, K, lda, ldw) or M <= SKINNY_MAX_ROWS:
         return False
-    _lib.call("bf16", "pi_gemm_mfma", out.data_ptr(), EPI_RELU2, out.stride(0), a.data_ptr(), lda, w.data_ptr(), ldw, M, N, K, 1,
+    _lib.call("bf16", "pi_gemm_mfma", out.data_ptr(), EPI_OF_ACTIVATION[activation], out.stride(0), a.data_ptr(), lda, w.data_ptr(), ldw, M, N, K, 1,
               _stream())
     return True
 
@@ -339,7 +341,7 @@ def head_gemm(out, a, w_rows, heads: int, K: int, N: int, a_head: int, out_head:
         return False
     group, row0, count = _head_tiles(M, heads, a.device)
     _lib.call("bf16", "pi_gemm_mfma_grouped", out.data_ptr(), EPI_BF16, ldc, a.data_ptr(), lda, w_rows.data_ptr(), K, N * K,
-              group.data_ptr(), row0.data_ptr(), count.data_ptr(), group.numel(), N, K, a_head, out_head, _stream())
+              group.data_ptr(), row0.data_ptr(), count.data_ptr(), group.numel(), N, K, a_head, out_head, 0.0, 0.0, _stream())
     return True
 
 
@@ -554,12 +556,14 @@ def _decode_splits_that_fit(ws, n_req: int, num_heads: int, num_kv_heads: int, h
 
 def paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_kv_heads, head_dim,
                     page_size, scale, window, pages, ws: Optional[KernelWorkspace] = None, slopes=None, sinks=None, gate=None,
-                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0) -> bool:
-    """``slopes`` / ``sinks`` (float32 [heads]) and ``gate`` (float32 [tokens, heads]): a distance bias, a sink in
-    the softmax and an output gate per head (None: none); ``softcap`` > 0: scaled scores s become
+                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0, gate_stride: int = 0) -> bool:
+    """``slopes`` / ``sinks`` (float32 [heads]) and ``gate`` (float32 [tokens, heads]; with ``gate_stride`` rows of one
+    unactivated gate per feature): a distance bias, a sink in the softmax and an output gate per head (None: none); ``softcap`` > 0: scaled scores s become
     softcap * tanh(s / softcap); ``out_scale``: a factor on every output."""
-    opt = tuple(None if t is None else t.data_ptr() for t in (slopes, sinks, gate)) + (float(softcap), float(out_scale), int(chunk))
+    opt = tuple(None if t is None else t.data_ptr() for t in (slopes, sinks, gate)) + (int(gate_stride), float(softcap), float(out_scale), int(chunk))
     if head_dim not in DECODE_HEAD_DIMS or page_size % 16 or q.data_ptr() % 16 or q.stride(0) % 8 or out.stride(0) % 4:
+        return False
+    if gate_stride and (gate_stride % 4 or gate.data_ptr() % 16):
         return False
     G = num_heads // num_kv_heads
     R = ctx.R
@@ -595,7 +599,7 @@ def paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_k
               num_kv_heads, head_dim, page_size, float(scale), int(window), pages, *opt, _stream())
     if plan.cut_tokens:
         _lib.call("bf16", "pi_attention_combine_rows", out.data_ptr(), out.stride(0), plan.rows.data_ptr(), plan.cut_tokens,
-                  tile_part.data_ptr(), num_heads, head_dim, plan.cuts, opt[1], opt[2], opt[4], _stream())
+                  tile_part.data_ptr(), num_heads, head_dim, plan.cuts, opt[1], opt[2], opt[3], opt[5], _stream())
     return True
 
 

@@ -51,10 +51,12 @@ class KeyRanges:
 
 @dataclass
 class PendingUpdate:
-    """``target += sum(pieces)`` that has not been applied yet."""
+    """``target += sum(pieces)`` (``accumulate`` False: ``target = sum(pieces)``, a sublayer's result that is still
+    in pieces) that has not been applied yet."""
 
     target: torch.Tensor
     pieces: Partials
+    accumulate: bool = True
 
     def is_for(self, x: torch.Tensor) -> bool:
         t = self.target
@@ -152,7 +154,15 @@ class KernelWorkspace:
     def take_pending(self, x: torch.Tensor) -> Optional[Partials]:
         """The pieces still to be added to ``x``, if any; they are the caller's to add."""
         p = self.pending
-        if p is not None and p.is_for(x):
+        if p is not None and p.accumulate and p.is_for(x):
+            self.pending = None
+            return p.pieces
+        return None
+
+    def take_result(self, y: torch.Tensor) -> Optional[Partials]:
+        """The pieces whose sum ``y`` is to hold, if they are still unadded (``y`` itself is then unwritten)."""
+        p = self.pending
+        if p is not None and not p.accumulate and p.is_for(y):
             self.pending = None
             return p.pieces
         return None

@@ -2,7 +2,7 @@
 from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, POSITION_ENCODINGS, Block, FeedForward,
                    KVCacheSpec, LayerCache, Mixer, Norm, PAGE, PagedCacheSpec, PagedTensor, Part, PositionEncoding, StateSpec,
                    StepContext)
-from .norm import LayerNorm, RMSNorm
+from .norm import LayerNorm, RMSNorm, StreamSumRMSNorm
 from .rope import RotaryEmbedding, rope_frequencies
 from .attention import PagedAttention
 from .sink_attention import SinkWindowAttention
@@ -12,9 +12,11 @@ from .state_space import StateSpaceMixer
 from .delta_rule import ChannelDeltaRule, GatedDeltaRule
 from .diff_attention import DifferentialAttention
 from .linear_attention import GatedLinearAttention
-from .mlp import ClampedGLU, SquaredReluMLP, SwiGLU
+from .min_gru import MinGRU
+from .token_shift import TokenShift
+from .mlp import ClampedGLU, GeluMLP, SquaredReluMLP, SwiGLU, UngatedMLP
 from .routed_experts import RoutedExperts
-from .block import OutputNormBlock, PreNormBlock, SandwichBlock, SideBySide
+from .block import HyperConnectionBlock, HyperConnections, OutputNormBlock, PreNormBlock, SandwichBlock, SideBySide
 from .embedding import LMHead, PositionedEmbedding, TokenEmbedding
 from .model import CachePlan, DecoderModel, ModelSpec, RunEntry, plan_cache
 
@@ -25,4 +27,5 @@ __all__ = [
     "PreNormBlock", "OutputNormBlock", "SinkWindowAttention", "MatrixMemory", "RoutedExperts", "LMHead", "TokenEmbedding", "CachePlan", "DecoderModel", "ModelSpec",
     "RunEntry", "plan_cache", "StateSpaceMixer", "ChannelDeltaRule", "ClampedGLU", "SideBySide", "PositionedEmbedding", "LatentAttention",
     "LayerNorm", "GatedDeltaRule", "DifferentialAttention", "GatedLinearAttention", "SquaredReluMLP", "SandwichBlock",
+    "StreamSumRMSNorm", "MinGRU", "TokenShift", "UngatedMLP", "GeluMLP", "HyperConnections", "HyperConnectionBlock",
 ]

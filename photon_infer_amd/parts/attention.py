@@ -22,6 +22,12 @@ its one rounding, so that the output projection needs no second pass), other ten
 q, k and v projections (``qkv_bias``) and on the output projection (``o_bias``; tensor names with ``bias_suffix``
 added; added in float32, the first three before the rotation), and ``accumulate`` False: the result is written into the
 tensor handed to ``forward`` instead of added to it.
+
+``values_are_keys``: there is no v projection; a token's values are its keys as projected (with their bias), before the
+rotation and any norm.  ``head_norm_eps``: after the rotation every head of q and k is divided by the root mean square
+of its entries (this eps inside the root, no weight).  ``feature_gate`` names a matrix [heads * value_dim, hidden]: the
+concatenated heads are multiplied, feature by feature, with ``sigmoid(W h)`` before the output projection, in float32
+before the one rounding.  The three come together (one kernel makes queries, keys and values from the projection).
 """
 from __future__ import annotations
 
@@ -37,6 +43,10 @@ from .base import MIXERS, PAGE, KVCacheSpec, LayerCache, Mixer, PagedCacheSpec, 
 
 
 POSITION_PREFIX = "position."
+
+
+def position_is_rotation(position: Optional[PositionEncoding]) -> bool:
+    return position is None or type(position).rotary_params is not PositionEncoding.rotary_params
 
 
 class PagedAttention(Mixer):
@@ -60,6 +70,9 @@ class PagedAttention(Mixer):
         bias_suffix: str = ".b",
         accumulate: bool = True,
         bias_to_caller: bool = False,
+        values_are_keys: bool = False,
+        head_norm_eps: Optional[float] = None,
+        feature_gate: Optional[str] = None,
     ):
         self.hidden_size = int(hidden_size)
         self.num_heads = int(num_heads)
@@ -78,6 +91,12 @@ class PagedAttention(Mixer):
         # and adds it in a pass of its own (an arrangement that normalises the result anyway)
         self.bias_to_caller = bool(bias_to_caller) and self.o_bias
         self.pending_bias: Optional[torch.Tensor] = None
+        self.values_are_keys, self.feature_gate = bool(values_are_keys), feature_gate
+        self.head_norm_eps = float(head_norm_eps) if head_norm_eps is not None else None
+        if not self.values_are_keys == (self.head_norm_eps is not None) == (self.feature_gate is not None):
+            raise UnsupportedModelError("attention: values that are keys, a norm per head and gates per feature are served together")
+        if self.values_are_keys and not (self.own_kv and self.value_dim == self.head_dim and position_is_rotation(position)):
+            raise UnsupportedModelError("attention: values that are keys need keys of the layer's own, as wide, with a rotation or no positions")
         self.q_size = self.num_heads * self.head_dim
         self.kv_size = self.num_kv_heads * self.head_dim
         self.v_size = self.num_kv_heads * self.value_dim
@@ -96,11 +115,14 @@ class PagedAttention(Mixer):
         if self.own_kv:
             specs += [
                 TensorSpec(self.names[1], (self.kv_size, self.hidden_size)),
-                TensorSpec(self.names[2], (self.v_size, self.hidden_size)),
             ]
+            if not self.values_are_keys:
+                specs.append(TensorSpec(self.names[2], (self.v_size, self.hidden_size)))
+        if self.feature_gate is not None:
+            specs.append(TensorSpec(self.feature_gate, (self.o_size, self.hidden_size)))
         specs.append(TensorSpec(self.names[3], (self.hidden_size, self.o_size)))
         if self.qkv_bias:
-            sizes = [self.q_size] + ([self.kv_size, self.v_size] if self.own_kv else [])
+            sizes = [self.q_size] + ([self.kv_size] if self.own_kv else []) + ([self.v_size] if self.own_kv and not self.values_are_keys else [])
             specs += [TensorSpec(n + self.bias_suffix, (size,), "small_bias") for n, size in zip(self.names, sizes)]
         if self.o_bias:
             specs.append(TensorSpec(self.names[3] + self.bias_suffix, (self.hidden_size,), "small_bias"))
@@ -121,7 +143,7 @@ class PagedAttention(Mixer):
         return self.position is None or bool(self.position.graph_safe)
 
     def step_planner(self, page_size: int):
-        if self.value_dim != self.head_dim:      # only the general kernel takes such heads; it needs no work lists
+        if self.value_dim != self.head_dim or self.head_dim % 16:      # only the general kernel takes such heads; it needs no work lists
             return None
         return ops.attention_planner(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim, page_size,
                                      self.window or 0, self.device)
@@ -130,14 +152,19 @@ class PagedAttention(Mixer):
         super().load(tensors, dtype, device)
         mats = [tensors[self.names[0]]]
         if self.own_kv:
-            mats += [tensors[self.names[1]], tensors[self.names[2]]]
-        # one projection for q, k and v: rows [q heads | k heads | v heads]
+            mats.append(tensors[self.names[1]])
+            if not self.values_are_keys:
+                mats.append(tensors[self.names[2]])
+        biased = len(mats)
+        if self.feature_gate is not None:
+            mats.append(tensors[self.feature_gate])
+        # one projection for q, k and v (and gates): rows [q heads | k heads | v heads | gates]
         common = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
         self.w_qkv = torch.cat([m.to(common) for m in mats], dim=0).contiguous()
         self.w_o = tensors[self.names[3]]
         self.b_qkv = self.b_o = None
         if self.qkv_bias:
-            self.b_qkv = torch.cat([tensors[n + self.bias_suffix].to(torch.float32) for n in self.names[:len(mats)]]).contiguous()
+            self.b_qkv = torch.cat([tensors[n + self.bias_suffix].to(torch.float32) for n in self.names[:biased]]).contiguous()
         if self.o_bias:
             self.b_o = tensors[self.names[3] + self.bias_suffix].to(torch.float32).contiguous()
             self.pending_bias = self.b_o if self.bias_to_caller else None
@@ -155,6 +182,9 @@ class PagedAttention(Mixer):
         fused_position = self.position is None or rotary is not None
         table = ctx.block_tables[cache.group]
         ws = ctx.workspace
+        if self.values_are_keys:
+            self._forward_values_are_keys(h, x, ctx, cache, rotary, table)
+            return
         if self.qkv_bias:
             if not fused_position:
                 raise UnsupportedModelError("biased projections go with a rotation (or none), not with another position encoding")
@@ -213,6 +243,20 @@ class PagedAttention(Mixer):
         # where the arrangement allows it, the product stays in pieces for the stream's next reader
         ops.gemm(x, attn, self.w_o, accumulate=self.accumulate,
                  may_defer=self.accumulate and not self.o_bias and getattr(ctx, "may_defer", False), ws=ws)
+        if self.o_bias and not self.bias_to_caller:
+            ops.add_row_bias(x, self.b_o)
+
+    def _forward_values_are_keys(self, h, x, ctx, cache, rotary, table) -> None:
+        T, ws = h.shape[0], ctx.workspace
+        # float32 results (a tensor, or the pieces of a product split over k): rounded once, behind the norm
+        proj = ops.qkv_projection(h, self.w_qkv, torch.float32, ws)
+        q = torch.empty((T, self.q_size), dtype=self.dtype, device=h.device)
+        gates = ops.qk_rope_norm_write(q, proj, self.b_qkv, rotary, ctx, self.head_norm_eps, self.num_heads, self.num_kv_heads, self.head_dim,
+                                       self.o_size, cache.k, cache.v, table, cache.page_size)
+        attn = torch.empty((T, self.o_size), dtype=self.dtype, device=h.device)
+        ops.paged_attention(attn, q, cache.k, cache.v, table, ctx, self.num_heads, self.num_kv_heads, self.head_dim, cache.page_size, self.scale,
+                            self.window or 0, ws, softcap=self.softcap, out_scale=self.out_scale, feature_gate=gates)
+        ops.gemm(x, attn, self.w_o, accumulate=self.accumulate, may_defer=not self.o_bias and getattr(ctx, "may_defer", False), ws=ws)
         if self.o_bias and not self.bias_to_caller:
             ops.add_row_bias(x, self.b_o)
 

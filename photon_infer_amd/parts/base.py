@@ -226,8 +226,9 @@ class Block(Part):
     reads_deferred = False     # True: the block's first reader of the stream is a norm that adds pending pieces
 
     def mixers(self) -> List[Mixer]:
-        """The block's mixers, each with a cache or state of its own.  With more than one,
-        ``forward`` receives a list of ``LayerCache`` in this order instead of a single one."""
+        """The block's mixers - and other parts of it that keep something per request (they have a mixer's
+        ``cache_spec`` and ``step_planner``) - each with a cache or state of its own.  With more than one, ``forward``
+        receives a list of ``LayerCache`` in this order instead of a single one."""
         m = getattr(self, "mixer", None)
         return [m] if m is not None else []
 

@@ -14,6 +14,8 @@ from .. import ops
 from ..errors import UnsupportedModelError
 from ..weights.loader import TensorSpec
 from .base import BLOCKS, MIXERS, Block, FeedForward, LayerCache, Mixer, Norm, Part, StepContext
+from .norm import LEFT_UPDATE
+from .token_shift import TokenShift
 
 
 class SideBySide(Mixer):
@@ -281,3 +283,109 @@ class SandwichBlock(Block):
 
 
 BLOCKS.register("sandwich", SandwichBlock)
+
+
+class HyperConnections(Part):
+    """How one sublayer is tied to several residual streams side by side (hyper-connections; Zhu et al.,
+    "Hyper-Connections"): it reads ``u = sum_s in[s] X_s``, and its result y joins all streams at once,
+    ``X_t <- sum_s mix[s, t] X_s + out[t] y`` (mix is indexed [from, to])."""
+
+    graph_safe = True
+
+    def __init__(self, streams: int):
+        self.streams = int(streams)
+        if not 0 < self.streams <= ops.HYPER_MAX_STREAMS:
+            raise UnsupportedModelError(f"{self.streams} residual streams (1 to {ops.HYPER_MAX_STREAMS} are served)")
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        n = self.streams
+        return [TensorSpec("in", (n,), "norm"), TensorSpec("out", (n,), "norm"), TensorSpec("mix", (n, n), "near_identity")]
+
+    def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
+        super().load(tensors, dtype, device)
+        f32 = lambda name: tensors[name].to(torch.float32).reshape(-1)
+        self.read = f32("in").contiguous()
+        self.post = torch.cat([f32("out"), f32("mix")]).contiguous()      # as the kernel takes them
+
+
+class HyperConnectionBlock(Block):
+    """Pre-norm sublayers on several residual streams side by side (the stream is [T, streams, D]); what the mixer reads
+    may be shifted towards the token before (``TokenShift``):
+
+        h = rms(sum_s in1[s] X_s; norm1), shifted;   X_t <- sum_s mix1[s, t] X_s + out1[t] * mixer(h)
+        h = rms(sum_s in2[s] X_s; norm2);            X_t <- sum_s mix2[s, t] X_s + out2[t] * ffn(h)     (no feed-forward: the first only)
+
+    The mixer and the feed-forward write their result (``accumulate=False``), or leave it in the pieces of its product.
+    The update by the mixer's result and the feed-forward's h are one kernel.  In a step of single tokens the update by
+    the feed-forward's result is left to the next reader of the streams (the next block's first kernel, or the final
+    norm); in other steps the token before belongs to another block of threads, and the update is a kernel of its own.
+
+    ``norm1`` / ``mixer`` / ``norm2`` / ``ffn``: (prefix, part); ``shift``: the name of the shift's tensor, or None;
+    ``connections``: the prefixes of the two sublayers' ``HyperConnections``."""
+
+    reads_deferred = False
+
+    def __init__(self, hidden_size: int, streams: int, norm1: Tuple[str, Norm], mixer: Tuple[str, Mixer], shift: Optional[str] = None,
+                 norm2: Optional[Tuple[str, Norm]] = None, ffn: Optional[Tuple[str, FeedForward]] = None, connections=("hc1.", "hc2.")):
+        if (ffn is None) != (norm2 is None):
+            raise UnsupportedModelError("a feed-forward and its norm come together")
+        for part in [mixer[1]] + ([ffn[1]] if ffn is not None else []):
+            if getattr(part, "accumulate", True):
+                raise UnsupportedModelError(f"{type(part).__name__} must be built with accumulate=False between streams side by side")
+        self.norm1, self.mixer = norm1[1], mixer[1]
+        self.norm2, self.ffn = (norm2[1], ffn[1]) if ffn is not None else (None, None)
+        self.shift = TokenShift(hidden_size, tensor_name="") if shift is not None else None
+        self.hc1, self.hc2 = HyperConnections(streams), HyperConnections(streams) if ffn is not None else None
+        self._named: List[Tuple[str, Part]] = [norm1, mixer, (connections[0], self.hc1)]
+        if shift is not None:
+            self._named.append((shift, self.shift))
+        if ffn is not None:
+            self._named += [norm2, ffn, (connections[1], self.hc2)]
+
+    def mixers(self) -> List[Part]:
+        return [self.mixer] + ([self.shift] if self.shift is not None else [])
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [s.with_prefix(p) for p, part in self._named for s in part.tensor_specs()]
+
+    def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
+        super().load(tensors, dtype, device)
+        for prefix, part in self._named:
+            names = [prefix + s.name for s in part.tensor_specs()]
+            part.load({n[len(prefix):]: tensors[n] for n in names}, dtype, device)
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(part.graph_safe for _, part in self._named)
+
+    def streamed_weights(self) -> List[torch.Tensor]:
+        return [w for _, part in self._named for w in part.streamed_weights()]
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache) -> None:
+        caches = cache if isinstance(cache, (list, tuple)) else [cache]
+        ws = ctx.workspace
+        left = ctx.scratch.pop(LEFT_UPDATE, None)
+        y, post = (left[1], left[2]) if left is not None and left[0] is x else (None, None)
+        if y is not None and not ctx.all_decode:      # an update and a shift in one kernel are for single tokens
+            ops.hyper_streams(x, y=y, post=post, ws=ws)
+            y = post = None
+        shift, state = (self.shift.share, caches[1].state) if self.shift is not None else (None, None)
+        h = ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.hc1.read, norm=self.norm1.weight_f32(), eps=self.norm1.eps,
+                              shift=shift, state=state, ctx=ctx, ws=ws)
+        result = lambda: torch.empty((x.shape[0], x.shape[2]), dtype=torch.float32, device=x.device)
+        y, post = result(), self.hc1.post
+        ctx.may_defer = True                          # the next kernel on the streams adds a product's pieces
+        self.mixer.forward(h, y, ctx, caches[0])
+        if self.ffn is not None:
+            h = ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.hc2.read, norm=self.norm2.weight_f32(), eps=self.norm2.eps,
+                                  ctx=ctx, ws=ws)
+            y, post = result(), self.hc2.post
+            self.ffn.forward(h, y, ctx)
+        ctx.may_defer = False
+        if ctx.all_decode:
+            ctx.scratch[LEFT_UPDATE] = (x, y, post)
+        else:
+            ops.hyper_streams(x, y=y, post=post, ws=ws)
+
+
+BLOCKS.register("hyper_connections", HyperConnectionBlock)

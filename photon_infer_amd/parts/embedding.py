@@ -19,9 +19,12 @@ from .base import Part
 class TokenEmbedding(Part):
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, tensor_name: str = "weight", scale: float = 1.0):
+    def __init__(self, vocab_size: int, hidden_size: int, tensor_name: str = "weight", scale: float = 1.0, copies: int = 0):
+        """``copies`` > 0: the stream is so many equal copies of the row, [T, copies, hidden] (for arrangements that keep
+        several streams side by side); 0: one stream, [T, hidden]."""
         self.vocab_size = int(vocab_size)
         self.hidden_size = int(hidden_size)
+        self.copies = int(copies)
         self.tensor_name = tensor_name          # after the part's prefix; may be empty
         self.scale = float(scale)               # a factor on every row as it enters the stream (the table itself stays as stored)
         self.weight: Optional[torch.Tensor] = None
@@ -34,9 +37,10 @@ class TokenEmbedding(Part):
         self.weight = tensors[self.tensor_name]
 
     def forward(self, token_ids: torch.Tensor, ctx=None) -> torch.Tensor:
-        """int32 [T] -> float32 residual stream [T, hidden].  ``ctx``: the step's context, for
+        """int32 [T] -> float32 residual stream [T, hidden] ([T, copies, hidden]).  ``ctx``: the step's context, for
         embeddings that look at more than the ids."""
-        x = torch.empty((token_ids.shape[0], self.hidden_size), dtype=torch.float32, device=token_ids.device)
+        shape = (token_ids.shape[0], self.copies, self.hidden_size) if self.copies else (token_ids.shape[0], self.hidden_size)
+        x = torch.empty(shape, dtype=torch.float32, device=token_ids.device)
         ops.embedding(x, self.weight, token_ids, self.scale)
         return x
 

@@ -135,15 +135,18 @@ class ClampedGLU(FeedForward):
 FEED_FORWARDS.register("clamped_glu", ClampedGLU)
 
 
-class SquaredReluMLP(FeedForward):
-    """A feed-forward without a gate: ``y = W_down act(W_up h)`` with ``act(z) = max(z, 0)^2``, no biases.  The square
-    is taken on the product's float32 result, before the one rounding.  ``accumulate`` False: the result is written
-    into the tensor handed to ``forward`` instead of added to it."""
+class UngatedMLP(FeedForward):
+    """A feed-forward without a gate: ``y = W_down act(W_up h)``, no biases; ``act`` is taken on the product's float32
+    result, before the one rounding.  ``activation``: "relu2", ``max(z, 0)^2``, or "gelu", the exact ``z Phi(z)`` with Phi
+    the normal distribution function.  ``accumulate`` False: the result is written into the tensor handed to
+    ``forward`` instead of added to it."""
 
     graph_safe = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int, names=("up", "down"), accumulate: bool = True):
-        self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str, names=("up", "down"), accumulate: bool = True):
+        if activation not in ops.ACTIVATIONS:
+            raise UnsupportedModelError(f"feed-forward activation '{activation}' is not supported ({', '.join(sorted(ops.ACTIVATIONS))})")
+        self.hidden_size, self.intermediate_size, self.activation = int(hidden_size), int(intermediate_size), activation
         self.names, self.accumulate = tuple(names), bool(accumulate)
 
     def tensor_specs(self) -> List[TensorSpec]:
@@ -160,9 +163,19 @@ class SquaredReluMLP(FeedForward):
     def forward(self, h: torch.Tensor, x: torch.Tensor, ctx: StepContext) -> None:
         ws = ctx.workspace if ctx is not None else None
         act = torch.empty((h.shape[0], self.intermediate_size), dtype=self.dtype, device=h.device)
-        ops.gemm_relu_squared(act, h, self.w_up, ws=ws)
-        ops.gemm(x, act, self.w_down, accumulate=self.accumulate,
-                 may_defer=self.accumulate and getattr(ctx, "may_defer", False), ws=ws)
+        ops.gemm_activation(act, h, self.w_up, self.activation, ws=ws)
+        ops.gemm(x, act, self.w_down, accumulate=self.accumulate, may_defer=getattr(ctx, "may_defer", False), ws=ws)
+
+
+class SquaredReluMLP(UngatedMLP):
+    def __init__(self, hidden_size: int, intermediate_size: int, names=("up", "down"), accumulate: bool = True):
+        super().__init__(hidden_size, intermediate_size, "relu2", names, accumulate)
+
+
+class GeluMLP(UngatedMLP):
+    def __init__(self, hidden_size: int, intermediate_size: int, names=("up", "down"), accumulate: bool = True):
+        super().__init__(hidden_size, intermediate_size, "gelu", names, accumulate)
 
 
 FEED_FORWARDS.register("squared_relu_mlp", SquaredReluMLP)
+FEED_FORWARDS.register("gelu_mlp", GeluMLP)

@@ -16,6 +16,11 @@ from ..weights.loader import TensorSpec
 from .base import NORMS, Norm
 
 
+# Key in a step's ``scratch``: (streams, a sublayer's result, the numbers it joins them by) - an update of streams that run
+# side by side, left to whoever reads them next.
+LEFT_UPDATE = "update of the streams left to their next reader"
+
+
 class RMSNorm(Norm):
     consumes_deferred = True   # reads the stream through ops.rmsnorm, which adds a pending update
     graph_safe = True
@@ -53,6 +58,31 @@ class RMSNorm(Norm):
 
 
 NORMS.register("rmsnorm", RMSNorm)
+
+
+class StreamSumRMSNorm(RMSNorm):
+    """The RMS norm of the sum of several streams that run side by side (``x`` is [T, streams, D]), read from them in the
+    norm's own pass.  An update that a block of such streams has left to the next reader (``HyperConnectionBlock``) is
+    applied on the way."""
+
+    consumes_deferred = False
+
+    def __init__(self, dim: int, eps: float, streams: int, offset: float = 0.0, tensor_name: str = "weight"):
+        super().__init__(dim, eps, offset, tensor_name)
+        self.streams = int(streams)
+
+    def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
+        super().load(tensors, dtype, device)
+        self.ones = torch.ones(self.streams, dtype=torch.float32, device=device)
+
+    def forward(self, x: torch.Tensor, ctx=None, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        left = ctx.scratch.pop(LEFT_UPDATE, None) if ctx is not None else None
+        y, post = (left[1], left[2]) if left is not None and left[0] is x else (None, None)
+        return ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.ones, norm=self.weight_f32(), eps=self.eps, rows=rows,
+                                 ctx=ctx, ws=ctx.workspace if ctx is not None else None)
+
+
+NORMS.register("stream_sum_rmsnorm", StreamSumRMSNorm)
 
 
 class LayerNorm(Norm):

@@ -5,13 +5,16 @@ Router logits ``z = Wr h`` in float32; scores ``s = softmax(z)`` over all expert
 experts of the ``keep`` best groups can be chosen.  Each token uses the ``top`` allowed experts
 with the largest scores, weighted by those scores as they are (``renormalize``: divided by
 their sum plus ``renorm_eps``).  An expert is a gated feed-forward ``Wdown (silu(Wgate h) * (Wup h))`` without
-biases (``activation`` "silu"), or ``Wdown max(Wup h, 0)^2`` (``activation`` "relu2": no gate matrix); the result is
+biases (``activation`` "silu"), or ``Wdown max(Wup h, 0)^2`` (``activation`` "relu2": no gate matrix), or the clamped
+gated unit of ``ClampedGLU`` without biases (``activation`` "clamped_glu", with ``limit`` and ``alpha``); the result is
 the weighted sum of the chosen experts' outputs (float32).
 
 Further options, each a constructor parameter: ``correction`` (a tensor of one number per router output that is
 added to the scores for the choice only; the weights stay the scores), ``identity`` (so many identity experts, which take
 the last places among the router's outputs, own no matrices and contribute ``weight * h``), and ``shared``
-((prefix, feed-forward): one more feed-forward that every token goes through, added to the routed sum).
+((prefix, feed-forward): one more feed-forward that every token goes through, added to the routed sum), ``scoring``
+"sigmoid" (an expert's score is its own logit's sigmoid instead of a share of the softmax), and ``weigh_input`` (the weight
+multiplies what the expert reads instead of what it gives: the sum of ``expert(weight * h)``).
 
 The step's (token, choice) entries are sorted by expert on the device and each expert's rows go
 through grouped products; nothing is counted on the host.
@@ -33,10 +36,16 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, groups: int = 1, keep: int = 1,
                  renormalize: bool = False, activation: str = "silu", accumulate: bool = True,
                  expert_prefix: str = "e", names=("gate", "up", "down"), router_name: str = "router", identity: int = 0,
-                 correction: str = "", renorm_eps: float = 0.0, shared=None):
-        if activation not in ("silu", "relu2"):
-            raise UnsupportedModelError(f"expert activation '{activation}' is not supported (silu, relu2)")
-        self.gated = activation == "silu"
+                 correction: str = "", renorm_eps: float = 0.0, shared=None, scoring: str = "softmax", weigh_input: bool = False,
+                 limit: float = 0.0, alpha: float = 1.702):
+        if activation not in ("silu", "relu2", "clamped_glu"):
+            raise UnsupportedModelError(f"expert activation '{activation}' is not supported (silu, relu2, clamped_glu)")
+        if activation == "clamped_glu" and not limit > 0.0:
+            raise UnsupportedModelError(f"routed experts: a clamped unit needs a positive limit, got {limit}")
+        self.gated, self.activation = activation != "relu2", activation
+        self.scoring, self.weigh_input, self.limit, self.alpha = scoring, bool(weigh_input), float(limit), float(alpha)
+        if self.weigh_input and identity:
+            raise UnsupportedModelError("routed experts: weights on the experts' inputs and identity experts do not go together")
         self.identity, self.correction_name, self.renorm_eps = int(identity), correction, float(renorm_eps)
         self.shared_prefix, self.shared = shared if shared is not None else ("", None)
         if self.identity < 0:
@@ -111,11 +120,14 @@ class RoutedExperts(FeedForward):
         T, ws = h.shape[0], ctx.workspace if ctx is not None else None
         logits = torch.empty((T, self.router_size), dtype=torch.float32, device=h.device)
         ops.gemm(logits, h, self.w_router, ws=ws)
-        ids, weights = ops.route(logits, self.top, self.groups, self.keep, self.renormalize, self.correction, self.renorm_eps)
+        ids, weights = ops.route(logits, self.top, self.groups, self.keep, self.renormalize, self.correction, self.renorm_eps,
+                                 self.scoring)
         rows = ops.group_entries(ids, self.num_experts, self.tile)
-        a = ops.gather_rows(h, rows)
+        a = ops.gather_rows(h, rows, weights.view(-1) if self.weigh_input else None)
         act = torch.empty((rows.rows, self.expert_size), dtype=self.dtype, device=h.device)
-        if self.gated:
+        if self.activation == "clamped_glu":
+            ops.grouped_gemm_clamped_glu(act, a, self.w_gate_up, rows, self.limit, self.alpha, self.interleave)
+        elif self.gated:
             ops.grouped_gemm_swiglu(act, a, self.w_gate_up, rows, self.interleave)
         else:
             ops.grouped_gemm_relu_squared(act, a, self.w_up, rows)
@@ -126,7 +138,7 @@ class RoutedExperts(FeedForward):
         if self.identity:
             ops.combine_choices(x, y, weights, rows, accumulate=self.accumulate, ids=ids, num_real=self.num_experts, h=h)
         else:
-            ops.combine_choices(x, y, weights, rows, accumulate=self.accumulate)
+            ops.combine_choices(x, y, None if self.weigh_input else weights, rows, accumulate=self.accumulate)
         if self.shared is not None:
             may_defer, ctx.may_defer = ctx.may_defer, False
             self.shared.forward(h, x, ctx)

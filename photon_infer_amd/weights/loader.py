@@ -29,7 +29,8 @@ class TensorSpec:
 
     ``role`` drives random initialisation only: "matrix" and "table" are drawn from
     N(0, std), "norm" follows the norm rule (ones or U(0.5, 1.5)), "norm_zero" the same
-    around zero (zeros or U(-0.5, 0.5)), "bias" is N(0, 1), "int_table" holds integers.
+    around zero (zeros or U(-0.5, 0.5)), "bias" is N(0, 1), "share" U(0, 1), "near_identity" the unit
+    matrix plus N(0, 0.2), "int_table" holds integers.
     """
 
     name: str

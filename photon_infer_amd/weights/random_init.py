@@ -44,6 +44,10 @@ def random_tensors(specs: Iterable[TensorSpec], seed: int, std: float = 0.02, no
             t = torch.randn(s.shape, generator=g, dtype=torch.float32) * 0.1
         elif s.role == "taps":           # a short convolution's weights: of order one, so that earlier inputs count
             t = torch.randn(s.shape, generator=g, dtype=torch.float32) * 0.5
+        elif s.role == "share":          # a share between two things, per feature
+            t = torch.rand(s.shape, generator=g)
+        elif s.role == "near_identity":  # a small square matrix that mixes a little
+            t = torch.eye(s.shape[0]) + torch.randn(s.shape, generator=g, dtype=torch.float32) * 0.2
         elif s.role == "int_table":
             out[s.name] = torch.randint(0, 2**15, s.shape, generator=g, dtype=torch.int32)
             continue
