@@ -1,7 +1,7 @@
 #!/usr/bin/python3
 """Decode and prefill throughput of the engine on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode1b|long1b|serve3b|mixed8b|dafidra|rorevik|dokanex|muretar]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode1b|long1b|serve3b|mixed8b|dafidra|rorevik|dokanex|muretar|semezen]
                     [--batch 8,1,64] [--context 4096] [--dtype bf16|fp32]
 
 Every workload prints ONE JSON line.  The default, ``decode1b`` (Llama 3.2 1B layer sizes):  ``value`` is decoded tokens per second at batch 8 with the context
@@ -55,6 +55,11 @@ attention, rotary attention with biases beside a gated delta rule; dense and rou
 experts) at layer sizes like Llama 3.2 1B's and 3B's, beside a Llama of the same width, depth and vocabulary, measured the
 same way.
 
+``--workload semezen``: the Semezen design (four residual streams side by side, a shift towards the token before; a minGRU
+in every second layer, windowed attention whose values are its keys and whose features are gated in the others; dense gelu
+feed-forwards and routed clamped ones) at layer sizes like Llama 3.2 1B's and 3B's, beside a Llama of the same width, depth
+and vocabulary, measured the same way.
+
 Weights are random (N(0, 0.02), norms 1), token ids uniform random; no dataset is involved.
 """
 from __future__ import annotations
@@ -107,6 +112,10 @@ def make_runner(cfg_raw, layers, dtype, max_batch, max_cache_tokens, seed=0, max
             tensors[s.name] = torch.ones(s.shape, dtype=tdtype, device="cuda")
         elif s.role == "norm_zero":       # weights used as 1 + w
             tensors[s.name] = torch.zeros(s.shape, dtype=tdtype, device="cuda")
+        elif s.role == "near_identity":   # how streams side by side mix
+            tensors[s.name] = torch.eye(s.shape[0], dtype=tdtype, device="cuda")
+        elif s.role == "share":
+            tensors[s.name] = torch.rand(s.shape, generator=gen, dtype=torch.float32, device="cuda").to(tdtype)
         else:
             tensors[s.name] = (torch.randn(s.shape, generator=gen, device="cuda", dtype=torch.float32) * 0.02).to(tdtype)
     opts = EngineOptions(dtype="bfloat16" if dtype == "bf16" else "float32", block_size=BLOCK_SIZE,
@@ -743,6 +752,76 @@ def workload_muretar(args) -> int:
     return 0
 
 
+def semezen_config(width, heads, kv_heads, head_dim, ff, vocab, layers):
+    """A Semezen of Llama-like layer sizes, four streams, layers in fours: minGRU as wide as the model with a dense
+    feed-forward (half as wide again as the Llama's: two matrices instead of three); attention of the Llama's heads within a
+    window of 1,024 (half a head rotated, frequencies scaled by 8) with routed experts; then minGRU with routed experts and
+    attention with the dense feed-forward.  Routed feed-forwards: 16 experts of a quarter of the Llama's width, 4 per token."""
+    gru = {"width": width}
+    attn = dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, mask={"size": 1024},
+                rot={"base": 500000.0, "dims": head_dim // 2, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}})
+    dense = {"kind": "dense", "ff": ff * 3 // 2}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4, "limit": 7.0}, "router": {"experts": 16, "top": 4}}
+    kinds = [("mingru", gru, dense), ("attention", attn, moe), ("mingru", gru, moe), ("attention", attn, dense)]
+    return {"architecture": "Semezen", "vocab": vocab, "width": width, "streams": 4, "norm": {"eps": 1e-5},
+            "layers": [dict(zip(("type", "mixer", "mlp"), kinds[i % 4])) for i in range(layers)]}
+
+
+def workload_semezen(args) -> int:
+    """Semezen beside a Llama of equal width, depth and vocabulary (see the module text)."""
+    import gc
+
+    import torch
+
+    layers = args.layers or 4
+    context = args.context
+    positions = max(context, PREFILL_TOKENS) + 64
+    sizes = {"1b": MODEL, "3b": MODEL_3B}
+    results = {}
+
+    def config(b):
+        return semezen_config(b["hidden_size"], b["num_attention_heads"], b["num_key_value_heads"], b["head_dim"],
+                              b["intermediate_size"], b["vocab_size"], layers)
+
+    def measured(raw):
+        return make_runner(raw, layers, args.dtype, args.batch, max(args.batch * (context + 64), PREFILL_TOKENS + 64), max_model_len=positions)[0]
+
+    if args.only:       # for profiles: the Semezen of the first size alone, a prompt or decode steps
+        runner = measured(config(sizes["1b"]))
+        if args.only == "prefill":
+            sec = time_prefill(runner, PREFILL_TOKENS, max(1, args.steps // 8))
+            print(json.dumps({"only": "prefill", "model": "semezen_1b", "tokens": PREFILL_TOKENS, "ms": round(sec * 1e3, 3)}), flush=True)
+        else:
+            sec, _ = time_decode(runner, args.batch, args.steps, args.warmup, context, synthetic_cache=True)
+            print(json.dumps({"only": "decode", "model": "semezen_1b", "batch": args.batch, "ms_per_step": round(sec * 1e3, 4),
+                              "cache": "random numbers, no prompt was run"}), flush=True)
+        return 0
+    for name, base in sizes.items():
+        for what, raw in (("semezen", config(base)), ("llama", dict(base, tie_word_embeddings=False))):
+            runner = measured(raw)
+            psec = time_prefill(runner, PREFILL_TOKENS, 3)
+            dsec, _ = time_decode(runner, args.batch, args.steps, args.warmup, context)
+            results[f"{what}_{name}"] = {"prefill_ms": round(psec * 1e3, 3), "prefill_tok_per_s": round(PREFILL_TOKENS / psec, 1),
+                                         "decode_ms_per_step": round(dsec * 1e3, 4), "decode_tok_per_s": round(args.batch / dsec, 1),
+                                         "graphs": len(runner._graphs)}
+            del runner
+            gc.collect()
+            torch.cuda.empty_cache()
+    first = results["semezen_1b"]
+    line = {
+        "metric": f"decode tok/s at batch {args.batch}, context {context} (Semezen at Llama 3.2 1B layer sizes, {layers} layers, random weights)",
+        "value": first["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": first["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": args.dtype, "data": "synthetic: random weights N(0, 0.02), streams mixed by the unit matrix, uniform random token ids",
+        "config": {"model": "semezen-at-llama-sizes", "layers": layers, "global_batch": args.batch, "seq_len": context,
+                   "prefill_tokens": PREFILL_TOKENS, "streams": 4, "window": 1024, "experts": 16, "top": 4, "kv_block": BLOCK_SIZE,
+                   "parallelism": "single-gpu"},
+        "models": results,
+    }
+    print(json.dumps(line), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -751,7 +830,7 @@ def main() -> int:
     ap.add_argument("--batch", default="8,1,64",
                     help="batch sizes of the decode steps: the first is the headline's, the others become points")
     ap.add_argument("--context", type=int, default=CONTEXT, help="context length that the decode steps end at")
-    ap.add_argument("--workload", choices=["decode1b", "long1b", "serve3b", "mixed8b", "dafidra", "rorevik", "dokanex", "muretar"], default="decode1b")
+    ap.add_argument("--workload", choices=["decode1b", "long1b", "serve3b", "mixed8b", "dafidra", "rorevik", "dokanex", "muretar", "semezen"], default="decode1b")
     ap.add_argument("--layers", type=int, default=None,
                     help="fewer layers than the model has, if memory or time needs it (both numbers are reported)")
     ap.add_argument("--dtype", default="bf16", choices=["bf16", "fp32"])
@@ -791,6 +870,8 @@ def main() -> int:
         return workload_dokanex(args)
     if args.workload == "muretar":
         return workload_muretar(args)
+    if args.workload == "semezen":
+        return workload_semezen(args)
     args.layers = args.layers or MODEL["num_hidden_layers"]
     elem = 2 if args.dtype == "bf16" else 4
     big = args.batch if (args.no_points or args.only) else max(batches)

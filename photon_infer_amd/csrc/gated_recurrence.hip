@@ -41,8 +41,9 @@ __device__ inline void gr_terms(float zp, float up, float& keep, float& add) {
   add = z * (up >= 0.f ? up + 0.5f : gr_sigmoid(up));
 }
 
+template <bool PIECES>
 __device__ inline float gr_column(const GruArgs& a, long t, int col) {
-  return a.part ? split_sum(a.part, a.splits, a.plane, t * a.proj_stride + col) : a.proj[t * a.proj_stride + col];
+  return PIECES ? split_sum(a.part, a.splits, a.plane, t * a.proj_stride + col) : a.proj[t * a.proj_stride + col];
 }
 
 // (request, chunk) of this block and its tokens; false: there is no such chunk
@@ -55,42 +56,58 @@ __device__ inline bool gr_range(const GruArgs& a, int& t0, int& t1, long& row) {
 }
 
 #define GR_AHEAD 8        // tokens whose loads are in flight together
+#define GR_RECORDS 16     // the same of the chunks' records
 
+// The tokens t0 .. t1 - 1 of feature c, in order: use(t, keep, add, gate) for each; GATE: with the gate's column.
+template <bool PIECES, bool GATE, typename Use>
+__device__ inline void gr_walk(const GruArgs& a, int c, int t0, int t1, Use&& use) {
+  const float bz = a.bias[c], bu = a.bias[a.W + c];
+  int t = t0;
+  for (; t + GR_AHEAD <= t1; t += GR_AHEAD) {
+    float zp[GR_AHEAD], up[GR_AHEAD], g[GR_AHEAD];
+#pragma unroll
+    for (int i = 0; i < GR_AHEAD; ++i) {
+      zp[i] = gr_column<PIECES>(a, t + i, c);
+      up[i] = gr_column<PIECES>(a, t + i, a.W + c);
+      g[i] = GATE ? gr_column<PIECES>(a, t + i, 2 * a.W + c) : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < GR_AHEAD; ++i) {
+      float keep, add;
+      gr_terms(zp[i] + bz, up[i] + bu, keep, add);
+      use(t + i, keep, add, g[i]);
+    }
+  }
+  for (; t < t1; ++t) {
+    float keep, add;
+    const float g = GATE ? gr_column<PIECES>(a, t, 2 * a.W + c) : 0.f;
+    gr_terms(gr_column<PIECES>(a, t, c) + bz, gr_column<PIECES>(a, t, a.W + c) + bu, keep, add);
+    use(t, keep, add, g);
+  }
+}
+
+template <bool PIECES>
 __global__ __launch_bounds__(GR_THREADS) void gru_chunk_kernel(GruArgs a) {
   int t0, t1;
   long row;
   if (!gr_range(a, t0, t1, row)) return;
   const int c = blockIdx.x * GR_THREADS + threadIdx.x;
   if (c >= a.W) return;
-  const float bz = a.bias[c], bu = a.bias[a.W + c];
   float A = 1.f, B = 0.f, S0 = 0.f;
   if (blockIdx.y == 0) {
     const int slot = a.slots[blockIdx.z];
     S0 = slot >= 0 && slot < a.num_slots ? a.state[(long)slot * a.state_stride + c] : 0.f;
   }
-  for (int t = t0; t < t1; t += GR_AHEAD) {
-    float zp[GR_AHEAD], up[GR_AHEAD];
-#pragma unroll
-    for (int i = 0; i < GR_AHEAD; ++i) {
-      const int tt = min(t + i, t1 - 1);
-      zp[i] = gr_column(a, tt, c);
-      up[i] = gr_column(a, tt, a.W + c);
-    }
-#pragma unroll
-    for (int i = 0; i < GR_AHEAD; ++i) {
-      if (t + i >= t1) break;
-      float keep, add;
-      gr_terms(zp[i] + bz, up[i] + bu, keep, add);
-      A *= keep;
-      B = fmaf(keep, B, add);
-    }
-  }
+  gr_walk<PIECES, false>(a, c, t0, t1, [&](int, float keep, float add, float) {
+    A *= keep;
+    B = fmaf(keep, B, add);
+  });
   float* ab = a.ab + (row + blockIdx.y) * 2 * a.W + c;
   ab[0] = blockIdx.y == 0 ? S0 : A;
   ab[a.W] = blockIdx.y == 0 ? fmaf(A, S0, B) : B;
 }
 
-template <typename T>
+template <typename T, bool PIECES>
 __global__ __launch_bounds__(GR_THREADS) void gru_walk_kernel(GruArgs a, T* __restrict__ out, long out_stride) {
   int t0, t1;
   long row;
@@ -100,7 +117,6 @@ __global__ __launch_bounds__(GR_THREADS) void gru_walk_kernel(GruArgs a, T* __re
   const int slot = a.slots[blockIdx.z];
   const bool has_state = slot >= 0 && slot < a.num_slots;
   float* st = a.state + (long)slot * a.state_stride + c;
-  const float bz = a.bias[c], bu = a.bias[a.W + c];
   float S;
   if (!a.ab) {
     S = has_state ? *st : 0.f;
@@ -110,41 +126,27 @@ __global__ __launch_bounds__(GR_THREADS) void gru_walk_kernel(GruArgs a, T* __re
     const float* ab = a.ab + row * 2 * a.W + c;
     S = ab[a.W];
     const int before = blockIdx.y;
-    for (int j = 1; j < before; j += GR_AHEAD) {
-      float A[GR_AHEAD], B[GR_AHEAD];
+    for (int j = 1; j < before; j += GR_RECORDS) {
+      float A[GR_RECORDS], B[GR_RECORDS];
 #pragma unroll
-      for (int i = 0; i < GR_AHEAD; ++i) {
+      for (int i = 0; i < GR_RECORDS; ++i) {
         const bool in = j + i < before;
         A[i] = in ? ab[(long)(j + i) * 2 * a.W] : 1.f;
         B[i] = in ? ab[(long)(j + i) * 2 * a.W + a.W] : 0.f;
       }
 #pragma unroll
-      for (int i = 0; i < GR_AHEAD; ++i) S = fmaf(A[i], S, B[i]);
+      for (int i = 0; i < GR_RECORDS; ++i) S = fmaf(A[i], S, B[i]);
     }
   }
-  for (int t = t0; t < t1; t += GR_AHEAD) {
-    float zp[GR_AHEAD], up[GR_AHEAD], g[GR_AHEAD];
-#pragma unroll
-    for (int i = 0; i < GR_AHEAD; ++i) {
-      const int tt = min(t + i, t1 - 1);
-      zp[i] = gr_column(a, tt, c);
-      up[i] = gr_column(a, tt, a.W + c);
-      g[i] = gr_column(a, tt, 2 * a.W + c);
-    }
-#pragma unroll
-    for (int i = 0; i < GR_AHEAD; ++i) {
-      if (t + i >= t1) break;
-      float keep, add;
-      gr_terms(zp[i] + bz, up[i] + bu, keep, add);
-      S = fmaf(keep, S, add);
-      out[(long)(t + i) * out_stride + c] = from_float<T>(S * g[i] / (1.0f + expf(-g[i])));
-    }
-  }
+  gr_walk<PIECES, true>(a, c, t0, t1, [&](int t, float keep, float add, float g) {
+    S = fmaf(keep, S, add);
+    out[(long)t * out_stride + c] = from_float<T>(S * g / (1.0f + expf(-g)));
+  });
   if (has_state && t1 == a.q_start[blockIdx.z + 1]) *st = S;
 }
 
 // A step of single tokens: a thread per (request, feature), nothing ahead.
-template <typename T>
+template <typename T, bool PIECES>
 __global__ __launch_bounds__(GR_THREADS) void gru_step_kernel(GruArgs a, T* __restrict__ out, long out_stride) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x, r = blockIdx.z;
   const long t = a.q_start[r];
@@ -153,7 +155,7 @@ __global__ __launch_bounds__(GR_THREADS) void gru_step_kernel(GruArgs a, T* __re
   const bool has_state = slot >= 0 && slot < a.num_slots;
   float* st = a.state + (long)slot * a.state_stride + c;
   const float S0 = has_state ? *st : 0.f;
-  const float zp = gr_column(a, t, c) + a.bias[c], up = gr_column(a, t, a.W + c) + a.bias[a.W + c], g = gr_column(a, t, 2 * a.W + c);
+  const float zp = gr_column<PIECES>(a, t, c) + a.bias[c], up = gr_column<PIECES>(a, t, a.W + c) + a.bias[a.W + c], g = gr_column<PIECES>(a, t, 2 * a.W + c);
   float keep, add;
   gr_terms(zp, up, keep, add);
   const float S = fmaf(keep, S0, add);
@@ -185,10 +187,19 @@ extern "C" int pi_min_gru(void* out, int out_dtype, long out_stride, const float
   if (T == 0 || R == 0) return 0;
   GruArgs a{proj, proj_stride, part, splits, (long)T * proj_stride, bias, q_start, slots, state, state_stride, num_slots, W, gru_chunk(longest), nullptr};
   const int threads = W >= 4 * GR_THREADS && longest > 1 ? GR_THREADS : PI_WAVE;
+#define GR_GO(K, GRID)                                                                                                     \
+  do {                                                                                                                     \
+    if (out_dtype == PI_F32) {                                                                                             \
+      if (part) hipLaunchKernelGGL((K<float, true>), GRID, dim3(threads), 0, stream, a, (float*)out, out_stride);          \
+      else hipLaunchKernelGGL((K<float, false>), GRID, dim3(threads), 0, stream, a, (float*)out, out_stride);              \
+    } else {                                                                                                               \
+      if (part) hipLaunchKernelGGL((K<bf16_t, true>), GRID, dim3(threads), 0, stream, a, (bf16_t*)out, out_stride);        \
+      else hipLaunchKernelGGL((K<bf16_t, false>), GRID, dim3(threads), 0, stream, a, (bf16_t*)out, out_stride);            \
+    }                                                                                                                      \
+  } while (0)
   if (longest == 1) {
     const dim3 grid(ceil_div(W, threads), 1, R);
-    if (out_dtype == PI_F32) hipLaunchKernelGGL(gru_step_kernel<float>, grid, dim3(threads), 0, stream, a, (float*)out, out_stride);
-    else hipLaunchKernelGGL(gru_step_kernel<bf16_t>, grid, dim3(threads), 0, stream, a, (bf16_t*)out, out_stride);
+    GR_GO(gru_step_kernel, grid);
     return pi_check_launch("gru_step");
   }
   const int chunks = ceil_div(longest, a.chunk);
@@ -196,11 +207,13 @@ extern "C" int pi_min_gru(void* out, int out_dtype, long out_stride, const float
   if (chunks > 1) {
     PI_REQUIRE(work && work_floats >= pi_min_gru_work_floats(T, R, longest, W), "min gru: the chunks' records do not fit");
     a.ab = work;
-    hipLaunchKernelGGL(gru_chunk_kernel, dim3(ceil_div(W, GR_THREADS), chunks, R), dim3(GR_THREADS), 0, stream, a);
+    const dim3 grid(ceil_div(W, GR_THREADS), chunks, R);
+    if (part) hipLaunchKernelGGL(gru_chunk_kernel<true>, grid, dim3(GR_THREADS), 0, stream, a);
+    else hipLaunchKernelGGL(gru_chunk_kernel<false>, grid, dim3(GR_THREADS), 0, stream, a);
     if (pi_check_launch("gru_chunk")) return -1;
   }
   const dim3 grid(ceil_div(W, threads), chunks, R);
-  if (out_dtype == PI_F32) hipLaunchKernelGGL(gru_walk_kernel<float>, grid, dim3(threads), 0, stream, a, (float*)out, out_stride);
-  else hipLaunchKernelGGL(gru_walk_kernel<bf16_t>, grid, dim3(threads), 0, stream, a, (bf16_t*)out, out_stride);
+  GR_GO(gru_walk_kernel, grid);
+#undef GR_GO
   return pi_check_launch("gru_walk");
 }

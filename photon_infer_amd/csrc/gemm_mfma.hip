@@ -58,6 +58,17 @@ __device__ inline float silu_mul(float g, float u) {
   return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g)) * u;
 }
 
+// x Phi(x) for a bfloat16 result, the error function by formula 7.1.26 of Abramowitz and Stegun's Handbook of
+// Mathematical Functions (absolute error of Phi below 1e-7): with q(|x|) = 1 - Phi(|x|) it is x (1 - q) above zero and
+// x q below, so that nothing cancels where x is far below zero.
+__device__ inline float gelu_mul(float x) {
+  const float a = fabsf(x) * 0.70710678118654752f;
+  const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, a, 1.0f));
+  const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.061405429f, -1.453152027f), 1.421413741f), -0.284496736f), 0.254829592f);
+  const float q = 0.5f * poly * __builtin_amdgcn_exp2f(-1.4426950408889634f * a * a);
+  return x * (x >= 0.f ? 1.0f - q : q);
+}
+
 // The epilogue of both kernels: 32 rows x 64 columns of a wave's result, held as two 32 x 32
 // accumulator tiles (lane = column, register = row), go through a patch of LDS that belongs to
 // the wave alone and come back with eight (bfloat16) or four (float32) neighbouring columns in
@@ -134,7 +145,7 @@ __device__ inline void store_rows32(float* patch, const f32x16_t& acc0, const f3
       }
       if (EPI == EPI_GELU) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) { a[e] = gelu_exact(a[e]); b[e] = gelu_exact(b[e]); }
+        for (int e = 0; e < 4; ++e) { a[e] = gelu_mul(a[e]); b[e] = gelu_mul(b[e]); }
       }
       bf16_t* dst = out + (row0 + r) * ld + c;
       if (wide && c + 8 <= cols_left) {

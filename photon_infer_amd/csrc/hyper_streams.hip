@@ -7,13 +7,10 @@
 // request's last h.
 //
 // One kernel does any of: the update of the streams with a sublayer's result y (a tensor, or the float32 pieces of a
-// product split over k), then the next sublayer's h from the new streams.  A block holds whole rows in registers: the
-// streams are read once and written once, everything is float32 until h is stored.
-//
-// The token before: a block walks `per_block` neighbouring tokens and carries h along; for its first token it makes
-// the one before again from the streams (which this form of the kernel does not change).  A request's state row is
-// read and written by one block only, the one that holds the request's first token: it makes the last token's h from
-// the streams as well.  Together with an update of the streams the shift is for steps of single tokens.
+// product split over k), then the next sublayer's h from the new streams.  A block holds a whole row in registers: the
+// streams are read once and written once, everything is float32 until h is stored.  In a step of single tokens the token
+// before is the state row's, and the shift is part of that kernel; in other steps h is left in float32 and a second
+// kernel shifts it.
 #include "common.h"
 
 #define HS_THREADS 512
@@ -40,10 +37,8 @@ struct HyperArgs {
   float* state;           // [slots, >= D]
   long state_stride;
   int num_slots;
-  const int* q_start;
   const int* slots;
   const int* req_of_token;
-  int per_block;
 };
 
 template <int V> struct Lanes { float v[V]; };
@@ -168,6 +163,8 @@ __device__ inline void hyper_row(const HyperArgs& a, long row, Lanes<V> (&h)[VPT
   }
 }
 
+__device__ inline float shifted(float h, float before, float share) { return fmaf(before - h, share, h); }
+
 template <int V, int VPT>
 __device__ inline void store_h(const HyperArgs& a, long row, const Lanes<V> (&h)[VPT]) {
   const int groups = a.D / V;
@@ -183,7 +180,7 @@ __device__ inline void store_h(const HyperArgs& a, long row, const Lanes<V> (&h)
 template <int S, int V, int VPT, bool POST, bool SHIFT, bool FIT>
 __global__ __launch_bounds__(HS_THREADS) void hyper_streams_kernel(HyperArgs a) {
   __shared__ float scratch[16];
-  const int groups = a.D / V;
+  [[maybe_unused]] const int groups = a.D / V;
   if (!SHIFT) {
     const long m = blockIdx.x;
     const long r = a.rows ? a.rows[m] : m;
@@ -192,49 +189,29 @@ __global__ __launch_bounds__(HS_THREADS) void hyper_streams_kernel(HyperArgs a) 
     if (a.h) store_h<V, VPT>(a, m, h);
     return;
   }
-  const int t0 = blockIdx.x * a.per_block, t1 = min(a.T, t0 + a.per_block);
-  Lanes<V> before[VPT], cur[VPT];
-  for (int t = t0; t < t1; ++t) {
-    const int r = a.req_of_token[t], slot = a.slots[r];
-    const bool first = t == a.q_start[r], has_state = slot >= 0 && slot < a.num_slots;
-    float* st = a.state + (long)slot * a.state_stride;
-    if (first) {
+  const int t = blockIdx.x, slot = a.slots[a.req_of_token[t]];
+  const bool has_state = slot >= 0 && slot < a.num_slots;
+  float* st = a.state + (long)slot * a.state_stride;
+  Lanes<V> before[VPT], cur[VPT], share[VPT];
 #pragma unroll
-      for (int k = 0; k < VPT; ++k) {
-        const int g = threadIdx.x + k * blockDim.x;
-        if (g < groups && has_state) before[k] = load_lanes<V>(st + g * V);
-        else
+  for (int k = 0; k < VPT; ++k) {
+    const int g = threadIdx.x + k * blockDim.x;
+    if (g < groups) share[k] = load_lanes<V>(a.share + g * V);
+    if (g < groups && has_state) before[k] = load_lanes<V>(st + g * V);
+    else
 #pragma unroll
-          for (int e = 0; e < V; ++e) before[k].v[e] = 0.f;
-      }
-    } else if (!POST && t == t0) {
-      hyper_row<S, V, VPT, false, FIT>(a, t - 1, before, scratch);
-    }
-    hyper_row<S, V, VPT, POST, FIT>(a, t, cur, scratch);
-    Lanes<V> moved[VPT];
-#pragma unroll
-    for (int k = 0; k < VPT; ++k) {
-      const int g = threadIdx.x + k * blockDim.x;
-      moved[k] = cur[k];
-      if (g >= groups) continue;
-      const Lanes<V> w = load_lanes<V>(a.share + g * V);
-#pragma unroll
-      for (int e = 0; e < V; ++e) moved[k].v[e] = fmaf(before[k].v[e] - cur[k].v[e], w.v[e], cur[k].v[e]);
-    }
-    store_h<V, VPT>(a, t, moved);
-#pragma unroll
-    for (int k = 0; k < VPT; ++k) before[k] = cur[k];
-    if (first) {
-      const int last = a.q_start[r + 1] - 1;
-      if (!POST && last > t) hyper_row<S, V, VPT, false, FIT>(a, last, cur, scratch);      // its own last token: cur is free again
-      if (has_state)
-#pragma unroll
-        for (int k = 0; k < VPT; ++k) {
-          const int g = threadIdx.x + k * blockDim.x;
-          if (g < groups) store_lanes<V>(st + g * V, cur[k]);
-        }
-    }
+      for (int e = 0; e < V; ++e) before[k].v[e] = 0.f;
   }
+  hyper_row<S, V, VPT, POST, FIT>(a, t, cur, scratch);
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int g = threadIdx.x + k * blockDim.x;
+    if (g >= groups) continue;
+    if (has_state) store_lanes<V>(st + g * V, cur[k]);
+#pragma unroll
+    for (int e = 0; e < V; ++e) cur[k].v[e] = shifted(cur[k].v[e], before[k].v[e], share[k].v[e]);
+  }
+  store_h<V, VPT>(a, t, cur);
 }
 
 template <int S, int V, int VPT, bool FIT>
@@ -247,23 +224,23 @@ static int launch_hyper(const HyperArgs& a, int blocks, int threads, bool post, 
 }
 
 // y or part: the sublayer's result to add (both null: no update).  h null: no next sublayer.  share null: no shift.
-// M: rows of h (with `rows`; else M == T).  single: every request of the step holds one token (needed for a shift together with an update).
+// M: rows of h (with `rows`; else M == T).  single: every request of the step holds one token (a shift is for such steps).
 extern "C" int pi_hyper_streams(float* x, int n, int D, int T, const float* y, const float* part, int splits, const float* post, int write_x,
                                 void* h, int h_dtype, const float* in, const float* w, float eps, const int* rows, int M, const float* share,
-                                float* state, long state_stride, int num_slots, const int* q_start, const int* slots,
-                                const int* req_of_token, int single, hipStream_t stream) {
+                                float* state, long state_stride, int num_slots, const int* slots, const int* req_of_token,
+                                int single, hipStream_t stream) {
   PI_REQUIRE(x && n > 0 && n <= HS_MAX_STREAMS && D > 0 && T >= 0 && M >= 0, "hyper streams: bad sizes streams=%d D=%d T=%d", n, D, T);
   const bool has_post = y || part, shift = share != nullptr;
   PI_REQUIRE(has_post || h, "hyper streams: nothing to do");
   PI_REQUIRE(!has_post || (post && !(y && part) && (!part || splits >= 1)), "hyper streams: bad description of the sublayer's result");
   PI_REQUIRE(!h || (in && w && (h_dtype == PI_F32 || h_dtype == PI_BF16)), "hyper streams: bad description of the next sublayer");
-  PI_REQUIRE(!shift || (h && !rows && state && q_start && slots && req_of_token && state_stride >= D), "hyper streams: bad description of the shift");
-  PI_REQUIRE(!(shift && has_post) || single, "hyper streams: shift and update together are for steps of single tokens");
+  PI_REQUIRE(!shift || (h && !rows && state && slots && req_of_token && state_stride >= D), "hyper streams: bad description of the shift");
+  PI_REQUIRE(!shift || single, "hyper streams: the shift in the same kernel is for steps of single tokens");
   PI_REQUIRE(rows || M == T, "hyper streams: %d rows of %d", M, T);
   PI_REQUIRE(!rows || !write_x, "hyper streams: chosen rows are read, not written");
   if (M == 0 || T == 0) return 0;
   HyperArgs a{x, n, D, T, y, part, splits, post, has_post ? write_x : 0, h, h_dtype == PI_BF16, in, w, eps, rows, share, state, state_stride,
-              num_slots, q_start, slots, req_of_token, 1};
+              num_slots, slots, req_of_token};
   bool wide = D % 4 == 0 && state_stride % 4 == 0;
   for (const void* p : {(const void*)x, (const void*)y, (const void*)part, (const void*)h, (const void*)w, (const void*)share, (const void*)state})
     wide = wide && (uintptr_t)p % 16 == 0;
@@ -273,9 +250,7 @@ extern "C" int pi_hyper_streams(float* x, int n, int D, int T, const float* y, c
   threads = threads > HS_THREADS ? HS_THREADS : ((threads + PI_WAVE - 1) / PI_WAVE) * PI_WAVE;
   const int vpt = (groups + threads - 1) / threads;
   PI_REQUIRE(vpt <= 8 && (n <= 4 || !wide || vpt <= 4), "hyper streams: rows of %d features in %d streams are too wide", D, n);
-  if (shift && !has_post) a.per_block = M >= 2048 ? 8 : (M >= 1024 ? 4 : 1);
-  const int blocks = ceil_div(M, a.per_block);
-#define HS_GO(S_, V_, N_, F_) return launch_hyper<S_, V_, N_, F_>(a, blocks, threads, has_post, shift, stream)
+#define HS_GO(S_, V_, N_, F_) return launch_hyper<S_, V_, N_, F_>(a, M, threads, has_post, shift, stream)
   if (!wide) HS_GO(HS_MAX_STREAMS, 1, 8, false);
 #define HS_PICK(S_)               \
   do {                            \
@@ -300,4 +275,56 @@ extern "C" int pi_hyper_streams(float* x, int n, int D, int T, const float* y, c
   HS_GO(16, 4, 4, false);
 #undef HS_PICK
 #undef HS_GO
+}
+
+// ---------------------------------------------------------------- the shift on its own, any number of tokens per request
+// out[t] = h[t] + (h of the request's token before - h[t]) * share.  The first token's predecessor is the request's
+// state row, which then takes the request's last h: read and written by the threads of the first token only.
+template <typename TO, int V>
+__global__ __launch_bounds__(256) void token_shift_kernel(TO* __restrict__ out, const float* __restrict__ h, const float* __restrict__ share,
+                                                          float* __restrict__ state, long state_stride, int num_slots,
+                                                          const int* __restrict__ q_start, const int* __restrict__ slots,
+                                                          const int* __restrict__ req_of_token, int D) {
+  const long t = blockIdx.x;
+  const int d = (blockIdx.y * 256 + threadIdx.x) * V;
+  if (d >= D) return;
+  const int r = req_of_token[t];
+  const Lanes<V> cur = load_lanes<V>(h + t * D + d), w = load_lanes<V>(share + d);
+  Lanes<V> before;
+  if (t == q_start[r]) {
+    const int slot = slots[r];
+    const bool has_state = slot >= 0 && slot < num_slots;
+    float* st = state + (long)slot * state_stride + d;
+    if (has_state) {
+      before = load_lanes<V>(st);
+      store_lanes<V>(st, load_lanes<V>(h + (long)(q_start[r + 1] - 1) * D + d));
+    } else {
+#pragma unroll
+      for (int e = 0; e < V; ++e) before.v[e] = 0.f;
+    }
+  } else {
+    before = load_lanes<V>(h + (t - 1) * D + d);
+  }
+  Lanes<V> o;
+#pragma unroll
+  for (int e = 0; e < V; ++e) o.v[e] = shifted(cur.v[e], before.v[e], w.v[e]);
+  store_lanes<V>(out + t * D + d, o);
+}
+
+extern "C" int pi_token_shift(void* out, int out_dtype, const float* h, const float* share, float* state, long state_stride, int num_slots,
+                              const int* q_start, const int* slots, const int* req_of_token, int T, int D, hipStream_t stream) {
+  PI_REQUIRE(T >= 0 && D > 0 && out && h && share && state && state_stride >= D && q_start && slots && req_of_token && out != (const void*)h,
+             "token shift: bad arguments T=%d D=%d", T, D);
+  PI_REQUIRE(out_dtype == PI_F32 || out_dtype == PI_BF16, "token shift: unsupported dtype %d", out_dtype);
+  if (T == 0) return 0;
+  bool wide = D % 4 == 0 && state_stride % 4 == 0;
+  for (const void* p : {(const void*)out, (const void*)h, (const void*)share, (const void*)state}) wide = wide && (uintptr_t)p % 16 == 0;
+  const int per_block = 256 * (wide ? 4 : 1);
+  PI_REQUIRE((D + per_block - 1) / per_block <= 65535, "token shift: rows of %d features are too wide", D);
+  const dim3 grid(T, (D + per_block - 1) / per_block), block(256);
+#define TS_GO(TO, V_) hipLaunchKernelGGL((token_shift_kernel<TO, V_>), grid, block, 0, stream, (TO*)out, h, share, state, state_stride, num_slots, q_start, slots, req_of_token, D)
+  if (out_dtype == PI_F32) { if (wide) TS_GO(float, 4); else TS_GO(float, 1); }
+  else { if (wide) TS_GO(bf16_t, 4); else TS_GO(bf16_t, 1); }
+#undef TS_GO
+  return pi_check_launch("token_shift");
 }

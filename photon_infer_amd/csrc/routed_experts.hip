@@ -31,7 +31,7 @@ __device__ inline void wave_argmax(float& v, int& idx) {
 }
 
 __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ logits,
-                                                        long logits_stride, int E, int top, int groups, int keep, int renorm,
+                                                        long logits_stride, int splits, long plane, int E, int top, int groups, int keep, int renorm,
                                                         const float* __restrict__ correction, float renorm_eps, int sigmoid) {
   __shared__ float s[RE_MAX_EXPERTS];
   __shared__ float c[RE_MAX_EXPERTS];      // what the choice goes by
@@ -39,7 +39,9 @@ __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, f
   __shared__ float gscore[RE_MAX_EXPERTS];
   const long t = blockIdx.x;
   const int lane = threadIdx.x;
-  const float* z = logits + t * logits_stride;
+  // the logits, or the pieces of their product (`splits` planes), added in split order
+  __shared__ float z[RE_MAX_EXPERTS];
+  for (int e = lane; e < E; e += PI_WAVE) z[e] = split_sum(logits, splits, plane, t * logits_stride + e);
   if (sigmoid) {
     // the sigmoid grows with z, so without a correction the choice goes by z itself: large logits whose scores round
     // to the same number keep their order
@@ -121,14 +123,15 @@ __global__ __launch_bounds__(PI_WAVE) void route_kernel(int* __restrict__ ids, f
   }
 }
 
-extern "C" int pi_route(int* ids, float* weights, const float* logits, long logits_stride, int T, int E, int top, int groups,
+extern "C" int pi_route(int* ids, float* weights, const float* logits, long logits_stride, int splits, int T, int E, int top, int groups,
                         int keep, int renorm, const float* correction, float renorm_eps, int sigmoid, hipStream_t stream) {
   PI_REQUIRE(T >= 0 && E > 0 && E <= RE_MAX_EXPERTS, "routing: %d experts (at most %d)", E, RE_MAX_EXPERTS);
+  PI_REQUIRE(splits >= 1 && logits_stride >= E, "routing: bad logits (%d pieces, rows of %ld)", splits, logits_stride);
   PI_REQUIRE(top > 0 && top <= E, "routing: %d choices among %d experts", top, E);
   PI_REQUIRE(groups <= 1 || (E % groups == 0 && keep > 0 && keep <= groups), "routing: %d experts in %d groups, %d kept", E, groups, keep);
   PI_REQUIRE(groups <= 1 || (long)keep * (E / groups) >= top, "routing: %d kept groups of %d experts hold fewer than %d choices", keep, groups > 0 ? E / groups : 0, top);
   if (T == 0) return 0;
-  hipLaunchKernelGGL(route_kernel, dim3(T), dim3(PI_WAVE), 0, stream, ids, weights, logits, logits_stride, E, top, groups, keep, renorm, correction, renorm_eps, sigmoid);
+  hipLaunchKernelGGL(route_kernel, dim3(T), dim3(PI_WAVE), 0, stream, ids, weights, logits, logits_stride, splits, (long)T * logits_stride, E, top, groups, keep, renorm, correction, renorm_eps, sigmoid);
   return pi_check_launch("route");
 }
 
@@ -139,62 +142,101 @@ extern "C" int pi_route(int* ids, float* weights, const float* logits, long logi
 //   tile_row0[i], tile_rows[i]; max_tiles = ceil(N / tile) + E bounds their number.
 // Entries whose id is not in 0 .. E - 1 (identity experts) own no row: their entry_row is 0, and the rows
 // that stay empty behind the last expert's name entry 0, so that whoever walks all N rows stays in bounds.
-// One block of 1024 threads; wave w places the experts w, w + 16, ...
+// One block of 1024 threads.  Wave w owns the w-th sixteenth of the entries and a row of counters [experts] in LDS: it
+// counts its entries per expert, the counters become every wave's first row per expert, and it places its entries in
+// order.  The lanes of a wave that hold the same expert find each other by votes on the bits of its number.
+#define RE_WAVES 16
+#define RE_AHEAD 8          // rounds of 64 entries whose ids are asked for together
+
+// calls use(entry, expert or -1, lanes with the same expert) for the wave's entries, 64 at a time and in order
+template <typename Use>
+__device__ inline void walk_entries(const int* __restrict__ ids, int first, int last, int E, int bits, int lane, Use&& use) {
+  for (int i0 = first; i0 < last; i0 += RE_AHEAD * PI_WAVE) {
+    int id[RE_AHEAD];
+#pragma unroll
+    for (int u = 0; u < RE_AHEAD; ++u) {
+      const int i = i0 + u * PI_WAVE + lane;
+      id[u] = i < last ? ids[i] : -1;
+    }
+#pragma unroll
+    for (int u = 0; u < RE_AHEAD; ++u) {
+      if (i0 + u * PI_WAVE >= last) break;
+      const int e = id[u] >= 0 && id[u] < E ? id[u] : -1;
+      unsigned long long same = __ballot(e >= 0);
+      for (int b = 0; b < bits; ++b) {
+        const unsigned long long ones = __ballot((e >> b) & 1);
+        same &= (e >> b) & 1 ? ones : ~ones;
+      }
+      use(i0 + u * PI_WAVE + lane, e, same);
+    }
+  }
+}
+
 __global__ __launch_bounds__(1024) void group_entries_kernel(const int* __restrict__ ids, int N, int E, int* __restrict__ row_entry,
                                                              int* __restrict__ entry_row, int* __restrict__ tile_expert,
                                                              int* __restrict__ tile_row0, int* __restrict__ tile_rows, int max_tiles,
-                                                             int tile) {
-  __shared__ int count[RE_MAX_EXPERTS];
-  __shared__ int start[RE_MAX_EXPERTS + 1];
-  __shared__ int tstart[RE_MAX_EXPERTS + 1];
+                                                             int tile, int bits) {
+  extern __shared__ int counters[];              // [waves][E]
+  __shared__ int rows_to[2][RE_MAX_EXPERTS];     // running sums over the experts, two buffers in turn: rows ...
+  __shared__ int tiles_to[2][RE_MAX_EXPERTS];    // ... and tiles
   const int tid = threadIdx.x, lane = tid % PI_WAVE, wave = tid / PI_WAVE;
-  for (int e = tid; e < E; e += 1024) count[e] = 0;
+  const int per = ((N + RE_WAVES - 1) / RE_WAVES + PI_WAVE - 1) / PI_WAVE * PI_WAVE;
+  const int first = min(N, wave * per), last = min(N, first + per);
+  volatile int* mine = counters + wave * E;      // read by all lanes of the wave before one of them changes it
+  for (int i = tid; i < RE_WAVES * E; i += 1024) counters[i] = 0;
   __syncthreads();
-  for (int i = tid; i < N; i += 1024) {
-    const int e = ids[i];
-    if (e >= 0 && e < E) atomicAdd(&count[e], 1);
+  walk_entries(ids, first, last, E, bits, lane, [&](int, int e, unsigned long long same) {
+    if (e >= 0 && lane == __ffsll(same) - 1) mine[e] = mine[e] + __popcll(same);
+  });
+  __syncthreads();
+  int rows = 0;                                  // thread e: expert e (RE_MAX_EXPERTS is the block's size)
+  if (tid < E)
+    for (int w = 0; w < RE_WAVES; ++w) rows += counters[w * E + tid];
+  const int tiles = (rows + tile - 1) / tile;
+  rows_to[0][tid] = rows;
+  tiles_to[0][tid] = tiles;
+  int b = 0;
+  for (int off = 1; off < E; off *= 2, b ^= 1) {
+    __syncthreads();
+    rows_to[b ^ 1][tid] = rows_to[b][tid] + (tid >= off ? rows_to[b][tid - off] : 0);
+    tiles_to[b ^ 1][tid] = tiles_to[b][tid] + (tid >= off ? tiles_to[b][tid - off] : 0);
   }
   __syncthreads();
-  if (tid == 0) {
-    int acc = 0, tacc = 0;
-    for (int e = 0; e < E; ++e) {
-      start[e] = acc;
-      tstart[e] = tacc;
-      acc += count[e];
-      tacc += (count[e] + tile - 1) / tile;
+  const int all_rows = rows_to[b][E - 1], all_tiles = tiles_to[b][E - 1];
+  if (tid < E) {
+    int at = rows_to[b][tid] - rows;
+    for (int w = 0; w < RE_WAVES; ++w) {         // every wave's first row of this expert
+      const int n = counters[w * E + tid];
+      counters[w * E + tid] = at;
+      at += n;
     }
-    start[E] = acc;
-    tstart[E] = tacc;
   }
-  __syncthreads();
-  for (int i = start[E] + tid; i < N; i += 1024) row_entry[i] = 0;
-  for (int i = tid; i < N; i += 1024)
-    if (ids[i] < 0 || ids[i] >= E) entry_row[i] = 0;
-  for (int i = tstart[E] + tid; i < max_tiles; i += 1024) {
+  for (int i = all_rows + tid; i < N; i += 1024) row_entry[i] = 0;
+  for (int i = all_tiles + tid; i < max_tiles; i += 1024) {
     tile_expert[i] = -1;
     tile_row0[i] = 0;
     tile_rows[i] = 0;
   }
-  for (int e = wave; e < E; e += 16) {
-    for (int i = lane; i < (count[e] + tile - 1) / tile; i += PI_WAVE) {
-      tile_expert[tstart[e] + i] = e;
-      tile_row0[tstart[e] + i] = start[e] + i * tile;
-      const int left = count[e] - i * tile;
-      tile_rows[tstart[e] + i] = left < tile ? left : tile;
-    }
-    int placed = start[e];
-    for (int i0 = 0; i0 < N; i0 += PI_WAVE) {
-      const int i = i0 + lane;
-      const bool mine = i < N && ids[i] == e;
-      const unsigned long long votes = __ballot(mine);
-      if (mine) {
-        const int row = placed + __popcll(votes & ((1ull << lane) - 1ull));
-        row_entry[row] = i;
-        entry_row[i] = row;
-      }
-      placed += __popcll(votes);
+  for (int e = wave; e < E; e += RE_WAVES) {
+    const int end = rows_to[b][e], row0 = e ? rows_to[b][e - 1] : 0, t0 = e ? tiles_to[b][e - 1] : 0;
+    for (int i = lane; t0 + i < tiles_to[b][e]; i += PI_WAVE) {
+      tile_expert[t0 + i] = e;
+      tile_row0[t0 + i] = row0 + i * tile;
+      tile_rows[t0 + i] = min(tile, end - row0 - i * tile);
     }
   }
+  __syncthreads();
+  walk_entries(ids, first, last, E, bits, lane, [&](int i, int e, unsigned long long same) {
+    const int at = e >= 0 ? mine[e] : 0;
+    if (e >= 0) {
+      const int row = at + __popcll(same & ((1ull << lane) - 1ull));
+      row_entry[row] = i;
+      entry_row[i] = row;
+      if (lane == __ffsll(same) - 1) mine[e] = at + __popcll(same);
+    } else if (i < last) {
+      entry_row[i] = 0;
+    }
+  });
 }
 
 extern "C" int pi_group_entries(const int* ids, int N, int E, int* row_entry, int* entry_row, int* tile_expert, int* tile_row0,
@@ -202,8 +244,18 @@ extern "C" int pi_group_entries(const int* ids, int N, int E, int* row_entry, in
   PI_REQUIRE(N >= 0 && E > 0 && E <= RE_MAX_EXPERTS && tile > 0, "grouping: bad sizes N=%d E=%d tile=%d", N, E, tile);
   PI_REQUIRE(max_tiles >= (N + tile - 1) / tile + E, "grouping: room for %d tiles is too little", max_tiles);
   if (N == 0) return 0;
-  hipLaunchKernelGGL(group_entries_kernel, dim3(1), dim3(1024), 0, stream, ids, N, E, row_entry, entry_row, tile_expert, tile_row0,
-                     tile_rows, max_tiles, tile);
+  int bits = 0;
+  while ((1 << bits) < E) ++bits;
+  const size_t lds = (size_t)RE_WAVES * E * sizeof(int);
+  static bool configured = false;
+  if (!configured) {
+    hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(group_entries_kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                         RE_WAVES * RE_MAX_EXPERTS * (int)sizeof(int));
+    if (err != hipSuccess) return pi_fail("grouping: cannot reserve LDS: %s", hipGetErrorString(err));
+    configured = true;
+  }
+  hipLaunchKernelGGL(group_entries_kernel, dim3(1), dim3(1024), lds, stream, ids, N, E, row_entry, entry_row, tile_expert, tile_row0,
+                     tile_rows, max_tiles, tile, bits);
   return pi_check_launch("group_entries");
 }
 
@@ -224,16 +276,47 @@ __global__ void gather_rows_kernel(T* __restrict__ out, const T* __restrict__ sr
   for (int d = threadIdx.x; d < D; d += blockDim.x) out[row * D + d] = src[t * D + d];
 }
 
+// The same for rows of whole 16-byte groups.
+template <typename T>
+__global__ void gather_rows_wide_kernel(T* __restrict__ out, const T* __restrict__ src, const int* __restrict__ row_entry, int top, int groups,
+                                        const float* __restrict__ weights) {
+  const long row = blockIdx.x;
+  const int entry = row_entry[row];
+  const uint4* from = reinterpret_cast<const uint4*>(src) + (long)(entry / top) * groups;
+  uint4* to = reinterpret_cast<uint4*>(out) + row * groups;
+  const float w = weights ? weights[entry] : 1.f;
+  for (int g = threadIdx.x; g < groups; g += blockDim.x) {
+    uint4 v = from[g];
+    if (weights) {
+      uint32_t* p = reinterpret_cast<uint32_t*>(&v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (sizeof(T) == 4) p[i] = __float_as_uint(__uint_as_float(p[i]) * w);
+        else p[i] = f32x2_to_bf16x2_bits(__uint_as_float(p[i] << 16) * w, __uint_as_float(p[i] & 0xffff0000u) * w);
+      }
+    }
+    to[g] = v;
+  }
+}
+
 extern "C" int pi_gather_rows(void* out, const void* src, int dtype, const int* row_entry, int N, int top, int D, const float* weights,
                               hipStream_t stream) {
   PI_REQUIRE(N >= 0 && top > 0 && D > 0, "gather: bad sizes");
+  PI_REQUIRE(dtype == PI_F32 || dtype == PI_BF16, "gather: unsupported dtype %d", dtype);
   if (N == 0) return 0;
+  const int per = dtype == PI_F32 ? 4 : 8;
+  if (D % per == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)src % 16 == 0) {
+    const int groups = D / per, threads = groups >= 256 ? 256 : ceil_div(groups, PI_WAVE) * PI_WAVE;
+    if (dtype == PI_F32)
+      hipLaunchKernelGGL(gather_rows_wide_kernel<float>, dim3(N), dim3(threads), 0, stream, (float*)out, (const float*)src, row_entry, top, groups, weights);
+    else
+      hipLaunchKernelGGL(gather_rows_wide_kernel<bf16_t>, dim3(N), dim3(threads), 0, stream, (bf16_t*)out, (const bf16_t*)src, row_entry, top, groups, weights);
+    return pi_check_launch("gather_rows_wide");
+  }
   if (dtype == PI_F32)
     hipLaunchKernelGGL(gather_rows_kernel<float>, dim3(N), dim3(256), 0, stream, (float*)out, (const float*)src, row_entry, top, D, weights);
-  else if (dtype == PI_BF16)
-    hipLaunchKernelGGL(gather_rows_kernel<bf16_t>, dim3(N), dim3(256), 0, stream, (bf16_t*)out, (const bf16_t*)src, row_entry, top, D, weights);
   else
-    return pi_fail("gather: unsupported dtype %d", dtype);
+    hipLaunchKernelGGL(gather_rows_kernel<bf16_t>, dim3(N), dim3(256), 0, stream, (bf16_t*)out, (const bf16_t*)src, row_entry, top, D, weights);
   return pi_check_launch("gather_rows");
 }
 

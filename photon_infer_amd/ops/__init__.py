@@ -936,22 +936,24 @@ def head_norm_gate(y: torch.Tensor, o: torch.Tensor, gates: torch.Tensor, weight
 # ----------------------------------------------------------------------------- routed experts
 def route(logits: torch.Tensor, top: int, groups: int = 1, keep: int = 1, renorm: bool = False,
           correction: Optional[torch.Tensor] = None, renorm_eps: float = 0.0, scoring: str = "softmax"):
-    """Choose ``top`` experts per row of float32 router logits: (ids int32 [T, top], weights float32
+    """Choose ``top`` experts per row of float32 router logits (a tensor, or ``Partials``, whose pieces are added here): (ids int32 [T, top], weights float32
     [T, top]).  Scores are the softmax over all experts, or (``scoring`` "sigmoid") every logit's own sigmoid; with ``groups`` > 1 only experts of the
     ``keep`` groups with the largest best score may be chosen; weights are the chosen scores
     (divided by their sum + ``renorm_eps`` when ``renorm``).  ``correction`` (float32 [E]): the choice goes
     by score + correction, the weights by the scores alone."""
-    _gpu(logits, correction)
-    T, E = logits.shape
+    pieces = logits if isinstance(logits, Partials) else None
+    src = pieces.part if pieces is not None else logits
+    _gpu(src, correction)
+    T, E = (pieces.M, pieces.N) if pieces is not None else logits.shape
     if scoring not in ("softmax", "sigmoid"):
         raise KernelError(f"routing: scores '{scoring}' are not known (softmax, sigmoid)")
     _f32_vector(correction, E, "routing correction")
-    if logits.dtype != torch.float32:
+    if src.dtype != torch.float32:
         raise KernelError("routing: logits must be float32")
-    ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
-    weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-    _lib.call("core", "pi_route", ids.data_ptr(), weights.data_ptr(), logits.data_ptr(), _rows(logits, "router logits"), T, E,
-              int(top), int(groups), int(keep), int(bool(renorm)), _ptr(correction), float(renorm_eps), int(scoring == "sigmoid"), _stream())
+    ids = torch.empty((T, top), dtype=torch.int32, device=src.device)
+    weights = torch.empty((T, top), dtype=torch.float32, device=src.device)
+    _lib.call("core", "pi_route", ids.data_ptr(), weights.data_ptr(), src.data_ptr(), E if pieces is not None else _rows(logits, "router logits"),
+              pieces.splits if pieces is not None else 1, T, E, int(top), int(groups), int(keep), int(bool(renorm)), _ptr(correction), float(renorm_eps), int(scoring == "sigmoid"), _stream())
     return ids, weights
 
 
@@ -1341,9 +1343,8 @@ def hyper_streams(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, post: Op
       of the new streams in that type - of the rows ``rows`` (int32) only, if given: the streams are then not
       written back.
 
-    ``shift`` (float32 [D]) with ``state`` (float32 [slots, >= D]) and ``ctx``: h is moved towards the h of the request's token
-    before, ``h + (h_before - h) * shift``; the state row holds the h of the last token of the step before and takes this
-    step's last.  Shift and update together are for steps of single tokens."""
+    ``shift`` (float32 [D]) with ``state`` (float32 [slots, >= D]) and ``ctx``, for a step of single tokens: h is shifted on the
+    way as ``token_shift`` does it."""
     pieces = ws.take_result(y) if y is not None and ws is not None else None
     _gpu(x, y, post, read, norm, rows, shift, state)
     if x.dim() != 3 or x.dtype != torch.float32 or not x.is_contiguous():
@@ -1372,15 +1373,33 @@ def hyper_streams(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, post: Op
     if shift is not None:
         _f32_vector(shift, D, "hyper streams shift")
         _state_rows(state, D, "hyper streams")
-        _i32(ctx.q_start, "q_start", ctx.R + 1)
         _i32(ctx.slots, "slots", ctx.R)
         _i32(ctx.req_of_token, "req_of_token", T)
     _lib.call("core", "pi_hyper_streams", x.data_ptr(), n, D, T, _ptr(y) if pieces is None else None, pieces.part.data_ptr() if pieces is not None else None,
               pieces.splits if pieces is not None else 0, _ptr(post), int(rows is None), _ptr(h), _dt(h) if h is not None else PI_F32, _ptr(read), _ptr(norm),
               float(eps), _ptr(rows), M, _ptr(shift), _ptr(state), state.stride(0) if state is not None else 0, state.shape[0] if state is not None else 0,
-              _ptr(ctx.q_start) if shift is not None else None, _ptr(ctx.slots) if shift is not None else None,
+              _ptr(ctx.slots) if shift is not None else None,
               _ptr(ctx.req_of_token) if shift is not None else None, int(bool(getattr(ctx, "all_decode", False))) if shift is not None else 0, _stream())
     return h
+
+
+def token_shift(h: torch.Tensor, shift: torch.Tensor, state: torch.Tensor, ctx, dtype: torch.dtype) -> torch.Tensor:
+    """``h + (h_before - h) * shift`` in ``dtype``, with ``h`` float32 [T, D] and h_before the h of the request's token before:
+    the state row (``state`` float32 [slots, >= D], rows ``ctx.slots``) before a request's first token of the step; the row
+    then takes the request's last h."""
+    _gpu(h, shift, state)
+    if h.dim() != 2 or h.dtype != torch.float32 or not h.is_contiguous():
+        raise KernelError(f"token shift: expected contiguous float32 [T, D], got {h.dtype} {tuple(h.shape)}")
+    T, D = h.shape
+    _f32_vector(shift, D, "token shift share")
+    _state_rows(state, D, "token shift")
+    _i32(ctx.q_start, "q_start", ctx.R + 1)
+    _i32(ctx.slots, "slots", ctx.R)
+    _i32(ctx.req_of_token, "req_of_token", T)
+    out = torch.empty((T, D), dtype=dtype, device=h.device)
+    _lib.call("core", "pi_token_shift", out.data_ptr(), _dt(out), h.data_ptr(), shift.data_ptr(), state.data_ptr(), state.stride(0), state.shape[0],
+              ctx.q_start.data_ptr(), ctx.slots.data_ptr(), ctx.req_of_token.data_ptr(), T, D, _stream())
+    return out
 
 
 def min_gru(out: torch.Tensor, proj, bias: torch.Tensor, ctx, state: torch.Tensor, width: int) -> None:

@@ -35,7 +35,7 @@ _SIGNATURES = {
         "pi_head_gemm": [P, L, I, P, L, I, P, I, I, I, I, I, I, P, I, P],
         "pi_matrix_memory_scan": [P, L, P, L, I, I, I, I, I, P, P, F, F, P, P, I, P, L, I, I, I, I, I, I, P, L, P],
         "pi_head_norm_gate": [P, I, P, L, P, L, P, F, I, I, I, F, I, P],
-        "pi_route": [P, P, P, L, I, I, I, I, I, I, P, F, I, P],
+        "pi_route": [P, P, P, L, I, I, I, I, I, I, I, P, F, I, P],
         "pi_group_entries": [P, I, I, P, P, P, P, P, I, I, P],
         "pi_gather_rows": [P, P, I, P, I, I, I, P, P],
         "pi_grouped_gemm_general": [P, I, L, P, I, L, P, I, L, L, P, P, P, I, I, I, P],
@@ -47,7 +47,8 @@ _SIGNATURES = {
         "pi_paged_attention_general_ranges": [I, I, I],
         "pi_rope_table": [P, P, P, I, I, F, P],
         "pi_qk_rope_norm_write": [P, L, I, P, L, P, I, P, P, I, I, F, I, I, I, I, I, P, P, P, P, P, P, I, I, L, P],
-        "pi_hyper_streams": [P, I, I, I, P, P, I, P, I, P, I, P, P, F, P, I, P, P, L, I, P, P, P, I, P],
+        "pi_hyper_streams": [P, I, I, I, P, P, I, P, I, P, I, P, P, F, P, I, P, P, L, I, P, P, I, P],
+        "pi_token_shift": [P, I, P, P, P, L, I, P, P, P, I, I, P],
         "pi_min_gru": [P, I, L, P, L, P, I, P, P, P, I, I, I, P, L, I, I, P, L, P],
         "pi_sample": [P, P, L, P, P, I, I, P, L, P],
         "pi_sample_static": [P, P, L, P, P, I, I, P],

@@ -316,9 +316,9 @@ class HyperConnectionBlock(Block):
         h = rms(sum_s in2[s] X_s; norm2);            X_t <- sum_s mix2[s, t] X_s + out2[t] * ffn(h)     (no feed-forward: the first only)
 
     The mixer and the feed-forward write their result (``accumulate=False``), or leave it in the pieces of its product.
-    The update by the mixer's result and the feed-forward's h are one kernel.  In a step of single tokens the update by
-    the feed-forward's result is left to the next reader of the streams (the next block's first kernel, or the final
-    norm); in other steps the token before belongs to another block of threads, and the update is a kernel of its own.
+    A sublayer's update of the streams and the next sublayer's h are one kernel, which reads and writes the streams
+    once; the last sublayer's update is left to whoever reads the streams next (the next block's first kernel, or the
+    final norm).  The shift is part of that kernel in a step of single tokens, and a kernel of its own in others.
 
     ``norm1`` / ``mixer`` / ``norm2`` / ``ffn``: (prefix, part); ``shift``: the name of the shift's tensor, or None;
     ``connections``: the prefixes of the two sublayers' ``HyperConnections``."""
@@ -363,29 +363,35 @@ class HyperConnectionBlock(Block):
 
     def forward(self, x: torch.Tensor, ctx: StepContext, cache) -> None:
         caches = cache if isinstance(cache, (list, tuple)) else [cache]
-        ws = ctx.workspace
+        ws, reads = ctx.workspace, (self.hc1.read, self.norm1.weight_f32(), self.norm1.eps)
         left = ctx.scratch.pop(LEFT_UPDATE, None)
         y, post = (left[1], left[2]) if left is not None and left[0] is x else (None, None)
-        if y is not None and not ctx.all_decode:      # an update and a shift in one kernel are for single tokens
-            ops.hyper_streams(x, y=y, post=post, ws=ws)
-            y = post = None
-        shift, state = (self.shift.share, caches[1].state) if self.shift is not None else (None, None)
-        h = ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.hc1.read, norm=self.norm1.weight_f32(), eps=self.norm1.eps,
-                              shift=shift, state=state, ctx=ctx, ws=ws)
-        result = lambda: torch.empty((x.shape[0], x.shape[2]), dtype=torch.float32, device=x.device)
-        y, post = result(), self.hc1.post
-        ctx.may_defer = True                          # the next kernel on the streams adds a product's pieces
-        self.mixer.forward(h, y, ctx, caches[0])
-        if self.ffn is not None:
-            h = ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.hc2.read, norm=self.norm2.weight_f32(), eps=self.norm2.eps,
-                                  ctx=ctx, ws=ws)
-            y, post = result(), self.hc2.post
-            self.ffn.forward(h, y, ctx)
-        ctx.may_defer = False
-        if ctx.all_decode:
-            ctx.scratch[LEFT_UPDATE] = (x, y, post)
+        if self.shift is None:
+            h = self._join_and_read(x, y, post, self.dtype, reads, ws)
+        elif ctx.all_decode:
+            h = self._join_and_read(x, y, post, self.dtype, reads, ws, shift=self.shift.share, state=caches[1].state, ctx=ctx)
         else:
-            ops.hyper_streams(x, y=y, post=post, ws=ws)
+            h = ops.token_shift(self._join_and_read(x, y, post, torch.float32, reads, ws), self.shift.share, caches[1].state, ctx, self.dtype)
+        ctx.may_defer = True                          # the next kernel on the streams adds a product's pieces
+        y = self._result(x)
+        self.mixer.forward(h, y, ctx, caches[0])
+        post = self.hc1.post
+        if self.ffn is not None:
+            h = self._join_and_read(x, y, post, self.dtype, (self.hc2.read, self.norm2.weight_f32(), self.norm2.eps), ws)
+            y = self._result(x)
+            self.ffn.forward(h, y, ctx)
+            post = self.hc2.post
+        ctx.may_defer = False
+        ctx.scratch[LEFT_UPDATE] = (x, y, post)
+
+    @staticmethod
+    def _join_and_read(x, y, post, dtype, reads, ws, **kw):
+        read, norm, eps = reads
+        return ops.hyper_streams(x, y=y, post=post, h_dtype=dtype, read=read, norm=norm, eps=eps, ws=ws, **kw)
+
+    @staticmethod
+    def _result(x: torch.Tensor) -> torch.Tensor:
+        return torch.empty((x.shape[0], x.shape[2]), dtype=torch.float32, device=x.device)
 
 
 BLOCKS.register("hyper_connections", HyperConnectionBlock)

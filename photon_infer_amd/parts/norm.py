@@ -79,7 +79,7 @@ class StreamSumRMSNorm(RMSNorm):
         left = ctx.scratch.pop(LEFT_UPDATE, None) if ctx is not None else None
         y, post = (left[1], left[2]) if left is not None and left[0] is x else (None, None)
         return ops.hyper_streams(x, y=y, post=post, h_dtype=self.dtype, read=self.ones, norm=self.weight_f32(), eps=self.eps, rows=rows,
-                                 ctx=ctx, ws=ctx.workspace if ctx is not None else None)
+                                 ws=ctx.workspace if ctx is not None else None)
 
 
 NORMS.register("stream_sum_rmsnorm", StreamSumRMSNorm)

@@ -118,8 +118,7 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h: torch.Tensor, x: torch.Tensor, ctx: StepContext) -> None:
         T, ws = h.shape[0], ctx.workspace if ctx is not None else None
-        logits = torch.empty((T, self.router_size), dtype=torch.float32, device=h.device)
-        ops.gemm(logits, h, self.w_router, ws=ws)
+        logits = ops.qkv_projection(h, self.w_router, torch.float32, ws)      # float32; pieces, where the product was split over k
         ids, weights = ops.route(logits, self.top, self.groups, self.keep, self.renormalize, self.correction, self.renorm_eps,
                                  self.scoring)
         rows = ops.group_entries(ids, self.num_experts, self.tile)
