@@ -135,3 +135,118 @@ def live_token_need(steps: List[dict], rounding: int = 64) -> int:
         for rid in s.get("end", []):
             held.pop(rid, None)
     return worst
+
+
+# ------------------------------------------------------------------ inputs, comparisons and contexts for kernels on their own
+def randn(*shape, seed=0, scale=1.0):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed), dtype=torch.float64) * scale
+
+
+def close(got, ref, what, tol=2e-5):
+    tol = tol * max(1.0, float(ref.abs().max()))
+    err = float((got.double().cpu() - ref).abs().max())
+    assert err <= tol, f"{what}: error {err:.3e} > {tol:.3e}"
+
+
+def dev32(t):
+    return t.float().to(DEV).contiguous()
+
+
+def state_ctx(q_lens, slots):
+    """The fields of a StepContext that the kernels of mixers with a state read."""
+    q_start = np.zeros(len(q_lens) + 1, np.int32)
+    np.cumsum(q_lens, out=q_start[1:])
+    return SimpleNamespace(T=int(sum(q_lens)), R=len(q_lens), max_q_len=max(q_lens), q_lens=list(q_lens),
+                           q_start=torch.from_numpy(q_start).to(DEV), slots=torch.tensor(slots, dtype=torch.int32, device=DEV))
+
+
+def in_steps(seqs, cuts):
+    """Steps over several sequences at once: ``cuts[name]`` are the portion sizes of sequence ``name`` (cycled); a step
+    holds the next portion of every sequence that has tokens left.  Yields [(name, begin, end)]."""
+    at = {n: 0 for n in seqs}
+    k = 0
+    while any(at[n] < seqs[n] for n in seqs):
+        step = []
+        for n in seqs:
+            if at[n] < seqs[n]:
+                size = min(cuts[n][k % len(cuts[n])], seqs[n] - at[n])
+                step.append((n, at[n], at[n] + size))
+                at[n] += size
+        k += 1
+        yield step
+
+
+def paged(lengths, page, seed=0):
+    """(block table [requests, width] on the device, pages in the pool): pages dealt out of order, three to spare."""
+    blocks = [-(-n // page) for n in lengths]
+    total = sum(blocks) + 3
+    order = torch.randperm(total, generator=torch.Generator().manual_seed(seed)).tolist()
+    table = torch.full((len(lengths), max(blocks)), -1, dtype=torch.int32)
+    it = iter(order)
+    for r, b in enumerate(blocks):
+        for j in range(b):
+            table[r, j] = next(it)
+    return table.to(DEV), total
+
+
+def make_part(kind, tensors, tdt, **params):
+    from photon_infer_amd.parts import MIXERS
+    part = MIXERS.make(kind, **params)
+    names = {s.name: s for s in part.tensor_specs()}
+    assert set(names) == set(tensors), (sorted(names), sorted(tensors))
+    part.load({n: t.to(tdt if t.dim() == 2 else torch.float32).to(DEV) for n, t in tensors.items()}, tdt, torch.device(DEV))
+    return part
+
+
+def run_paged_part(part, h, want, cuts_list, tdt, page, tol, what, D):
+    """A mixer with pages as a part, on pages dealt out of order: under each cutting of the sequence its result must be the plain one."""
+    from photon_infer_amd.parts import LayerCache
+    T = h.shape[0]
+    table, pages = paged([T], page, seed=2)
+    spec = part.cache_spec()
+    pools = {t.name: torch.zeros((pages, *t.page_shape(page)), dtype=tdt, device=DEV) for t in spec.tensors}
+    cache = LayerCache(group=0, k=pools["k"], v=pools["v"], page_size=page, writes=True, tensors=pools)
+    for cuts in cuts_list:
+        for t in pools.values():
+            t.fill_(50.0)                     # what a page held before must not show
+        done = 0
+        for n in cuts:
+            ctx = attention_ctx([n], [done + n], tdt)
+            ctx.block_tables, ctx.may_defer = {0: table}, False
+            x = torch.full((n, D), 3.0, dtype=torch.float32, device=DEV)          # the part writes its result, it does not add
+            part.forward(h[done:done + n].to(tdt).to(DEV).contiguous(), x, ctx, cache)
+            close(x, want[done:done + n], f"{what} tokens {done} .. {done + n} of cuts {cuts[:4]}", tol)
+            done += n
+
+
+class RouteRecorder:
+    """Records the experts the engine chooses (every call of ``ops.route``, in order), so that the plain implementation can be
+    asked for the logits of the same choices: among hundreds of routing decisions some are near ties, which bfloat16 rounding
+    decides either way, and one flipped expert changes everything after it."""
+
+    def __enter__(self):
+        from photon_infer_amd import ops
+        self.ops, self.real, self.calls = ops, ops.route, []
+
+        def route(*a, **k):
+            ids, w = self.real(*a, **k)
+            self.calls.append(ids.cpu())
+            return ids, w
+        ops.route = route
+        return self
+
+    def __exit__(self, *exc):
+        self.ops.route = self.real
+
+    def by_request(self, steps, config):
+        """{request: {routed layer: [tokens, top] expert ids}} from the calls, given the trace's steps."""
+        layers = [i for i, l in enumerate(config["layers"]) if l["mlp"] and l["mlp"]["kind"] == "moe"]
+        out, k = {}, 0
+        for s in steps:
+            sizes = [len(e["tokens"]) for e in s["entries"]]
+            for i in layers:
+                for e, part in zip(s["entries"], torch.split(self.calls[k], sizes)):
+                    out.setdefault(e["id"], {}).setdefault(i, []).append(part)
+                k += 1
+        assert k == len(self.calls)
+        return {rid: {i: [r.tolist() for r in torch.cat(p)] for i, p in per.items()} for rid, per in out.items()}
