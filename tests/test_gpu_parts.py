@@ -347,7 +347,7 @@ def register_routed_toy():
                 if rows.numel():
                     x[rows] += self.scale * (torch.relu(hf[rows] @ self.up[e].t()) @ self.down[e].t())
 
-    FEED_FORWARDS.register("routed_experts", RoutedExperts)
+    FEED_FORWARDS.register("toy_routed_experts", RoutedExperts)
 
     class AddedPositions(PositionEncoding):
         """q and k of the token at position p get table[p] added, the same vector for every head."""
@@ -402,7 +402,7 @@ def register_routed_toy():
             mixer = MIXERS.make("attention", hidden_size=D, num_heads=cfg.heads, num_kv_heads=cfg.heads, head_dim=hd,
                                 position=POSITION_ENCODINGS.make("added_positions", head_dim=hd, max_positions=40))
             return BLOCKS.make("prenorm", norm1=("n1.", norm()), mixer=("attn.", mixer), norm2=("n2.", norm()), ffn=("ffn.", ffn))
-        layers = [("l0.", block(FEED_FORWARDS.make("routed_experts", hidden_size=D, expert_size=cfg.expert_width,
+        layers = [("l0.", block(FEED_FORWARDS.make("toy_routed_experts", hidden_size=D, expert_size=cfg.expert_width,
                                                     num_experts=cfg.experts, output_scale=cfg.expert_scale))),
                   ("l1.", block(FEED_FORWARDS.make("swiglu", hidden_size=D, intermediate_size=3 * D)))]
         return ModelSpec(hidden_size=D, vocab_size=cfg.vocab, max_positions=40, embedding=("emb.", TokenEmbedding(cfg.vocab, D)),
