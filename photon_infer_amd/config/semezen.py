@@ -3,8 +3,8 @@
 The file names every size and every constant that may differ between models of the design:
 ``vocab``, ``width``, ``streams`` (how many copies of the residual stream run side by side), ``norm.eps``
 and a list ``layers`` whose entries give the layer's ``type`` (which mixer it has: ``attention`` or
-``mingru``), the mixer's sizes (``mixer``) and its feed-forward (``mlp``: ``kind`` ``dense`` or ``moe``, or
-null for none).
+``mingru``), the mixer's sizes (``mixer``) and, where the layer has one, its feed-forward (``mlp``: ``kind`` ``dense`` or
+``moe``).
 """
 from __future__ import annotations
 

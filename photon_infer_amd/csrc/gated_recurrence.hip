@@ -1,4 +1,4 @@
-// A gated recurrence that keeps one number per feature and whose gates read the current token only (minGRU):
+// A recurrence of one number per feature whose gate and candidate do not look at the state (minGRU):
 //   z = sigmoid(zp + bz),  u = up + bu,  c = u + 1/2 where u >= 0, sigmoid(u) where u < 0
 //   S <- (1 - z) S + z c;   out = S * silu(g)
 // from float32 projection rows [zp: W | up: W | g: W] (a tensor, or the pieces of a product split over k), from and

@@ -1,8 +1,8 @@
 // Several residual streams side by side (hyper-connections), X [T, n, D] float32.  Around a sublayer:
 //   u = sum_s in[s] X_s;   h = u / sqrt(mean(u^2) + eps) * w       (what the sublayer reads, in the activation type)
-//   X_t <- sum_s mix[s, t] X_s + out[t] * y                        (all streams at once from the old ones)
+//   X_t <- sum_s mix[s, t] X_s + out[t] * y                        (no new stream is read while any is made)
 // and, for a sublayer that also sees the token before its own,
-//   h <- h + (h_before - h) * share                                (per feature; h_before as it was before this line)
+//   h <- h + (h_before - h) * share                                (per feature; h_before: the neighbour's h, itself unshifted)
 // with h_before of a request's first token of the step taken from the request's state row, which then takes the
 // request's last h.
 //

@@ -1,6 +1,6 @@
 """Semezen: a decoder with several residual streams side by side.  Every sublayer reads a weighted sum of them and
 writes to all of them through a small matrix; a token's mixer also sees the token before it; mixers are windowed
-attention whose values are its keys, or a gated recurrence that keeps one number per feature; feed-forwards are
+attention whose values are its keys, or minGRU, a recurrence of one number per feature; feed-forwards are
 dense (gelu) or routed.
 
     X_s = embed[token]   (s = 1 .. streams)

@@ -23,8 +23,8 @@ q, k and v projections (``qkv_bias``) and on the output projection (``o_bias``; 
 added; added in float32, the first three before the rotation), and ``accumulate`` False: the result is written into the
 tensor handed to ``forward`` instead of added to it.
 
-``values_are_keys``: there is no v projection; a token's values are its keys as projected (with their bias), before the
-rotation and any norm.  ``head_norm_eps``: after the rotation every head of q and k is divided by the root mean square
+``values_are_keys``: there is no v projection; a token's value vectors are its key vectors straight from the biased
+projection.  ``head_norm_eps``: after the rotation every head of q and k is divided by the root mean square
 of its entries (this eps inside the root, no weight).  ``feature_gate`` names a matrix [heads * value_dim, hidden]: the
 concatenated heads are multiplied, feature by feature, with ``sigmoid(W h)`` before the output projection, in float32
 before the one rounding.  The three come together (one kernel makes queries, keys and values from the projection).

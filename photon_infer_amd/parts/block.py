@@ -287,8 +287,8 @@ BLOCKS.register("sandwich", SandwichBlock)
 
 class HyperConnections(Part):
     """How one sublayer is tied to several residual streams side by side (hyper-connections; Zhu et al.,
-    "Hyper-Connections"): it reads ``u = sum_s in[s] X_s``, and its result y joins all streams at once,
-    ``X_t <- sum_s mix[s, t] X_s + out[t] y`` (mix is indexed [from, to])."""
+    "Hyper-Connections"): it reads ``u = sum_s in[s] X_s``, and its result y joins every stream while they mix,
+    ``X_t <- sum_s mix[s, t] X_s + out[t] y`` (rows of mix: where from; columns: where to)."""
 
     graph_safe = True
 

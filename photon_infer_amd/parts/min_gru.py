@@ -1,4 +1,4 @@
-"""minGRU: a gated recurrence that keeps one number per feature, whose gates read the current token only
+"""minGRU: a recurrence of one number per feature whose gate and candidate do not look at the state
 (Feng et al., "Were RNNs All We Needed?").
 
 With input h: ``z = sigmoid(Wz h + bz)``, ``u = Wx h + bx``; the candidate is ``c = u + 1/2`` where u >= 0 and

@@ -2,8 +2,8 @@
 
     h <- h + (h_before - h) * share
 
-with h_before the previous token's h as it was before this line (zeros before a sequence's first token).  A
-request's state row holds the h of its last token in float32; a prompt may be cut anywhere.
+h_before is the unshifted h of the neighbour on the left; a sequence starts with a neighbour of zeros.  A
+request's state row holds the unshifted h of its last token in float32, so a prompt may be cut anywhere.
 
 The arrangement that uses it makes h, the shift and the state update in one kernel (``ops.hyper_streams``); this part
 holds the weights and declares the state.

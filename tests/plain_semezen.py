@@ -7,13 +7,13 @@ the raw config.json mapping and a dict of tensors by their names in a model fold
         u = sum_s in_s X_s;   y = sublayer(rms(u; norm));   X_t <- sum_s mix[s, t] X_s + out_t y
     logits = head . rms(sum_s X_s; final.norm)
 
-What a mixer reads is h + (h' - h) * shift, with h the normalised u of the token and h' that of the
-token before it (zeros before the first).  A layer's mixer is one of
+What a mixer reads is h + (h' - h) * shift, with h the normalised u of the token and h' that of its left
+neighbour (the first token's is zero).  A layer's mixer is one of
 
 * ``attention``: grouped-query attention within a sliding window; queries and keys with biases,
   a part of each head rotated (paired halves, frequencies scaled by wavelength), then every head
-  of both divided by its root mean square; the values are the keys as projected; every feature of
-  the result times a sigmoid gate;
+  of both divided by its root mean square; value vectors are the biased keys, unturned and at their own length; every
+  feature of the result times a sigmoid gate;
 * ``mingru``: ``S <- (1 - z) S + z c`` per feature with ``z = sigmoid(Wz h + bz)``, ``u = Wx h + bx``,
   ``c = u + 1/2`` for u >= 0 and ``sigmoid(u)`` below; the result is ``Wo (S * silu(Wg h))``.
 
@@ -79,7 +79,7 @@ def shift_in(h: torch.Tensor, share: torch.Tensor) -> torch.Tensor:
 
 
 def mix_streams(X: List[torch.Tensor], y: torch.Tensor, mix: torch.Tensor, out: torch.Tensor) -> List[torch.Tensor]:
-    """All new streams from the old ones: X_t <- sum_s mix[s, t] X_s + out[t] y."""
+    """Every new stream from the streams as they were: X_t <- sum_s mix[s, t] X_s + out[t] y."""
     n = len(X)
     return [sum(mix[s, t] * X[s] for s in range(n)) + out[t] * y for t in range(n)]
 

@@ -82,7 +82,7 @@ def test_folder_with_random_weights(tmp_path):
 
 
 # ----------------------------------------------------------------------------- the plain implementation's own closed forms
-def test_streams_are_mixed_all_at_once_from_the_old_ones():
+def test_streams_are_mixed_from_the_streams_as_they_were():
     X = [torch.tensor([1.0, 2.0], dtype=F64), torch.tensor([10.0, 20.0], dtype=F64)]
     y = torch.tensor([100.0, 200.0], dtype=F64)
     swap = torch.tensor([[0.0, 1.0], [1.0, 0.0]], dtype=F64)
