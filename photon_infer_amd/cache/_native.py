@@ -20,7 +20,7 @@ _SIGNATURES = {
     "pi_pool_allocate": (c_int, [c_void_p, c_int, _IP]),
     "pi_pool_free": (c_int, [c_void_p, _IP, c_int]),
     "pi_pool_reset": (None, [c_void_p]),
-    "pi_cache_create": (c_void_p, [c_int, _IP, c_int, _IP, c_int, c_int]),
+    "pi_cache_create": (c_void_p, [c_int, _IP, _IP, c_int, _IP, c_int, c_int]),
     "pi_cache_destroy": (None, [c_void_p]),
     "pi_cache_error": (c_char_p, [c_void_p]),
     "pi_cache_max_blocks": (c_int, [c_void_p]),

@@ -9,7 +9,8 @@ Reference: src/runtime/kv_cache_manager.cpp (one pool, same block id in all laye
 * pages are taken on demand, one step at a time (the reference reserves a request's
   whole lifetime up front, include/photon/scheduler/continuous_batch_engine.hpp:98-103);
 * a group with a window gives a page back as soon as every position in it is out of
-  reach of all later queries;
+  reach of all later queries; a group that also keeps a sequence's first tokens keeps the
+  pages they lie in until the request ends;
 * every live request owns a *slot*: the row of its block tables and the index of its
   fixed-size state, if any mixer keeps one.
 
@@ -47,11 +48,11 @@ class _GroupPool:
 
 
 class _Group:
-    """A view of one cache group: its window, pool and block tables (numpy views of native memory)."""
+    """A view of one cache group: its window, kept first tokens, pool and block tables (numpy views of native memory)."""
 
-    def __init__(self, manager: "CacheManager", index: int, window: Optional[int], num_pages: int):
+    def __init__(self, manager: "CacheManager", index: int, window: Optional[int], keep_first: int, num_pages: int):
         lib, h = manager._lib, manager._h
-        self.window = window
+        self.window, self.keep_first = window, keep_first
         self.pool = _GroupPool(manager, index, num_pages)
         shape = (manager.max_slots, manager.max_blocks)
         self.table = np.ctypeslib.as_array(lib.pi_cache_table(h, index), shape=shape)          # -1 = no page
@@ -61,9 +62,10 @@ class _Group:
 
 class CacheManager:
     def __init__(self, windows: Sequence[Optional[int]], page_size: int, num_pages: int | Sequence[int],
-                 max_slots: int, max_model_len: int):
+                 max_slots: int, max_model_len: int, keep_first: Optional[Sequence[int]] = None):
         """``windows``: one entry per cache group (None = keep all keys).
-        ``num_pages``: pages of each group's pool (one number = the same for all)."""
+        ``num_pages``: pages of each group's pool (one number = the same for all).
+        ``keep_first``: per group, how many of a sequence's first tokens stay beside its window (None: none)."""
         if page_size <= 0 or max_slots <= 0 or max_model_len <= 0:
             raise CacheError("page_size, max_slots and max_model_len must be positive")
         self.page_size = int(page_size)
@@ -76,12 +78,15 @@ class CacheManager:
         if any(int(n) <= 0 for n in counts):
             raise CacheError(f"a page pool needs at least one page, got {counts}")
         self._lib = _native.lib()
+        keeps = [0] * len(windows) if keep_first is None else [int(k) for k in keep_first]
+        if len(keeps) != len(windows) or any(k < 0 for k in keeps):
+            raise CacheError(f"{len(windows)} cache groups with kept first tokens {keeps}")
         self._h = self._lib.pi_cache_create(len(windows), _native.int_array(-1 if w is None else int(w) for w in windows),
-                                            self.page_size, _native.int_array(int(n) for n in counts), self.max_slots,
+                                            _native.int_array(keeps), self.page_size, _native.int_array(int(n) for n in counts), self.max_slots,
                                             self.max_model_len)
         if not self._h:
             raise CacheError("the native cache manager refused its sizes")
-        self.groups: List[_Group] = [_Group(self, i, w, int(n)) for i, (w, n) in enumerate(zip(windows, counts))]
+        self.groups: List[_Group] = [_Group(self, i, w, k, int(n)) for i, (w, k, n) in enumerate(zip(windows, keeps, counts))]
         self._lengths = np.ctypeslib.as_array(self._lib.pi_cache_lengths(self._h), shape=(self.max_slots,))
         self._slots: Dict[Hashable, int] = {}
         self._need = _native.int_array([0] * len(self.groups))
@@ -155,7 +160,7 @@ class CacheManager:
 
     def commit(self, rid: Hashable, new_tokens: int) -> None:
         """The step wrote ``new_tokens`` more keys: advance the length and give back the
-        pages that every window has passed."""
+        pages that every window has passed (pages of kept first tokens stay)."""
         status = self._lib.pi_cache_commit(self._h, self.slot(rid), int(new_tokens))
         if status:
             self._fail(status, rid)

@@ -196,11 +196,17 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 2
   st.lo[0] = lo;
   st.bias[0] = (OPT && valid && opt.slopes) ? opt.slopes[g * G + lr] / scale : 0.f;
   attn_set_cap(st, OPT ? opt.softcap : 0.f, scale);
-  // this wave's keys: chunk `split` of the 32-key chunks between lo and p
-  const int first_chunk = lo / 32, last_chunk = p / 32;
-  const int chunks = last_chunk - first_chunk + 1;
+  st.keep = OPT ? opt.keep : 0;
+  // this wave's keys: range `split` of the list of 32-key chunks that hold keys to see - those between lo and p, and in front
+  // of them those of the kept first keys (places below `kept`; from there on a chunk is its place + gap)
+  const int first_chunk = lo / 32;
+  const int kept = OPT ? min((opt.keep + 31) / 32, first_chunk) : 0;
+  const int gap = OPT && kept > 0 ? first_chunk - kept : 0;
+  const int first_place = OPT && kept > 0 ? 0 : first_chunk;
+  const int last_chunk = p / 32 - gap;             // as a place
+  const int chunks = last_chunk - first_place + 1;
   const int per = (chunks + splits - 1) / splits;
-  const int c0 = first_chunk + split * per;
+  const int c0 = first_place + split * per;
   const int c1 = min(last_chunk + 1, c0 + per);
   // The wave whose keys end at the new token writes that token into the cache first and waits
   // for the stores; after that it reads the token like any other key, in the same order of
@@ -221,7 +227,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 2
                        float unused[1];
                        rotated_fragments<HD, 0>(st.q[0], src, row, src.q_col + (g * G + lr) * HD, valid, lane, none, false, unused);
                      }
-                   });
+                   }, kept, gap);
   attn_finish(st);
 
   const int head = g * G + lr;
@@ -430,12 +436,12 @@ extern "C" int pi_attention_decode(void* out, long out_stride, const void* q, lo
                                    const int* kv_len, const int* req_ids, int R, int nh, int nkv, int hd, int page_size,
                                    float scale, int window, long num_pages, int splits, void* part, long part_elems,
                                    const float* slopes, const float* sinks, const float* gate, long gate_stride, float softcap,
-                                   float out_mult, int chunk, hipStream_t stream) {
-  PI_REQUIRE(chunk >= 0, "attention_decode: chunk must be >= 0, got %d", chunk);
+                                   float out_mult, int chunk, int keep, hipStream_t stream) {
+  PI_REQUIRE(chunk >= 0 && keep >= 0, "attention_decode: chunk and kept first keys must be >= 0, got %d and %d", chunk, keep);
   PI_REQUIRE(gate_stride == 0 || (gate && gate_stride % 4 == 0 && (uintptr_t)gate % 16 == 0), "attention_decode: gates per feature must lie in 16-byte groups");
   return launch_decode(false, DecodeSource{}, out, out_stride, q, q_stride, k_cache, v_cache, block_table, table_width, q_start,
                        kv_len, req_ids, R, nh, nkv, hd, page_size, scale, window, num_pages, splits, part, part_elems, true, stream,
-                       AttnOptions{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk});
+                       AttnOptions{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk, keep});
 }
 
 // The same for a step of single tokens only (T == R tokens, request r at row q_start[r]),

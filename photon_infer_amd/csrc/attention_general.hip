@@ -7,7 +7,9 @@
 //   o = sum_t P_t V[t]
 // with lo = 0, or p - window + 1 when a window is given, or the start of p's chunk,
 // floor(p / chunk) * chunk, when positions are cut into chunks that do not see one another
-// (both given: the later of the two).  Causality is the loop bound.
+// (both given: the later of the two).  Causality is the loop bound.  With keep > 0 the keys 0..keep-1
+// are seen besides (a window that keeps a sequence's first tokens): the walk goes over the kept keys
+// before lo and then over lo..p, as one list.
 // The softmax is exact: no constant is added to the denominator (the reference's paged
 // kernel adds 1e-6, src/ops/kernels/cuda/paged_attention.cu:71).
 //
@@ -38,7 +40,7 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
     const T* __restrict__ v_cache, const int* __restrict__ block_table, int table_width,
     const int* __restrict__ req_of_token, const int* __restrict__ positions, int nh, int nkv, int hd, int page_size,
     float scale, int window, long num_pages, float* __restrict__ part, int vd, const float* __restrict__ slopes,
-    const float* __restrict__ sinks, const float* __restrict__ gate, long gate_stride, float softcap, float out_mult, int chunk) {
+    const float* __restrict__ sinks, const float* __restrict__ gate, long gate_stride, float softcap, float out_mult, int chunk, int keep) {
   __shared__ float qs[NACC * PI_WAVE];
   __shared__ float ps[PI_WAVE];
   __shared__ long voff[PI_WAVE];   // values are stored [page, kv_head, head_dim, slot]
@@ -60,16 +62,21 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
   __syncthreads();
   // this wave's keys: all of lo..p, or the z-th of gridDim.z ranges of whole 64-key groups
   const int splits = gridDim.z;
-  const int groups = (p - lo) / PI_WAVE + 1;
+  // places in the list of seen keys: place i holds key i below kp, and key i + gap from there on; without kept keys
+  // (kp = 0) the list is lo..p.  Places are counted so that gap = 0 there (i from lo).
+  const int kp = keep < lo ? keep : lo;
+  const int gap = kp > 0 ? lo - kp : 0, from = kp > 0 ? 0 : lo, end = p - gap;
+  auto key_at = [&](int place) { return place < kp ? place : place + gap; };
+  const int groups = (end - from) / PI_WAVE + 1;
   const int per = (groups + splits - 1) / splits;
-  const int first = lo + (int)blockIdx.z * per * PI_WAVE;
+  const int first = from + (int)blockIdx.z * per * PI_WAVE;
   const long last_l = (long)first + (long)per * PI_WAVE - 1;
-  const int last = last_l < p ? (int)last_l : p;
+  const int last = last_l < end ? (int)last_l : end;
   for (int k0 = first; k0 <= last; k0 += PI_WAVE) {
-    const int key = k0 + lane;
+    const int key = key_at(k0 + lane);
     float s = -INFINITY;
     long off = -1, vo = -1;
-    if (key <= p) {
+    if (k0 + lane <= end) {
       const int blk = key / page_size;
       const long page = blk < table_width ? bt[blk] : -1;
       if (page >= 0 && page < num_pages) {
@@ -97,7 +104,7 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
       }
     }
     const float m_new = fmaxf(m, wave_max(s));
-    const float pe = (key <= p) ? expf(s - m_new) : 0.f;
+    const float pe = (k0 + lane <= end) ? expf(s - m_new) : 0.f;
     const float corr = expf(m - m_new);
     l = l * corr + wave_sum(pe);
     ps[lane] = pe;
@@ -105,12 +112,13 @@ __global__ __launch_bounds__(PI_WAVE) void paged_attention_general_kernel(
 #pragma unroll
     for (int i = 0; i < NACC; ++i) acc[i] *= corr;
     __syncthreads();
-    const int nk = (p - k0 + 1) < PI_WAVE ? (p - k0 + 1) : PI_WAVE;
+    const int nk = (end - k0 + 1) < PI_WAVE ? (end - k0 + 1) : PI_WAVE;
     // keys in ascending order; four at a time where they lie side by side in a page (values are
     // stored with the slot as the last axis), in the same order of additions
     for (int kk = 0; kk < nk;) {
       const long o2 = voff[kk];
-      const bool four = page_size % 4 == 0 && ((k0 + kk) & 3) == 0 && kk + 3 < nk;
+      const int at = k0 + kk;      // four neighbouring places hold neighbouring keys, except across the end of the kept ones
+      const bool four = page_size % 4 == 0 && (key_at(at) & 3) == 0 && kk + 3 < nk && (at >= kp || at + 3 < kp);
       if (o2 >= 0) {
         const T* vr = v_cache + o2;
         if (four) {
@@ -229,7 +237,8 @@ extern "C" int pi_paged_attention_general(void* out, long out_stride, const void
                                           const int* req_of_token, const int* positions, int T, int nh, int nkv, int hd,
                                           int page_size, float scale, int window, long num_pages, int splits, void* part,
                                           long part_elems, int vd, const float* slopes, const float* sinks, const float* gate, long gate_stride,
-                                          float softcap, float out_mult, int chunk, hipStream_t stream) {
+                                          float softcap, float out_mult, int chunk, int keep, hipStream_t stream) {
+  PI_REQUIRE(keep >= 0, "attention: kept first keys must be >= 0, got %d", keep);
   PI_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention: heads %d must be a positive multiple of kv heads %d", nh, nkv);
   PI_REQUIRE(hd > 0 && hd <= PI_MAX_HEAD_DIM, "attention: head_dim %d must be at most %d", hd, PI_MAX_HEAD_DIM);
   PI_REQUIRE(page_size > 0 && table_width > 0 && num_pages > 0, "attention: bad cache geometry page_size=%d table_width=%d pages=%ld", page_size, table_width, num_pages);
@@ -248,11 +257,11 @@ extern "C" int pi_paged_attention_general(void* out, long out_stride, const void
     if (dtype == PI_F32)
       hipLaunchKernelGGL((paged_attention_general_kernel<float, PI_ATTN_WIDE>), grid, block, 0, stream, (float*)out, out_stride, (const float*)q,
                          q_stride, (const float*)k_cache, (const float*)v_cache, block_table, table_width, req_of_token,
-                         positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
+                         positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk, keep);
     else if (dtype == PI_BF16)
       hipLaunchKernelGGL((paged_attention_general_kernel<bf16_t, PI_ATTN_WIDE>), grid, block, 0, stream, (bf16_t*)out, out_stride,
                          (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, table_width,
-                         req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
+                         req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk, keep);
     else
       return pi_fail("attention: unsupported dtype %d", dtype);
     if (pi_check_launch("paged_attention_general")) return -1;
@@ -266,11 +275,11 @@ extern "C" int pi_paged_attention_general(void* out, long out_stride, const void
   if (dtype == PI_F32)
     hipLaunchKernelGGL((paged_attention_general_kernel<float, 4>), grid, block, 0, stream, (float*)out, out_stride, (const float*)q,
                        q_stride, (const float*)k_cache, (const float*)v_cache, block_table, table_width, req_of_token,
-                       positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
+                       positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk, keep);
   else if (dtype == PI_BF16)
     hipLaunchKernelGGL((paged_attention_general_kernel<bf16_t, 4>), grid, block, 0, stream, (bf16_t*)out, out_stride,
                        (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, table_width,
-                       req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk);
+                       req_of_token, positions, nh, nkv, hd, page_size, scale, window, num_pages, (float*)part, vd, slopes, sinks, gate, gate_stride, softcap, out_mult, chunk, keep);
   else
     return pi_fail("attention: unsupported dtype %d", dtype);
   if (pi_check_launch("paged_attention_general")) return -1;

@@ -48,6 +48,7 @@ struct AttnState {
                         // (slope / scale); read only by the BIAS variants of the arithmetic
   float cap_raw;        // the cap on the scores in raw score units (cap / scale; 0: none), the same for every
   float cap_rate;       // column; and 2 log2(e) scale / cap.  Read only by the BIAS variants.
+  int keep;             // keys below this one are seen whatever lo says (read only by the BIAS variants)
 };
 
 // Options of a head beyond plain softmax attention, each off when its pointer is null:
@@ -65,7 +66,8 @@ struct AttnOptions {
   float out_mult = 1.f;
   long gate_stride = 0;   // > 0: gates per feature
   int chunk = 0;          // C > 0: a token sees the keys of its own chunk of C positions only (a bound like the window's: no option of the arithmetic)
-  bool any() const { return slopes || sinks || gate || softcap > 0.f || out_mult != 1.f; }
+  int keep = 0;           // N > 0: a token sees the sequence's first N keys besides those of its window or chunk
+  bool any() const { return slopes || sinks || gate || softcap > 0.f || out_mult != 1.f || keep > 0; }
 };
 
 // the factors that the gates of four neighbouring features (as projected) put on them
@@ -169,6 +171,15 @@ struct PageCursor {
   ScalarIntPtr bt;    // block-table row, uniform
   int table_width, kv_len, page_size;
   int key, blk, slot; // next tile
+  int jump, land;     // a walk in two stretches: at key `jump` (a multiple of 32) it goes on at key `land`; -1: in one
+  __device__ inline void jump_at(int from, int to) {
+    jump = __builtin_amdgcn_readfirstlane(from);
+    land = __builtin_amdgcn_readfirstlane(to);
+    cross();
+  }
+  __device__ inline void cross() {
+    if (key == jump) { key = land; blk = land / page_size; slot = land - blk * page_size; }
+  }
   __device__ inline void start(const int* row, int width, int len, int psize, int key0) {
     const uint64_t v = reinterpret_cast<uint64_t>(row);
     const uint32_t lo = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(v));
@@ -180,8 +191,11 @@ struct PageCursor {
     key = __builtin_amdgcn_readfirstlane(key0);
     blk = __builtin_amdgcn_readfirstlane(key0 / psize);
     slot = key - blk * page_size;
+    jump = -1;
+    land = 0;
   }
-  // A tile beyond the keys or beyond the table has no page.
+  // A tile beyond the keys or beyond the table has no page.  JUMPS: the walk may have two stretches.
+  template <bool JUMPS = false>
   __device__ inline ChunkPages next() {
     ChunkPages cp;
 #pragma unroll
@@ -194,6 +208,7 @@ struct PageCursor {
       slot += 16;
       if (slot >= page_size) { slot = 0; ++blk; }
     }
+    if (JUMPS) cross();
     return cp;
   }
 };
@@ -284,7 +299,7 @@ __device__ inline void attn_compute(AttnState<HD, CB>& st, const KV& kv, int k0,
       for (int i = 0; i < 4; ++i) {
         if (MASKED) {
           const int key = k0 + t * 16 + lg * 4 + i;
-          if (!(kv.have[t] && key <= st.pos[c] && key >= st.lo[c])) s[t][c][i] = -INFINITY;
+          if (!(kv.have[t] && key <= st.pos[c] && (key >= st.lo[c] || (BIAS && key < st.keep)))) s[t][c][i] = -INFINITY;
         }
         mx = fmaxf(mx, s[t][c][i]);
       }
@@ -466,13 +481,15 @@ __device__ inline void attn_compute(AttnState<HD, CB>& st, const KV& kv, int k0,
 // Walk chunks c0 .. c1-1 (32 keys each) with the next chunk's loads in flight during the
 // current chunk's arithmetic.  Chunks from `first_unmasked` up to `last_unmasked` (inclusive)
 // are known to be fully visible to every column.
+// The chunks are places in a list: place c is chunk c + gap from `head` on, and chunk c below it (kept first keys in front of
+// a window; BIAS variants only; head = gap = 0: place and chunk are the same).  The unmasked bounds are chunks.
 // `meanwhile` is called once the first chunk's loads are on their way (also when the range is
 // empty): work that the walk needs but the loads do not, such as fetching the queries.
 template <int HD, int CB, bool BIAS = false, class Meanwhile>
 __device__ inline void attn_walk(AttnState<HD, CB>& st, int c0, int c1, int first_unmasked, int last_unmasked,
                                  const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
                                  const int* __restrict__ bt, int table_width, int kv_len, int nkv, int g, int page_size,
-                                 long num_pages_l, float scale_log2, int lane, Meanwhile&& meanwhile) {
+                                 long num_pages_l, float scale_log2, int lane, Meanwhile&& meanwhile, int head = 0, int gap = 0) {
   // the range is the same in every lane; saying so keeps the loop's branches scalar, and a
   // divergent break would make the compiler wait for every load at the loop's head
   c0 = __builtin_amdgcn_readfirstlane(c0);
@@ -487,8 +504,16 @@ __device__ inline void attn_walk(AttnState<HD, CB>& st, int c0, int c1, int firs
   KVLaneOffsets<HD> off;
   off.set(page_size, lane);
   const int num_pages = (int)(num_pages_l < 0x7fffffffL ? num_pages_l : 0x7fffffffL);
+  head = __builtin_amdgcn_readfirstlane(head);
+  gap = __builtin_amdgcn_readfirstlane(gap);
+  auto chunk_of = [&](int c) { return BIAS && c >= head ? c + gap : c; };
   PageCursor cur;
-  cur.start(bt, table_width, kv_len, page_size, c0 * 32);
+  cur.start(bt, table_width, kv_len, page_size, chunk_of(c0) * 32);
+  if (BIAS && gap > 0 && c0 < head) cur.jump_at(head * 32, (head + gap) * 32);
+  auto compute = [&](const KVChunk<HD>& kv, int place) {
+    const int c = chunk_of(place);
+    attn_compute<HD, CB, KVChunk<HD>, BIAS>(st, kv, c * 32, scale_log2, c < first_unmasked || c > last_unmasked, lane);
+  };
   // Page ids run two chunks ahead, keys and values one chunk ahead of the arithmetic.  Two
   // chunks per turn with fixed roles for the two buffers and no way out of the loop between
   // them: the loads of one buffer are then always the youngest in flight when the other is
@@ -498,27 +523,27 @@ __device__ inline void attn_walk(AttnState<HD, CB>& st, int c0, int c1, int firs
     // Heads this wide: one chunk's keys and values are 128 registers, two chunks in flight beside the accumulators
     // do not fit the register file (the kernel spilled to memory).  One buffer: a chunk is asked for when the one
     // before it has been used; page ids still run a chunk ahead.
-    ChunkPages pn = cur.next();
+    ChunkPages pn = cur.next<BIAS>();
     attn_load<HD>(a, pn, k_cache, v_cache, off, nkv, g, page_size, num_pages);
     meanwhile();
     for (int c = c0; c < c1; ++c) {
-      pn = cur.next();
-      attn_compute<HD, CB, KVChunk<HD>, BIAS>(st, a, c * 32, scale_log2, c < first_unmasked || c > last_unmasked, lane);
+      pn = cur.next<BIAS>();
+      compute(a, c);
       if (c + 1 < c1) attn_load<HD>(a, pn, k_cache, v_cache, off, nkv, g, page_size, num_pages);
     }
     return;
   }
   KVChunk<HD> b;
-  ChunkPages pa = cur.next(), pb = cur.next();
+  ChunkPages pa = cur.next<BIAS>(), pb = cur.next<BIAS>();
   attn_load<HD>(a, pa, k_cache, v_cache, off, nkv, g, page_size, num_pages);
   meanwhile();
   for (int c = c0; c < c1; c += 2) {
-    pa = cur.next();
+    pa = cur.next<BIAS>();
     attn_load<HD>(b, pb, k_cache, v_cache, off, nkv, g, page_size, num_pages);
-    attn_compute<HD, CB, KVChunk<HD>, BIAS>(st, a, c * 32, scale_log2, c < first_unmasked || c > last_unmasked, lane);
-    pb = cur.next();
+    compute(a, c);
+    pb = cur.next<BIAS>();
     attn_load<HD>(a, pa, k_cache, v_cache, off, nkv, g, page_size, num_pages);
-    if (c + 1 < c1) attn_compute<HD, CB, KVChunk<HD>, BIAS>(st, b, (c + 1) * 32, scale_log2, c + 1 < first_unmasked || c + 1 > last_unmasked, lane);
+    if (c + 1 < c1) compute(b, c + 1);
   }
 }
 

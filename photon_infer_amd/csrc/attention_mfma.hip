@@ -68,8 +68,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
     // shares' results are merged by the combine kernel, as for decode attention)
     const int cut = tile_cut[tile] & 0xff, cuts = tile_cut[tile] >> 8;
     const int all0 = first_key(pos0) / KEYS_PER_ROUND, all1 = (pos0 + n_tok - 1) / KEYS_PER_ROUND + 1;
-    const int share = (all1 - all0 + cuts - 1) / cuts;
-    const int sc0 = all0 + cut * share, sc1 = min(all1, sc0 + share);   // may be empty: nothing seen, m stays -inf
+    // with kept first keys the rounds are places in a list: the rounds that hold kept keys, then the window's; from `head`
+    // on a round is its place + gap (head = gap = 0: place and round are the same)
+    const int keep = OPT ? opt.keep : 0;
+    const int head = OPT ? min((keep + KEYS_PER_ROUND - 1) / KEYS_PER_ROUND, all0) : 0;
+    const int gap = OPT && head > 0 ? all0 - head : 0;
+    const int from = OPT && head > 0 ? 0 : all0, end = all1 - gap;
+    auto round_of = [&](int place) { return OPT && place >= head ? place + gap : place; };
+    const int share = (end - from + cuts - 1) / cuts;
+    const int sc0 = from + cut * share, sc1 = min(end, sc0 + share);   // may be empty: nothing seen, m stays -inf
     // tokens of this wave's columns, and the keys all / any of them see
     const int tok_a = (wave * CB * 16) / G, tok_b = min(((wave + 1) * CB * 16 - 1) / G, n_tok - 1);
     const bool active = tok_a < n_tok;
@@ -79,6 +86,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
     AttnState<HD, CB> st;
     attn_init(st);
     attn_set_cap(st, OPT ? opt.softcap : 0.f, scale);
+    st.keep = keep;
     long rows[CB];
     int heads[CB];
     bool valid[CB];
@@ -102,7 +110,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
     // instead of 53 for a 2,048-token prompt at head size 64)
     const bool fetches = NCH == 4 || wave < NCH;
     PageCursor cur;
-    cur.start(block_table + (long)r * table_width, table_width, kv_len, page_size, sc0 * KEYS_PER_ROUND + wave * 32);
+    cur.start(block_table + (long)r * table_width, table_width, kv_len, page_size, round_of(sc0) * KEYS_PER_ROUND + wave * 32);
+    // where the fetch of the window's first round lands, if kept rounds come before it
+    const int jump_key = OPT && gap > 0 && sc0 < head ? head * KEYS_PER_ROUND + wave * 32 : -1;
+    const int land_key = all0 * KEYS_PER_ROUND + wave * 32, land_blk = land_key / page_size, land_slot = land_key - land_blk * page_size;
     KVChunk<HD> pre;
     auto fetch = [&]() {
       if (!fetches) return;
@@ -113,6 +124,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
       cur.blk += step_blk;
       cur.slot += step_slot;
       if (cur.slot >= page_size) { cur.slot -= page_size; ++cur.blk; }
+      if (OPT) {
+        const bool lands = cur.key == jump_key;
+        cur.key = lands ? land_key : cur.key;
+        cur.blk = lands ? land_blk : cur.blk;
+        cur.slot = lands ? land_slot : cur.slot;
+      }
     };
     auto stash = [&](int buf) {
       if (!fetches) return;
@@ -135,22 +152,23 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(HD <= 64 ? 
       fetch();                                     // the next 128 keys (past the end: no pages, page 0 is read)
       // a round that every column of the wave sees whole, with every page there: straight-line
       // code without the per-key tests (the accumulators then stay in place from chunk to chunk)
-      const int round0 = sc * KEYS_PER_ROUND;
+      const int round0 = round_of(sc) * KEYS_PER_ROUND;
       const bool missing = __builtin_amdgcn_ballot_w64(lane < 2 * NCH && !(&present[buf][0][0])[lane % 8]) != 0;
       constexpr int NJ = NCH < PLAIN_NJ ? NCH : PLAIN_NJ;
-      if (active && !missing && round0 >= see_all_lo && round0 + KEYS_PER_ROUND - 1 <= see_all_hi) {
+      const bool whole = round0 >= see_all_lo || (OPT && round0 + KEYS_PER_ROUND <= keep);
+      if (active && !missing && whole && round0 + KEYS_PER_ROUND - 1 <= see_all_hi) {
         attn_compute_plain<HD, CB, NJ, OPT>(st, staged + (buf * NCH * F) * 64 + lane, F * 64, scale_log2, round0, lane);
         if (NJ < NCH) attn_compute_plain<HD, CB, NJ, OPT>(st, staged + ((buf * NCH + 2) * F) * 64 + lane, F * 64, scale_log2, round0 + 64, lane);
       } else if (active) {
 #pragma unroll 1
         for (int j = 0; j < NCH; ++j) {
-          const int key0 = sc * KEYS_PER_ROUND + j * 32;
-          if (key0 > see_any_hi || key0 + 31 < see_any_lo) continue;
+          const int key0 = round0 + j * 32;
+          if (key0 > see_any_hi || (key0 + 31 < see_any_lo && !(OPT && key0 < keep))) continue;
           StagedChunk<HD> kv;
           kv.from = staged + ((buf * NCH + j) * F) * 64 + lane;
           kv.have[0] = __builtin_amdgcn_readfirstlane(present[buf][j][0]) != 0;
           kv.have[1] = __builtin_amdgcn_readfirstlane(present[buf][j][1]) != 0;
-          const bool masked = key0 < see_all_lo || key0 + 31 > see_all_hi || !kv.have[0] || !kv.have[1];
+          const bool masked = (key0 < see_all_lo && !(OPT && key0 + 32 <= keep)) || key0 + 31 > see_all_hi || !kv.have[0] || !kv.have[1];
           attn_compute<HD, CB, StagedChunk<HD>, OPT>(st, kv, key0, scale_log2, masked, lane);
         }
       }
@@ -219,8 +237,8 @@ extern "C" int pi_attention_prefill_mfma(void* out, long out_stride, const void*
                                          const int* tile_z0, void* part, const int* order, int rounds, int seats, int nh,
                                          int nkv, int hd, int page_size, float scale, int window, long num_pages,
                                          const float* slopes, const float* sinks, const float* gate, long gate_stride,
-                                         float softcap, float out_mult, int chunk, hipStream_t stream) {
-  PI_REQUIRE(chunk >= 0, "attention_prefill: chunk must be >= 0, got %d", chunk);
+                                         float softcap, float out_mult, int chunk, int keep, hipStream_t stream) {
+  PI_REQUIRE(chunk >= 0 && keep >= 0, "attention_prefill: chunk and kept first keys must be >= 0, got %d and %d", chunk, keep);
   PI_REQUIRE(rounds > 0 && seats > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_prefill: bad sizes rounds=%d seats=%d heads=%d kv_heads=%d", rounds, seats, nh, nkv);
   PI_REQUIRE(hd >= 16 && hd <= 256 && hd % 16 == 0, "attention_prefill: head_dim %d is not a multiple of 16 up to 256", hd);
   PI_REQUIRE(page_size >= 16 && page_size % 16 == 0, "attention_prefill: page size %d must be a multiple of 16", page_size);
@@ -232,7 +250,7 @@ extern "C" int pi_attention_prefill_mfma(void* out, long out_stride, const void*
   const size_t lds = tiles_lds_bytes(hd);
   const dim3 grid(nkv, seats), block(256);
   PI_REQUIRE(gate_stride == 0 || (gate && gate_stride % 4 == 0 && (uintptr_t)gate % 16 == 0), "attention_prefill: gates per feature must lie in 16-byte groups");
-  const AttnOptions opt{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk};
+  const AttnOptions opt{slopes, sinks, gate, softcap, out_mult, gate_stride, chunk, keep};
   const bool with_options = opt.any();
   PI_REQUIRE(!with_options || scale > 0.f, "attention_prefill: a distance bias or a cap needs a positive scale");
 #define GO(H, C, N)                    \

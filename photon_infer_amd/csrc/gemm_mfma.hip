@@ -30,19 +30,22 @@ PI_DEFINE_MODULE(bf16)
 #define BK 64
 #define TILE_ELEMS (BM * BK)                // a tile's slab in LDS: rows of 128 bytes
 
-enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ACCUM = 2, EPI_SWIGLU = 3, EPI_CLAMPED_GLU = 4, EPI_RELU2 = 5, EPI_GELU = 6 };
+enum { EPI_BF16 = 0, EPI_F32 = 1, EPI_ACCUM = 2, EPI_SWIGLU = 3, EPI_CLAMPED_GLU = 4, EPI_RELU2 = 5, EPI_GELU = 6, EPI_GATE = 7 };
 
-// results that leave as bfloat16, one per input column: as they are, through max(c, 0)^2, or through the exact gelu
-#define EPI_HALF(E) ((E) == EPI_BF16 || (E) == EPI_RELU2 || (E) == EPI_GELU)
+// results that leave as bfloat16, one per input column: as they are, through max(c, 0)^2, through the exact gelu, or times
+// the sigmoid of a gate of their own
+#define EPI_HALF(E) ((E) == EPI_BF16 || (E) == EPI_RELU2 || (E) == EPI_GELU || (E) == EPI_GATE)
 
 // the gated epilogues store one output column per pair of input columns, in bfloat16
 #define EPI_GATED(E) ((E) == EPI_SWIGLU || (E) == EPI_CLAMPED_GLU)
 
 // What the clamped gated unit needs beside the products: biases in the order of W's rows (gate and up
-// interleaved by 16), the clamp and the sigmoid's factor.
+// interleaved by 16), the clamp and the sigmoid's factor.  For EPI_GATE, `bias` points at the gates (float32, before
+// their sigmoid, one per output; rows gate_stride apart).
 struct GluArgs {
   const float* bias;
   float limit, alpha;
+  long gate_stride;
 };
 
 // g' = min(g + bg, limit), u' = clamp(u + bu, -limit, limit): g' * sigmoid(alpha * g') * (u' + 1)
@@ -57,6 +60,8 @@ __device__ inline float clamped_glu_mul(float g, float u, float bg, float bu, fl
 __device__ inline float silu_mul(float g, float u) {
   return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g)) * u;
 }
+
+__device__ inline float sigmoid_fast(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
 
 // x Phi(x) for a bfloat16 result, the error function by formula 7.1.26 of Abramowitz and Stegun's Handbook of
 // Mathematical Functions (absolute error of Phi below 1e-7): with q(|x|) = 1 - Phi(|x|) it is x (1 - q) above zero and
@@ -82,7 +87,7 @@ __device__ inline uint32_t pack2(float a, float b) { return f32x2_to_bf16x2_bits
 
 template <int EPI>
 __device__ inline void store_rows32(float* patch, const f32x16_t& acc0, const f32x16_t& acc1, void* C, int ld, int row0,
-                                    int rows_left, int cols_left, int lane, bool wide, GluArgs glu = GluArgs{nullptr, 0.f, 0.f},
+                                    int rows_left, int cols_left, int lane, bool wide, GluArgs glu = GluArgs{nullptr, 0.f, 0.f, 0},
                                     long col0 = 0) {
   const int half = lane / 32, ccol = lane % 32;
 #pragma unroll
@@ -146,6 +151,14 @@ __device__ inline void store_rows32(float* patch, const f32x16_t& acc0, const f3
       if (EPI == EPI_GELU) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) { a[e] = gelu_mul(a[e]); b[e] = gelu_mul(b[e]); }
+      }
+      if (EPI == EPI_GATE) {
+        const float* g = glu.bias + (row0 + r) * glu.gate_stride + c;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float f = c + e < cols_left ? sigmoid_fast(g[e]) : 0.f;
+          if (e < 4) a[e] *= f; else b[e - 4] *= f;
+        }
       }
       bf16_t* dst = out + (row0 + r) * ld + c;
       if (wide && c + 8 <= cols_left) {
@@ -241,6 +254,7 @@ __global__ __launch_bounds__(256) void gemm_mfma_kernel(void* __restrict__ Cv, l
     A += r0 * lda + grp * group_a_step;
     W += (long)grp * group_stride;
     Cv = reinterpret_cast<char*>(Cv) + (r0 * ldc + grp * group_c_step) * (EPI_HALF(EPI) || EPI_GATED(EPI) ? 2 : 4);
+    if (EPI == EPI_GATE) glu.bias += r0 * glu.gate_stride + grp * group_c_step;       // a gate per column of the result's rows
   }
   const long m0 = (long)tile_m * BM, n0 = (long)tile_n * BN;
 
@@ -356,6 +370,7 @@ __global__ __launch_bounds__(256) void gemm_mfma_kernel(void* __restrict__ Cv, l
   {
     const long mw = m0 + wm * 64, nw = n0 + wn * 64;
     const int rows_left = (int)min((long)64, M - mw), cols_left = (int)min((long)64, N - nw);   // may be <= 0
+    if (EPI == EPI_GATE) glu.bias += mw * glu.gate_stride + nw;
     float* patch = reinterpret_cast<float*>(lds) + wave * PATCH_FLOATS;
     const int esize = EPI_HALF(EPI) || EPI_GATED(EPI) ? 2 : 4;
     char* corner = reinterpret_cast<char*>(Cv) + (mw * ldc + (EPI_GATED(EPI) ? nw / 2 : nw)) * esize;
@@ -511,6 +526,7 @@ __global__ __launch_bounds__(512) void gemm_mfma_big_kernel(void* __restrict__ C
   {
     const long mw = m0 + wm * 128, nw = n0 + wn * 64;
     const int rows_left = (int)min((long)128, M - mw), cols_left = (int)min((long)64, N - nw);   // may be <= 0
+    if (EPI == EPI_GATE) glu.bias += mw * glu.gate_stride + nw;
     float* patch = reinterpret_cast<float*>(lds) + wave * PATCH_FLOATS;
     const int esize = EPI_HALF(EPI) || EPI_GATED(EPI) ? 2 : 4;
     char* corner = reinterpret_cast<char*>(Cv) + (mw * ldc + (EPI_GATED(EPI) ? nw / 2 : nw)) * esize;
@@ -537,7 +553,7 @@ static const size_t kLdsBytes = 4 * TILE_ELEMS * sizeof(uint16_t);   // 65,536 b
 
 template <int EPI>
 static int launch(void* C, long ldc, const void* A, long lda, const void* W, long ldw, int M, int N, int K, int splits,
-                  hipStream_t stream, GluArgs glu = GluArgs{nullptr, 0.f, 0.f}) {
+                  hipStream_t stream, GluArgs glu = GluArgs{nullptr, 0.f, 0.f, 0}) {
   static bool configured = false;
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_mfma_kernel<EPI>),
@@ -574,11 +590,12 @@ extern "C" int pi_gemm_mfma_group_tile_rows() { return BM; }
 // C[row, :] = A[row, :] . W[group of row]^T over a device-side list of `tiles` row tiles (see the
 // kernel); W is [groups, N, K] with `group_stride` elements from one group's matrix to the next.
 // epilogue: 0 store bf16, 1 store f32, 3 SwiGLU (every group's rows interleaved by 16; C is [rows, N / 2] bf16), 4 the clamped
-// gated unit without biases (rows as for 3; `limit` and `alpha`), 5 max(c, 0)^2 as bf16.
+// gated unit without biases (rows as for 3; `limit` and `alpha`), 5 max(c, 0)^2 as bf16, 7 c * sigmoid(gate) as bf16 (`gate`
+// float32, rows `gate_stride` apart, a gate per column of C's rows).
 template <int EPI>
 static int launch_grouped(void* C, long ldc, const void* A, long lda, const void* W, long ldw, long group_stride,
                           const int* group_of_tile, const int* tile_row0, const int* tile_rows, int tiles, int N, int K,
-                          long group_a_step, long group_c_step, hipStream_t stream, GluArgs glu = GluArgs{nullptr, 0.f, 0.f}) {
+                          long group_a_step, long group_c_step, hipStream_t stream, GluArgs glu = GluArgs{nullptr, 0.f, 0.f, 0}) {
   static bool configured = false;
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_mfma_kernel<EPI>),
@@ -596,11 +613,11 @@ static int launch_grouped(void* C, long ldc, const void* A, long lda, const void
 extern "C" int pi_gemm_mfma_grouped(void* C, int epilogue, long ldc, const void* A, long lda, const void* W, long ldw,
                                     long group_stride, const int* group_of_tile, const int* tile_row0, const int* tile_rows,
                                     int tiles, int N, int K, long group_a_step, long group_c_step, float limit, float alpha,
-                                    hipStream_t stream) {
+                                    const float* gate, long gate_stride, hipStream_t stream) {
   PI_REQUIRE(tiles >= 0 && N > 0 && K > 0, "gemm_mfma_grouped: bad sizes tiles=%d N=%d K=%d", tiles, N, K);
   PI_REQUIRE(group_a_step >= 0 && group_c_step >= 0 && group_a_step % 8 == 0 && group_c_step % 8 == 0,
              "gemm_mfma_grouped: a group's columns in the rows (%ld, %ld) must start at multiples of 8", group_a_step, group_c_step);
-  PI_REQUIRE(group_c_step == 0 || epilogue == EPI_BF16 || epilogue == EPI_F32, "gemm_mfma_grouped: groups side by side in the result's rows store plainly");
+  PI_REQUIRE(group_c_step == 0 || epilogue == EPI_BF16 || epilogue == EPI_F32 || epilogue == EPI_GATE, "gemm_mfma_grouped: groups side by side in the result's rows store plainly");
   PI_REQUIRE(K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && group_stride % 8 == 0, "gemm_mfma_grouped: K (%d) and strides must be multiples of 8", K);
   PI_REQUIRE(256 * lda < (1L << 29) && 256 * ldw < (1L << 29), "gemm_mfma_grouped: row strides (%ld, %ld) are too long", lda, ldw);
   PI_REQUIRE(ldc > 0 && ldc < (1L << 23), "gemm_mfma_grouped: the result's row stride (%ld) is too long", ldc);
@@ -608,11 +625,13 @@ extern "C" int pi_gemm_mfma_grouped(void* C, int epilogue, long ldc, const void*
   PI_REQUIRE(!EPI_GATED(epilogue) || N % 32 == 0, "gemm_mfma_grouped: the gated epilogues need N (%d) to be a multiple of 32", N);
   PI_REQUIRE((long)tiles * ceil_div(N, BN) < 2147483647L, "gemm_mfma_grouped: too many tiles");
   PI_REQUIRE(group_of_tile && tile_row0 && tile_rows, "gemm_mfma_grouped: the tile list is missing");
+  PI_REQUIRE(epilogue != EPI_GATE || (gate && gate_stride > 0), "gemm_mfma_grouped: the gates are missing");
   if (tiles == 0) return 0;
   switch (epilogue) {
     case EPI_BF16: return launch_grouped<EPI_BF16>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
     case EPI_F32: return launch_grouped<EPI_F32>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
-    case EPI_CLAMPED_GLU: return launch_grouped<EPI_CLAMPED_GLU>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream, GluArgs{nullptr, limit, alpha});
+    case EPI_CLAMPED_GLU: return launch_grouped<EPI_CLAMPED_GLU>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream, GluArgs{nullptr, limit, alpha, 0});
+    case EPI_GATE: return launch_grouped<EPI_GATE>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream, GluArgs{gate, 0.f, 0.f, gate_stride});
     case EPI_RELU2: return launch_grouped<EPI_RELU2>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
     case EPI_SWIGLU: return launch_grouped<EPI_SWIGLU>(C, ldc, A, lda, W, ldw, group_stride, group_of_tile, tile_row0, tile_rows, tiles, N, K, group_a_step, group_c_step, stream);
   }
@@ -662,5 +681,5 @@ extern "C" int pi_gemm_mfma_clamped_glu(void* C, long ldc, const void* A, long l
   PI_REQUIRE(((uintptr_t)A % 16 == 0) && ((uintptr_t)W % 16 == 0), "gemm_mfma: operands must be 16-byte aligned");
   PI_REQUIRE(N % 32 == 0, "gemm_mfma: the gated epilogue needs N (%d) to be a multiple of 32", N);
   PI_REQUIRE((long)ceil_div(M, BM) * ceil_div(N, BN) < 2147483647L, "gemm_mfma: too many tiles");
-  return launch<EPI_CLAMPED_GLU>(C, ldc, A, lda, W, ldw, M, N, K, 1, stream, GluArgs{bias, limit, alpha});
+  return launch<EPI_CLAMPED_GLU>(C, ldc, A, lda, W, ldw, M, N, K, 1, stream, GluArgs{bias, limit, alpha, 0});
 }

@@ -10,6 +10,8 @@
 // same cached rows [c | k_r] (one key/value head for all query heads) with c as the value, and
 // Wuv_h is applied to the attention's result afterwards (a product per head).
 //
+// A design may gate every feature of the heads' results: their sigmoid multiplies in the last product's kernel.
+//
 // Norms, angles and rotations are float32; rms(v) = sqrt(mean(v^2) + eps).
 #include "common.h"
 
@@ -17,19 +19,21 @@
 // Cache: keys [page, 1, slot, kv_rank + rot] = [c | k_r]; values transposed [page, 1, v_rows, slot], rows 0 .. kv_rank - 1
 // = c and, when v_rows = kv_rank + rot (values kept as wide as keys, for kernels that want them so), then k_r.
 // table: the step's [T, rot] cosines then sines (rot / 2 each), already scaled; pairs are neighbours (2j, 2j + 1).
+// The rows may go on with `ng` gates; those of a product in pieces are summed into gate_out (float32 [T, ng]), as they are.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(
     T* __restrict__ cq_out, long cq_stride, const float* __restrict__ proj, long proj_stride, const float* __restrict__ wq,
     const float* __restrict__ wkv, const float* __restrict__ table, const int* __restrict__ positions,
     const int* __restrict__ req_of_token, float eps, int q_rank, int kv_rank, int rot, int v_rows, T* __restrict__ k_cache,
     T* __restrict__ v_cache, const int* __restrict__ block_table, int table_width, int page_size, long num_pages,
-    const float* __restrict__ part, int splits, long part_stride) {
+    const float* __restrict__ part, int splits, long part_stride, int ng, float* __restrict__ gate_out) {
   __shared__ float scratch[32];
   extern __shared__ float staged[];
   const long t = blockIdx.x;
   const float* row = proj + t * proj_stride;
   const int N = q_rank + kv_rank + rot;
   if (part) {
+    for (int i = threadIdx.x; i < ng; i += blockDim.x) gate_out[t * ng + i] = split_sum(part, splits, part_stride, t * proj_stride + N + i);
     for (int i = threadIdx.x; i < N; i += blockDim.x) staged[i] = split_sum(part, splits, part_stride, t * proj_stride + i);
     __syncthreads();
     row = staged;
@@ -72,11 +76,12 @@ extern "C" int pi_latent_kv_write(void* cq_out, long cq_stride, int dtype, const
                                   const float* wkv, const float* table, const int* positions, const int* req_of_token, float eps,
                                   int T, int q_rank, int kv_rank, int rot, int v_rows, void* k_cache, void* v_cache,
                                   const int* block_table, int table_width, int page_size, long num_pages, const float* part,
-                                  int splits, long part_stride, hipStream_t stream) {
+                                  int splits, long part_stride, int ng, float* gate_out, hipStream_t stream) {
   PI_REQUIRE(T >= 0 && q_rank >= 0 && kv_rank > 0 && rot >= 0 && rot % 2 == 0, "latent: bad sizes q_rank=%d kv_rank=%d rot=%d", q_rank, kv_rank, rot);
   PI_REQUIRE(v_rows == kv_rank || v_rows == kv_rank + rot, "latent: value rows %d are neither the latent's %d nor the key's %d", v_rows, kv_rank, kv_rank + rot);
   const long row_floats = (long)q_rank + kv_rank + rot;
-  PI_REQUIRE(proj_stride >= row_floats, "latent: projection rows of %ld hold no %ld columns", proj_stride, row_floats);
+  PI_REQUIRE(ng >= 0 && proj_stride >= row_floats + ng, "latent: projection rows of %ld hold no %ld columns and %d gates", proj_stride, row_floats, ng);
+  PI_REQUIRE(!part || ng == 0 || gate_out, "latent: gates in pieces need a place");
   PI_REQUIRE((proj != nullptr) != (part != nullptr), "latent: give the projection as a tensor or as pieces");
   PI_REQUIRE(!part || (splits >= 1 && part_stride >= (long)T * proj_stride), "latent: bad pieces (%d planes of %ld floats)", splits, part_stride);
   PI_REQUIRE(!part || row_floats * 4 <= 60000, "latent: rows of %ld floats in pieces do not fit the staging memory", row_floats);
@@ -88,7 +93,7 @@ extern "C" int pi_latent_kv_write(void* cq_out, long cq_stride, int dtype, const
   const size_t lds = part ? (size_t)row_floats * sizeof(float) : 0;
 #define LKV_GO(TT) hipLaunchKernelGGL(latent_kv_write_kernel<TT>, dim3(T), dim3(256), lds, stream, (TT*)cq_out, cq_stride, proj, proj_stride, \
                                       wq, wkv, table, positions, req_of_token, eps, q_rank, kv_rank, rot, v_rows, (TT*)k_cache,            \
-                                      (TT*)v_cache, block_table, table_width, page_size, num_pages, part, splits, part_stride)
+                                      (TT*)v_cache, block_table, table_width, page_size, num_pages, part, splits, part_stride, ng, gate_out)
   if (dtype == PI_F32) LKV_GO(float);
   else if (dtype == PI_BF16) LKV_GO(bf16_t);
   else return pi_fail("latent: unsupported dtype %d", dtype);
@@ -103,7 +108,7 @@ extern "C" int pi_latent_kv_write(void* cq_out, long cq_stride, int dtype, const
 // columns): the tokens' inputs sit in LDS and are read four at a time; a lane owns one output column, neighbouring lanes
 // read neighbouring weights, sixteen loads in flight; the block's eight waves each take an eighth of k (in whole eights) and
 // their float32 sums - each in ascending k - are added in wave order.  A token's result does not depend on the tokens
-// beside it.  `skip_product`: only the rotated tails are made (the product comes from another kernel).
+// beside it.  `gate`: every result is multiplied by the sigmoid of the gate at its column (rows gate_stride apart).  `skip_product`: only the rotated tails are made (the product comes from another kernel).
 #define HG_TOKENS 8
 #define HG_WAVES 8
 #define HG_LOADS 16        // weights a lane asks for before it waits: a wave's whole share of k at the usual sizes
@@ -111,7 +116,8 @@ template <typename T>
 __global__ __launch_bounds__(HG_WAVES * PI_WAVE) void head_gemm_kernel(T* __restrict__ out, long out_stride, int out_head,
                                                                        const T* __restrict__ a, long a_stride, int a_head,
                                                                        const T* __restrict__ w, int M, int K, int N, int rot,
-                                                                       const float* __restrict__ table, int skip_product) {
+                                                                       const float* __restrict__ table, int skip_product,
+                                                                       const float* __restrict__ gate, long gate_stride) {
   extern __shared__ __attribute__((aligned(16))) float as[];          // [HG_TOKENS][KP], KP = K + rot rounded up to four
   __shared__ float sums[HG_WAVES][HG_TOKENS][PI_WAVE];
   const int h = blockIdx.y, lane = threadIdx.x % PI_WAVE, wave = threadIdx.x / PI_WAVE;
@@ -183,6 +189,7 @@ __global__ __launch_bounds__(HG_WAVES * PI_WAVE) void head_gemm_kernel(T* __rest
         float v = sums[0][tt][lane];
 #pragma unroll
         for (int u = 1; u < HG_WAVES; ++u) v += sums[u][tt][lane];
+        if (gate) v *= 1.0f / (1.0f + expf(-gate[(t0 + tt) * gate_stride + (long)h * out_head + n]));
         out[(t0 + tt) * out_stride + (long)h * out_head + n] = from_float<T>(v);
       }
     }
@@ -201,7 +208,8 @@ __global__ __launch_bounds__(HG_WAVES * PI_WAVE) void head_gemm_kernel(T* __rest
 
 extern "C" int pi_head_gemm(void* out, long out_stride, int out_head, const void* a, long a_stride, int a_head, const void* w,
                             int dtype, int M, int heads, int K, int N, int rot, const float* table, int skip_product,
-                            hipStream_t stream) {
+                            const float* gate, long gate_stride, hipStream_t stream) {
+  PI_REQUIRE(!gate || gate_stride >= (long)(heads - 1) * out_head + N, "head product: gate rows of %ld hold no %d heads", gate_stride, heads);
   PI_REQUIRE(M >= 0 && heads > 0 && K > 0 && N > 0 && rot >= 0 && rot % 2 == 0, "head product: bad sizes M=%d heads=%d K=%d N=%d rot=%d", M, heads, K, N, rot);
   PI_REQUIRE(heads <= 65535 && N <= 65535 * PI_WAVE, "head product: too many heads or columns (%d, %d)", heads, N);
   PI_REQUIRE(a_head >= K + rot && out_head >= N + rot, "head product: heads of %d / %d numbers hold no %d / %d", a_head, out_head, K + rot, N + rot);
@@ -215,10 +223,10 @@ extern "C" int pi_head_gemm(void* out, long out_stride, int out_head, const void
   const dim3 grid(ceil_div(M, HG_TOKENS), heads, skip_product ? 1 : ceil_div(N, PI_WAVE)), block(HG_WAVES * PI_WAVE);
   if (dtype == PI_F32)
     hipLaunchKernelGGL(head_gemm_kernel<float>, grid, block, lds, stream, (float*)out, out_stride, out_head, (const float*)a, a_stride,
-                       a_head, (const float*)w, M, K, N, rot, table, skip_product);
+                       a_head, (const float*)w, M, K, N, rot, table, skip_product, gate, gate_stride);
   else if (dtype == PI_BF16)
     hipLaunchKernelGGL(head_gemm_kernel<bf16_t>, grid, block, lds, stream, (bf16_t*)out, out_stride, out_head, (const bf16_t*)a, a_stride,
-                       a_head, (const bf16_t*)w, M, K, N, rot, table, skip_product);
+                       a_head, (const bf16_t*)w, M, K, N, rot, table, skip_product, gate, gate_stride);
   else
     return pi_fail("head product: unsupported dtype %d", dtype);
   return pi_check_launch("head_gemm");

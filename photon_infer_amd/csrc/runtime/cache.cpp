@@ -73,10 +73,16 @@ int pool_free(Pool& pool, const int* pages, int n, std::string& error) {
 
 struct Group {
   int window = -1;                     // -1: keep every key
+  int kept_blocks = 0;                 // a window's group: the first blocks of every sequence, which are kept while it lives
   Pool pool;
   std::vector<int32_t> table;          // [max_slots][max_blocks], -1 = no page
   std::vector<int32_t> next_block;     // [max_slots] blocks ever handed out (index of the next one)
-  std::vector<int32_t> first_block;    // [max_slots] first block still held
+  std::vector<int32_t> first_block;    // [max_slots] first block still held apart from the kept ones (all of them are held at first)
+
+  // the blocks a slot holds: [0, kept_end) and [rest_begin, next_block)
+  int kept_end(int slot) const { return first_block[slot] < kept_blocks ? first_block[slot] : kept_blocks; }
+  int rest_begin(int slot) const { return first_block[slot]; }
+  int held(int slot) const { return kept_end(slot) + next_block[slot] - rest_begin(slot); }
 };
 
 struct Cache {
@@ -135,10 +141,13 @@ int pi_pool_free(void* h, const int* pages, int n) {
 void pi_pool_reset(void* h) { static_cast<Pool*>(h)->reset(); }
 
 // ---------------------------------------------------------------- the cache manager
-void* pi_cache_create(int n_groups, const int* windows, int page_size, const int* num_pages, int max_slots, int max_model_len) {
+// windows[g]: -1, or how many of a sequence's last positions group g's layers see; keep_first[g] (keep_first may be null): how
+// many of its first positions they see besides, however far the sequence has grown.
+void* pi_cache_create(int n_groups, const int* windows, const int* keep_first, int page_size, const int* num_pages, int max_slots,
+                      int max_model_len) {
   if (n_groups < 0 || page_size <= 0 || max_slots <= 0 || max_model_len <= 0) return nullptr;
   for (int g = 0; g < n_groups; ++g)
-    if (num_pages[g] <= 0) return nullptr;
+    if (num_pages[g] <= 0 || (keep_first && keep_first[g] < 0)) return nullptr;
   Cache* c = new Cache;
   c->page_size = page_size;
   c->max_slots = max_slots;
@@ -148,6 +157,7 @@ void* pi_cache_create(int n_groups, const int* windows, int page_size, const int
   for (int g = 0; g < n_groups; ++g) {
     Group& grp = c->groups[g];
     grp.window = windows[g];
+    grp.kept_blocks = keep_first ? (keep_first[g] - 1 + page_size) / page_size : 0;      // (keep_first - 1 may be -1: no blocks)
     grp.pool.num_pages = num_pages[g];
     grp.pool.reset();
     grp.table.assign((size_t)max_slots * c->max_blocks, -1);
@@ -246,7 +256,8 @@ int pi_cache_commit(void* h, int slot, int new_tokens) {
     // the next query sits at position >= length and reads keys >= length - window + 1
     int first_key = c->length[slot] - grp.window + 1;
     if (first_key < 0) first_key = 0;
-    const int lo = grp.first_block[slot];
+    int lo = grp.first_block[slot];
+    if (lo < grp.kept_blocks) lo = grp.kept_blocks;
     int hi = first_key / c->page_size;
     if (hi > grp.next_block[slot]) hi = grp.next_block[slot];
     if (hi > lo) {
@@ -266,7 +277,11 @@ int pi_cache_release(void* h, int slot) {
   if (!c->is_live(slot)) { c->error = format("slot %d is not live in the cache", slot); return MISUSE; }
   for (Group& grp : c->groups) {
     int32_t* row = c->row(grp, slot);
-    const int lo = grp.first_block[slot], hi = grp.next_block[slot];
+    const int kept = grp.kept_end(slot), lo = grp.rest_begin(slot), hi = grp.next_block[slot];
+    if (kept > 0) {
+      const int st = pool_free(grp.pool, row, kept, c->error);
+      if (st != OK) return st;
+    }
     if (hi > lo) {
       const int st = pool_free(grp.pool, row + lo, hi - lo, c->error);
       if (st != OK) return st;
@@ -345,7 +360,7 @@ int pi_cache_check(void* h) {
         const int p = row[b];
         if (p < 0) continue;
         ++pages;
-        if (b < grp.first_block[s] || b >= grp.next_block[s]) {
+        if ((b >= grp.kept_end(s) && b < grp.rest_begin(s)) || b >= grp.next_block[s]) {
           c->error = format("group %d: slot %d table does not match its block range", (int)gi, s);
           return MISUSE;
         }
@@ -357,7 +372,7 @@ int pi_cache_check(void* h) {
         seen[p] = 1;
       }
       if (!c->live[s] && pages) { c->error = format("group %d: free slot %d still holds pages", (int)gi, s); return MISUSE; }
-      if (pages != grp.next_block[s] - grp.first_block[s]) {
+      if (pages != grp.held(s)) {
         c->error = format("group %d: slot %d table does not match its block range", (int)gi, s);
         return MISUSE;
       }

@@ -432,6 +432,174 @@ extern "C" int pi_sandwich_norm_add(float* x, void* h, int h_dtype, const float*
   return pi_check_launch("sandwich_norm_add");
 }
 
+// ---------------------------------------------------------------- a sublayer's result between two RMS norms
+// A sublayer's result joins the stream through an RMS norm, and the next sublayer's input is made on the way:
+//   x <- x + rms(y; pw);   h = rms(x; nw)       (nw null: no h),   rms(v; w) = v / sqrt(mean(v^2) + eps) * w
+// y is a tensor [T, D]; or the float32 pieces of a product split over k, added here in split order; or the sum over a
+// token's `top` choices of weight * (the row of `a` that the choice got), in choice order (routed experts).
+// With `rows` only those rows of h are made (h row m from stream row rows[m]) and the stream is not written back.
+struct JoinArgs {
+  float* x;
+  const float* a;          // the result, or the experts' rows
+  const float* part;       // pieces [splits, T, D]
+  int splits;
+  const int* entry_row;    // [T, top]: where each choice's row lies
+  const float* weights;    // [T, top]
+  int top;
+  const int* rows;
+  const float* pw;
+  float post_eps;
+  const float* nw;
+  float next_eps;
+  int T, D, entries;
+};
+
+__device__ inline float4 fma4(float w, const float4& v, const float4& s) { return make_float4(fmaf(w, v.x, s.x), fmaf(w, v.y, s.y), fmaf(w, v.z, s.z), fmaf(w, v.w, s.w)); }
+__device__ inline float4 add4(const float4& a, const float4& b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
+
+// columns 4 g .. 4 g + 3 of the result's row t
+__device__ inline float4 join_value4(const JoinArgs& j, long t, int g) {
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (j.part) {
+    const float4* p = reinterpret_cast<const float4*>(j.part + t * j.D) + g;
+    const long plane = (long)j.T * j.D / 4;
+    for (int s0 = 0; s0 < j.splits; s0 += 8) {
+      float4 l[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) l[u] = s0 + u < j.splits ? p[(s0 + u) * plane] : make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v = add4(v, l[u]);
+    }
+    return v;
+  }
+  if (j.entry_row) {
+    for (int c0 = 0; c0 < j.top; c0 += 4) {
+      float4 l[4];
+      float w[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int row = c0 + u < j.top ? j.entry_row[t * j.top + c0 + u] : -1;
+        const bool ok = row >= 0 && row < j.entries;
+        w[u] = ok ? j.weights[t * j.top + c0 + u] : 0.f;
+        l[u] = ok ? reinterpret_cast<const float4*>(j.a + (long)row * j.D)[g] : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v = fma4(w[u], l[u], v);
+    }
+    return v;
+  }
+  return reinterpret_cast<const float4*>(j.a + t * j.D)[g];
+}
+
+__device__ inline float join_value(const JoinArgs& j, long t, int d) {
+  if (j.part) return split_sum(j.part, j.splits, (long)j.T * j.D, t * j.D + d);
+  if (j.entry_row) {
+    float v = 0.f;
+    for (int c = 0; c < j.top; ++c) {
+      const int row = j.entry_row[t * j.top + c];
+      if (row >= 0 && row < j.entries) v = fmaf(j.weights[t * j.top + c], j.a[(long)row * j.D + d], v);
+    }
+    return v;
+  }
+  return j.a[t * j.D + d];
+}
+
+template <typename TH, int VPT>
+__global__ __launch_bounds__(1024) void rms_join_wide_kernel(JoinArgs j, TH* __restrict__ h) {
+  __shared__ float scratch[16];
+  const long m = blockIdx.x, t = j.rows ? j.rows[m] : m;
+  const int groups = j.D / 4;
+  const bool ok = t >= 0 && t < j.T;                // a row outside the stream gives NaN, no fault
+  float4 y[VPT], xo[VPT], w[VPT];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int g = threadIdx.x + i * blockDim.x;
+    const bool in = g < groups;
+    const float4 none = make_float4(0.f, 0.f, 0.f, 0.f), nan = make_float4(NAN, NAN, NAN, NAN);
+    y[i] = !in ? none : ok ? join_value4(j, t, g) : nan;
+    xo[i] = !in ? none : ok ? reinterpret_cast<const float4*>(j.x + t * j.D)[g] : nan;
+    w[i] = in ? reinterpret_cast<const float4*>(j.pw)[g] : none;
+    ss += dot4(y[i]);
+  }
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / j.D + j.post_eps);
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int g = threadIdx.x + i * blockDim.x;
+    xo[i] = make_float4(fmaf(y[i].x * r, w[i].x, xo[i].x), fmaf(y[i].y * r, w[i].y, xo[i].y), fmaf(y[i].z * r, w[i].z, xo[i].z),
+                        fmaf(y[i].w * r, w[i].w, xo[i].w));
+    ss += dot4(xo[i]);
+    if (g >= groups) continue;
+    if (!j.rows) reinterpret_cast<float4*>(j.x + t * j.D)[g] = xo[i];
+    if (j.nw) w[i] = reinterpret_cast<const float4*>(j.nw)[g];
+  }
+  if (!j.nw) return;
+  const float rn = 1.0f / sqrtf(block_sum(ss, scratch) / j.D + j.next_eps);
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int g = threadIdx.x + i * blockDim.x;
+    if (g < groups)
+      store4<TH>(h + m * j.D + 4 * (long)g, make_float4(xo[i].x * rn * w[i].x, xo[i].y * rn * w[i].y, xo[i].z * rn * w[i].z, xo[i].w * rn * w[i].w));
+  }
+}
+
+// the same for any width: the row stays in LDS
+template <typename TH>
+__global__ __launch_bounds__(256) void rms_join_kernel(JoinArgs j, TH* __restrict__ h) {
+  extern __shared__ float row[];
+  __shared__ float scratch[16];
+  const long m = blockIdx.x, t = j.rows ? j.rows[m] : m;
+  const bool ok = t >= 0 && t < j.T;
+  float ss = 0.f;
+  for (int d = threadIdx.x; d < j.D; d += blockDim.x) {
+    const float v = ok ? join_value(j, t, d) : NAN;
+    row[d] = v;
+    ss = fmaf(v, v, ss);
+  }
+  const float r = 1.0f / sqrtf(block_sum(ss, scratch) / j.D + j.post_eps);
+  ss = 0.f;
+  for (int d = threadIdx.x; d < j.D; d += blockDim.x) {       // a thread meets its own entries only
+    const float v = fmaf(row[d] * r, j.pw[d], ok ? j.x[t * j.D + d] : NAN);
+    row[d] = v;
+    if (ok && !j.rows) j.x[t * j.D + d] = v;
+    ss = fmaf(v, v, ss);
+  }
+  if (!j.nw) return;
+  const float rn = 1.0f / sqrtf(block_sum(ss, scratch) / j.D + j.next_eps);
+  for (int d = threadIdx.x; d < j.D; d += blockDim.x) h[m * j.D + d] = from_float<TH>(row[d] * rn * j.nw[d]);
+}
+
+extern "C" int pi_rms_join(float* x, void* h, int h_dtype, const float* a, const float* part, int splits, const int* entry_row,
+                           const float* weights, int top, int entries, const int* rows, int M, const float* pw, float post_eps,
+                           const float* nw, float next_eps, int T, int D, hipStream_t stream) {
+  PI_REQUIRE(T >= 0 && M >= 0 && D > 0 && D <= 16000, "rms join: bad sizes T=%d M=%d D=%d", T, M, D);
+  PI_REQUIRE(x && pw && (a != nullptr) != (part != nullptr), "rms join: the stream, the norm's weight and one result (a tensor or pieces) are needed");
+  PI_REQUIRE(!part || (splits >= 1 && !entry_row), "rms join: %d pieces", splits);
+  PI_REQUIRE(!entry_row || (weights && top > 0 && entries >= 0), "rms join: choices need their weights");
+  PI_REQUIRE(!nw || (h && (h_dtype == PI_F32 || h_dtype == PI_BF16)), "rms join: the next norm needs a place for its result (dtype %d)", h_dtype);
+  PI_REQUIRE(rows ? nw != nullptr : M == T, "rms join: %d rows of %d", M, T);
+  if (M == 0) return 0;
+  const JoinArgs j{x, a, part, splits, entry_row, weights, top, rows, pw, post_eps, nw, next_eps, T, D, entries};
+  const bool f32 = !nw || h_dtype == PI_F32;
+  int wide_threads = 0, vpt = 0;
+  bool aligned = true;
+  for (const void* p : {(const void*)x, (const void*)h, (const void*)a, (const void*)part, (const void*)pw, (const void*)nw}) aligned = aligned && (uintptr_t)p % 16 == 0;
+  if (aligned && wide_row_shape(M, D, wide_threads, vpt)) {
+#define RJ_GO(TH, V) hipLaunchKernelGGL((rms_join_wide_kernel<TH, V>), dim3(M), dim3(wide_threads), 0, stream, j, (TH*)h)
+#define RJ_PICK(TH) do { if (vpt <= 1) RJ_GO(TH, 1); else if (vpt <= 2) RJ_GO(TH, 2); else RJ_GO(TH, 4); } while (0)
+    if (f32) RJ_PICK(float); else RJ_PICK(bf16_t);
+#undef RJ_PICK
+#undef RJ_GO
+    return pi_check_launch("rms_join_wide");
+  }
+  const int threads = D >= 1024 ? 256 : (D >= 256 ? 128 : 64);
+  const size_t lds = (size_t)D * sizeof(float);
+  if (f32) hipLaunchKernelGGL(rms_join_kernel<float>, dim3(M), dim3(threads), lds, stream, j, (float*)h);
+  else hipLaunchKernelGGL(rms_join_kernel<bf16_t>, dim3(M), dim3(threads), lds, stream, j, (bf16_t*)h);
+  return pi_check_launch("rms_join");
+}
+
 // ---------------------------------------------------------------- two attention maps into one head
 // Differential attention: head n of kv group g holds the results a1 and a2 of two softmax maps over the same
 // values.  In `attn` the maps are heads of their own, and a head's value vector may come in `split` equal pieces

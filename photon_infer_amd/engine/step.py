@@ -196,7 +196,7 @@ class ModelRunner:
             self.max_model_len = min(self.max_model_len, num_pages * self.page_size)
         self.num_pages = num_pages
         self.cache = CacheManager([g.window for g in self.plan.groups], self.page_size, num_pages,
-                                  o.max_batch, self.max_model_len)
+                                  o.max_batch, self.max_model_len, keep_first=[g.keep_first for g in self.plan.groups])
         self.states = StateSlots(self.plan.states, o.max_batch, self.device)
         # one pool per paged tensor of every mixer that owns pages, [pages, *page shape]: for
         # attention, keys [pages, kv_heads, page, head_dim] and values [pages, kv_heads, head_dim,

@@ -440,7 +440,7 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
                     value_dim: Optional[int] = None, slopes: Optional[torch.Tensor] = None,
                     sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                     softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0,
-                    feature_gate: Optional[torch.Tensor] = None) -> None:
+                    feature_gate: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
     """Causal attention of every token of the step over its request's pages.
 
     ``ctx`` carries ``positions`` and ``req_of_token`` ([T] int32), the step's shape on the host
@@ -454,12 +454,15 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
     ``out_scale`` (a factor on every output, applied in float32 before the one rounding), ``chunk`` (C > 0: positions
     are cut into chunks of C, counted from 0, and a token sees the keys of its own chunk only), ``feature_gate``
     (float32 [T, heads * value_dim], rows may lie apart; instead of ``gate``: feature i of the output is multiplied by
-    sigmoid(feature_gate[t, i]), in float32 before the one rounding).
+    sigmoid(feature_gate[t, i]), in float32 before the one rounding), ``keep_first`` (N > 0: the sequence's first N keys
+    are seen besides those of the window or chunk).
     """
     _gpu(out, q, k_cache, v_cache, block_table, ctx.positions, ctx.req_of_token)
-    chunk = int(chunk or 0)
-    if chunk < 0:
-        raise KernelError(f"attention: a chunk must be positive, got {chunk}")
+    chunk, keep = int(chunk or 0), int(keep_first or 0)
+    if chunk < 0 or keep < 0:
+        raise KernelError(f"attention: a chunk must be positive and kept first keys not negative, got {chunk} and {keep}")
+    if not (window or chunk):
+        keep = 0                      # every key is seen anyway
     T = q.shape[0]
     vd = head_dim if value_dim is None else int(value_dim)
     softcap, out_scale = float(softcap or 0.0), float(out_scale)
@@ -471,7 +474,7 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
             raise KernelError("attention: gates per head and per feature do not go together")
         gate_stride, gate = _f32_rows(feature_gate, T, num_heads * vd, "attention gates"), feature_gate
         _gpu(feature_gate)
-    plain = value_dim is None and slopes is None and sinks is None and gate is None and softcap == 0.0 and out_scale == 1.0
+    plain = value_dim is None and slopes is None and sinks is None and gate is None and softcap == 0.0 and out_scale == 1.0 and keep == 0
     if plain:
         check_attention_sizes(num_heads, num_kv_heads, head_dim)
     else:
@@ -493,18 +496,18 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
         # the matrix-core kernels take heads whose values are as wide as their keys, options included
         from . import fast
         if fast.paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_kv_heads, head_dim,
-                                page_size, scale, window, pages, ws, slopes, sinks, gate, softcap, out_scale, chunk, gate_stride):
+                                page_size, scale, window, pages, ws, slopes, sinks, gate, softcap, out_scale, chunk, gate_stride, keep):
             return
     # a step of few tokens over long contexts: its keys cut into ranges, merged by a second kernel
     # (as many as the context-length bucket asks for, so that a step gives the same bits eagerly and replayed)
     # (chunks bound a token's keys whatever the context: one range)
-    ranges = general_attention_ranges(T, num_heads, min(int(ctx.max_kv_len), chunk) if chunk else int(ctx.max_kv_len))
+    ranges = general_attention_ranges(T, num_heads, min(int(ctx.max_kv_len), chunk + keep) if chunk else int(ctx.max_kv_len))
     part = torch.empty(T * num_heads * ranges * (vd + 2), dtype=torch.float32, device=q.device) if ranges > 1 else None
     _lib.call("core", "pi_paged_attention_general", out.data_ptr(), _rows(out, "attention out"), q.data_ptr(),
               _rows(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), _dt(q), block_table.data_ptr(),
               block_table.shape[1], ctx.req_of_token.data_ptr(), ctx.positions.data_ptr(), T, num_heads,
               num_kv_heads, head_dim, page_size, float(scale), int(window), pages, ranges, _ptr(part),
-              0 if part is None else part.numel(), vd, _ptr(slopes), _ptr(sinks), _ptr(gate), gate_stride, softcap, out_scale, chunk, _stream())
+              0 if part is None else part.numel(), vd, _ptr(slopes), _ptr(sinks), _ptr(gate), gate_stride, softcap, out_scale, chunk, keep, _stream())
 
 
 def general_attention_ranges(tokens: int, num_heads: int, max_kv_len: int) -> int:
@@ -546,12 +549,12 @@ def decode_length_bucket(max_kv_len: int) -> int:
 
 
 def attention_planner(dtype: torch.dtype, num_heads: int, num_kv_heads: int, head_dim: int, page_size: int,
-                      window: int, device, chunk: int = 0):
+                      window: int, device, chunk: int = 0, keep_first: int = 0):
     """What makes a step's work lists for an attention mixer of these sizes (a hashable object with
     ``plan(q_lens, kv_lens)``; equal ones share a plan), or None when its kernels need none."""
     if _FAST and dtype == torch.bfloat16 and _lib.build.MODULES["bf16"]:
         from . import fast
-        return fast.attention_planner(dtype, num_heads, num_kv_heads, head_dim, page_size, int(window), torch.device(device), int(chunk or 0))
+        return fast.attention_planner(dtype, num_heads, num_kv_heads, head_dim, page_size, int(window), torch.device(device), int(chunk or 0), int(keep_first or 0))
     return None
 
 
@@ -616,6 +619,61 @@ def sandwich_norm_add(x: torch.Tensor, a: torch.Tensor, post, eps: float, nxt=No
     _lib.call("core", "pi_sandwich_norm_add", x.data_ptr(), _ptr(h), _dt(h) if h is not None else PI_F32, a.data_ptr(), _ptr(a_bias),
               _ptr(w_a), _ptr(b), _ptr(w_b), post[0].data_ptr(), post[1].data_ptr(), _ptr(nxt[0]) if nxt is not None else None,
               _ptr(nxt[1]) if nxt is not None else None, float(eps), T, D, _stream())
+    return h
+
+
+# Key in a step's ``scratch``: the ``LeftChoices`` of a routed feed-forward whose arrangement sums them itself.
+LEFT_CHOICES = "choices left to whoever reads the result"
+
+
+class LeftChoices:
+    """A sublayer's result [T, D] that is still a sum over each token's chosen experts: ``y`` float32 [entries, D] in expert
+    order, one weight per entry, and where each (token, choice) lies (``ExpertRows``)."""
+
+    def __init__(self, target, y, weights, rows):
+        self.target, self.y, self.weights, self.rows = target, y, weights, rows
+
+
+def rms_join(x: torch.Tensor, y: torch.Tensor, post: torch.Tensor, post_eps: float, nxt: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+             h_dtype: Optional[torch.dtype] = None, rows: Optional[torch.Tensor] = None, ws: Optional[KernelWorkspace] = None,
+             choices: Optional[LeftChoices] = None) -> Optional[torch.Tensor]:
+    """x += rms(y; post), rms(v; w) = v / sqrt(mean(v^2) + eps) * w, float32; with ``nxt`` (float32 [D]) and ``h_dtype`` the
+    RMS norm of the new stream is returned in that type, made in the same pass - of the rows ``rows`` (int32) only, if
+    given: the stream is then not written back.  ``y`` is a sublayer's float32 result [T, D]; when its product is still in
+    pieces in ``ws`` they are added here, and ``choices`` gives it as a sum over experts' rows instead."""
+    pieces = ws.take_result(y) if ws is not None and choices is None else None
+    _gpu(x, y, post, nxt, rows)
+    T, D = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous():
+        raise KernelError(f"rms join: the stream must be contiguous float32, got {x.dtype} {tuple(x.shape)}")
+    _f32_vector(post, D, "rms join norm weight")
+    _f32_vector(nxt, D, "rms join next norm weight")
+    a, entry_row, weights, top, entries = None, None, None, 0, 0
+    if choices is not None:
+        a, top, entries = choices.y, choices.rows.top, choices.rows.rows
+        entry_row, weights = choices.rows.entry_row, choices.weights
+        if a.dtype != torch.float32 or not a.is_contiguous() or tuple(a.shape) != (entries, D) or entries != T * top:
+            raise KernelError(f"rms join: expert rows must be contiguous float32 [{T * top}, {D}], got {a.dtype} {tuple(a.shape)}")
+        _f32_vector(weights.view(-1), entries, "rms join choice weights")
+    elif pieces is not None:
+        ws.counts["added_by_join"] += 1
+        if (pieces.M, pieces.N) != (T, D):
+            raise KernelError(f"rms join: pieces [{pieces.M}, {pieces.N}] of a result [{T}, {D}]")
+    else:
+        a = y
+        if y.dtype != torch.float32 or not y.is_contiguous() or tuple(y.shape) != (T, D):
+            raise KernelError(f"rms join: the result must be contiguous float32 [{T}, {D}]")
+    h, M = None, T
+    if rows is not None:
+        M = rows.numel()
+        _i32(rows, "rms join rows", M)
+        if nxt is None:
+            raise KernelError("rms join: rows without a norm to make of them")
+    if nxt is not None:
+        h = torch.empty((M, D), dtype=h_dtype or torch.float32, device=x.device)
+    _lib.call("core", "pi_rms_join", x.data_ptr(), _ptr(h), _dt(h) if h is not None else PI_F32, _ptr(a), pieces.part.data_ptr() if pieces is not None else None,
+              pieces.splits if pieces is not None else 0, _ptr(entry_row), _ptr(weights), top, entries, _ptr(rows), M, post.data_ptr(), float(post_eps),
+              _ptr(nxt), float(next_eps), T, D, _stream())
     return h
 
 
@@ -791,22 +849,24 @@ def qk_rope_norm_write(q_out: torch.Tensor, proj, bias: Optional[torch.Tensor], 
 # ----------------------------------------------------------------------------- attention through a latent
 def latent_kv_write(cq_out: Optional[torch.Tensor], proj, w_q: Optional[torch.Tensor], w_kv: torch.Tensor, table: Optional[torch.Tensor],
                     ctx, eps: float, q_rank: int, kv_rank: int, rot: int, k_cache: Optional[torch.Tensor],
-                    v_cache: Optional[torch.Tensor], block_table: Optional[torch.Tensor], page_size: int) -> None:
+                    v_cache: Optional[torch.Tensor], block_table: Optional[torch.Tensor], page_size: int, num_gates: int = 0) -> Optional[torch.Tensor]:
     """From float32 projection rows [query latent: q_rank | key/value latent: kv_rank | shared rotated key part: rot]
     (a tensor, or ``Partials``): the query latent RMS-normalised with ``w_q`` into ``cq_out`` ([T, q_rank], the
     activation type); the key/value latent RMS-normalised with ``w_kv`` and the rotated part turned by the token's
     angles (``table``: the step's [T, rot] cosines and sines, neighbouring pairs) into the pages: keys
-    [pages, 1, page, kv_rank + rot] = [latent | rotated part], values transposed [pages, 1, kv_rank (+ rot), page]."""
+    [pages, 1, page, kv_rank + rot] = [latent | rotated part], values transposed [pages, 1, kv_rank (+ rot), page].
+    ``num_gates``: the rows go on with so many gates; they are returned as they are, float32 [T, num_gates] (a view of a
+    projection that is a tensor, otherwise their pieces summed; None without gates)."""
     pieces = proj if isinstance(proj, Partials) else None
     _gpu(cq_out, pieces.part if pieces is not None else proj, w_q, w_kv, table, k_cache, v_cache, block_table)
     N = q_rank + kv_rank + rot
     if pieces is not None:
         T = pieces.M
-        if pieces.N < N:
+        if pieces.N < N + num_gates:
             raise KernelError(f"latent: pieces [{pieces.M}, {pieces.N}] do not hold {N} columns")
     else:
         T = proj.shape[0]
-        if proj.dtype != torch.float32 or proj.dim() != 2 or proj.shape[1] < N:
+        if proj.dtype != torch.float32 or proj.dim() != 2 or proj.shape[1] < N + num_gates:
             raise KernelError(f"latent: projection must be float32 [{T}, >= {N}], got {proj.dtype} {tuple(proj.shape)}")
     if q_rank and (cq_out is None or cq_out.shape != (T, q_rank)):
         raise KernelError(f"latent: the query latent's place must be [{T}, {q_rank}]")
@@ -825,25 +885,31 @@ def latent_kv_write(cq_out: Optional[torch.Tensor], proj, w_q: Optional[torch.Te
             raise KernelError("latent: block table must be contiguous int32 [requests, width]")
     _i32(ctx.positions, "positions", T)
     _i32(ctx.req_of_token, "req_of_token", T)
+    gates = None
+    if num_gates:
+        gates = torch.empty((T, num_gates), dtype=torch.float32, device=w_kv.device) if pieces is not None else proj[:, N:N + num_gates]
     _lib.call("core", "pi_latent_kv_write", _ptr(cq_out), _rows(cq_out, "query latent") if cq_out is not None else 0,
               PI_F32 if dtype == torch.float32 else PI_BF16, None if pieces is not None else proj.data_ptr(),
               pieces.N if pieces is not None else _rows(proj, "projection"), _ptr(w_q), w_kv.data_ptr(), _ptr(table),
               ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(), float(eps), T, q_rank, kv_rank, rot, v_rows, _ptr(k_cache),
               _ptr(v_cache), _ptr(block_table), block_table.shape[1] if k_cache is not None else 0, page_size, pages,
               pieces.part.data_ptr() if pieces is not None else None, pieces.splits if pieces is not None else 0,
-              pieces.M * pieces.N if pieces is not None else 0, _stream())
+              pieces.M * pieces.N if pieces is not None else 0, int(num_gates), _ptr(gates) if pieces is not None else None, _stream())
+    return gates
 
 
 def head_gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, heads: int, a_head: Optional[int] = None,
               out_head: Optional[int] = None, rot: int = 0, table: Optional[torch.Tensor] = None,
-              w_rows: Optional[torch.Tensor] = None) -> None:
+              w_rows: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """A product per head: ``out[t, h * out_head + n] = sum_k a[t, h * a_head + k] * w[h, k, n]`` with ``w``
     [heads, K, N] (a head's matrix stored with its inputs as rows), float32 sums.  ``a_head`` / ``out_head``: the
     distance between two heads in a row of ``a`` / ``out`` (default K + rot / N + rot).  ``rot`` > 0: the ``rot`` numbers
     behind a head's K inputs are turned by the token's angles (``table``: the step's [T, rot] cosines and sines,
     neighbouring pairs) and placed behind the head's N results.  ``w_rows``: the same matrices stored [heads, N, K]
-    (a head's outputs as rows), which the matrix-core kernel reads for steps of many tokens (bfloat16)."""
-    _gpu(out, a, w, table, w_rows)
+    (a head's outputs as rows), which the matrix-core kernel reads for steps of many tokens (bfloat16).  ``gate`` (float32 [tokens, columns of ``out``],
+    rows may lie apart; not with ``rot``): every result is multiplied by the sigmoid of the gate at its column, in float32
+    before the one rounding."""
+    _gpu(out, a, w, table, w_rows, gate)
     if w.dim() != 3 or w.shape[0] != heads or not w.is_contiguous():
         raise KernelError(f"head product: weights must be contiguous [{heads}, K, N], got {tuple(w.shape)}")
     K, N = int(w.shape[1]), int(w.shape[2])
@@ -858,17 +924,23 @@ def head_gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, heads: int, a
         raise KernelError(f"head product: cos / sin table must be contiguous float32 [{M}, {rot}]")
     if M == 0:
         return
+    gate_stride = 0
+    if gate is not None:
+        if rot:
+            raise KernelError("head product: gates and a rotated tail do not go together")
+        gate_stride = _f32_rows(gate, M, (heads - 1) * out_head + N, "head product gates")
     skip = 0
     if _FAST and a.dtype == torch.bfloat16 and w_rows is not None:
         if w_rows.shape != (heads, N, K) or w_rows.dtype != a.dtype or not w_rows.is_contiguous():
             raise KernelError(f"head product: the row-major weights must be contiguous [{heads}, {N}, {K}] {a.dtype}")
         from . import fast
-        if fast.head_gemm(out, a, w_rows, heads, K, N, a_head, out_head, _rows(a, "head product a"), _rows(out, "head product out")):
+        if fast.head_gemm(out, a, w_rows, heads, K, N, a_head, out_head, _rows(a, "head product a"), _rows(out, "head product out"),
+                          gate, gate_stride):
             if rot == 0:
                 return
             skip = 1          # the rotated tails are still to make
     _lib.call("core", "pi_head_gemm", out.data_ptr(), _rows(out, "head product out"), out_head, a.data_ptr(), _rows(a, "head product a"),
-              a_head, w.data_ptr(), _dt(a), M, heads, K, N, int(rot), _ptr(table), skip, _stream())
+              a_head, w.data_ptr(), _dt(a), M, heads, K, N, int(rot), _ptr(table), skip, _ptr(gate), gate_stride, _stream())
 
 
 # ----------------------------------------------------------------------------- matrix memory
@@ -1019,7 +1091,7 @@ def _grouped_fast(out, a, w, rows: ExpertRows, epilogue: int, limit: float = 0.0
         return False
     _lib.call("bf16", "pi_gemm_mfma_grouped", out.data_ptr(), epilogue, _rows(out, "out"), a.data_ptr(), _rows(a, "a"), w.data_ptr(),
               K, w.shape[1] * K, rows.tile_expert.data_ptr(), rows.tile_row0.data_ptr(), rows.tile_rows.data_ptr(),
-              rows.tile_expert.numel(), w.shape[1], K, 0, 0, float(limit), float(alpha), _stream())
+              rows.tile_expert.numel(), w.shape[1], K, 0, 0, float(limit), float(alpha), None, 0, _stream())
     return True
 
 
@@ -1400,6 +1472,48 @@ def token_shift(h: torch.Tensor, shift: torch.Tensor, state: torch.Tensor, ctx, 
     _lib.call("core", "pi_token_shift", out.data_ptr(), _dt(out), h.data_ptr(), shift.data_ptr(), state.data_ptr(), state.stride(0), state.shape[0],
               ctx.q_start.data_ptr(), ctx.slots.data_ptr(), ctx.req_of_token.data_ptr(), T, D, _stream())
     return out
+
+
+def retention(y: torch.Tensor, proj, rotary, decay: torch.Tensor, k_scale: float, eps: float, ctx, state: torch.Tensor, heads: int,
+              key_dim: int, value_dim: int) -> None:
+    """Retention over the step's tokens, request by request, from and into the requests' state rows (``state`` float32
+    [slots, >= heads * key_dim * value_dim], rows ``ctx.slots``): from float32 projection rows [q | k | v | gates] (a tensor; in
+    a step of single tokens also ``Partials``) ``S <- decay S + k' v^T; o = S^T q'`` with q and k rotated (``rotary`` as for
+    ``rope_kv_write``) and k times ``k_scale``; ``y`` [T, heads * value_dim] = o / rms(o) (per head) * silu(gate).
+    ``decay``: float32 [2, heads], the decays and their base-2 logarithms (``decay_table``)."""
+    pieces = proj if isinstance(proj, Partials) else None
+    _gpu(y, pieces.part if pieces is not None else proj, decay, state)
+    T, cols = y.shape[0], 2 * heads * (key_dim + value_dim)
+    single = bool(getattr(ctx, "all_decode", False))
+    if pieces is not None:
+        if not single:
+            raise KernelError("retention: only a step of single tokens takes a projection in pieces")
+        if pieces.M != T or pieces.N < cols:
+            raise KernelError(f"retention: pieces [{pieces.M}, {pieces.N}] do not hold {cols} columns of {T} tokens")
+    if y.dim() != 2 or y.shape[1] != heads * value_dim or not y.is_contiguous():
+        raise KernelError(f"retention: output must be contiguous [{T}, {heads * value_dim}], got {tuple(y.shape)}")
+    _f32_vector(decay, 2 * heads, "retention decays")
+    _state_rows(state, heads * key_dim * value_dim, "retention")
+    _i32(ctx.q_start, "q_start", ctx.R + 1)
+    _i32(ctx.slots, "slots", ctx.R)
+    table_ptr, rdim, inter, _keep = _rotary_args(rotary, ctx.positions, T)
+    longest = 1 if single else max(2, int(getattr(ctx, "max_q_len", 0) or T))
+    lib = _lib.load("core")
+    lib.pi_retention_work_floats.restype = ctypes.c_long
+    floats = int(lib.pi_retention_work_floats(T, ctx.R, longest, heads, key_dim, value_dim))
+    work = torch.empty(floats, dtype=torch.float32, device=y.device) if floats else None
+    _lib.call("core", "pi_retention", y.data_ptr(), _dt(y), None if pieces is not None else proj.data_ptr(),
+              pieces.N if pieces is not None else _f32_rows(proj, T, cols, "retention projection"), pieces.part.data_ptr() if pieces is not None else None,
+              pieces.splits if pieces is not None else 0, table_ptr, rdim, int(bool(inter)), decay.data_ptr(), float(k_scale), float(eps),
+              ctx.q_start.data_ptr(), ctx.slots.data_ptr(), ctx.R, T, longest, state.data_ptr(), state.stride(0), state.shape[0], heads, key_dim,
+              value_dim, _ptr(work), floats, _stream())
+
+
+def decay_table(decays, device) -> torch.Tensor:
+    """float32 [2, heads]: fixed decays and their base-2 logarithms (of a decay of zero: a number whose powers are zero)."""
+    d = torch.tensor([float(x) for x in decays], dtype=torch.float64)
+    logs = torch.where(d > 0, torch.log2(d.clamp(min=1e-300)), torch.full_like(d, -1e30))
+    return torch.stack([d, logs]).to(torch.float32).to(device).contiguous()
 
 
 def min_gru(out: torch.Tensor, proj, bias: torch.Tensor, ctx, state: torch.Tensor, width: int) -> None:

@@ -27,12 +27,12 @@ _SIGNATURES = {
         "pi_swiglu": [P, P, I, I, I, I, P],
         "pi_rope_kv_write": [P, L, P, L, P, L, I, P, P, P, I, I, I, I, I, I, I, P, P, P, I, I, L, P, I, I, I, I, I, I, P, P],
         "pi_gemm_general": [P, I, L, P, I, L, P, I, L, I, I, I, I, P],
-        "pi_paged_attention_general": [P, L, P, L, P, P, I, P, I, P, P, I, I, I, I, I, F, I, L, I, P, L, I, P, P, P, L, F, F, I, P],
+        "pi_paged_attention_general": [P, L, P, L, P, P, I, P, I, P, P, I, I, I, I, I, F, I, L, I, P, L, I, P, P, P, L, F, F, I, I, P],
         "pi_branch_norm_add": [P, P, I, P, P, P, P, P, F, F, I, I, P],
         "pi_cast_stream": [P, I, P, L, P],
         "pi_qk_norm_kv_write": [P, L, P, I, P, L, P, P, P, P, F, F, I, I, I, I, I, I, I, P, P, P, I, I, L, P, I, L, I, I, P],
-        "pi_latent_kv_write": [P, L, I, P, L, P, P, P, P, P, F, I, I, I, I, I, P, P, P, I, I, L, P, I, L, P],
-        "pi_head_gemm": [P, L, I, P, L, I, P, I, I, I, I, I, I, P, I, P],
+        "pi_latent_kv_write": [P, L, I, P, L, P, P, P, P, P, F, I, I, I, I, I, P, P, P, I, I, L, P, I, L, I, P, P],
+        "pi_head_gemm": [P, L, I, P, L, I, P, I, I, I, I, I, I, P, I, P, L, P],
         "pi_matrix_memory_scan": [P, L, P, L, I, I, I, I, I, P, P, F, F, P, P, I, P, L, I, I, I, I, I, I, P, L, P],
         "pi_head_norm_gate": [P, I, P, L, P, L, P, F, I, I, I, F, I, P],
         "pi_route": [P, P, P, L, I, I, I, I, I, I, I, P, F, I, P],
@@ -43,6 +43,8 @@ _SIGNATURES = {
         "pi_activation": [P, I, P, L, I, I, P],
         "pi_layer_norm": [P, I, P, P, P, P, F, I, I, I, P],
         "pi_sandwich_norm_add": [P, P, I, P, P, P, P, P, P, P, P, P, F, I, I, P],
+        "pi_rms_join": [P, P, I, P, P, I, P, P, I, I, P, I, P, F, P, F, I, I, P],
+        "pi_retention": [P, I, P, L, P, I, P, I, I, P, F, F, P, P, I, I, I, P, L, I, I, I, I, P, L, P],
         "pi_diff_combine": [P, I, P, I, F, F, F, I, I, I, I, I, P],
         "pi_paged_attention_general_ranges": [I, I, I],
         "pi_rope_table": [P, P, P, I, I, F, P],
@@ -57,13 +59,13 @@ _SIGNATURES = {
         "pi_gemm_mfma": [P, I, L, P, L, P, L, I, I, I, I, P],
         "pi_gemm_mfma_pieces": [I, I],
         "pi_gemm_mfma_clamped_glu": [P, L, P, L, P, L, I, I, I, P, F, F, P],
-        "pi_gemm_mfma_grouped": [P, I, L, P, L, P, L, L, P, P, P, I, I, I, L, L, F, F, P],
+        "pi_gemm_mfma_grouped": [P, I, L, P, L, P, L, L, P, P, P, I, I, I, L, L, F, F, P, L, P],
         "pi_gemm_skinny": [P, I, L, P, L, P, L, I, I, I, I, P, L, P, I, P],
         "pi_splitk_reduce": [P, I, L, P, I, I, I, P],
         "pi_attention_tile_rows": [I, I, I],
-        "pi_attention_prefill_mfma": [P, L, P, L, P, P, P, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, L, P, P, P, L, F, F, I, P],
+        "pi_attention_prefill_mfma": [P, L, P, L, P, P, P, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I, L, P, P, P, L, F, F, I, I, P],
         "pi_attention_combine_rows": [P, L, P, I, P, I, I, I, P, P, L, F, P],
-        "pi_attention_decode": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, L, I, P, L, P, P, P, L, F, F, I, P],
+        "pi_attention_decode": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, L, I, P, L, P, P, P, L, F, F, I, I, P],
         "pi_attention_decode_fused": [P, L, P, L, P, I, I, I, P, I, P, P, P, I, P, P, I, I, I, I, I, F, I, L, I, P, L, I, P],
         "pi_gemm_skinny_ranges": [P, I, L, P, I, I, I, P, L, I, I, I, P, L, P, I, P],
     },

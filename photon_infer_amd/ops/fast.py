@@ -280,6 +280,7 @@ def gemm_pieces(a, w, ws: Optional[KernelWorkspace]) -> Optional[Partials]:
     return _skinny(0, EPI_F32, N, a, w, M, N, K, lda, ldw, splits, ws)
 
 
+EPI_GATE = 7
 EPI_OF_ACTIVATION = {"relu2": 5, "gelu": 6}
 
 
@@ -330,7 +331,7 @@ def _head_tiles(M: int, heads: int, device) -> Tuple[torch.Tensor, torch.Tensor,
     return tuple(torch.from_numpy(x).to(device) for x in (group, row0, count))
 
 
-def head_gemm(out, a, w_rows, heads: int, K: int, N: int, a_head: int, out_head: int, lda: int, ldc: int) -> bool:
+def head_gemm(out, a, w_rows, heads: int, K: int, N: int, a_head: int, out_head: int, lda: int, ldc: int, gate=None, gate_stride: int = 0) -> bool:
     """A product per head (``w_rows`` [heads, N, K]) as one launch of the grouped tile kernel, every head a group that
     sits at columns of its own in the rows of ``a`` and ``out``; False: not for these sizes (few tokens, or heads that
     do not start at multiples of 8 columns)."""
@@ -340,8 +341,9 @@ def head_gemm(out, a, w_rows, heads: int, K: int, N: int, a_head: int, out_head:
     if 256 * lda >= (1 << 29) or ldc >= (1 << 23) or out.data_ptr() % 4:
         return False
     group, row0, count = _head_tiles(M, heads, a.device)
-    _lib.call("bf16", "pi_gemm_mfma_grouped", out.data_ptr(), EPI_BF16, ldc, a.data_ptr(), lda, w_rows.data_ptr(), K, N * K,
-              group.data_ptr(), row0.data_ptr(), count.data_ptr(), group.numel(), N, K, a_head, out_head, 0.0, 0.0, _stream())
+    _lib.call("bf16", "pi_gemm_mfma_grouped", out.data_ptr(), EPI_BF16 if gate is None else EPI_GATE, ldc, a.data_ptr(), lda, w_rows.data_ptr(), K, N * K,
+              group.data_ptr(), row0.data_ptr(), count.data_ptr(), group.numel(), N, K, a_head, out_head, 0.0, 0.0,
+              None if gate is None else gate.data_ptr(), gate_stride, _stream())
     return True
 
 
@@ -385,6 +387,7 @@ class AttentionPlanner:
     units: int                # compute units of the device
     blocks_per_unit: int = 2  # blocks that a unit holds at a time (attention_blocks_per_unit)
     chunk: int = 0            # C > 0: a token sees the keys of its own chunk of C positions only
+    keep: int = 0             # N > 0: a token sees the first N keys besides
 
     def plan(self, q_lens: Sequence[int], kv_lens: Sequence[int]):
         """None for a step of single tokens only (the key-split kernel needs no list); otherwise
@@ -408,7 +411,7 @@ class AttentionPlanner:
                     lo = max(0, first - window + 1) if window > 0 else 0
                     if chunk > 0:
                         lo = max(lo, first - first % chunk)
-                    walks.append(last // 128 - lo // 128 + 1)
+                    walks.append(last // 128 - lo // 128 + 1 + min(-(-self.keep // 128), lo // 128))
                     first_row.append(row0 + start)
                     n_tok.append(min(tile_rows, n - start))
             row0 += n
@@ -443,7 +446,7 @@ class AttentionPlanner:
 
 @functools.lru_cache(maxsize=None)
 def attention_planner(dtype, num_heads: int, num_kv_heads: int, head_dim: int, page_size: int, window: int,
-                      device, chunk: int = 0) -> Optional[AttentionPlanner]:
+                      device, chunk: int = 0, keep: int = 0) -> Optional[AttentionPlanner]:
     """The planner for a mixer of these sizes, or None when the general kernel serves it."""
     if dtype != torch.bfloat16 or head_dim not in TILE_HEAD_DIMS or page_size % 16:
         return None
@@ -452,7 +455,7 @@ def attention_planner(dtype, num_heads: int, num_kv_heads: int, head_dim: int, p
         return None
     units = torch.cuda.get_device_properties(device).multi_processor_count
     return AttentionPlanner(tile_rows, int(window), num_kv_heads, num_heads // num_kv_heads <= 16, units,
-                            attention_blocks_per_unit(head_dim), int(chunk))
+                            attention_blocks_per_unit(head_dim), int(chunk), int(keep))
 
 
 def upload_arrays(arrays: Dict[str, np.ndarray], device) -> Dict[str, torch.Tensor]:
@@ -556,11 +559,11 @@ def _decode_splits_that_fit(ws, n_req: int, num_heads: int, num_kv_heads: int, h
 
 def paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_kv_heads, head_dim,
                     page_size, scale, window, pages, ws: Optional[KernelWorkspace] = None, slopes=None, sinks=None, gate=None,
-                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0, gate_stride: int = 0) -> bool:
+                    softcap: float = 0.0, out_scale: float = 1.0, chunk: int = 0, gate_stride: int = 0, keep: int = 0) -> bool:
     """``slopes`` / ``sinks`` (float32 [heads]) and ``gate`` (float32 [tokens, heads]; with ``gate_stride`` rows of one
     unactivated gate per feature): a distance bias, a sink in the softmax and an output gate per head (None: none); ``softcap`` > 0: scaled scores s become
-    softcap * tanh(s / softcap); ``out_scale``: a factor on every output."""
-    opt = tuple(None if t is None else t.data_ptr() for t in (slopes, sinks, gate)) + (int(gate_stride), float(softcap), float(out_scale), int(chunk))
+    softcap * tanh(s / softcap); ``out_scale``: a factor on every output; ``keep`` > 0: the first so many keys are seen besides."""
+    opt = tuple(None if t is None else t.data_ptr() for t in (slopes, sinks, gate)) + (int(gate_stride), float(softcap), float(out_scale), int(chunk), int(keep))
     if head_dim not in DECODE_HEAD_DIMS or page_size % 16 or q.data_ptr() % 16 or q.stride(0) % 8 or out.stride(0) % 4:
         return False
     if gate_stride and (gate_stride % 4 or gate.data_ptr() % 16):
@@ -570,7 +573,7 @@ def paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_k
 
     def decode_kernel(n_req: int, req_ids: int, longest: int) -> None:
         if chunk:                      # a token's keys end at its chunk's start, whatever the context
-            longest = min(longest, chunk)
+            longest = min(longest, chunk + keep)
         splits = _decode_splits_that_fit(ws, n_req, num_heads, num_kv_heads, head_dim, longest)
         part = _attn_part(ws, n_req * num_heads * splits * (head_dim + 4), q.device)
         _lib.call("bf16", "pi_attention_decode", out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0),
@@ -581,7 +584,7 @@ def paged_attention(out, q, k_cache, v_cache, block_table, ctx, num_heads, num_k
     if ctx.all_decode and G <= 16:
         decode_kernel(R, 0, ctx.max_kv_len)
         return True
-    planner = attention_planner(q.dtype, num_heads, num_kv_heads, head_dim, page_size, window, q.device, int(chunk))
+    planner = attention_planner(q.dtype, num_heads, num_kv_heads, head_dim, page_size, window, q.device, int(chunk), int(keep))
     if planner is None:
         return False
     # A step of prompt portions and single tokens: the single tokens, whose keys no other token

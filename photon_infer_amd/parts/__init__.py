@@ -12,11 +12,12 @@ from .state_space import StateSpaceMixer
 from .delta_rule import ChannelDeltaRule, GatedDeltaRule
 from .diff_attention import DifferentialAttention
 from .linear_attention import GatedLinearAttention
+from .retention import Retention
 from .min_gru import MinGRU
 from .token_shift import TokenShift
 from .mlp import ClampedGLU, GeluMLP, SquaredReluMLP, SwiGLU, UngatedMLP
 from .routed_experts import RoutedExperts
-from .block import HyperConnectionBlock, HyperConnections, OutputNormBlock, PreNormBlock, SandwichBlock, SideBySide
+from .block import HyperConnectionBlock, HyperConnections, OutputNormBlock, PreNormBlock, RMSSandwichBlock, SandwichBlock, SideBySide
 from .embedding import LMHead, PositionedEmbedding, TokenEmbedding
 from .model import CachePlan, DecoderModel, ModelSpec, RunEntry, plan_cache
 
@@ -27,5 +28,5 @@ __all__ = [
     "PreNormBlock", "OutputNormBlock", "SinkWindowAttention", "MatrixMemory", "RoutedExperts", "LMHead", "TokenEmbedding", "CachePlan", "DecoderModel", "ModelSpec",
     "RunEntry", "plan_cache", "StateSpaceMixer", "ChannelDeltaRule", "ClampedGLU", "SideBySide", "PositionedEmbedding", "LatentAttention",
     "LayerNorm", "GatedDeltaRule", "DifferentialAttention", "GatedLinearAttention", "SquaredReluMLP", "SandwichBlock",
-    "StreamSumRMSNorm", "MinGRU", "TokenShift", "UngatedMLP", "GeluMLP", "HyperConnections", "HyperConnectionBlock",
+    "StreamSumRMSNorm", "MinGRU", "TokenShift", "UngatedMLP", "GeluMLP", "HyperConnections", "HyperConnectionBlock", "Retention", "RMSSandwichBlock",
 ]

@@ -55,11 +55,13 @@ class PagedTensor:
 class PagedCacheSpec:
     """What a mixer keeps per token, in pages: any number of named tensors, each with its own
     shape and layout.  ``window`` = None keeps every token; an integer W keeps the last W
-    positions, so the cache manager may hand back pages that the window has passed.  Mixers with
-    the same window share a cache group (one page pool's bookkeeping, one block table)."""
+    positions, so the cache manager may hand back pages that the window has passed, and
+    ``keep_first`` N keeps a sequence's first N positions besides.  Mixers with the same window and
+    kept tokens share a cache group (one page pool's bookkeeping, one block table)."""
 
     tensors: Tuple[PagedTensor, ...]
     window: Optional[int] = None
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -70,6 +72,7 @@ class KVCacheSpec:
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
+    keep_first: int = 0
 
     @property
     def tensors(self) -> Tuple[PagedTensor, ...]:
@@ -117,6 +120,7 @@ class StepContext:
     # the stream in pieces (``ops.gemm(..., may_defer=True)``) because the stream's next reader
     # adds them.  False unless an arrangement says so, so a part never defers by itself.
     may_defer: bool = False
+    may_leave_choices: bool = False       # likewise: a routed feed-forward may leave its result as the experts' rows (``ops.LeftChoices``)
     after_block_consumes: bool = False    # set by the model per block: whoever reads the stream after this block adds pending pieces
     workspace: Any = None                 # the runner's ops.KernelWorkspace: scratch memory of the kernels
     plans: Dict[Any, Any] = field(default_factory=dict)     # step planner -> what it made for this step
@@ -223,6 +227,7 @@ class Block(Part):
     nothing of deferred updates therefore never meets one."""
 
     mixer: Mixer
+    takes_left_join = False    # True: the block's first reader applies a result that a sandwich block has left (``norm.LEFT_JOIN``)
     reads_deferred = False     # True: the block's first reader of the stream is a norm that adds pending pieces
 
     def mixers(self) -> List[Mixer]:

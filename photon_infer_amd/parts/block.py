@@ -14,7 +14,7 @@ from .. import ops
 from ..errors import UnsupportedModelError
 from ..weights.loader import TensorSpec
 from .base import BLOCKS, MIXERS, Block, FeedForward, LayerCache, Mixer, Norm, Part, StepContext
-from .norm import LEFT_UPDATE
+from .norm import LEFT_JOIN, LEFT_UPDATE, LeftJoin
 from .token_shift import TokenShift
 
 
@@ -216,6 +216,7 @@ class SandwichBlock(Block):
     """
 
     reads_deferred = False
+    NORMS_ARE = ("weight_bias_f32", "layer norms with weight and bias")
 
     def __init__(self, branches, pre1: Tuple[str, Norm], post1: Tuple[str, Norm], pre2=None, post2=None, ffn=None):
         if not 1 <= len(branches) <= 2:
@@ -234,8 +235,8 @@ class SandwichBlock(Block):
             if getattr(part, "accumulate", True):
                 raise UnsupportedModelError(f"{type(part).__name__} must be built with accumulate=False inside a sandwich block")
         for n in (self.pre1, self.post1, self.pre2, self.post2):
-            if n is not None and not hasattr(n, "weight_bias_f32"):
-                raise UnsupportedModelError(f"a sandwich block's norms are layer norms with weight and bias, not {type(n).__name__}")
+            if n is not None and not hasattr(n, self.NORMS_ARE[0]):
+                raise UnsupportedModelError(f"this sandwich block's norms are {self.NORMS_ARE[1]}, not {type(n).__name__}")
 
     def mixers(self) -> List[Mixer]:
         return [m for _, m, _ in self.branches]
@@ -283,6 +284,44 @@ class SandwichBlock(Block):
 
 
 BLOCKS.register("sandwich", SandwichBlock)
+
+
+class RMSSandwichBlock(SandwichBlock):
+    """The sandwich with RMS norms (``RMSNorm``) and one mixer:
+
+        x <- x + rms(mix(rms(x; pre1)); post1);   x <- x + rms(ffn(rms(x; pre2)); post2)     (no feed-forward: the first only)
+
+    A sublayer's result joins the stream through its norm, and the next sublayer's input is made, in one kernel; the kernel
+    adds the pieces of a product that was split over k, and sums a token's experts, on the way.  The last sublayer's result
+    is left to whoever reads the stream next (``LEFT_JOIN``: the next block's first norm, or the final norm)."""
+
+    takes_left_join = True
+    NORMS_ARE = ("weight_f32", "RMS norms")
+
+    def __init__(self, branches, pre1: Tuple[str, Norm], post1: Tuple[str, Norm], pre2=None, post2=None, ffn=None):
+        if len(branches) != 1 or branches[0][2] is not None:
+            raise UnsupportedModelError("a sandwich block with RMS norms holds one mixer")
+        super().__init__(branches, pre1, post1, pre2, post2, ffn)
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache) -> None:
+        h = self.pre1.forward(x, ctx)
+        left = self._sublayer(self.branches[0][1], h, x, ctx, self.post1, (cache[0] if isinstance(cache, (list, tuple)) else cache,))
+        if self.ffn is not None:
+            h = left.apply(ctx.workspace, self.pre2.weight_f32(), self.pre2.eps, self.dtype)
+            left = self._sublayer(self.ffn, h, x, ctx, self.post2, ())
+        ctx.scratch[LEFT_JOIN] = left
+
+    @staticmethod
+    def _sublayer(part: Part, h: torch.Tensor, x: torch.Tensor, ctx: StepContext, post: Norm, cache: tuple) -> LeftJoin:
+        y = torch.empty_like(x)
+        ctx.may_defer = ctx.may_leave_choices = True
+        part.forward(h, y, ctx, *cache)
+        ctx.may_defer = ctx.may_leave_choices = False
+        choices = ctx.scratch.pop(ops.LEFT_CHOICES, None)
+        return LeftJoin(x, y, post.weight_f32(), post.eps, choices if choices is not None and choices.target is y else None)
+
+
+BLOCKS.register("rms_sandwich", RMSSandwichBlock)
 
 
 class HyperConnections(Part):

@@ -19,7 +19,13 @@ and ``W_uv_n`` is applied to the result, head by head.  Norms, angles, rotations
 softmax are float32 in both compute modes.
 
 The rotation is a ``PositionEncoding`` over ``rot_dim`` (any pairing rule and frequency scaling the
-rotary part offers; its cos / sin table is made once per step).
+rotary part offers; its cos / sin table is made once per step).  The kernels turn neighbouring pairs; a rotation
+that pairs halves is theirs after the rotated rows of ``W_uq`` and ``W_dkv`` are put in another order at load (i beside
+i + rot_dim / 2), the same in queries and keys, which leaves every score what it is.
+
+``gate`` names a matrix [num_heads * value_dim, hidden]: the concatenated heads are multiplied, feature by feature,
+with ``sigmoid(W h)`` before the output projection, in float32 before the one rounding.  Its rows ride in the
+first product; the last product per head applies them.
 """
 from __future__ import annotations
 
@@ -38,22 +44,22 @@ class LatentAttention(Mixer):
 
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, q_rank: int, kv_rank: int,
                  scale: float, eps: float, position: Optional[PositionEncoding] = None, accumulate: bool = True,
-                 names=("dq", "dq.norm", "uq", "dkv", "dkv.norm", "uk", "uv", "o")):
+                 names=("dq", "dq.norm", "uq", "dkv", "dkv.norm", "uk", "uv", "o"), gate: Optional[str] = None):
         self.hidden_size, self.num_heads = int(hidden_size), int(num_heads)
         self.head_dim, self.rot_dim, self.value_dim = int(head_dim), int(rot_dim), int(value_dim)
         self.q_rank, self.kv_rank = int(q_rank), int(kv_rank)
         self.scale, self.eps = float(scale), float(eps)
         self.position = position
         self.accumulate = bool(accumulate)
-        self.names = tuple(names)
+        self.names, self.gate = tuple(names), gate
         if self.rot_dim % 2:
             raise UnsupportedModelError(f"latent attention: the rotated width {self.rot_dim} must be even")
         if self.rot_dim and position is None:
             raise UnsupportedModelError("latent attention: a rotated part needs its position encoding")
         if position is not None:
             params = position.rotary_params if hasattr(position, "rotary_params") else None
-            if params is None or getattr(position, "rotary_dim", self.rot_dim) != self.rot_dim or not getattr(position, "interleaved", True):
-                raise UnsupportedModelError("latent attention: the rotation must turn neighbouring pairs over the whole rotated part")
+            if params is None or getattr(position, "rotary_dim", self.rot_dim) != self.rot_dim:
+                raise UnsupportedModelError("latent attention: the rotation must turn the whole rotated part")
         self.latent_dim = self.kv_rank + self.rot_dim          # what a cached key row holds
         self.q_size = self.num_heads * (self.head_dim + self.rot_dim)
         self.o_size = self.num_heads * self.value_dim
@@ -61,7 +67,8 @@ class LatentAttention(Mixer):
 
     def tensor_specs(self) -> List[TensorSpec]:
         D, n = self.hidden_size, self.names
-        return [TensorSpec(n[0], (self.q_rank, D)), TensorSpec(n[1], (self.q_rank,), "norm"),
+        gate = [TensorSpec(self.gate, (self.o_size, D))] if self.gate is not None else []
+        return gate + [TensorSpec(n[0], (self.q_rank, D)), TensorSpec(n[1], (self.q_rank,), "norm"),
                 TensorSpec(n[2], (self.q_size, self.q_rank)),
                 TensorSpec(n[3], (self.kv_rank + self.rot_dim, D)), TensorSpec(n[4], (self.kv_rank,), "norm"),
                 TensorSpec(n[5], (self.num_heads * self.head_dim, self.kv_rank)),
@@ -89,14 +96,20 @@ class LatentAttention(Mixer):
     def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
         super().load(tensors, dtype, device)
         n = self.names
-        mats = [tensors[n[0]], tensors[n[3]]]
+        H, d, dr, dv, r = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank
+        w_uq, w_dkv = tensors[n[2]], tensors[n[3]]
+        if self.position is not None and not getattr(self.position, "interleaved", True):
+            pairs = torch.arange(dr, device=w_uq.device).view(2, dr // 2).t().reshape(-1)         # 0, dr/2, 1, dr/2 + 1, ..
+            heads = w_uq.view(H, d + dr, -1)
+            w_uq = torch.cat([heads[:, :d], heads[:, d:][:, pairs]], dim=1).reshape(H * (d + dr), -1).contiguous()
+            w_dkv = torch.cat([w_dkv[:r], w_dkv[r:][pairs]], dim=0).contiguous()
+        mats = [tensors[n[0]], w_dkv] + ([tensors[self.gate]] if self.gate is not None else [])
         common = torch.float32 if any(m.dtype == torch.float32 for m in mats) else mats[0].dtype
-        # one projection into [query latent | key/value latent | shared rotated part]
+        # one projection into [query latent | key/value latent | shared rotated part (| gates)]
         self.w_in = torch.cat([m.to(common) for m in mats], dim=0).contiguous()
-        self.w_uq = tensors[n[2]]
+        self.w_uq = w_uq
         f32 = lambda t: t.to(torch.float32).contiguous()
         self.w_qn, self.w_kvn = f32(tensors[n[1]]), f32(tensors[n[4]])
-        H, d, dv, r = self.num_heads, self.head_dim, self.value_dim, self.kv_rank
         # per head, inputs as rows: W_uk_n as stored ([head_dim, kv_rank]: the query's plain part goes in, latent
         # coordinates come out) and W_uv_n transposed ([kv_rank, value_dim]: the attended latent goes in)
         self.w_uk = tensors[n[5]].to(dtype).reshape(H, d, r).contiguous()
@@ -119,8 +132,9 @@ class LatentAttention(Mixer):
         # a float32 tensor, or - where the product was split over k - its pieces, which the next kernel adds
         proj = ops.qkv_projection(h, self.w_in, torch.float32, ws)
         cq = torch.empty((T, self.q_rank), dtype=self.dtype, device=h.device)
-        ops.latent_kv_write(cq, proj, self.w_qn, self.w_kvn, rot_table, ctx, self.eps, self.q_rank, self.kv_rank, self.rot_dim,
-                            cache.k if cache.writes else None, cache.v if cache.writes else None, table, cache.page_size)
+        gates = ops.latent_kv_write(cq, proj, self.w_qn, self.w_kvn, rot_table, ctx, self.eps, self.q_rank, self.kv_rank, self.rot_dim,
+                            cache.k if cache.writes else None, cache.v if cache.writes else None, table, cache.page_size,
+                            num_gates=self.o_size if self.gate is not None else 0)
         q = torch.empty((T, self.q_size), dtype=self.dtype, device=h.device)
         ops.gemm(q, cq, self.w_uq, ws=ws)
         # queries in the latent's coordinates, the rotated part behind them
@@ -134,9 +148,8 @@ class LatentAttention(Mixer):
             ops.paged_attention(att, q_lat, cache.k, cache.v, table, ctx, H, 1, self.latent_dim, cache.page_size, self.scale, 0, ws,
                                 value_dim=v_rows)
         out = torch.empty((T, self.o_size), dtype=self.dtype, device=h.device)
-        ops.head_gemm(out, att, self.w_uv, H, a_head=v_rows, w_rows=self.w_uv_rows)
-        ops.gemm(x, out, self.w_o, accumulate=self.accumulate,
-                 may_defer=self.accumulate and getattr(ctx, "may_defer", False), ws=ws)
+        ops.head_gemm(out, att, self.w_uv, H, a_head=v_rows, w_rows=self.w_uv_rows, gate=gates)
+        ops.gemm(x, out, self.w_o, accumulate=self.accumulate, may_defer=getattr(ctx, "may_defer", False), ws=ws)
 
 
 MIXERS.register("latent_attention", LatentAttention)

@@ -67,8 +67,7 @@ class SwiGLU(FeedForward):
         act = torch.empty((h.shape[0], self.intermediate_size), dtype=self.dtype, device=h.device)
         ws = ctx.workspace if ctx is not None else None
         ops.gemm_swiglu(act, h, self.w_gate_up, self.interleave, ws=ws)
-        ops.gemm(x, act, self.w_down, accumulate=self.accumulate,
-                 may_defer=self.accumulate and getattr(ctx, "may_defer", False), ws=ws)
+        ops.gemm(x, act, self.w_down, accumulate=self.accumulate, may_defer=getattr(ctx, "may_defer", False), ws=ws)
 
 
 FEED_FORWARDS.register("swiglu", SwiGLU)

@@ -18,6 +18,7 @@ from ..errors import ConfigError
 from ..weights.loader import TensorSpec
 from .base import Block, KVCacheSpec, LayerCache, Norm, PagedCacheSpec, PagedTensor, StateSpec, StepContext
 from .embedding import LMHead, TokenEmbedding
+from .norm import settle_left_join
 
 
 @dataclass(frozen=True)
@@ -69,11 +70,12 @@ CacheKey = Tuple[int, int]
 
 @dataclass(frozen=True)
 class CacheGroupPlan:
-    """Mixers whose paged tensors follow one block table (the same window)."""
+    """Mixers whose paged tensors follow one block table (the same window and kept first tokens)."""
 
     window: Optional[int]
     owners: Tuple[CacheKey, ...]                        # the mixers that own pages
     tensors: Tuple[Tuple[PagedTensor, ...], ...]        # per owner: what it keeps per token
+    keep_first: int = 0                                 # a sequence's first tokens that stay beside the window
 
 
 @dataclass(frozen=True)
@@ -85,8 +87,8 @@ class CachePlan:
 
 
 def plan_cache(spec: ModelSpec) -> CachePlan:
-    """Group the run order's cache needs: one block table per distinct window."""
-    by_window: Dict[Optional[int], List[Tuple[CacheKey, tuple]]] = {}
+    """Group the run order's cache needs: one block table per distinct window and number of kept first tokens."""
+    by_window: Dict[Tuple[Optional[int], int], List[Tuple[CacheKey, tuple]]] = {}
     states: List[Tuple[CacheKey, StateSpec]] = []
     owner_of: Dict[CacheKey, CacheKey] = {}
     for i, e in enumerate(spec.run_order):
@@ -100,14 +102,15 @@ def plan_cache(spec: ModelSpec) -> CachePlan:
                                   f"must name the entry whose cache it reads")
             need = mixer.cache_spec()
             if isinstance(need, (KVCacheSpec, PagedCacheSpec)):
-                by_window.setdefault(need.window, []).append(((i, j), tuple(need.tensors)))
+                # without a window everything is kept anyway
+                by_window.setdefault((need.window, need.keep_first if need.window is not None else 0), []).append(((i, j), tuple(need.tensors)))
             elif isinstance(need, StateSpec):
                 states.append(((i, j), need))
             elif need is not None:
                 raise ConfigError(f"mixer {j} of layer {e.layer} returned an unknown cache spec {need!r}")
     groups, group_of = [], {}
-    for g, (window, items) in enumerate(sorted(by_window.items(), key=lambda kv: (kv[0] is not None, kv[0] or 0))):
-        groups.append(CacheGroupPlan(window, tuple(k for k, _ in items), tuple(t for _, t in items)))
+    for g, ((window, keep), items) in enumerate(sorted(by_window.items(), key=lambda kv: (kv[0][0] is not None, kv[0][0] or 0, kv[0][1]))):
+        groups.append(CacheGroupPlan(window, tuple(k for k, _ in items), tuple(t for _, t in items), keep))
         for k, _ in items:
             group_of[k] = g
     for key, owner in owner_of.items():
@@ -155,6 +158,8 @@ class DecoderModel:
             block = self.blocks[entry.layer]
             # A block meets an update of the stream that is still in pieces only if it says that
             # its first reader adds them, and may leave one behind only for such a reader.
+            if not block.takes_left_join:
+                settle_left_join(x, ctx)
             if not block.reads_deferred:
                 ops.materialize(x, ws)
             if i + 1 < len(order):
@@ -163,10 +168,12 @@ class DecoderModel:
                 ctx.after_block_consumes = not wanted or bool(getattr(self.final_norm, "consumes_deferred", False))
             ctx.may_defer = False
             block.forward(x, ctx, caches[i])
-        ctx.may_defer = ctx.after_block_consumes = False
+        ctx.may_defer = ctx.may_leave_choices = ctx.after_block_consumes = False
         if not wanted:
             ops.discard_deferred(x, ws)    # the stream is not read again
             return None
+        if not getattr(self.final_norm, "takes_left_join", False):
+            settle_left_join(x, ctx)
         if not getattr(self.final_norm, "consumes_deferred", False):
             ops.materialize(x, ws)
         return self.head.forward(self.final_norm.forward(x, ctx, rows=ctx.logit_rows), ctx)

@@ -7,6 +7,7 @@ rounded once to the compute dtype.
 """
 from __future__ import annotations
 
+from dataclasses import dataclass
 from typing import Dict, List, Optional
 
 import torch
@@ -20,18 +21,50 @@ from .base import NORMS, Norm
 # side by side, left to whoever reads them next.
 LEFT_UPDATE = "update of the streams left to their next reader"
 
+# Key in a step's ``scratch``: a ``LeftJoin``, a sublayer's result that joins the stream through a norm of its own and has been left
+# to the stream's next reader, which makes its own norm in the same pass.
+LEFT_JOIN = "result left to the stream's next reader"
+
+
+@dataclass
+class LeftJoin:
+    x: torch.Tensor                  # the stream
+    y: torch.Tensor                  # the result (its product may still be in pieces in the workspace)
+    weight: torch.Tensor             # the norm it goes through, float32
+    eps: float
+    choices: Optional[object] = None  # ops.LeftChoices: the result is still a sum over experts' rows
+
+    def apply(self, ws, nxt=None, next_eps: float = 0.0, dtype=None, rows=None):
+        return ops.rms_join(self.x, self.y, self.weight, self.eps, nxt, next_eps, dtype, rows, ws, self.choices)
+
+
+def take_left_join(x: torch.Tensor, ctx) -> Optional[LeftJoin]:
+    left = ctx.scratch.get(LEFT_JOIN) if ctx is not None else None
+    if left is None or left.x is not x:
+        return None
+    return ctx.scratch.pop(LEFT_JOIN)
+
+
+def settle_left_join(x: torch.Tensor, ctx) -> None:
+    """Apply a result that was left for ``x``, if there is one (before a reader that knows nothing of it)."""
+    left = take_left_join(x, ctx)
+    if left is not None:
+        left.apply(ctx.workspace)
+
 
 class RMSNorm(Norm):
     consumes_deferred = True   # reads the stream through ops.rmsnorm, which adds a pending update
+    takes_left_join = True     # and a result that a sandwich block has left
     graph_safe = True
 
-    def __init__(self, dim: int, eps: float, offset: float = 0.0, tensor_name: str = "weight"):
+    def __init__(self, dim: int, eps: float, offset: float = 0.0, tensor_name: str = "weight", mult: float = 1.0):
         """``offset``: what is added to the stored weight (1.0 for weights stored around zero, used
-        as 1 + w); the sum is made and kept in float32.  ``tensor_name``: the weight's name
+        as 1 + w); the sum is made and kept in float32.  ``mult``: a factor on the normalised row, made part of
+        the float32 weight (for a head whose logits carry a factor).  ``tensor_name``: the weight's name
         after the part's prefix (may be empty: the prefix is the name)."""
         self.dim = int(dim)
         self.eps = float(eps)
-        self.offset = float(offset)
+        self.offset, self.mult = float(offset), float(mult)
         self.tensor_name = tensor_name
         self.weight: Optional[torch.Tensor] = None
 
@@ -41,8 +74,8 @@ class RMSNorm(Norm):
     def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
         super().load(tensors, dtype, device)
         self.weight = tensors[self.tensor_name]
-        if self.offset:
-            self.weight = (self.weight.to(torch.float32) + self.offset).contiguous()
+        if self.offset or self.mult != 1.0:
+            self.weight = ((self.weight.to(torch.float32) + self.offset) * self.mult).contiguous()
 
     def weight_f32(self) -> torch.Tensor:
         """The weight as the kernels that want float32 weights take it (made once)."""
@@ -51,6 +84,9 @@ class RMSNorm(Norm):
         return self._w32
 
     def forward(self, x: torch.Tensor, ctx=None, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        left = take_left_join(x, ctx)
+        if left is not None:
+            return left.apply(ctx.workspace, self.weight_f32(), self.eps, self.dtype, rows)
         m = x.shape[0] if rows is None else rows.shape[0]
         out = torch.empty((m, self.dim), dtype=self.dtype, device=x.device)
         ops.rmsnorm(out, x, self.weight, self.eps, rows, ws=ctx.workspace if ctx is not None else None)
@@ -65,7 +101,7 @@ class StreamSumRMSNorm(RMSNorm):
     norm's own pass.  An update that a block of such streams has left to the next reader (``HyperConnectionBlock``) is
     applied on the way."""
 
-    consumes_deferred = False
+    consumes_deferred = takes_left_join = False
 
     def __init__(self, dim: int, eps: float, streams: int, offset: float = 0.0, tensor_name: str = "weight"):
         super().__init__(dim, eps, offset, tensor_name)

@@ -134,6 +134,9 @@ class RoutedExperts(FeedForward):
         ops.grouped_gemm(y, act, self.w_down, rows)
         if self.accumulate:
             ops.materialize(x, ws)
+        elif getattr(ctx, "may_leave_choices", False) and not (self.identity or self.weigh_input or self.shared is not None):
+            ctx.scratch[ops.LEFT_CHOICES] = ops.LeftChoices(x, y, weights, rows)      # whoever reads x sums them in its own pass
+            return
         if self.identity:
             ops.combine_choices(x, y, weights, rows, accumulate=self.accumulate, ids=ids, num_real=self.num_experts, h=h)
         else:

@@ -21,7 +21,11 @@ Further options, each a constructor parameter:
 
 * ``norm_per_head``: every head of q and of k is divided by the root mean square of its own
   ``head_dim`` entries instead of the whole projection's; ``norm_weights`` False: the norms have
-  no weights (no tensors ``q.norm`` / ``k.norm``);
+  no weights (no tensors ``q.norm`` / ``k.norm``); with weights they are one per entry of the projection, or
+  (``norm_shared``) ``head_dim`` of them for all heads;
+* ``sink_score``: the sink's score is this number for every head, not a tensor (0: a one in the softmax's denominator);
+* ``keep_first`` N: a token sees the sequence's first N keys besides those of its window or chunk; the cache keeps
+  the pages they lie in;
 * ``softcap`` c: the scaled score s becomes ``c * tanh(s / c)`` before the softmax;
 * ``chunk`` C: positions are cut into chunks of C, counted from position 0 of the sequence, and a
   token sees the keys ``floor(p / C) * C <= t <= p`` of its own chunk only;
@@ -57,7 +61,8 @@ class SinkWindowAttention(Mixer):
                  window: Optional[int], eps: float, temp_coef: float = 0.0, temp_every: int = 1, qk_norm: bool = True,
                  distance_bias: bool = True, sink: bool = True, output_gate: bool = True, accumulate: bool = True,
                  norm_per_head: bool = False, norm_weights: bool = True, softcap: Optional[float] = None,
-                 chunk: Optional[int] = None, own_kv: bool = True, cache_reach="own"):
+                 chunk: Optional[int] = None, own_kv: bool = True, cache_reach="own", norm_shared: bool = False,
+                 sink_score: Optional[float] = None, keep_first: int = 0):
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.head_dim, self.value_dim = int(head_dim), int(value_dim)
         self.scale, self.eps = float(scale), float(eps)
@@ -68,6 +73,11 @@ class SinkWindowAttention(Mixer):
         self.norm_per_head, self.norm_weights = bool(norm_per_head), bool(norm_weights)
         if self.qk_norm and not self.norm_per_head and not self.norm_weights:
             raise UnsupportedModelError("the norm over a whole projection comes with weights; without them it is made per head")
+        self.norm_shared = bool(norm_shared)
+        if self.norm_shared and not (self.norm_per_head and self.norm_weights):
+            raise UnsupportedModelError("one norm weight for all heads goes with norms per head that have weights")
+        self.sink_score = float(sink_score) if sink_score is not None else None
+        self.keep_first = int(keep_first)
         self.softcap = float(softcap) if softcap else 0.0
         self.chunk = int(chunk) if chunk else None
         self.own_kv = bool(own_kv)             # False: no k / v projection; reads the cache of another layer
@@ -86,10 +96,10 @@ class SinkWindowAttention(Mixer):
         if self.own_kv:
             specs += [TensorSpec("k", (self.k_size, D)), TensorSpec("v", (self.v_size, D))]
         if self.qk_norm and self.norm_weights:
-            specs.append(TensorSpec("q.norm", (self.q_size,), "norm"))
+            specs.append(TensorSpec("q.norm", (self.head_dim if self.norm_shared else self.q_size,), "norm"))
             if self.own_kv:
-                specs.append(TensorSpec("k.norm", (self.k_size,), "norm"))
-        if self.sink:
+                specs.append(TensorSpec("k.norm", (self.head_dim if self.norm_shared else self.k_size,), "norm"))
+        if self.sink and self.sink_score is None:
             specs.append(TensorSpec("sink", (self.num_heads,), "bias"))
         if self.output_gate:
             specs.append(TensorSpec("g", (self.num_heads, D)))
@@ -98,13 +108,13 @@ class SinkWindowAttention(Mixer):
 
     def cache_spec(self):
         return PagedCacheSpec((PagedTensor("k", (self.num_kv_heads, PAGE, self.head_dim)),
-                               PagedTensor("v", (self.num_kv_heads, self.value_dim, PAGE))), self.cache_reach)
+                               PagedTensor("v", (self.num_kv_heads, self.value_dim, PAGE))), self.cache_reach, self.keep_first)
 
     def step_planner(self, page_size: int):
         if self.value_dim != self.head_dim or self.head_dim % 16:     # only the general kernel takes such heads; it needs no work lists
             return None
         return ops.attention_planner(self.dtype, self.num_heads, self.num_kv_heads, self.head_dim, page_size, self.window or 0,
-                                     self.device, self.chunk or 0)
+                                     self.device, self.chunk or 0, self.keep_first if self.window or self.chunk else 0)
 
     def load(self, tensors: Dict[str, torch.Tensor], dtype, device) -> None:
         super().load(tensors, dtype, device)
@@ -115,9 +125,12 @@ class SinkWindowAttention(Mixer):
         self.w_o = tensors["o"]
         f32 = lambda t: t.to(torch.float32).contiguous()
         weighted = self.qk_norm and self.norm_weights
-        self.w_qn = f32(tensors["q.norm"]) if weighted else None
-        self.w_kn = f32(tensors["k.norm"]) if weighted and self.own_kv else None
-        self.sinks = f32(tensors["sink"]) if self.sink else None
+        per = lambda t, heads: f32(t).repeat(heads) if self.norm_shared else f32(t)       # one weight per entry, as the kernel reads them
+        self.w_qn = per(tensors["q.norm"], self.num_heads) if weighted else None
+        self.w_kn = per(tensors["k.norm"], self.num_kv_heads) if weighted and self.own_kv else None
+        self.sinks = None
+        if self.sink:
+            self.sinks = f32(tensors["sink"]) if self.sink_score is None else torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=device)
         self.slopes = distance_slopes(self.num_heads).to(device) if self.distance_bias else None
 
     def streamed_weights(self) -> List[torch.Tensor]:
@@ -139,9 +152,8 @@ class SinkWindowAttention(Mixer):
         attn = torch.empty((T, self.o_size), dtype=self.dtype, device=h.device)
         ops.paged_attention(attn, q, cache.k, cache.v, table, ctx, self.num_heads, self.num_kv_heads, self.head_dim,
                             cache.page_size, self.scale, self.window or 0, ws, value_dim=self.value_dim,
-                            slopes=self.slopes, sinks=self.sinks, gate=gate, softcap=self.softcap, chunk=self.chunk or 0)
-        ops.gemm(x, attn, self.w_o, accumulate=self.accumulate,
-                 may_defer=self.accumulate and getattr(ctx, "may_defer", False), ws=ws)
+                            slopes=self.slopes, sinks=self.sinks, gate=gate, softcap=self.softcap, chunk=self.chunk or 0, keep_first=self.keep_first)
+        ops.gemm(x, attn, self.w_o, accumulate=self.accumulate, may_defer=getattr(ctx, "may_defer", False), ws=ws)
 
 
 MIXERS.register("sink_window_attention", SinkWindowAttention)

@@ -10,7 +10,7 @@
 #include <vector>
 
 extern "C" {
-void* pi_cache_create(int n_groups, const int* windows, int page_size, const int* num_pages, int max_slots, int max_model_len);
+void* pi_cache_create(int n_groups, const int* windows, const int* keep_first, int page_size, const int* num_pages, int max_slots, int max_model_len);
 void pi_cache_destroy(void* h);
 const char* pi_cache_error(void* h);
 int pi_cache_free_slots(void* h);
@@ -44,10 +44,11 @@ static int run(unsigned seed) {
   auto pick = [&](int lo, int hi) { return lo + (int)(rng() % (unsigned)(hi - lo + 1)); };
   const int groups = pick(1, 2);
   const int windows[2] = {-1, pick(4, 24)};            // all keys; a window of a few pages
+  const int keeps[2] = {0, pick(0, 1) * pick(1, 40)};  // first tokens kept beside the window: none, or a few pages
   const int page = 1 << pick(1, 4);
   const int pages[2] = {pick(6, 40), pick(6, 40)};
   const int slots = pick(1, 6), max_len = pick(16, 200);
-  void* c = pi_cache_create(groups, windows, page, pages, slots, max_len);
+  void* c = pi_cache_create(groups, windows, keeps, page, pages, slots, max_len);
   REQUIRE(c != nullptr);
   std::vector<int> live;
   for (int step = 0; step < 400; ++step) {
