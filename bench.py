@@ -1,7 +1,7 @@
 #!/usr/bin/python3
 """Decode and prefill throughput of the engine on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode1b|long1b|serve3b|mixed8b|dafidra|rorevik|dokanex|muretar|semezen]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode1b|long1b|serve3b|mixed8b|dafidra|rorevik|dokanex|muretar|semezen|roserax]
                     [--batch 8,1,64] [--context 4096] [--dtype bf16|fp32]
 
 Every workload prints ONE JSON line.  The default, ``decode1b`` (Llama 3.2 1B layer sizes):  ``value`` is decoded tokens per second at batch 8 with the context
@@ -59,6 +59,10 @@ same way.
 in every second layer, windowed attention whose values are its keys and whose features are gated in the others; dense gelu
 feed-forwards and routed clamped ones) at layer sizes like Llama 3.2 1B's and 3B's, beside a Llama of the same width, depth
 and vocabulary, measured the same way.
+
+``--workload roserax``: the Roserax design (RMS norms around every sublayer; attention within 1,024 positions that keeps the
+first tokens, attention through a latent with gates, retention; dense squared-relu and routed feed-forwards) at layer sizes
+like Llama 3.2 1B's and 3B's, beside a Llama of the same width, depth and vocabulary, measured the same way.
 
 Weights are random (N(0, 0.02), norms 1), token ids uniform random; no dataset is involved.
 """
@@ -822,6 +826,81 @@ def workload_semezen(args) -> int:
     return 0
 
 
+def roserax_config(width, heads, kv_heads, head_dim, ff, vocab, layers):
+    """A Roserax of Llama-like layer sizes, layers in fours: attention of the Llama's heads within a window of 1,024 that keeps
+    the first 16 tokens, with a dense feed-forward (half as wide again as the Llama's: two matrices instead of three);
+    attention through a latent (16 heads of 128 plain and 64 rotated dimensions, cached rows of 192 + 64, a query latent of
+    three eighths of the width, values that fill the width) with routed experts; retention (heads of 128, as many as fill the
+    width) with the dense feed-forward; the first attention with routed experts.  Routed: 16 experts of a quarter of the
+    Llama's width in four groups of which two are kept, 4 per token."""
+    attn = dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, mask={"size": 1024, "keep_first": 16})
+    latent = dict(heads=16, dim=128, rot_dim=64, vdim=width // 16, q_rank=width * 3 // 8, kv_rank=192, scale=192 ** -0.5,
+                  rot={"base": 500000.0, "dims": 64})
+    nr = width // 128
+    retention = dict(heads=nr, dim=128, vdim=128, decay=[1.0 - 2.0 ** (-5.0 - 7.0 * i / max(1, nr - 1)) for i in range(nr)],
+                     rot={"base": 10000.0, "dims": 128})
+    dense = {"kind": "dense", "ff": ff * 3 // 2}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2}}}
+    kinds = [("attention", attn, dense), ("latent_attention", latent, moe), ("retention", retention, dense), ("attention", attn, moe)]
+    return {"architecture": "Roserax", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "logit_scale": 1.0, "norm": {"eps": 1e-5},
+            "layers": [dict(zip(("type", "mixer", "mlp"), kinds[i % 4])) for i in range(layers)]}
+
+
+def workload_roserax(args) -> int:
+    """Roserax beside a Llama of equal width, depth and vocabulary (see the module text)."""
+    import gc
+
+    import torch
+
+    layers = args.layers or 4
+    context = args.context
+    positions = max(context, PREFILL_TOKENS) + 64
+    sizes = {"1b": MODEL, "3b": MODEL_3B}
+    results = {}
+
+    def config(b):
+        return roserax_config(b["hidden_size"], b["num_attention_heads"], b["num_key_value_heads"], b["head_dim"],
+                              b["intermediate_size"], b["vocab_size"], layers)
+
+    def measured(raw):
+        return make_runner(raw, layers, args.dtype, args.batch, max(args.batch * (context + 64), PREFILL_TOKENS + 64), max_model_len=positions)[0]
+
+    if args.only:       # for profiles: the Roserax of the first size alone, a prompt or decode steps
+        runner = measured(config(sizes["1b"]))
+        if args.only == "prefill":
+            sec = time_prefill(runner, PREFILL_TOKENS, max(1, args.steps // 8))
+            print(json.dumps({"only": "prefill", "model": "roserax_1b", "tokens": PREFILL_TOKENS, "ms": round(sec * 1e3, 3)}), flush=True)
+        else:
+            sec, _ = time_decode(runner, args.batch, args.steps, args.warmup, context, synthetic_cache=True)
+            print(json.dumps({"only": "decode", "model": "roserax_1b", "batch": args.batch, "ms_per_step": round(sec * 1e3, 4),
+                              "cache": "random numbers, no prompt was run"}), flush=True)
+        return 0
+    for name, base in sizes.items():
+        for what, raw in (("roserax", config(base)), ("llama", dict(base, tie_word_embeddings=False))):
+            runner = measured(raw)
+            psec = time_prefill(runner, PREFILL_TOKENS, 3)
+            dsec, _ = time_decode(runner, args.batch, args.steps, args.warmup, context)
+            results[f"{what}_{name}"] = {"prefill_ms": round(psec * 1e3, 3), "prefill_tok_per_s": round(PREFILL_TOKENS / psec, 1),
+                                         "decode_ms_per_step": round(dsec * 1e3, 4), "decode_tok_per_s": round(args.batch / dsec, 1),
+                                         "graphs": len(runner._graphs)}
+            del runner
+            gc.collect()
+            torch.cuda.empty_cache()
+    first = results["roserax_1b"]
+    line = {
+        "metric": f"decode tok/s at batch {args.batch}, context {context} (Roserax at Llama 3.2 1B layer sizes, {layers} layers, random weights)",
+        "value": first["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": first["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": args.dtype, "data": "synthetic: random weights N(0, 0.02), uniform random token ids",
+        "config": {"model": "roserax-at-llama-sizes", "layers": layers, "global_batch": args.batch, "seq_len": context,
+                   "prefill_tokens": PREFILL_TOKENS, "window": 1024, "keep_first": 16, "experts": 16, "top": 4, "kv_block": BLOCK_SIZE,
+                   "parallelism": "single-gpu"},
+        "models": results,
+    }
+    print(json.dumps(line), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -830,7 +909,7 @@ def main() -> int:
     ap.add_argument("--batch", default="8,1,64",
                     help="batch sizes of the decode steps: the first is the headline's, the others become points")
     ap.add_argument("--context", type=int, default=CONTEXT, help="context length that the decode steps end at")
-    ap.add_argument("--workload", choices=["decode1b", "long1b", "serve3b", "mixed8b", "dafidra", "rorevik", "dokanex", "muretar", "semezen"], default="decode1b")
+    ap.add_argument("--workload", choices=["decode1b", "long1b", "serve3b", "mixed8b", "dafidra", "rorevik", "dokanex", "muretar", "semezen", "roserax"], default="decode1b")
     ap.add_argument("--layers", type=int, default=None,
                     help="fewer layers than the model has, if memory or time needs it (both numbers are reported)")
     ap.add_argument("--dtype", default="bf16", choices=["bf16", "fp32"])
@@ -872,6 +951,8 @@ def main() -> int:
         return workload_muretar(args)
     if args.workload == "semezen":
         return workload_semezen(args)
+    if args.workload == "roserax":
+        return workload_roserax(args)
     args.layers = args.layers or MODEL["num_hidden_layers"]
     elem = 2 if args.dtype == "bf16" else 4
     big = args.batch if (args.no_points or args.only) else max(batches)
