@@ -21,7 +21,7 @@
 // table: the step's [T, rot] cosines then sines (rot / 2 each), already scaled; pairs are neighbours (2j, 2j + 1).
 // The rows may go on with `ng` gates; those of a product in pieces are summed into gate_out (float32 [T, ng]), as they are.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_kv_write_kernel(
+__global__ __launch_bounds__(1024) void latent_kv_write_kernel(
     T* __restrict__ cq_out, long cq_stride, const float* __restrict__ proj, long proj_stride, const float* __restrict__ wq,
     const float* __restrict__ wkv, const float* __restrict__ table, const int* __restrict__ positions,
     const int* __restrict__ req_of_token, float eps, int q_rank, int kv_rank, int rot, int v_rows, T* __restrict__ k_cache,
@@ -32,8 +32,12 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
   const long t = blockIdx.x;
   const float* row = proj + t * proj_stride;
   const int N = q_rank + kv_rank + rot;
+  if (blockIdx.y > 0) {                           // the gates of a product in pieces: a thread per gate
+    const int i = (blockIdx.y - 1) * blockDim.x + threadIdx.x;
+    if (i < ng) gate_out[t * ng + i] = split_sum(part, splits, part_stride, t * proj_stride + N + i);
+    return;
+  }
   if (part) {
-    for (int i = threadIdx.x; i < ng; i += blockDim.x) gate_out[t * ng + i] = split_sum(part, splits, part_stride, t * proj_stride + N + i);
     for (int i = threadIdx.x; i < N; i += blockDim.x) staged[i] = split_sum(part, splits, part_stride, t * proj_stride + i);
     __syncthreads();
     row = staged;
@@ -91,7 +95,9 @@ extern "C" int pi_latent_kv_write(void* cq_out, long cq_stride, int dtype, const
              "latent: bad cache geometry");
   if (T == 0) return 0;
   const size_t lds = part ? (size_t)row_floats * sizeof(float) : 0;
-#define LKV_GO(TT) hipLaunchKernelGGL(latent_kv_write_kernel<TT>, dim3(T), dim3(256), lds, stream, (TT*)cq_out, cq_stride, proj, proj_stride, \
+  const int threads = T <= 64 ? 1024 : 256;       // few tokens (decode steps): the row's passes are a matter of latency
+  const dim3 grid(T, part ? 1 + ceil_div(ng, threads) : 1);
+#define LKV_GO(TT) hipLaunchKernelGGL(latent_kv_write_kernel<TT>, grid, dim3(threads), lds, stream, (TT*)cq_out, cq_stride, proj, proj_stride, \
                                       wq, wkv, table, positions, req_of_token, eps, q_rank, kv_rank, rot, v_rows, (TT*)k_cache,            \
                                       (TT*)v_cache, block_table, table_width, page_size, num_pages, part, splits, part_stride, ng, gate_out)
   if (dtype == PI_F32) LKV_GO(float);
@@ -125,25 +131,36 @@ __global__ __launch_bounds__(HG_WAVES * PI_WAVE) void head_gemm_kernel(T* __rest
   const int nt = (M - t0) < HG_TOKENS ? (int)(M - t0) : HG_TOKENS;
   const int KR = K + rot, KP = (KR + 3) & ~3;
   const int k_from = skip_product ? K : 0;
+  const int n = blockIdx.z * PI_WAVE + lane;
+  const int per = ((K + HG_WAVES - 1) / HG_WAVES + 7) & ~7;            // a wave's share of k, in whole eights
+  const int k0 = wave * per, k1 = min(K, k0 + per);
+  const T* wh = w + (long)h * K * N + n;
+  // the first weights are asked for before the inputs are staged: nothing in them waits for the tokens
+  T first[HG_LOADS];
+  const bool primed = !skip_product && n < N && k0 + HG_LOADS <= k1;
+  if (primed) {
+#pragma unroll
+    for (int u = 0; u < HG_LOADS; ++u) first[u] = wh[(long)(k0 + u) * N];
+  }
   for (int i = threadIdx.x; i < HG_TOKENS * KP; i += blockDim.x) {
     const int tt = i / KP, k = i % KP;
     as[i] = (tt < nt && k >= k_from && k < KR) ? to_float(a[(t0 + tt) * a_stride + (long)h * a_head + k]) : 0.f;
   }
   __syncthreads();
   if (!skip_product) {
-    const int n = blockIdx.z * PI_WAVE + lane;
-    const int per = ((K + HG_WAVES - 1) / HG_WAVES + 7) & ~7;          // a wave's share of k, in whole eights
-    const int k0 = wave * per, k1 = min(K, k0 + per);
     float acc[HG_TOKENS];
 #pragma unroll
     for (int tt = 0; tt < HG_TOKENS; ++tt) acc[tt] = 0.f;
     if (n < N) {
-      const T* wh = w + (long)h * K * N + n;
       int k = k0;
       for (; k + HG_LOADS <= k1; k += HG_LOADS) {
+        if (k != k0) {
+#pragma unroll
+          for (int u = 0; u < HG_LOADS; ++u) first[u] = wh[(long)(k + u) * N];
+        }
         float wv[HG_LOADS];
 #pragma unroll
-        for (int u = 0; u < HG_LOADS; ++u) wv[u] = to_float(wh[(long)(k + u) * N]);
+        for (int u = 0; u < HG_LOADS; ++u) wv[u] = to_float(first[u]);
 #pragma unroll
         for (int tt = 0; tt < HG_TOKENS; ++tt) {
 #pragma unroll

@@ -70,15 +70,42 @@ __global__ __launch_bounds__(1024) void retention_step_kernel(RetentionArgs a, T
   float* const q = lds;
   float* const k = q + d;
   float* const v = k + d;
-  float* const o = v + dv;
-  float* const sums = lds + ((2 * d + 2 * dv + 3) & ~3);
+  float* const gate = v + dv;
+  float* const o = gate + dv;
+  float* const sums = lds + ((2 * d + 3 * dv + 3) & ~3);
+  float* const row = state_row(a, r);
+  if (!row) return;                                  // the same for the whole block
+  float* const S = row + (long)h * d * dv;
+  const float g = a.decay[h];
+  const int groups = dv / VEC;                       // column groups; VEC divides dv
+  int lanes_c = 1;
+  while (lanes_c < groups && lanes_c < NT) lanes_c *= 2;
+  const int rg = tid / lanes_c, nrg = NT / lanes_c;
+  constexpr int U = 8;                               // rows in flight
+  float s[U][VEC];
+  auto fetch = [&](int cg, int c0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = c0 + u * nrg;
+      const bool ok = cg < groups && c < d;
+      const float* src = S + (long)(ok ? c : 0) * dv + (ok ? cg : 0) * VEC;
+      if constexpr (VEC == 4) {
+        const float4 f = *reinterpret_cast<const float4*>(src);
+        s[u][0] = f.x; s[u][1] = f.y; s[u][2] = f.z; s[u][3] = f.w;
+      } else {
+        s[u][0] = *src;
+      }
+    }
+  };
+  fetch(tid % lanes_c, rg);                          // the first rows, on their way while the token's vectors are made
   auto at = [&](long col) { return a.part ? split_sum(a.part, a.splits, a.plane, t * a.stride + col) : a.proj[t * a.stride + col]; };
   const long k_col = (long)a.H * d, v_col = 2 * k_col, g_col = v_col + (long)a.H * dv;
-  for (int i = tid; i < d; i += NT) {
-    q[i] = at((long)h * d + i);
-    k[i] = at(k_col + (long)h * d + i) * a.k_scale;
+  for (int i = tid; i < 2 * d + 2 * dv; i += NT) {   // q, k, v and gate lie in a row in LDS
+    const long col = i < d ? (long)h * d + i : i < 2 * d ? k_col + (long)h * d + (i - d)
+                     : i < 2 * d + dv ? v_col + (long)h * dv + (i - 2 * d) : g_col + (long)h * dv + (i - 2 * d - dv);
+    const float x = at(col);
+    lds[i] = i >= d && i < 2 * d ? x * a.k_scale : x;
   }
-  for (int i = tid; i < dv; i += NT) v[i] = at(v_col + (long)h * dv + i);
   __syncthreads();
   const float* cs = a.table + t * a.rd;
   for (int j = tid; j < a.rd / 2; j += NT) {         // a thread owns a pair
@@ -90,35 +117,14 @@ __global__ __launch_bounds__(1024) void retention_step_kernel(RetentionArgs a, T
     k[lo_i] = lo; k[hi_i] = hi;
   }
   __syncthreads();
-  float* const row = state_row(a, r);
-  if (!row) return;                                  // the same for the whole block
-  float* const S = row + (long)h * d * dv;
-  const float g = a.decay[h];
-  const int groups = dv / VEC;                       // column groups; VEC divides dv
-  int lanes_c = 1;
-  while (lanes_c < groups && lanes_c < NT) lanes_c *= 2;
-  const int rg = tid / lanes_c, nrg = NT / lanes_c;
   for (int cb = 0; cb < groups; cb += lanes_c) {
     const int cg = cb + tid % lanes_c;
     const bool in = cg < groups;
     float acc[VEC], vv[VEC];
 #pragma unroll
     for (int e = 0; e < VEC; ++e) { acc[e] = 0.f; vv[e] = in ? v[cg * VEC + e] : 0.f; }
-    constexpr int U = 8;                             // rows in flight
     for (int c0 = rg; c0 < d; c0 += U * nrg) {
-      float s[U][VEC];
-#pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int c = c0 + u * nrg;
-        const bool ok = in && c < d;
-        const float* src = S + (long)(ok ? c : 0) * dv + (ok ? cg : 0) * VEC;
-        if constexpr (VEC == 4) {
-          const float4 f = *reinterpret_cast<const float4*>(src);
-          s[u][0] = f.x; s[u][1] = f.y; s[u][2] = f.z; s[u][3] = f.w;
-        } else {
-          s[u][0] = *src;
-        }
-      }
+      if (cb > 0 || c0 > rg) fetch(cg, c0);
 #pragma unroll
       for (int u = 0; u < U; ++u) {
         const int c = c0 + u * nrg;
@@ -151,7 +157,7 @@ __global__ __launch_bounds__(1024) void retention_step_kernel(RetentionArgs a, T
   for (int e = tid; e < dv; e += NT) ss = fmaf(o[e], o[e], ss);
   const float rinv = 1.0f / sqrtf(block_sum(ss, scratch) / dv + a.eps);
   for (int e = tid; e < dv; e += NT)
-    y[t * a.H * dv + (long)h * dv + e] = from_float<TY>(o[e] * rinv * silu_full(at(g_col + (long)h * dv + e)));
+    y[t * a.H * dv + (long)h * dv + e] = from_float<TY>(o[e] * rinv * silu_full(gate[e]));
 }
 
 // ------------------------------------------------------------------ chunks
@@ -168,7 +174,10 @@ __device__ inline long first_record(const RetentionArgs& a, int r) { return a.q_
 template <class Factor>
 __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0, int len, long col, int f0, Factor&& factor) {
   if (a.vec) {
-    for (int i = threadIdx.x; i < RT_CHUNK * (RT_SLAB / 4); i += RT_THREADS) {
+    const bool by_fours = !a.interleaved && (a.rd / 2) % 4 == 0 && (uintptr_t)a.table % 16 == 0;
+#pragma unroll
+    for (int it = 0; it < RT_CHUNK * (RT_SLAB / 4) / RT_THREADS; ++it) {
+      const int i = threadIdx.x + it * RT_THREADS;
       const int j = i / (RT_SLAB / 4), f = (i % (RT_SLAB / 4)) * 4, c = f0 + f;
       float x[4] = {0.f, 0.f, 0.f, 0.f};
       if (j < len && c < a.d) {
@@ -177,19 +186,26 @@ __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0
         x[0] = own.x; x[1] = own.y; x[2] = own.z; x[3] = own.w;
         if (c < a.rd) {
           const float* cs = a.table + (t0 + j) * a.rd;
-          float other[4] = {x[1], x[0], x[3], x[2]};            // neighbouring pairs
-          if (!a.interleaved) {
-            if ((a.rd / 2) % 4 == 0) {
-              const float4 p = *reinterpret_cast<const float4*>(src + partner_of(a, c));
-              other[0] = p.x; other[1] = p.y; other[2] = p.z; other[3] = p.w;
-            } else {
+          if (by_fours) {                            // four features on one side, their partners side by side on the other
+            const int half = a.rd / 2;
+            const bool low = c < half;
+            const float4 p = *reinterpret_cast<const float4*>(src + (low ? c + half : c - half));
+            const float4 cv = *reinterpret_cast<const float4*>(cs + (low ? c : c - half)), sv = *reinterpret_cast<const float4*>(cs + (low ? c + half : c));
+            const float o[4] = {p.x, p.y, p.z, p.w}, cc[4] = {cv.x, cv.y, cv.z, cv.w}, ss[4] = {sv.x, sv.y, sv.z, sv.w};
 #pragma unroll
-              for (int e = 0; e < 4; ++e) other[e] = c + e < a.rd ? src[partner_of(a, c + e)] : 0.f;
+            for (int e = 0; e < 4; ++e) {
+              float lo, hi;
+              rope_pair(low ? x[e] : o[e], low ? o[e] : x[e], cc[e], ss[e], lo, hi);
+              x[e] = low ? lo : hi;
             }
-          }
+          } else {
+            float other[4];
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            if (c + e < a.rd) x[e] = rotated(a, cs, c + e, x[e], other[e]);
+            for (int e = 0; e < 4; ++e) other[e] = c + e < a.rd ? src[partner_of(a, c + e)] : 0.f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (c + e < a.rd) x[e] = rotated(a, cs, c + e, x[e], other[e]);
+          }
         }
         const float w = factor(j);
 #pragma unroll
@@ -217,7 +233,11 @@ __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0
 template <int ROWS, int COLS>
 __device__ inline void stage_rows(float* dst, const float* __restrict__ src, long ld_src, int n, int e0, int cols, bool vec) {
   if (vec) {
-    for (int i = threadIdx.x; i < ROWS * (COLS / 4); i += RT_THREADS) {
+    constexpr int N = ROWS * (COLS / 4), IT = (N + RT_THREADS - 1) / RT_THREADS;
+#pragma unroll
+    for (int it = 0; it < IT; ++it) {
+      const int i = threadIdx.x + it * RT_THREADS;
+      if (N % RT_THREADS != 0 && i >= N) break;
       const int j = i / (COLS / 4), e = (i % (COLS / 4)) * 4;
       float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
       if (j < n && e0 + e < cols) x = *reinterpret_cast<const float4*>(src + j * ld_src + e0 + e);
@@ -490,7 +510,7 @@ extern "C" int pi_retention(void* y, int y_dtype, const float* proj, long stride
     const int per = wide_state ? 4 : 1;
     int threads = 256;
     while (threads < 1024 && (long)threads * per * 8 < (long)d * dv) threads *= 2;
-    const size_t lds = (size_t)(((2 * d + 2 * dv + 3) & ~3) + threads * per) * sizeof(float);
+    const size_t lds = (size_t)(((2 * d + 3 * dv + 3) & ~3) + threads * per) * sizeof(float);
     PI_REQUIRE(lds <= 60000, "retention: heads of %d and %d features do not fit the staging memory", d, dv);
 #define RT_STEP(TY, V) hipLaunchKernelGGL((retention_step_kernel<TY, V>), dim3(H, R), dim3(threads), lds, stream, a, (TY*)y)
     if (y_dtype == PI_F32) { if (per == 4) RT_STEP(float, 4); else RT_STEP(float, 1); }

@@ -782,12 +782,14 @@ extern "C" int pi_qk_norm_kv_write(void* q_out, long q_stride, float* gate_out, 
   return pi_check_launch("qk_norm_kv_write");
 }
 
-// ---------------------------------------------------------------- queries and keys rotated, then normalised per head; values are the keys
-// Projection rows (float32, a tensor or the pieces of a product split over k) hold [q: nh*hd | k: nkv*hd | gates: ng].
+// ---------------------------------------------------------------- queries and keys rotated, then normalised per head
+// Projection rows (float32, a tensor or the pieces of a product split over k) hold [q: nh*hd | k: nkv*hd | v: nkv*vd | gates: ng],
+// or no v: values are then the keys (vd = hd, v_col = the keys' first column).
 //   q, k <- + bias (by column; null: none), rotated by the token's angles on the first rd features of each head
-//           (halves paired, or neighbours), then every head divided by the root mean square of its hd entries
-//   values: the keys with their bias, neither rotated nor normalised
-// Queries go to q_out, keys to the key pages [page, kv head, slot, hd], values to the value pages [page, kv head, hd, slot].
+//           (halves paired, or neighbours), then every head divided by the root mean square of its hd entries, times
+//           wq / wk (one weight of hd for all heads; null: none)
+//   values: their columns (with their bias), neither rotated nor normalised
+// Queries go to q_out, keys to the key pages [page, kv head, slot, hd], values to the value pages [page, kv head, vd, slot].
 // Pieces only: the gates' columns are summed into gate_out (float32 [T, ng]) as they are, for whoever applies them.
 // Everything is float32 until the one rounding on store.
 struct QkRopeArgs {
@@ -796,7 +798,10 @@ struct QkRopeArgs {
   const float* part;       // [splits, T, stride]
   int splits;
   long plane;
-  const float* bias;       // [(nh + nkv) * hd] or null
+  const float* bias;       // one per column of q, k and v, or null
+  const float* wq;         // [hd] or null
+  const float* wk;
+  int v_col, vd, g_col;    // where the values and the gates start in a row; a value head's width
   const float* table;      // [T, rd]: cosines, then sines
   int rd, interleaved;
   float eps;
@@ -869,6 +874,7 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
       dst = k_cache + ((page * a.nkv + (u - a.nh)) * a.page_size + slot) * hd;
     }
     const float* cs = a.table + t * a.rd;
+    const float* wn = u < a.nh ? a.wq : a.wk;
     if constexpr (LANES > 0) {
       const int d = 4 * lane;
       const bool in = d < hd;
@@ -901,6 +907,7 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
           o[e] = low ? lo : hi;
         }
         o[e] *= r;
+        if (wn) o[e] *= wn[i];
       }
       store4<T>(dst + d, make_float4(o[0], o[1], o[2], o[3]));
     } else {
@@ -920,15 +927,16 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
           rope_pair(low ? v : b, low ? b : v, cs[j], cs[half + j], lo, hi);
           v = low ? lo : hi;
         }
-        dst[i] = from_float<T>(v * r);
+        v *= r;
+        dst[i] = from_float<T>(wn ? v * wn[i] : v);
       }
     }
     return;
   }
   if ((int)blockIdx.x < head_blocks + value_blocks) {
     const long idx = ((long)blockIdx.x - head_blocks) * 256 + threadIdx.x;
-    const int row = a.nkv * hd;
-    const int c = (int)(idx % row), g = c / hd, d = c % hd;
+    const int vd = a.vd, row = a.nkv * vd;
+    const int c = (int)(idx % row), g = c / vd, d = c % vd;
     const long t0 = idx / row * PT;
     if (t0 >= a.T) return;
     const int n = (int)min((long)PT, a.T - t0);
@@ -937,7 +945,7 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
 #pragma unroll
     for (int i = 0; i < PT; ++i) {
       const long t = t0 + (i < n ? i : 0);
-      val[i] = from_float<T>(qkr_value(a, t, a.nh * hd + c));
+      val[i] = from_float<T>(qkr_value(a, t, a.v_col + c));
       pos[i] = a.positions[t];
       req[i] = a.req_of_token[t];
     }
@@ -949,7 +957,7 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
         int slot;
         if (!qkr_place(a, t0, page, slot)) return;
         const uint16_t* b = reinterpret_cast<const uint16_t*>(val);
-        *reinterpret_cast<uint2*>(v_cache + ((page * a.nkv + g) * hd + d) * a.page_size + slot) =
+        *reinterpret_cast<uint2*>(v_cache + ((page * a.nkv + g) * vd + d) * a.page_size + slot) =
             make_uint2((uint32_t)b[0] | ((uint32_t)b[1] << 16), (uint32_t)b[2] | ((uint32_t)b[3] << 16));
         return;
       }
@@ -958,7 +966,7 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
     for (int i = 0; i < PT; ++i) {
       long page;
       int slot;
-      if (i < n && qkr_place(a, t0 + i, page, slot)) v_cache[((page * a.nkv + g) * hd + d) * a.page_size + slot] = val[i];
+      if (i < n && qkr_place(a, t0 + i, page, slot)) v_cache[((page * a.nkv + g) * vd + d) * a.page_size + slot] = val[i];
     }
     return;
   }
@@ -967,9 +975,9 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
   const long t = idx / per;
   const int c = (int)(idx % per) * 4;
   if (t >= a.T) return;
-  const int col = (a.nh + a.nkv) * hd + c;
+  const int col = a.g_col + c;
   if constexpr (LANES > 0) {
-    if (a.ng % 4 == 0) {
+    if (a.ng % 4 == 0 && a.g_col % 4 == 0) {
       *reinterpret_cast<float4*>(a.gate_out + t * a.ng + c) = qkr_value4(a, t, col, false);
       return;
     }
@@ -978,27 +986,31 @@ __global__ __launch_bounds__(256) void qk_rope_norm_write_kernel(QkRopeArgs a, T
 }
 
 extern "C" int pi_qk_rope_norm_write(void* q_out, long q_stride, int dtype, const float* proj, long stride, const float* part, int splits,
-                                     const float* bias, const float* table, int rd, int interleaved, float eps, int T, int nh, int nkv,
-                                     int hd, int ng, float* gate_out, const int* positions, const int* req_of_token, void* k_cache,
+                                     const float* bias, const float* table, int rd, int interleaved, float eps, const float* wq,
+                                     const float* wk, int T, int nh, int nkv, int hd, int vd, int ng, float* gate_out, const int* positions, const int* req_of_token, void* k_cache,
                                      void* v_cache, const int* block_table, int table_width, int page_size, long num_pages,
                                      hipStream_t stream) {
   PI_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && hd > 0 && hd <= 640 && ng >= 0, "qk rope norm: bad sizes T=%d heads=%d kv_heads=%d head_dim=%d", T, nh, nkv, hd);
   PI_REQUIRE((proj != nullptr) != (part != nullptr) && (!part || splits >= 1), "qk rope norm: give the projection as a tensor or as pieces");
-  PI_REQUIRE(stride >= (long)(nh + nkv) * hd + (part ? ng : 0), "qk rope norm: rows of %ld hold no queries, keys and gates", stride);
+  // vd == 0: the values are the keys
+  const int g_col = (nh + nkv) * hd + (vd > 0 ? nkv * vd : 0), v_col = vd > 0 ? (nh + nkv) * hd : nh * hd;
+  if (vd == 0) vd = hd;
+  PI_REQUIRE(vd > 0 && vd <= 640, "qk rope norm: values of %d", vd);
+  PI_REQUIRE(stride >= (long)g_col + (part ? ng : 0), "qk rope norm: rows of %ld hold no queries, keys and gates", stride);
   PI_REQUIRE(rd >= 0 && rd <= hd && rd % 2 == 0 && (rd == 0 || table), "qk rope norm: rotation of %d features", rd);
   PI_REQUIRE(q_out && positions && req_of_token && k_cache && v_cache && block_table && table_width > 0 && page_size > 0 && num_pages > 0,
              "qk rope norm: bad cache geometry");
   PI_REQUIRE(!part || ng == 0 || gate_out, "qk rope norm: gates in pieces need a place");
   PI_REQUIRE(dtype == PI_F32 || dtype == PI_BF16, "qk rope norm: unsupported dtype %d", dtype);
   if (T == 0) return 0;
-  QkRopeArgs a{proj, stride, part, splits, (long)T * stride, bias, table, rd, interleaved, eps, T, nh, nkv, hd, ng, positions, req_of_token,
+  QkRopeArgs a{proj, stride, part, splits, (long)T * stride, bias, wq, wk, v_col, vd, g_col, table, rd, interleaved, eps, T, nh, nkv, hd, ng, positions, req_of_token,
                block_table, table_width, page_size, num_pages, gate_out};
   const int bytes = dtype == PI_F32 ? 16 : 8;
   bool wide = hd % 4 == 0 && hd <= 256 && stride % 4 == 0 && q_stride % 4 == 0 && (uintptr_t)q_out % bytes == 0 && (uintptr_t)k_cache % bytes == 0;
   for (const void* p : {(const void*)proj, (const void*)part, (const void*)bias, (const void*)gate_out}) wide = wide && (uintptr_t)p % 16 == 0;
   const int lanes = !wide ? 0 : (hd <= 64 ? 16 : (hd <= 128 ? 32 : 64));
   const bool four = T >= 16 && (uintptr_t)v_cache % 8 == 0;
-  const long items = (long)T * (nh + nkv), values = (long)ceil_div(T, four ? 4 : 1) * nkv * hd, gates = part ? (long)T * ceil_div(ng, 4) : 0;
+  const long items = (long)T * (nh + nkv), values = (long)ceil_div(T, four ? 4 : 1) * nkv * vd, gates = part ? (long)T * ceil_div(ng, 4) : 0;
   const long hb = (items * (lanes ? lanes : PI_WAVE) + 255) / 256, vb = (values + 255) / 256, gb = (gates + 255) / 256;
   PI_REQUIRE(hb + vb + gb < 2147483647L, "qk rope norm: too many tokens (%d)", T);
   const dim3 grid((unsigned)(hb + vb + gb)), block(256);

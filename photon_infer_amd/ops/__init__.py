@@ -811,16 +811,19 @@ def qk_norm_kv_write(q_out: torch.Tensor, gate_out: Optional[torch.Tensor], proj
 
 def qk_rope_norm_write(q_out: torch.Tensor, proj, bias: Optional[torch.Tensor], rotary, ctx, eps: float, num_heads: int, num_kv_heads: int,
                        head_dim: int, num_gates: int, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
-                       page_size: int) -> Optional[torch.Tensor]:
-    """From float32 projection rows [q heads | k heads | gates] (a tensor, or ``Partials``), with ``bias`` (float32, one per
-    column of q and k, or None) added: queries and keys rotated (``rotary`` as for ``rope_kv_write``), then every head divided
-    by its root mean square, queries into ``q_out``, keys into their pages; the keys as projected, neither rotated nor
-    normalised, into the value pages.  Returns the gates' columns as they are, float32 [T, num_gates]: a view of a
+                       page_size: int, value_dim: Optional[int] = None, w_q: Optional[torch.Tensor] = None,
+                       w_k: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """From float32 projection rows [q heads | k heads | v heads | gates] (a tensor, or ``Partials``), with ``bias`` (float32,
+    one per column of q, k and v, or None) added: queries and keys rotated (``rotary`` as for ``rope_kv_write``), then every
+    head divided by its root mean square (times ``w_q`` / ``w_k``, float32 [head_dim], one weight for all heads), queries
+    into ``q_out``, keys into their pages; the values of ``value_dim`` into theirs.  ``value_dim`` None: the rows hold no v,
+    and the keys as projected, neither rotated nor normalised, are the values.  Returns the gates' columns as they are, float32 [T, num_gates]: a view of a
     projection that is a tensor, otherwise their pieces summed (None without gates)."""
     pieces = proj if isinstance(proj, Partials) else None
     _gpu(q_out, pieces.part if pieces is not None else proj, bias, k_cache, v_cache, block_table)
-    check_general_attention_sizes(num_heads, num_kv_heads, head_dim, head_dim)
-    T, QK = q_out.shape[0], (num_heads + num_kv_heads) * head_dim
+    vd = head_dim if value_dim is None else int(value_dim)
+    check_general_attention_sizes(num_heads, num_kv_heads, head_dim, vd)
+    T, QK = q_out.shape[0], (num_heads + num_kv_heads) * head_dim + (0 if value_dim is None else num_kv_heads * vd)
     if pieces is not None:
         if pieces.M != T or pieces.N < QK + num_gates:
             raise KernelError(f"qk rope norm: pieces [{pieces.M}, {pieces.N}] do not hold q, k and gates of {T} tokens")
@@ -829,7 +832,9 @@ def qk_rope_norm_write(q_out: torch.Tensor, proj, bias: Optional[torch.Tensor], 
     if q_out.shape[1] != num_heads * head_dim:
         raise KernelError(f"qk rope norm: q has {q_out.shape[1]} columns, expected {num_heads * head_dim}")
     _f32_vector(bias, QK, "qk rope norm bias")
-    pages = _check_cache(k_cache, v_cache, num_kv_heads, head_dim, page_size, q_out.dtype)
+    _f32_vector(w_q, head_dim, "qk rope norm query weight")
+    _f32_vector(w_k, head_dim, "qk rope norm key weight")
+    pages = _check_cache(k_cache, v_cache, num_kv_heads, head_dim, page_size, q_out.dtype, vd)
     if block_table.dim() != 2 or block_table.dtype != torch.int32 or not block_table.is_contiguous():
         raise KernelError("qk rope norm: block table must be contiguous int32 [requests, width]")
     _i32(ctx.positions, "positions", T)
@@ -840,8 +845,8 @@ def qk_rope_norm_write(q_out: torch.Tensor, proj, bias: Optional[torch.Tensor], 
         gates = torch.empty((T, num_gates), dtype=torch.float32, device=q_out.device) if pieces is not None else proj[:, QK:QK + num_gates]
     _lib.call("core", "pi_qk_rope_norm_write", q_out.data_ptr(), _rows(q_out, "q"), _dt(q_out), None if pieces is not None else proj.data_ptr(),
               pieces.N if pieces is not None else _rows(proj, "projection"), pieces.part.data_ptr() if pieces is not None else None,
-              pieces.splits if pieces is not None else 0, _ptr(bias), table_ptr, rdim, int(bool(inter)), float(eps), T, num_heads, num_kv_heads,
-              head_dim, num_gates, _ptr(gates) if pieces is not None else None, ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(),
+              pieces.splits if pieces is not None else 0, _ptr(bias), table_ptr, rdim, int(bool(inter)), float(eps), _ptr(w_q), _ptr(w_k), T, num_heads, num_kv_heads,
+              head_dim, 0 if value_dim is None else vd, num_gates, _ptr(gates) if pieces is not None else None, ctx.positions.data_ptr(), ctx.req_of_token.data_ptr(),
               k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, pages, _stream())
     return gates
 

@@ -48,7 +48,7 @@ _SIGNATURES = {
         "pi_diff_combine": [P, I, P, I, F, F, F, I, I, I, I, I, P],
         "pi_paged_attention_general_ranges": [I, I, I],
         "pi_rope_table": [P, P, P, I, I, F, P],
-        "pi_qk_rope_norm_write": [P, L, I, P, L, P, I, P, P, I, I, F, I, I, I, I, I, P, P, P, P, P, P, I, I, L, P],
+        "pi_qk_rope_norm_write": [P, L, I, P, L, P, I, P, P, I, I, F, P, P, I, I, I, I, I, I, P, P, P, P, P, P, I, I, L, P],
         "pi_hyper_streams": [P, I, I, I, P, P, I, P, I, P, I, P, P, F, P, I, P, P, L, I, P, P, I, P],
         "pi_token_shift": [P, I, P, P, P, L, I, P, P, P, I, I, P],
         "pi_min_gru": [P, I, L, P, L, P, I, P, P, P, I, I, I, P, L, I, I, P, L, P],

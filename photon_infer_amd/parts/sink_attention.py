@@ -125,7 +125,11 @@ class SinkWindowAttention(Mixer):
         self.w_o = tensors["o"]
         f32 = lambda t: t.to(torch.float32).contiguous()
         weighted = self.qk_norm and self.norm_weights
-        per = lambda t, heads: f32(t).repeat(heads) if self.norm_shared else f32(t)       # one weight per entry, as the kernel reads them
+        # the kernel that has a group of lanes per head knows neither temperature nor gates per head, and one weight for all heads
+        self.per_head_kernel = (self.qk_norm and self.norm_per_head and self.temp_coef == 0.0 and not self.output_gate
+                                and self.own_kv and (self.norm_shared or not weighted))
+        # the other one reads a weight per entry of the projection
+        per = lambda t, heads: f32(t).repeat(heads) if self.norm_shared and not self.per_head_kernel else f32(t)
         self.w_qn = per(tensors["q.norm"], self.num_heads) if weighted else None
         self.w_kn = per(tensors["k.norm"], self.num_kv_heads) if weighted and self.own_kv else None
         self.sinks = None
@@ -144,11 +148,15 @@ class SinkWindowAttention(Mixer):
         q = torch.empty((T, self.q_size), dtype=self.dtype, device=h.device)
         gate = torch.empty((T, self.num_heads), dtype=torch.float32, device=h.device) if self.output_gate else None
         writes = self.own_kv and cache.writes
-        ops.qk_norm_kv_write(q, gate, proj, self.w_qn, self.w_kn, ctx, self.eps, self.temp_coef, self.temp_every,
-                             self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
-                             self.num_heads if self.output_gate else 0, cache.k if writes else None,
-                             cache.v if writes else None, table, cache.page_size,
-                             per_head=self.qk_norm and self.norm_per_head, has_kv=self.own_kv)
+        if self.per_head_kernel and writes:
+            ops.qk_rope_norm_write(q, proj, None, None, ctx, self.eps, self.num_heads, self.num_kv_heads, self.head_dim, 0, cache.k, cache.v,
+                                   table, cache.page_size, value_dim=self.value_dim, w_q=self.w_qn, w_k=self.w_kn)
+        else:
+            ops.qk_norm_kv_write(q, gate, proj, self.w_qn, self.w_kn, ctx, self.eps, self.temp_coef, self.temp_every,
+                                 self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
+                                 self.num_heads if self.output_gate else 0, cache.k if writes else None,
+                                 cache.v if writes else None, table, cache.page_size,
+                                 per_head=self.qk_norm and self.norm_per_head, has_kv=self.own_kv)
         attn = torch.empty((T, self.o_size), dtype=self.dtype, device=h.device)
         ops.paged_attention(attn, q, cache.k, cache.v, table, ctx, self.num_heads, self.num_kv_heads, self.head_dim,
                             cache.page_size, self.scale, self.window or 0, ws, value_dim=self.value_dim,

@@ -176,18 +176,21 @@ def choice_margin(scores: torch.Tensor, top: int, groups: int, keep: int) -> flo
     return min(gaps, default=math.inf)
 
 
-def routed_ff(h: torch.Tensor, mlp: dict, W: Dict[str, torch.Tensor], act_round: Round = None, experts=None, margins=None) -> torch.Tensor:
-    """``experts``: the choices to make instead of the router's own ([T][top] expert numbers); ``margins`` collects how far
-    apart the last chosen and the first passed-over score lie."""
+def routed_ff(h: torch.Tensor, mlp: dict, W: Dict[str, torch.Tensor], act_round: Round = None, experts=None, margins: Optional[list] = None,
+              chosen: Optional[list] = None) -> torch.Tensor:
+    """``experts``: the choices to make instead of the router's own ([T][top] expert numbers); ``margins`` collects how far each
+    token's own choice is from another (``choice_margin``), ``chosen`` the own choices."""
     r = mlp["router"]
     groups = r.get("groups") or {"count": 1, "keep": 1}
     scores = torch.softmax(h @ W["router"].T, dim=-1)
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
-        chosen = choose_experts(scores[t], r["top"], groups["count"], groups["keep"]) if experts is None else experts[t]
+        own = choose_experts(scores[t], r["top"], groups["count"], groups["keep"])
         if margins is not None:
             margins.append(choice_margin(scores[t], r["top"], groups["count"], groups["keep"]))
-        for e in chosen:
+        if chosen is not None:
+            chosen.append(own)
+        for e in own if experts is None else experts[t]:
             act = _r(silu(h[t] @ W[f"e{e}.gate"].T) * (h[t] @ W[f"e{e}.up"].T), act_round)
             out[t] += scores[t, e] * (act @ W[f"e{e}.down"].T)
     return out
@@ -201,9 +204,10 @@ def _sub(tensors: Dict[str, torch.Tensor], prefix: str) -> Dict[str, torch.Tenso
 
 
 def forward(config: dict, tensors: Dict[str, torch.Tensor], tokens, act_round: Round = None, streams: Optional[list] = None,
-            experts: Optional[dict] = None, margins: Optional[list] = None) -> torch.Tensor:
+            experts: Optional[dict] = None, margins: Optional[dict] = None, chosen: Optional[dict] = None) -> torch.Tensor:
     """float64 logits [T, vocab] of one whole sequence; ``streams`` collects the stream after every layer; ``experts``:
-    {layer: [T][top]} choices to make instead of the routers' own."""
+    {layer: [T][top]} choices to make instead of the routers' own; ``margins`` and ``chosen`` collect per layer what
+    ``routed_ff`` collects."""
     eps = float(config["norm"]["eps"])
     embed = tensors["embed"].to(F64)
     norm = lambda x, name: rms_norm(x, tensors[name].to(F64), eps)
@@ -216,7 +220,11 @@ def forward(config: dict, tensors: Dict[str, torch.Tensor], tokens, act_round: R
         if mlp is not None:
             h = _r(norm(x, f"l{i}.norm2"), act_round)
             W = _sub(tensors, f"l{i}.mlp.")
-            y = dense_ff(h, W, act_round) if mlp["kind"] == "dense" else routed_ff(h, mlp, W, act_round, (experts or {}).get(i), margins)
+            if mlp["kind"] == "dense":
+                y = dense_ff(h, W, act_round)
+            else:
+                keep = lambda d: d.setdefault(i, []) if d is not None else None
+                y = routed_ff(h, mlp, W, act_round, (experts or {}).get(i), keep(margins), keep(chosen))
             x = x + norm(y, f"l{i}.norm2b")
         if streams is not None:
             streams.append(x.clone())
