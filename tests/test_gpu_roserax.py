@@ -3,6 +3,7 @@ that a fault shows (keys that stand out just inside and just outside a window an
 write that must be recalled after hundreds of tokens, a loud latent far back), then whole models under every cutting,
 batching, page and slot reuse, long decoding, and greedy generation through the engine's own entry point."""
 import json
+import math
 import os
 from types import SimpleNamespace
 
@@ -470,14 +471,11 @@ _plain = {}
 CLOSE_CALL = 0.05      # a bfloat16 choice that differs from the plain one must be this close to a tie (in the scores' logarithms)
 
 
-def plain_logits(model_dir, tokens, emulate=False, forced=None):
+def plain_logits(model_dir, tokens, emulate=False):
     key = (model_dir, tuple(tokens), emulate)
-    if forced or key not in _plain:
+    if key not in _plain:
         cfg, W = P.read_model_folder(model_dir)
-        out = P.forward(cfg, W, list(tokens), P.bf16_round if emulate else None, experts=forced).float()
-        if forced:
-            return out
-        _plain[key] = out
+        _plain[key] = P.forward(cfg, W, list(tokens), P.bf16_round if emulate else None).float()
     return _plain[key]
 
 
@@ -494,13 +492,17 @@ def check(got, model_dir, reqs, dtype, what, choices=None):
         forced = choices.get(rid) if choices else None
         if forced:
             cfg, W = P.read_model_folder(model_dir)
-            margins, chosen = {}, {}
+            margins, chosen, exact = {}, {}, {}
             emulated = P.forward(cfg, W, list(toks), P.bf16_round, experts=forced, margins=margins, chosen=chosen).float()
+            ref = P.forward(cfg, W, list(toks), experts=forced, margins=exact).float()
             for i, ids in forced.items():
+                # a close call: within three times of what the rounding moves this layer's margins by
+                close_call = max(CLOSE_CALL, 3.0 * max((abs(a - b) for a, b in zip(margins[i], exact[i]) if math.isfinite(a)), default=0.0))
                 for t in range(len(toks)):
                     if sorted(ids[t]) != sorted(chosen[i][t]):
-                        assert margins[i][t] < CLOSE_CALL, f"{what}: layer {i} token {t}: experts {ids[t]} instead of {chosen[i][t]} (margin {margins[i][t]:.4f})"
-        ref = plain_logits(model_dir, toks, forced=forced)
+                        assert margins[i][t] < close_call, f"{what}: layer {i} token {t}: experts {ids[t]} instead of {chosen[i][t]} (margin {margins[i][t]:.4f})"
+        else:
+            ref = plain_logits(model_dir, toks)
         if dtype == "float32":
             tol = 1e-4 * max(1.0, float(ref.abs().max()))
         else:       # three times what rounding activations to bfloat16 does to the plain implementation itself
@@ -665,10 +667,14 @@ def test_greedy_generation_through_the_engine(name, dtype, model_dirs):
         want = P.greedy(cfg, W, prompt, 10)
         if dtype == "float32":
             assert list(out) == want
-        else:       # bfloat16: a near tie may fall the other way; the differing token must be a close second of the plain logits
+        else:       # bfloat16: a near tie may fall the other way; the differing token must be a close second of the
+            # plain logits
             for i, (a, b) in enumerate(zip(out, want)):
                 if a != b:
-                    lg = P.forward(cfg, W, prompt + want[:i])[-1]
+                    margins = {}
+                    lg = P.forward(cfg, W, prompt + want[:i], margins=margins)[-1]
+                    if min((m for v in margins.values() for m in v), default=1.0) < CLOSE_CALL:
+                        break                          # a routing choice on the way was a close call: another expert, another token
                     tol = 3.0 * float((P.forward(cfg, W, prompt + want[:i], P.bf16_round)[-1] - lg).abs().max())
                     assert float(lg[b] - lg[a]) <= 2.0 * tol, f"token {i}: {a} instead of {b} ({float(lg[b] - lg[a]):.3f} apart, bound {tol:.3f})"
                     break
