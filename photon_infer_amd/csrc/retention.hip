@@ -100,6 +100,9 @@ __global__ __launch_bounds__(1024) void retention_step_kernel(RetentionArgs a, T
   fetch(tid % lanes_c, rg);                          // the first rows, on their way while the token's vectors are made
   auto at = [&](long col) { return a.part ? split_sum(a.part, a.splits, a.plane, t * a.stride + col) : a.proj[t * a.stride + col]; };
   const long k_col = (long)a.H * d, v_col = 2 * k_col, g_col = v_col + (long)a.H * dv;
+  const float* cs = a.table + t * a.rd;
+  const int half = a.rd / 2;
+  const float cos0 = tid < half ? cs[tid] : 1.f, sin0 = tid < half ? cs[half + tid] : 0.f;
   for (int i = tid; i < 2 * d + 2 * dv; i += NT) {   // q, k, v and gate lie in a row in LDS
     const long col = i < d ? (long)h * d + i : i < 2 * d ? k_col + (long)h * d + (i - d)
                      : i < 2 * d + dv ? v_col + (long)h * dv + (i - 2 * d) : g_col + (long)h * dv + (i - 2 * d - dv);
@@ -107,13 +110,13 @@ __global__ __launch_bounds__(1024) void retention_step_kernel(RetentionArgs a, T
     lds[i] = i >= d && i < 2 * d ? x * a.k_scale : x;
   }
   __syncthreads();
-  const float* cs = a.table + t * a.rd;
-  for (int j = tid; j < a.rd / 2; j += NT) {         // a thread owns a pair
-    const int lo_i = a.interleaved ? 2 * j : j, hi_i = a.interleaved ? 2 * j + 1 : j + a.rd / 2;
+  for (int j = tid; j < half; j += NT) {             // a thread owns a pair
+    const int lo_i = a.interleaved ? 2 * j : j, hi_i = a.interleaved ? 2 * j + 1 : j + half;
+    const float c = j == tid ? cos0 : cs[j], s1 = j == tid ? sin0 : cs[half + j];
     float lo, hi;
-    rope_pair(q[lo_i], q[hi_i], cs[j], cs[a.rd / 2 + j], lo, hi);
+    rope_pair(q[lo_i], q[hi_i], c, s1, lo, hi);
     q[lo_i] = lo; q[hi_i] = hi;
-    rope_pair(k[lo_i], k[hi_i], cs[j], cs[a.rd / 2 + j], lo, hi);
+    rope_pair(k[lo_i], k[hi_i], c, s1, lo, hi);
     k[lo_i] = lo; k[hi_i] = hi;
   }
   __syncthreads();
@@ -169,16 +172,16 @@ __device__ inline f32x4_t mfma_f32(float a, float b, f32x4_t c) { return __built
 // first record of request r's chunks: requests never meet, whatever their lengths
 __device__ inline long first_record(const RetentionArgs& a, int r) { return a.q_start[r] / RT_CHUNK + r; }
 
-// 64 tokens' features f0 .. f0 + 63 of q or k of head h (`col`: the head's first column), rotated, into LDS; token j times
+// 64 tokens' features f0 .. f0 + SLAB - 1 of q or k of head h (`col`: the head's first column), rotated, into LDS; token j times
 // `factor(j)`.  Tokens from len on and features from d on are zero.
-template <class Factor>
+template <int SLAB, int THREADS, class Factor>
 __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0, int len, long col, int f0, Factor&& factor) {
   if (a.vec) {
     const bool by_fours = !a.interleaved && (a.rd / 2) % 4 == 0 && (uintptr_t)a.table % 16 == 0;
 #pragma unroll
-    for (int it = 0; it < RT_CHUNK * (RT_SLAB / 4) / RT_THREADS; ++it) {
-      const int i = threadIdx.x + it * RT_THREADS;
-      const int j = i / (RT_SLAB / 4), f = (i % (RT_SLAB / 4)) * 4, c = f0 + f;
+    for (int it = 0; it < RT_CHUNK * (SLAB / 4) / THREADS; ++it) {
+      const int i = threadIdx.x + it * THREADS;
+      const int j = i / (SLAB / 4), f = (i % (SLAB / 4)) * 4, c = f0 + f;
       float x[4] = {0.f, 0.f, 0.f, 0.f};
       if (j < len && c < a.d) {
         const float* src = a.proj + (t0 + j) * a.stride + col;
@@ -211,12 +214,12 @@ __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0
 #pragma unroll
         for (int e = 0; e < 4; ++e) x[e] *= w;
       }
-      *reinterpret_cast<float4*>(dst + j * RT_QK_LD + f) = make_float4(x[0], x[1], x[2], x[3]);
+      *reinterpret_cast<float4*>(dst + j * (SLAB + 4) + f) = make_float4(x[0], x[1], x[2], x[3]);
     }
     return;
   }
-  for (int i = threadIdx.x; i < RT_CHUNK * RT_SLAB; i += RT_THREADS) {
-    const int j = i / RT_SLAB, f = i % RT_SLAB, c = f0 + f;
+  for (int i = threadIdx.x; i < RT_CHUNK * SLAB; i += THREADS) {
+    const int j = i / SLAB, f = i % SLAB, c = f0 + f;
     float x = 0.f;
     if (j < len && c < a.d) {
       const float* src = a.proj + (t0 + j) * a.stride + col;
@@ -224,50 +227,65 @@ __device__ inline void stage_rotated(const RetentionArgs& a, float* dst, long t0
       if (c < a.rd) x = rotated(a, a.table + (t0 + j) * a.rd, c, x, src[partner_of(a, c)]);
       x *= factor(j);
     }
-    dst[j * RT_QK_LD + f] = x;
+    dst[j * (SLAB + 4) + f] = x;
   }
 }
 
-// ROWS rows of `ld_src` floats apart, COLS columns from column e0 on, into LDS rows of COLS + 4; rows from n on and columns
-// from `cols` on are zero
-template <int ROWS, int COLS>
-__device__ inline void stage_rows(float* dst, const float* __restrict__ src, long ld_src, int n, int e0, int cols, bool vec) {
-  if (vec) {
-    constexpr int N = ROWS * (COLS / 4), IT = (N + RT_THREADS - 1) / RT_THREADS;
+// ROWS rows of `ld_src` floats apart, COLS columns from column e0 on, on their way into LDS rows of COLS + 4; rows from n on and
+// columns from `cols` on are zero.  Fetching and storing are two steps, so that the next rows can be in flight while the
+// ones before them are used (rows that are no whole 16-byte groups are copied by store()).
+template <int ROWS, int COLS, int THREADS>
+struct StagedRows {
+  static constexpr int N = ROWS * (COLS / 4), IT = (N + THREADS - 1) / THREADS;
+  float4 v[IT];
+  const float* src;
+  long ld;
+  int n, e0, cols;
+  bool vec;
+  __device__ inline void fetch(const float* __restrict__ from, long ld_src, int rows, int first_col, int num_cols, bool wide) {
+    src = from; ld = ld_src; n = rows; e0 = first_col; cols = num_cols; vec = wide;
+    if (!vec) return;
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
-      const int i = threadIdx.x + it * RT_THREADS;
-      if (N % RT_THREADS != 0 && i >= N) break;
-      const int j = i / (COLS / 4), e = (i % (COLS / 4)) * 4;
-      float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (j < n && e0 + e < cols) x = *reinterpret_cast<const float4*>(src + j * ld_src + e0 + e);
-      *reinterpret_cast<float4*>(dst + j * (COLS + 4) + e) = x;
+      const int i = threadIdx.x + it * THREADS, j = i / (COLS / 4), e = (i % (COLS / 4)) * 4;
+      v[it] = (j < n && j < ROWS && e0 + e < cols) ? *reinterpret_cast<const float4*>(src + j * ld + e0 + e) : make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    return;
   }
-  for (int i = threadIdx.x; i < ROWS * COLS; i += RT_THREADS) {
-    const int j = i / COLS, e = i % COLS;
-    dst[j * (COLS + 4) + e] = (j < n && e0 + e < cols) ? src[j * ld_src + e0 + e] : 0.f;
+  __device__ inline void store(float* dst) const {
+    if (vec) {
+#pragma unroll
+      for (int it = 0; it < IT; ++it) {
+        const int i = threadIdx.x + it * THREADS, j = i / (COLS / 4), e = (i % (COLS / 4)) * 4;
+        if (N % THREADS == 0 || j < ROWS) *reinterpret_cast<float4*>(dst + j * (COLS + 4) + e) = v[it];
+      }
+      return;
+    }
+    for (int i = threadIdx.x; i < ROWS * COLS; i += THREADS) {
+      const int j = i / COLS, e = i % COLS;
+      dst[j * (COLS + 4) + e] = (j < n && e0 + e < cols) ? src[j * ld + e0 + e] : 0.f;
+    }
   }
-}
+};
 
-// U of one chunk and head: blocks of 64 key features x 16 * NT value columns; a wave has 16 features.
-template <int NT>
-__global__ __launch_bounds__(RT_THREADS) void retention_sums_kernel(RetentionArgs a) {
-  constexpr int COLS = 16 * NT;
-  __shared__ __attribute__((aligned(16))) float Ks[RT_CHUNK * RT_QK_LD];
+// U of one chunk and head: blocks of NW waves, 16 * NW key features x 16 * NT value columns; a wave has 16 features.
+template <int NT, int NW>
+__global__ __launch_bounds__(NW * PI_WAVE) void retention_sums_kernel(RetentionArgs a) {
+  constexpr int COLS = 16 * NT, SLAB = 16 * NW, KLD = SLAB + 4;
+  __shared__ __attribute__((aligned(16))) float Ks[RT_CHUNK * KLD];
   __shared__ __attribute__((aligned(16))) float Vs[RT_CHUNK * (COLS + 4)];
-  const int tiles_e = (a.dv + COLS - 1) / COLS, tiles = tiles_e * ((a.d + RT_SLAB - 1) / RT_SLAB);
+  const int tiles_e = (a.dv + COLS - 1) / COLS, tiles = tiles_e * ((a.d + SLAB - 1) / SLAB);
   const int chunk = blockIdx.x / tiles, tile = blockIdx.x % tiles, h = blockIdx.y, r = blockIdx.z;
-  const int f0 = tile / tiles_e * RT_SLAB, e0 = tile % tiles_e * COLS;
+  const int f0 = tile / tiles_e * SLAB, e0 = tile % tiles_e * COLS;
   const int qs = a.q_start[r], n = a.q_start[r + 1] - qs;
   if (chunk * RT_CHUNK >= n) return;
   const long t0 = qs + chunk * RT_CHUNK;
   const int len = min(RT_CHUNK, n - chunk * RT_CHUNK);
   const int lane = threadIdx.x % PI_WAVE, wave = threadIdx.x / PI_WAVE, lr = lane % 16, lg = lane / 16;
   const float l2 = a.decay[a.H + h];
-  stage_rotated(a, Ks, t0, len, (long)(a.H + h) * a.d, f0, [&](int j) { return a.k_scale * power2((float)(len - 1 - j), l2); });
-  stage_rows<RT_CHUNK, COLS>(Vs, a.proj + t0 * a.stride + 2L * a.H * a.d + (long)h * a.dv, a.stride, len, e0, a.dv, a.vec != 0);
+  StagedRows<RT_CHUNK, COLS, NW * PI_WAVE> values;
+  values.fetch(a.proj + t0 * a.stride + 2L * a.H * a.d + (long)h * a.dv, a.stride, len, e0, a.dv, a.vec != 0);
+  stage_rotated<SLAB, NW * PI_WAVE>(a, Ks, t0, len, (long)(a.H + h) * a.d, f0, [&](int j) { return a.k_scale * power2((float)(len - 1 - j), l2); });
+  values.store(Vs);
   __syncthreads();
   f32x4_t u[NT];
 #pragma unroll
@@ -277,7 +295,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_sums_kernel(RetentionArg
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
       const int j = jt * 16 + lg * 4 + v;
-      const float kf = Ks[j * RT_QK_LD + wave * 16 + lr];
+      const float kf = Ks[j * KLD + wave * 16 + lr];
 #pragma unroll
       for (int e = 0; e < NT; ++e) u[e] = mfma_f32(kf, Vs[j * (COLS + 4) + e * 16 + lr], u[e]);
     }
@@ -368,14 +386,24 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   for (int e = 0; e < VT; ++e) o[e] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int kt = 0; kt < 4; ++kt) p[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  // the rows of the state, then the values, BR at a time; the next ones are fetched while the present ones are used
+  const int state_parts = (a.d + BR - 1) / BR;
+  StagedRows<BR, COLS, RT_THREADS> rows;
+  auto fetch_rows = [&](int part) {
+    if (part < state_parts) rows.fetch(S + (long)part * BR * a.dv, a.dv, a.d - part * BR, e0, a.dv, a.vec != 0);
+    else rows.fetch(a.proj + (t0 + (part - state_parts) * BR) * a.stride + v_col, a.stride, len - (part - state_parts) * BR, e0, a.dv, a.vec != 0);
+  };
+  fetch_rows(0);
+  int part = 0;
   for (int f0 = 0; f0 < a.d; f0 += RT_SLAB) {
     if (f0 > 0) __syncthreads();
-    stage_rotated(a, Qs, t0, len, (long)h * a.d, f0, [](int) { return 1.0f; });
-    stage_rotated(a, Ks, t0, len, k_col, f0, [&](int) { return a.k_scale; });
+    stage_rotated<RT_SLAB, RT_THREADS>(a, Qs, t0, len, (long)h * a.d, f0, [](int) { return 1.0f; });
+    stage_rotated<RT_SLAB, RT_THREADS>(a, Ks, t0, len, k_col, f0, [&](int) { return a.k_scale; });
     for (int b0 = 0; b0 < RT_SLAB && f0 + b0 < a.d; b0 += BR) {
       if (b0 > 0) __syncthreads();
-      stage_rows<BR, COLS>(Bs, S + (long)(f0 + b0) * a.dv, a.dv, a.d - f0 - b0, e0, a.dv, a.vec != 0);
+      rows.store(Bs);
       __syncthreads();
+      fetch_rows(++part);
       if (live) {
 #pragma unroll
         for (int kk = 0; kk < BR / 16; ++kk) {
@@ -411,8 +439,9 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   for (int jb = 0; jb < RT_CHUNK / BR; ++jb) {
     if (jb * BR >= len) break;
     __syncthreads();
-    stage_rows<BR, COLS>(Bs, a.proj + (t0 + jb * BR) * a.stride + v_col, a.stride, len - jb * BR, e0, a.dv, a.vec != 0);
+    rows.store(Bs);
     __syncthreads();
+    if ((jb + 1) * BR < len) fetch_rows(++part);
     if (!live) continue;
 #pragma unroll
     for (int k2 = 0; k2 < BR / 16; ++k2) {
@@ -521,10 +550,11 @@ extern "C" int pi_retention(void* y, int y_dtype, const float* proj, long stride
   PI_REQUIRE(work, "retention: scratch memory is missing");
   a.vec = wide_state && d % 4 == 0 && stride % 4 == 0 && (uintptr_t)proj % 16 == 0 && (uintptr_t)work % 16 == 0 && (uintptr_t)y % 16 == 0;
   const int chunks = ceil_div(longest, RT_CHUNK);
-  const int slabs = ceil_div(d, RT_SLAB);
-#define RT_SUMS(N_) hipLaunchKernelGGL((retention_sums_kernel<N_>), dim3(chunks * slabs * ceil_div(dv, 16 * N_), H, R), dim3(RT_THREADS), 0, stream, a)
+#define RT_SUMS1(N_, W_) hipLaunchKernelGGL((retention_sums_kernel<N_, W_>), dim3(chunks * ceil_div(d, 16 * W_) * ceil_div(dv, 16 * N_), H, R), dim3(W_ * PI_WAVE), 0, stream, a)
+#define RT_SUMS(N_) do { if (d <= 64) RT_SUMS1(N_, 4); else RT_SUMS1(N_, 8); } while (0)
   if (dv <= 32) RT_SUMS(2); else if (dv <= 64) RT_SUMS(4); else RT_SUMS(8);
 #undef RT_SUMS
+#undef RT_SUMS1
   if (pi_check_launch("retention_sums")) return -1;
   const long size = (long)d * dv;
   if (a.vec)
