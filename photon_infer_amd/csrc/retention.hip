@@ -359,14 +359,15 @@ __global__ __launch_bounds__(RT_THREADS) void retention_states_kernel(RetentionA
   for (int e = 0; e < VEC; ++e) st[e] = s[e];
 }
 
-// The results of one chunk and head, value columns e0 .. e0 + 16 * VT - 1.  A wave has 16 queries; everything is transposed
-// (value columns or keys as rows, queries as columns), so that the tile of decayed scores is the operand of the product with
+// The results of one chunk and head, value columns e0 .. e0 + 16 * VT * CW - 1.  A wave has 16 queries and 16 * VT columns
+// (CW waves share the queries, and the tiles of scores, which they exchange through LDS); everything is transposed (value columns or keys as rows, queries as columns), so that the tile of decayed scores is the operand of the product with
 // the values as it lies, and a query's results lie in the four lanes l, l + 16, l + 32, l + 48.  A wave's queries
 // meet the key tiles up to their own only.  With all columns in one block (col_tiles 1) the head's norm and the gate
 // follow on the spot into y; otherwise the results go to o as float32.
-template <typename TY, int VT>
-__global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs a, TY* __restrict__ y, float* __restrict__ o_out) {
-  constexpr int COLS = 16 * VT, LD = COLS + 4, BR = VT > 8 ? 16 : 32;      // BR: rows of the state, or of values, staged at a time
+template <typename TY, int VT, int CW>
+__global__ __launch_bounds__(RT_THREADS * CW) __attribute__((amdgpu_waves_per_eu(VT <= 4 ? 4 : 2))) void retention_out_kernel(RetentionArgs a, TY* __restrict__ y, float* __restrict__ o_out) {
+  constexpr int COLS = 16 * VT * CW, LD = COLS + 4, BR = COLS > 128 ? 16 : 32;      // BR: rows of the state, or of values, staged at a time
+  static_assert(CW == 1 || CW == 2, "one or two waves share their queries");
   __shared__ __attribute__((aligned(16))) float Qs[RT_CHUNK * RT_QK_LD];
   __shared__ __attribute__((aligned(16))) float Ks[RT_CHUNK * RT_QK_LD];
   __shared__ __attribute__((aligned(16))) float Bs[BR * LD];
@@ -375,7 +376,9 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   if (chunk * RT_CHUNK >= n) return;
   const long t0 = qs + chunk * RT_CHUNK;
   const int len = min(RT_CHUNK, n - chunk * RT_CHUNK);
-  const int lane = threadIdx.x % PI_WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / PI_WAVE), lr = lane % 16, lg = lane / 16;
+  const int lane = threadIdx.x % PI_WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / PI_WAVE) % 4, lr = lane % 16, lg = lane / 16;
+  const int cw = CW == 1 ? 0 : __builtin_amdgcn_readfirstlane(threadIdx.x / RT_THREADS), w0 = cw * 16 * VT;      // the wave's first column
+  __shared__ float squares[CW][RT_CHUNK];
   const float l2 = a.decay[a.H + h];
   const float* S = a.work + ((first_record(a, r) + chunk) * a.H + h) * (long)a.d * a.dv;
   const long k_col = (long)(a.H + h) * a.d, v_col = 2L * a.H * a.d + (long)h * a.dv;
@@ -388,7 +391,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   for (int kt = 0; kt < 4; ++kt) p[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   // the rows of the state, then the values, BR at a time; the next ones are fetched while the present ones are used
   const int state_parts = (a.d + BR - 1) / BR;
-  StagedRows<BR, COLS, RT_THREADS> rows;
+  StagedRows<BR, COLS, RT_THREADS * CW> rows;
   auto fetch_rows = [&](int part) {
     if (part < state_parts) rows.fetch(S + (long)part * BR * a.dv, a.dv, a.d - part * BR, e0, a.dv, a.vec != 0);
     else rows.fetch(a.proj + (t0 + (part - state_parts) * BR) * a.stride + v_col, a.stride, len - (part - state_parts) * BR, e0, a.dv, a.vec != 0);
@@ -397,8 +400,8 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   int part = 0;
   for (int f0 = 0; f0 < a.d; f0 += RT_SLAB) {
     if (f0 > 0) __syncthreads();
-    stage_rotated<RT_SLAB, RT_THREADS>(a, Qs, t0, len, (long)h * a.d, f0, [](int) { return 1.0f; });
-    stage_rotated<RT_SLAB, RT_THREADS>(a, Ks, t0, len, k_col, f0, [&](int) { return a.k_scale; });
+    stage_rotated<RT_SLAB, RT_THREADS * CW>(a, Qs, t0, len, (long)h * a.d, f0, [](int) { return 1.0f; });
+    stage_rotated<RT_SLAB, RT_THREADS * CW>(a, Ks, t0, len, k_col, f0, [&](int) { return a.k_scale; });
     for (int b0 = 0; b0 < RT_SLAB && f0 + b0 < a.d; b0 += BR) {
       if (b0 > 0) __syncthreads();
       rows.store(Bs);
@@ -411,7 +414,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
           const f32x4_t qf = *reinterpret_cast<const f32x4_t*>(Qs + i * RT_QK_LD + b0 + f);
 #pragma unroll
           for (int kt = 0; kt < 4; ++kt) {
-            if (kt > wave) continue;
+            if (kt > wave || (CW == 2 && (kt & 1) != cw)) continue;
             const f32x4_t kf = *reinterpret_cast<const f32x4_t*>(Ks + (kt * 16 + lr) * RT_QK_LD + b0 + f);
 #pragma unroll
             for (int v = 0; v < 4; ++v) p[kt] = mfma_f32(kf[v], qf[v], p[kt]);
@@ -419,7 +422,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
 #pragma unroll
           for (int v = 0; v < 4; ++v)
 #pragma unroll
-            for (int e = 0; e < VT; ++e) o[e] = mfma_f32(Bs[(f + v) * LD + e * 16 + lr], qf[v], o[e]);
+            for (int e = 0; e < VT; ++e) o[e] = mfma_f32(Bs[(f + v) * LD + w0 + e * 16 + lr], qf[v], o[e]);
         }
       }
     }
@@ -435,6 +438,18 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
       const int j = kt * 16 + lg * 4 + v;
       p[kt][v] = j <= i ? p[kt][v] * power2((float)(i - j), l2) : 0.f;
     }
+  if constexpr (CW == 2) {                           // each of the two waves has every second tile
+    f32x4_t* const shared = reinterpret_cast<f32x4_t*>(Qs) + wave * 4 * PI_WAVE + lane;
+    static_assert(sizeof(Qs) >= 4 * 4 * PI_WAVE * sizeof(f32x4_t), "the tiles of scores take the queries' place");
+    __syncthreads();
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+      if ((kt & 1) == cw) shared[kt * PI_WAVE] = p[kt];
+    __syncthreads();
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+      if ((kt & 1) != cw) p[kt] = shared[kt * PI_WAVE];
+  }
 #pragma unroll
   for (int jb = 0; jb < RT_CHUNK / BR; ++jb) {
     if (jb * BR >= len) break;
@@ -450,16 +465,21 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
 #pragma unroll
       for (int v = 0; v < 4; ++v)
 #pragma unroll
-        for (int e = 0; e < VT; ++e) o[e] = mfma_f32(Bs[(k2 * 16 + lg * 4 + v) * LD + e * 16 + lr], p[kt][v], o[e]);
+        for (int e = 0; e < VT; ++e) o[e] = mfma_f32(Bs[(k2 * 16 + lg * 4 + v) * LD + w0 + e * 16 + lr], p[kt][v], o[e]);
     }
   }
-  // o[e][v] is column e0 + 16 e + 4 lg + v of query i; columns beyond dv are zero
+  // o[e][v] is column e0 + w0 + 16 e + 4 lg + v of query i; columns beyond dv are zero
   float ss = 0.f;
 #pragma unroll
   for (int e = 0; e < VT; ++e)
 #pragma unroll
     for (int v = 0; v < 4; ++v) ss = fmaf(o[e][v], o[e][v], ss);
   ss = column_sum(ss);
+  if constexpr (CW == 2) {
+    if (lg == 0) squares[cw][i] = ss;
+    __syncthreads();
+    ss = squares[0][i] + squares[1][i];
+  }
   if (i >= len) return;
   const long t = t0 + i;
   if (o_out) {
@@ -467,7 +487,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
     for (int e = 0; e < VT; ++e)
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
-        const int col = e0 + e * 16 + lg * 4 + v;
+        const int col = e0 + w0 + e * 16 + lg * 4 + v;
         if (col < a.dv) o_out[(t * a.H + h) * a.dv + col] = o[e][v];
       }
     return;
@@ -477,7 +497,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_out_kernel(RetentionArgs
   TY* yr = y + (t * a.H + h) * a.dv;
 #pragma unroll
   for (int e = 0; e < VT; ++e) {
-    const int col = e * 16 + lg * 4;
+    const int col = w0 + e * 16 + lg * 4;
     if (a.vec) {
       if (col >= a.dv) continue;
       const float4 g = *reinterpret_cast<const float4*>(gates + col);
@@ -567,13 +587,13 @@ extern "C" int pi_retention(void* y, int y_dtype, const float* proj, long stride
     a.col_tiles = ceil_div(dv, 128);
     o = work + ((((long)(T / RT_CHUNK + R) * H * size) + 3) & ~3L);
   }
-#define RT_OUT(TY, V_) hipLaunchKernelGGL((retention_out_kernel<TY, V_>), dim3(chunks * a.col_tiles, H, R), dim3(RT_THREADS), 0, stream, a, (TY*)y, o)
-#define RT_OUT_PICK(TY)                   \
-  do {                                    \
-    if (dv <= 32) RT_OUT(TY, 2);          \
-    else if (dv <= 64) RT_OUT(TY, 4);     \
-    else if (dv <= 128 || o) RT_OUT(TY, 8); \
-    else RT_OUT(TY, 16);                  \
+#define RT_OUT(TY, V_, C_) hipLaunchKernelGGL((retention_out_kernel<TY, V_, C_>), dim3(chunks * a.col_tiles, H, R), dim3(RT_THREADS * C_), 0, stream, a, (TY*)y, o)
+#define RT_OUT_PICK(TY)                      \
+  do {                                       \
+    if (dv <= 32) RT_OUT(TY, 2, 1);          \
+    else if (dv <= 64) RT_OUT(TY, 2, 2);     \
+    else if (dv <= 128 || o) RT_OUT(TY, 4, 2); \
+    else RT_OUT(TY, 8, 2);                   \
   } while (0)
   if (y_dtype == PI_F32) RT_OUT_PICK(float); else RT_OUT_PICK(bf16_t);
 #undef RT_OUT_PICK
