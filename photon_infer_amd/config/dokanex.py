@@ -2,8 +2,8 @@
 
 The file names every size and every constant that may differ between models of the design:
 ``vocab``, ``width``, ``embedding.scale``, ``norm.eps``, ``logit_softcap`` and a list ``layers`` whose
-entries give the layer's ``type`` (which mixer it has), the mixer's sizes (``mixer``) and its
-feed-forward (``mlp``, or null for none).  Nothing here has a default that a model could
+entries give a ``type`` (the kind of mixer), the sizes of that mixer (``mixer``) and, where there is one,
+a feed-forward (``mlp``).  Nothing here has a default that a model could
 contradict, except where a whole feature may be left out (no chunks, no cap on the scores or on
 the logits, no frequency scaling, keys and values of the layer's own).
 """

@@ -2,8 +2,8 @@
 
 The file names every size and every constant that may differ between models of the design:
 ``vocab``, ``width``, ``max_positions`` (rows of the learned position table), ``embedding.scale``,
-``norm.eps``, a list ``layers`` whose entries give the layer's ``type`` (which mixer it has), the
-mixer's sizes (``mixer``) and its feed-forward (``mlp``, or null for none), and ``loop``: the
+``norm.eps``, a list ``layers`` whose entries give a ``type`` (the kind of mixer),
+the sizes of that mixer (``mixer``) and, where there is one, a feed-forward (``mlp``), and ``loop``: the
 layers ``start .. stop - 1`` run ``times`` times in a row before the rest follow.  Nothing here
 has a default that a model could contradict, except where a whole feature may be left out (no
 loop, no rotation, no cap on the scores).

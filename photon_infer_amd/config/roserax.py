@@ -1,9 +1,9 @@
 """Typed configuration of the Roserax architecture, read from its config.json.
 
 The file names every size and every constant that may differ between models of the design: ``vocab``, ``width``,
-``embedding.scale``, ``logit_scale``, ``norm.eps`` and a list ``layers`` whose entries give the layer's ``type`` (which mixer it
-has: ``attention``, ``latent_attention`` or ``retention``), the mixer's sizes and constants (``mixer``) and its feed-forward
-(``mlp``: ``kind`` ``dense`` or ``moe``, or null for none).  Features that may be left out: an attention layer's ``mask`` (it then
+``embedding.scale``, ``logit_scale``, ``norm.eps`` and a list ``layers`` whose entries give a ``type`` (the kind of
+mixer: ``attention``, ``latent_attention`` or ``retention``), the sizes and constants of that mixer (``mixer``) and, where
+there is one, a feed-forward (``mlp``: ``kind`` ``dense`` or ``moe``).  Features that may be left out: an attention layer's ``mask`` (it then
 sees every earlier position), the mask's ``keep_first``, a router's ``groups``, a retention layer's ``rot``.
 """
 from __future__ import annotations

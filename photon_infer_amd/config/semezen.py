@@ -2,8 +2,8 @@
 
 The file names every size and every constant that may differ between models of the design:
 ``vocab``, ``width``, ``streams`` (how many copies of the residual stream run side by side), ``norm.eps``
-and a list ``layers`` whose entries give the layer's ``type`` (which mixer it has: ``attention`` or
-``mingru``), the mixer's sizes (``mixer``) and, where the layer has one, its feed-forward (``mlp``: ``kind`` ``dense`` or
+and a list ``layers`` whose entries give a ``type`` (the kind of mixer: ``attention`` or
+``mingru``), the sizes of that mixer (``mixer``) and, where the layer has one, its feed-forward (``mlp``: ``kind`` ``dense`` or
 ``moe``).
 """
 from __future__ import annotations

@@ -1,4 +1,4 @@
-// Retention: linear attention with a fixed decay per head, no softmax and no denominator (Sun et al., "Retentive Network: A
+// Retention, a linear attention whose state decays by a constant of its head (Sun et al., "Retentive Network: A
 // Successor to Transformer for Large Language Models").  Per head, with state S [d, dv] (float32, zero at the start):
 //   q' = rotate(q);  k' = rotate(k) * k_scale;   S <- decay S + k' v^T;   o = S^T q'
 //   y = o / sqrt(mean(o^2) + eps) * silu(gate)

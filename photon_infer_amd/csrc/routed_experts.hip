@@ -3,9 +3,9 @@
 // count ever travels to the host, so a step's launches depend on its number of tokens only.
 //
 // Routing, per token, from float32 router logits z [E]:
-//   s = softmax(z) over all experts, or sigmoid(z) of each on its own;
-//   experts form `groups` equal groups of neighbours, a group's score is its largest s, and
-//   only experts of the `keep` best groups may be chosen (groups <= 1: all may);
+//   s = softmax(z), or sigmoid(z) of each on its own;
+//   with groups > 1: the experts are cut into `groups` runs of equal length, ranked by their best s, and
+//   those outside the first `keep` runs leave the choice;
 //   the `top` allowed experts with the largest s are chosen, weights = their s (as they are,
 //   or divided by their sum + renorm_eps when `renorm`).  Equal scores: the lower index wins.
 //   With a `correction` [E] the choice (of groups and of experts) goes by s + correction; the

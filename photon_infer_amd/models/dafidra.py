@@ -8,7 +8,7 @@ feed-forward.
     logits = head . norm(x; final.norm)
 
 ``norm1``, ``norm2`` and ``final.norm`` store their weights around zero (used as 1 + w); the two
-branch norms have plain weights.  Layer i's tensors start with ``l<i>.``; the mixers' with
+branch norms have plain weights.  The names of layer i's tensors begin with ``l<i>.``; the mixers' with
 ``mix.left.`` / ``mix.right.``, the feed-forward's with ``mlp.``.
 """
 from __future__ import annotations

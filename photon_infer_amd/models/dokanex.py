@@ -8,7 +8,7 @@ for all heads (neighbouring pairs, frequencies scaled by a ramp).
     per layer:  x <- x + mixer(norm(x; norm1));  x <- x + ffn(norm(x; norm2))     (layers with a feed-forward)
     logits = cap * tanh((embed . norm(x; final.norm)) / cap)
 
-Layer i's tensors start with ``l<i>.``; the mixer's with ``mix.``, the feed-forward's with ``mlp.``;
+The names of layer i's tensors begin with ``l<i>.``; the mixer's with ``mix.``, the feed-forward's with ``mlp.``;
 norms are named by themselves (``l<i>.norm1``, ``final.norm``); the head is the embedding's table.
 """
 from __future__ import annotations

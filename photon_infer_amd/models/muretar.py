@@ -11,7 +11,7 @@ gated or routed (real and identity experts, a shared expert).
     mixer of a "gla" layer:         gated linear attention with a decay per key channel
 
 A layer with ``weights_of: j`` has no tensors: the run order names layer j's block again, and every entry of the
-run order gets a cache or state of its own.  Layer i's tensors start with ``l<i>.``; the mixers' with ``mix.``
+run order gets a cache or state of its own.  The names of layer i's tensors begin with ``l<i>.``; the mixers' with ``mix.``
 (``mix.left.`` / ``mix.right.``), the feed-forward's with ``mlp.``; norms are named by themselves (``l<i>.norm1``,
 ``final.norm``) with their bias at ``<name>.b``.
 """

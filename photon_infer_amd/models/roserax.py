@@ -11,7 +11,7 @@ are dense (squared relu) or routed; a scaled embedding and a tied head whose log
     mixer of a "latent_attention" layer:   a rotated key part for all heads (paired halves), gates per feature
     mixer of a "retention" layer:          a matrix state per head with a fixed decay
 
-Layer i's tensors start with ``l<i>.``; the mixer's with ``mix.``, the feed-forward's with ``mlp.``; norms are named by themselves
+The names of layer i's tensors begin with ``l<i>.``; the mixer's with ``mix.``, the feed-forward's with ``mlp.``; norms are named by themselves
 (``l<i>.norm1``, ``final.norm``); the head is the embedding's table.
 """
 from __future__ import annotations

@@ -9,7 +9,7 @@ dense (gelu) or routed.
         X_t <- sum_s mix_q[s, t] X_s + out_q[t] * sublayer(h)
     logits = head . rms(sum_s X_s; final.norm)
 
-Layer i's tensors start with ``l<i>.``: ``norm1`` / ``norm2``, ``shift``, ``hc1.`` / ``hc2.`` (in, out, mix), ``mix.`` (the
+The names of layer i's tensors begin with ``l<i>.``: ``norm1`` / ``norm2``, ``shift``, ``hc1.`` / ``hc2.`` (in, out, mix), ``mix.`` (the
 mixer) and ``mlp.``.
 """
 from __future__ import annotations

@@ -3,10 +3,10 @@ part that all heads share.
 
 For a token at position p with input h (sizes and constants are constructor parameters):
 
-* queries through a latent of ``q_rank``: ``c_q = norm(W_dq h; dq.norm)``, ``q = W_uq c_q``, laid out head
-  by head as [``head_dim`` plain | ``rot_dim`` rotated];
-* ``W_dkv h`` has ``kv_rank + rot_dim`` rows: the first ``kv_rank``, normalised with ``dkv.norm``, are the
-  latent ``c``; the last ``rot_dim`` (not normalised) are the rotated key part ``k_r`` of every head;
+* queries through a latent of ``q_rank``: ``c_q = norm(W_dq h; dq.norm)``, ``q = W_uq c_q``, a head's
+  share of it [``head_dim`` plain | ``rot_dim`` rotated];
+* ``[c_raw | k_r] = W_dkv h`` with ``kv_rank`` and ``rot_dim`` numbers: ``c = norm(c_raw; dkv.norm)`` is the latent;
+  ``k_r``, which no norm touches, is rotated and serves every head as the other part of its key;
 * head n's key is ``[W_uk_n c | k_r]`` and its value ``W_uv_n c``;
   ``score(p, t) = scale * (<q_plain, W_uk_n c_t> + <rotate(q_rot, p), rotate(k_r, t)>)`` for ``t <= p``;
 * ordinary softmax; ``W_o`` on the concatenated heads.
@@ -23,8 +23,8 @@ rotary part offers; its cos / sin table is made once per step).  The kernels tur
 that pairs halves is theirs after the rotated rows of ``W_uq`` and ``W_dkv`` are put in another order at load (i beside
 i + rot_dim / 2), the same in queries and keys, which leaves every score what it is.
 
-``gate`` names a matrix [num_heads * value_dim, hidden]: the concatenated heads are multiplied, feature by feature,
-with ``sigmoid(W h)`` before the output projection, in float32 before the one rounding.  Its rows ride in the
+``gate`` names a matrix [num_heads * value_dim, hidden]: what goes into the output projection carries, feature by
+feature, a factor ``sigmoid(W h)``, in float32 before the one rounding.  Its rows ride in the
 first product; the last product per head applies them.
 """
 from __future__ import annotations

@@ -8,7 +8,7 @@ State S [d, dv], n [d] and a running maximum m, all zero at the start of a seque
     m' = max(f + m, i);  S' = exp(f + m - m') S + exp(i - m') k v^T;  n' likewise with k alone;
     o = S'^T q / (max(|n' . q|, exp(-m')) + 1e-6)
 
-Each head's o is divided by its root mean square, the heads are concatenated and multiplied by
+A head's o goes through an RMS norm of its own without weight, the heads are concatenated and multiplied by
 a weight ``norm`` and by ``sigmoid(Wg h)``, then projected by ``Wo``.  Gates, state and the cell
 are float32 in both compute modes; the state lives in the request's slot and is carried from
 step to step, so a prompt may be cut anywhere.

@@ -1,9 +1,9 @@
-"""Retention: linear attention with a fixed decay per head (Sun et al., "Retentive Network: A Successor to Transformer for
+"""Retention, a linear attention whose state decays by a constant (Sun et al., "Retentive Network: A Successor to Transformer for
 Large Language Models").
 
 With input h, ``heads`` heads with keys of ``key_dim`` and values of ``value_dim``:
 
-* ``q = W_q h``, ``k = W_k h``, ``v = W_v h`` (no biases); q and k rotated by the token's position (``position``, a rotation over
+* ``q, k, v = W_q h, W_k h, W_v h``; q and k rotated by the token's position (``position``, a rotation over
   any leading part of a head; None: none), then ``k <- k * key_dim^-1/2``;
 * per head, state S [key_dim, value_dim]: ``S <- decay S + k v^T``, ``o = S^T q``, with ``decays[head]`` a constant;
 * ``y = W_o (silu(W_g h) * concat_n(o_n / rms(o_n)))``, the root mean square per head, no weight.

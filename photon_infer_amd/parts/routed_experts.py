@@ -1,13 +1,12 @@
 """Routed experts (mixture of experts) feed-forward.
 
-Router logits ``z = Wr h`` in float32; scores ``s = softmax(z)`` over all experts.  Experts form
-``groups`` equal groups of neighbours; a group's score is its largest expert score and only
-experts of the ``keep`` best groups can be chosen.  Each token uses the ``top`` allowed experts
-with the largest scores, weighted by those scores as they are (``renormalize``: divided by
-their sum plus ``renorm_eps``).  An expert is a gated feed-forward ``Wdown (silu(Wgate h) * (Wup h))`` without
+Router logits ``z = Wr h`` in float32; an expert's score is its share of ``softmax(z)``.  With ``groups`` > 1 the
+experts are cut into so many runs of equal length, the runs are ranked by their best expert, and the
+first ``keep`` of them stay in the choice.  The ``top`` best experts that are left take the token, each
+weighed by its score as it is (``renormalize``: divided by the sum of theirs plus ``renorm_eps``).  An expert is a gated feed-forward ``Wdown (silu(Wgate h) * (Wup h))`` without
 biases (``activation`` "silu"), or ``Wdown max(Wup h, 0)^2`` (``activation`` "relu2": no gate matrix), or the clamped
-gated unit of ``ClampedGLU`` without biases (``activation`` "clamped_glu", with ``limit`` and ``alpha``); the result is
-the weighted sum of the chosen experts' outputs (float32).
+gated unit of ``ClampedGLU`` without biases (``activation`` "clamped_glu", with ``limit`` and ``alpha``); their
+outputs, weighed, are summed in float32.
 
 Further options, each a constructor parameter: ``correction`` (a tensor of one number per router output that is
 added to the scores for the choice only; the weights stay the scores), ``identity`` (so many identity experts, which take

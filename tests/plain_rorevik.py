@@ -81,7 +81,7 @@ def rotate_interleaved(x: torch.Tensor, pos: int, dims: int, base: float) -> tor
 
 
 def attend(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, scale: float, cap: Optional[float]) -> torch.Tensor:
-    """q [T, H, d], k [T, G, d], v [T, G, dv] of one sequence -> [T, H, dv]: position i sees every j <= i;
+    """q [T, H, d], k [T, G, d], v [T, G, dv] of one sequence -> [T, H, dv]: causal;
     the scaled score s becomes cap * tanh(s / cap); ordinary softmax."""
     T, H, G = q.shape[0], q.shape[1], k.shape[1]
     out = torch.zeros((T, H, v.shape[2]), dtype=F64)

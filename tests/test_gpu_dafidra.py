@@ -479,7 +479,7 @@ def test_portions_of_changing_size(name, dtype, sizes, model_dirs, tmp_path):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", list(TD.ALL))
 def test_mixed_batches_with_pages_and_slots_used_again(name, dtype, model_dirs, tmp_path):
-    """Seven unequal requests through four slots: portions of some beside single tokens of others; a request may sit
+    """Seven unequal requests through four slots: some bring portions while others decode; a request may sit
     out a step; a finished request's pages and slot go to the next one.  Each must come out as it does alone."""
     vocab = TD.ALL[name][0]["vocab"]
     lengths = [70, 33, 5, 120, 64, 18, 91]

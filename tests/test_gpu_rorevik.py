@@ -384,7 +384,7 @@ def test_whole_prompts_and_every_layer_runs_stream(name, dtype, model_dirs, tmp_
         steps += cut_steps(rid, toks, [len(toks)], first_step=len(steps))
     runner = runner_for(model_dirs[name], name, dtype, live_token_need(steps))
     check(run_trace(runner, steps, str(tmp_path)), model_dirs[name], reqs, dtype, "whole")
-    if dtype == "float32":         # the stream after every layer run (a looped layer counts each time), for the longest request
+    if dtype == "float32":         # the stream behind every entry of the run order, for the longest request
         from photon_infer_amd import ops
         from photon_infer_amd.engine.step import StepEntry
         toks = reqs["r2"]
@@ -431,7 +431,7 @@ def test_portions_of_changing_size(name, dtype, sizes, model_dirs, tmp_path):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", list(TR.ALL))
 def test_mixed_batches_with_pages_and_slots_used_again(name, dtype, model_dirs, tmp_path):
-    """Seven unequal requests through four slots: portions of some beside single tokens of others; a request may sit
+    """Seven unequal requests through four slots: some bring portions while others decode; a request may sit
     out a step; a finished request's pages and slot go to the next one.  Each must come out as it does alone."""
     vocab = TR.ALL[name][0]["vocab"]
     lengths = [70, 33, 5, 120, 64, 18, 91]
